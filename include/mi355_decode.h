@@ -297,16 +297,19 @@ int32_t mi355_paged_attn_prefill(void* out, int64_t out_stride, const void* q,
  * query at position p sees the keys j with (p / chunk) * chunk <= j <= p (chunk 0: all j <= p);
  * sink (fp32 [num_heads], may be null): one more term exp(sink[h]) in the softmax denominator,
  * without a value; gate (dtype, rows gate_stride apart, may be null): the output of (token, head) is
- * multiplied by sigmoid(gate[token, head]).  Pages as above with v_dim == head_dim.
+ * multiplied by sigmoid(gate[token, head]).  window > 0: the keys j > p - window only, and (chunk 0)
+ * the first `keep` keys of the sequence.  The output is multiplied by out_scale.  K pages
+ * [blocks, kv_heads, 16, head_dim], V pages [blocks, kv_heads, v_dim, 16], head_dim and v_dim each 64 or 128.
  */
 int32_t mi355_paged_attn_prefill_ext(void* out, int64_t out_stride, const void* q, int64_t q_stride,
                                      const void* k_cache, const void* v_cache, int32_t num_blocks,
                                      const int32_t* block_tables, int32_t max_blocks_per_seq,
                                      const int32_t* cu_seqlens, const int32_t* context_lens,
                                      int32_t num_seqs, int32_t max_q_len, int32_t num_heads,
-                                     int32_t num_kv_heads, int32_t head_dim, float scale,
-                                     int32_t chunk, const float* sink, const void* gate,
-                                     int64_t gate_stride, int32_t dtype, void* stream);
+                                     int32_t num_kv_heads, int32_t head_dim, int32_t v_dim, float scale,
+                                     int32_t chunk, int32_t window, int32_t keep, const float* sink,
+                                     const void* gate, int64_t gate_stride, float out_scale,
+                                     int32_t dtype, void* stream);
 
 /*
  * SwiGLU gate:  out[t, :] = round(round(silu(x[t, :F])) * x[t, F:2F]).
@@ -754,7 +757,7 @@ int32_t mi355_allreduce_oneshot_destroy(void* comm);
  * Decoders with an fp32 residual stream (no counterpart in the reference: the engine it launches
  * keeps the residual in the model's 16-bit type).  `dtype` is the storage type of activations and
  * weights: MI355_BF16, MI355_F16 or MI355_F32; sums, means and transcendentals are fp32 always.
- *   embed_scale_f32       resid[t] = embed[ids[t]] * scale
+ *   embed_scale_f32       resid[t] = embed[ids[t]] * scale; act_out (dtype, may be null): the same rows once more
  *   embed_scale_pos_f32   resid[t] = embed[ids[t]] * scale + pos_table[positions[t]] (learned positions,
  *                         [max_pos, width] in `dtype`)
  *   resid_add_f32         resid[t] += other[t] (fp32) + rows[t] (dtype) + vec (one row, dtype); each may be null
@@ -764,11 +767,13 @@ int32_t mi355_allreduce_oneshot_destroy(void* comm);
  *   gelu_tanh_and_mul     out[t] = gelu_tanh(x[t, :inter]) * x[t, inter:2 inter]
  *   gated_head_rms_norm   out[t, h] = o[t, h] / rms(o[t, h]) * weight * act(gate[t, h]); o fp32
  *                         [tokens, heads, head_dim]; activation 0: silu, 1: sigmoid; weight [head_dim]
- *                         shared by the heads (weight_heads 1) or [heads, head_dim] (weight_heads == heads)
+ *                         shared by the heads (weight_heads 1) or [heads, head_dim] (weight_heads == heads);
+ *                         output rows out_stride apart
  *   softcap               z = cap * tanh(z / cap), in place
  */
-int32_t mi355_embed_scale_f32(float* out, const void* embed, const int64_t* ids, int64_t num_tokens,
-                              int32_t width, int64_t vocab, float scale, int32_t dtype, void* stream);
+int32_t mi355_embed_scale_f32(float* out, void* act_out, const void* embed, const int64_t* ids,
+                              int64_t num_tokens, int32_t width, int64_t vocab, float scale,
+                              int32_t dtype, void* stream);
 int32_t mi355_embed_scale_pos_f32(float* out, const void* embed, const void* pos_table, const int64_t* ids,
                                   const int64_t* positions, int64_t num_tokens, int32_t width,
                                   int64_t vocab, int64_t max_pos, float scale, int32_t dtype, void* stream);
@@ -782,7 +787,7 @@ int32_t mi355_rms_norm_mix_f32(float* resid, const void* xa, const void* wa, con
                                float alpha, int32_t dtype, void* stream);
 int32_t mi355_gelu_tanh_and_mul(void* out, const void* x, int64_t x_stride, int64_t num_tokens,
                                 int32_t inter, int32_t dtype, void* stream);
-int32_t mi355_gated_head_rms_norm(void* out, const float* o, const void* gate, int64_t gate_stride,
+int32_t mi355_gated_head_rms_norm(void* out, int64_t out_stride, const float* o, const void* gate, int64_t gate_stride,
                                   const float* weight, int32_t weight_heads, int64_t num_tokens,
                                   int32_t num_heads, int32_t head_dim, float eps, int32_t activation,
                                   int32_t dtype, void* stream);
@@ -1028,9 +1033,13 @@ int32_t mi355_moe_combine(void* out, const void* y, const int32_t* inv, const fl
  *   relu_squared          out = max(x, 0)^2
  *   qk_norm_kv_write      q <- rms(q) * q_weight per head, in place; K pages <- rms(k) * k_weight per
  *                         head; V pages <- v (rows of the caller's choice).  Weights fp32 [head_dim]
+ *   row_norm_rope_kv_write  q <- rotate(rms(q row) * q_weight) in place, the RMS norm over all heads of the row at
+ *                         once (weights fp32 [heads * head_dim]); K pages <- the same of the k row; V pages <- v;
+ *                         rotation of the first rot_dims coordinates of every head, pairs (i, i + rot_dims / 2), by
+ *                         cos_sin fp32 [max_pos, rot_dims] = cos | sin
  *   softmax_bias_attn     out[t,h] = sigmoid(gate) * sum_j softmax_j(q.k_j * scale - r1[h] ln(1 + r2[h]
  *                         (p - j))) v_j over the keys j <= p with j >= (p / block) * block (block 0: all)
- *                         and, window > 0, j > p - window.  gate: one number per head or
+ *                         and, window > 0, j > p - window or (block 0) j < keep; times out_scale.  gate: one number per head or
  *                         (gate_per_channel) per output channel; r1 / r2 null: no penalty.  sink (fp32
  *                         [heads], may be null): one more term exp(sink[h]) in the softmax denominator,
  *                         without a value.  Output rows are out_stride elements apart.  tiles as for
@@ -1058,6 +1067,14 @@ int32_t mi355_qk_norm_kv_write(void* q, int64_t q_stride, const void* k, int64_t
                                const int64_t* slot_mapping, void* k_cache, void* v_cache,
                                int64_t num_tokens, int32_t num_heads, int32_t num_kv_heads,
                                int32_t head_dim, int32_t v_dim, float eps, int32_t dtype, void* stream);
+int32_t mi355_row_norm_rope_kv_write(void* q, int64_t q_stride, const void* k, int64_t k_stride,
+                                     const void* v, int64_t v_stride, const float* q_weight,
+                                     const float* k_weight, const float* cos_sin, int64_t max_pos,
+                                     const int64_t* positions, const int64_t* slot_mapping,
+                                     void* k_cache, void* v_cache, int64_t num_tokens,
+                                     int32_t num_heads, int32_t num_kv_heads, int32_t head_dim,
+                                     int32_t v_dim, int32_t rot_dims, float eps, int32_t dtype,
+                                     void* stream);
 int64_t mi355_softmax_bias_attn_workspace(int64_t num_tokens, int32_t num_heads, int32_t v_dim,
                                           int32_t num_splits);
 int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_stride, const void* k_cache,
@@ -1066,9 +1083,10 @@ int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_stride, cons
                                 const float* r2, const void* gate, int64_t gate_stride,
                                 int32_t gate_per_channel, int64_t num_tokens, int32_t num_heads,
                                 int32_t num_kv_heads, int32_t head_dim, int32_t v_dim, int32_t block,
-                                int32_t window, float scale, const int32_t* tiles, int32_t num_tiles,
-                                float* workspace, int32_t num_splits, const float* sink,
-                                int64_t out_stride, int32_t dtype, void* stream);
+                                int32_t window, int32_t keep, float scale, const int32_t* tiles,
+                                int32_t num_tiles, float* workspace, int32_t num_splits,
+                                const float* sink, int64_t out_stride, float out_scale, int32_t dtype,
+                                void* stream);
 int32_t mi355_mingru_scan(void* out, const void* proj, int64_t stride, int32_t z_off, int32_t x_off,
                           int32_t g_off, const float* z_bias, const float* x_bias, float* state,
                           const int32_t* cu_seqlens, const int64_t* positions,
@@ -1076,6 +1094,74 @@ int32_t mi355_mingru_scan(void* out, const void* proj, int64_t stride, int32_t z
                           int32_t channels, int32_t long_chunks, float* workspace, int32_t num_parts,
                           int32_t dtype, void* stream);
 int64_t mi355_mingru_scan_workspace(int32_t num_seqs, int32_t channels, int32_t num_parts);
+
+/*
+ * Decoders whose sub-layers read the fp32 residual itself and whose norms sit on their outputs, with a
+ * token's own row of numbers for every layer; linear attention with a scalar decay per head and token.
+ *   norm_resid_f32        resid += y' / sqrt(mean(y'^2) + eps) * weight, y' = y * y_scale (y in `dtype`, weight
+ *                         fp32); act_out (dtype, may be null): the new residual rows
+ *   token_gate_rows       out[t, c] = gelu_tanh(z[t, c]) * table[ids[t], offset + c], c < n
+ *   token_side_f32        g = gelu_tanh(gate_w resid) * table[ids[t], offset ..]; y = proj_w g;
+ *                         resid += y / sqrt(mean(y^2) + eps) * norm; act_out as above.  gate_w [n, width],
+ *                         proj_w [width, n] in `dtype`; one workgroup per row (few rows), width <= 8192
+ *   decay_attn_step       S <- exp(log_decay[h]) S + k v^T, o = S^T q per token and head with q, k, v the silu of the
+ *                         given rows; o fp32 [tokens, heads, v_dim]; every chunk's tokens in order, the state
+ *                         (fp32 [slots, heads, linear_attn_state_floats]) updated in place, zeros for a chunk that
+ *                         starts at position 0
+ *   mlstm_step            a = cap tanh((gate_w[h] x + b[h]) / cap), f = log sigmoid(cap tanh((gate_w[H + h] x +
+ *                         b[H + h]) / cap)); m' = max(f + m, a); S <- e^(f + m - m') S + e^(a - m') k v^T, n likewise
+ *                         with k alone; o = S^T q / (max(|n . q|, e^-m') + 1e-6), q times q_scale; out = o / rms(o) *
+ *                         norm[h] * sigmoid(g) in `dtype`.  State: S, then n; m_state [slots, heads]
+ *   mlstm_gates           for chunks of many tokens, from z [tokens, 2 heads] (the gate products without biases), by
+ *                         tiles of up to tile_rows rows of a chunk: log_in = a, log_decay_sum = f summed from the
+ *                         tile's first row, running_max = m, all [heads, tokens]; tile_max = m ahead of every tile
+ *                         [tiles, heads]; m_state is updated
+ *   linear_attn_chunks    both recurrences over chunks of any length by such tiles (tiles: chunk, first row, rows;
+ *                         tile_start [chunks + 1]): log_decay for the constant decay (silu on q, k, v), null and the
+ *                         four arrays of mlstm_gates otherwise.  o fp32 [tokens, heads, v_dim] (not normed or gated).
+ *                         workspace: tiles * heads * linear_attn_state_floats floats
+ *   linear_attn_tile_rows  rows of a tile that fit (64, 32 or 16); 0: heads too large
+ */
+int32_t mi355_norm_resid_f32(float* resid, void* act_out, const void* y, const float* weight,
+                             int64_t num_tokens, int32_t width, float eps, float y_scale, int32_t dtype,
+                             void* stream);
+int32_t mi355_token_gate_rows(void* out, const void* z, int64_t z_stride, const void* table,
+                              int64_t table_stride, int64_t offset, const int64_t* ids, int64_t vocab,
+                              int64_t num_tokens, int32_t n, int32_t dtype, void* stream);
+int32_t mi355_token_side_f32(float* resid, void* act_out, const void* gate_w, const void* proj_w,
+                             const float* norm, const void* table, int64_t table_stride, int64_t offset,
+                             const int64_t* ids, int64_t vocab, int64_t num_tokens, int32_t width,
+                             int32_t n, float eps, int32_t dtype, void* stream);
+int64_t mi355_linear_attn_state_floats(int32_t head_dim, int32_t v_dim, int32_t normalizer);
+int32_t mi355_linear_attn_tile_rows(int32_t head_dim, int32_t v_dim);
+int32_t mi355_mlstm_gates(float* log_in, double* log_decay_sum, float* running_max, float* tile_max,
+                          const float* z, const float* bias, float cap, float* m_state,
+                          const int32_t* cu_seqlens, const int64_t* positions,
+                          const int32_t* state_slots, const int32_t* tile_start, int32_t num_seqs,
+                          int32_t num_heads, int32_t tile_rows, int64_t num_tokens, void* stream);
+int32_t mi355_linear_attn_chunks(float* o, const void* q, int64_t q_stride, const void* k,
+                                 int64_t k_stride, const void* v, int64_t v_stride, float q_scale,
+                                 const double* log_decay, const float* log_in,
+                                 const double* log_decay_sum, const float* running_max,
+                                 const float* tile_max, float* state, const int32_t* cu_seqlens,
+                                 const int64_t* positions, const int32_t* state_slots,
+                                 const int32_t* tiles, const int32_t* tile_start, int32_t num_tiles,
+                                 int32_t tile_rows, int32_t num_seqs, int32_t num_heads,
+                                 int32_t head_dim, int32_t v_dim, int64_t num_tokens, float* workspace,
+                                 int64_t workspace_floats, int32_t dtype, void* stream);
+int32_t mi355_decay_attn_step(float* o, const void* q, int64_t q_stride, const void* k,
+                              int64_t k_stride, const void* v, int64_t v_stride,
+                              const double* log_decay, float* state, const int32_t* cu_seqlens,
+                              const int64_t* positions, const int32_t* state_slots, int32_t num_seqs,
+                              int32_t num_heads, int32_t head_dim, int32_t v_dim, int32_t dtype,
+                              void* stream);
+int32_t mi355_mlstm_step(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* k,
+                         int64_t k_stride, const void* v, int64_t v_stride, float q_scale,
+                         const float* x, int64_t x_stride, const void* gate_w, const float* gate_b,
+                         int32_t width, float cap, const void* g, int64_t g_stride, const float* norm,
+                         float eps, float* state, float* m_state, const int32_t* cu_seqlens,
+                         const int64_t* positions, const int32_t* state_slots, int32_t num_seqs,
+                         int32_t num_heads, int32_t head_dim, int32_t v_dim, int32_t dtype, void* stream);
 
 #ifdef __cplusplus
 }

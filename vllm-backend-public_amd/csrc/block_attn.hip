@@ -5,10 +5,13 @@
 //   qk_norm_kv_write      q <- rms(q) * wq per head, in place; K pages <- rms(k) * wk per head; V pages <- v
 //                         (any rows of the caller's choice: a design whose values are its unnormed keys
 //                         passes k again)
+//   row_norm_rope_kv_write   q <- rotate(rms(q row) * wq), in place, the norm over all heads of the row at once; K pages <-
+//                         the same of the k row; V pages <- v.  Rotation of the first rot coordinates of every head by a
+//                         fp32 table (pairs i, i + rot / 2)
 //   softmax_bias_attn     out[t,h] = gate[t,h,:] * sum_j softmax_j(q.k_j * scale - r1[h] ln(1 + r2[h] (p - j))) v_j
 //                         over the keys j <= p of p's block: lo = (p / block) * block (block 0: lo = 0), and
-//                         with a window also j > p - window.  Blocks are counted from position 0 of the
-//                         sequence.  gate: sigmoid of one number per head or per output channel.
+//                         with a window also j > p - window or (keep first) j < keep.  Blocks are counted from
+//                         position 0 of the sequence.  The output is multiplied by out_scale.  gate: sigmoid of one number per head or per output channel.
 //                         sink (fp32, one score per head, may be null): the softmax denominator holds one
 //                         more term exp(sink[h]) that carries no value.  Output rows are out_stride apart
 //                         (a column slice of a wider buffer is fine).
@@ -62,6 +65,72 @@ __global__ __launch_bounds__(256) void qk_norm_kv_write_kernel(
   }
 }
 
+// One workgroup per packed row: the mean squares of the whole q row and the whole k row, then pair by pair
+// norm, weight and rotation.
+template <typename T>
+__global__ __launch_bounds__(256) void row_norm_rope_kv_write_kernel(
+    typename Elem<T>::S* __restrict__ q, int64_t q_stride, const typename Elem<T>::S* __restrict__ k, int64_t k_stride,
+    const typename Elem<T>::S* __restrict__ v, int64_t v_stride, const float* __restrict__ wq, const float* __restrict__ wk,
+    const float* __restrict__ cos_sin, int64_t max_pos, const int64_t* __restrict__ positions,
+    const int64_t* __restrict__ slot_mapping, typename Elem<T>::S* __restrict__ k_cache,
+    typename Elem<T>::S* __restrict__ v_cache, int H, int G, int d, int dv, int rot, float eps) {
+  typedef typename Elem<T>::S E;
+  __shared__ float scratch[32];
+  const int64_t t = blockIdx.x;
+  int64_t p = MI355_LD(int64_t, positions, positions + t);
+  p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
+  const int64_t slot = MI355_LD(int64_t, slot_mapping, slot_mapping + t);
+  const int64_t page = slot / kPageB, off = slot % kPageB;
+  const int half = rot >> 1, units = d - half;           // a head is `half` pairs and d - rot single coordinates
+  const float* cs = cos_sin + p * rot;                    // cos[0..half) | sin[0..half)
+  E* qr = q + t * q_stride;
+  const E* kr = k + t * k_stride;
+  float sq = 0.f, sk = 0.f;
+  for (int i = threadIdx.x; i < H * d; i += blockDim.x) {
+    const float x = MI355_LDF(T, q, qr + i);
+    sq += x * x;
+  }
+  for (int i = threadIdx.x; i < G * d; i += blockDim.x) {
+    const float x = MI355_LDF(T, k, kr + i);
+    sk += x * x;
+  }
+  const float rq = 1.0f / sqrtf(block_sum32(sq, scratch) / static_cast<float>(H * d) + eps);
+  const float rk = 1.0f / sqrtf(block_sum32(sk, scratch) / static_cast<float>(G * d) + eps);
+  for (int i = threadIdx.x; i < (slot < 0 ? H : H + G) * units; i += blockDim.x) {
+    const int hh = i / units, u = i - hh * units;
+    const bool is_q = hh < H;
+    const int head = is_q ? hh : hh - H;
+    const int a = u < half ? u : u + half;                // first coordinate of the pair, or the single one
+    const E* src = (is_q ? static_cast<const E*>(qr) : kr) + static_cast<int64_t>(head) * d + a;
+    const float* w = (is_q ? wq : wk) + static_cast<int64_t>(head) * d + a;
+    [[maybe_unused]] const void* base = is_q ? static_cast<const void*>(q) : static_cast<const void*>(k);
+    [[maybe_unused]] const void* wbase = is_q ? wq : wk;
+    const float r = is_q ? rq : rk;
+    float x = MI355_LDF(T, base, src) * r * MI355_LD(float, wbase, w), y = 0.f;
+    if (u < half) {
+      const float b = MI355_LDF(T, base, src + half) * r * MI355_LD(float, wbase, w + half);
+      const float c = MI355_LD(float, cos_sin, cs + u), s = MI355_LD(float, cos_sin, cs + half + u);
+      const float x0 = x;
+      x = x0 * c - b * s;
+      y = b * c + x0 * s;
+    }
+    if (is_q) {
+      E* o = qr + static_cast<int64_t>(head) * d + a;
+      MI355_STF(T, q, o, x);
+      if (u < half) MI355_STF(T, q, o + half, y);
+    } else {
+      E* o = k_cache + ((page * G + head) * kPageB + off) * d + a;
+      MI355_STF(T, k_cache, o, x);
+      if (u < half) MI355_STF(T, k_cache, o + half, y);
+    }
+  }
+  if (slot < 0) return;
+  for (int i = threadIdx.x; i < G * dv; i += blockDim.x) {
+    const int g = i / dv, j = i % dv;
+    MI355_ST(E, v_cache, v_cache + ((page * G + g) * dv + j) * kPageB + off, MI355_LD(E, v, v + t * v_stride + i));
+  }
+}
+
 __device__ __forceinline__ int64_t first_visible(int64_t p, int block, int window) {
   int64_t lo = block > 0 ? (p / block) * block : 0;
   if (window > 0 && p - window + 1 > lo) lo = p - window + 1;
@@ -78,7 +147,7 @@ __global__ __launch_bounds__(64) void softmax_bias_attn_kernel(
     const int32_t* __restrict__ block_tables, int max_blocks, const int32_t* __restrict__ tok_seq,
     const int64_t* __restrict__ positions, const float* __restrict__ r1, const float* __restrict__ r2,
     const typename Elem<T>::S* __restrict__ gate, int64_t gate_stride, int gate_per_channel, int H, int G, int d, int dv,
-    int block, int window, float scale, const float* __restrict__ sink, int64_t out_stride) {
+    int block, int window, int keep, float scale, const float* __restrict__ sink, int64_t out_stride, float out_scale) {
   extern __shared__ float lds[];                        // q [d] | w [64]
   float* qs = lds;
   float* ws = lds + d;
@@ -96,11 +165,16 @@ __global__ __launch_bounds__(64) void softmax_bias_attn_kernel(
   for (int i = 0; i < DV_PER_LANE; ++i) acc[i] = 0.f;
   float m = -__builtin_inff(), l = 0.f;
   const int64_t lo = first_visible(p, block, window);
+  // the kept first keys that lie before the window, 64 at a time, then the window's keys
+  const int64_t kept = keep < lo ? keep : lo, kept_up = (kept + 63) / 64 * 64;
   __syncthreads();
-  for (int64_t base = lo; base <= p; base += 64) {
+  for (int64_t at = 0; at <= kept_up + p - lo; at += 64) {
+    const bool first = at < kept_up;
+    const int64_t base = first ? at : lo + at - kept_up;
+    const int64_t end = first ? kept - 1 : p;             // last key of this run
     const int64_t j = base + lane;
     float s = -__builtin_inff();
-    if (j <= p) {
+    if (j <= end) {
       const int64_t page = MI355_LD(int32_t, block_tables, bt + j / kPageB);
       const typename Elem<T>::S* kr = k_cache + ((page * G + g) * kPageB + j % kPageB) * d;
       float dot = 0.f;
@@ -112,12 +186,12 @@ __global__ __launch_bounds__(64) void softmax_bias_attn_kernel(
     for (int o = 32; o > 0; o >>= 1) tm = fmaxf(tm, __shfl_xor(tm, o, 64));
     const float mn = fmaxf(m, tm);                      // (finite: the tile's first key is visible)
     const float corr = expf(m - mn);
-    const float w = j <= p ? expf(s - mn) : 0.f;
+    const float w = j <= end ? expf(s - mn) : 0.f;
     l = l * corr + wave_sum(w);
     m = mn;
     ws[lane] = w;
     __syncthreads();
-    const int n = static_cast<int>((p - base + 1) < 64 ? (p - base + 1) : 64);
+    const int n = static_cast<int>((end - base + 1) < 64 ? (end - base + 1) : 64);
 #pragma unroll
     for (int i = 0; i < DV_PER_LANE; ++i) acc[i] *= corr;
     for (int jj = 0; jj < n; ++jj) {
@@ -141,7 +215,7 @@ __global__ __launch_bounds__(64) void softmax_bias_attn_kernel(
 #pragma unroll
     for (int i = 0; i < DV_PER_LANE; ++i) acc[i] *= corr;
   }
-  const float inv = 1.0f / l;
+  const float inv = out_scale / l;
 #pragma unroll
   for (int i = 0; i < DV_PER_LANE; ++i) {
     const int c = lane + 64 * i;
@@ -171,8 +245,8 @@ __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
     const uint16_t* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tiles, int num_tiles, const int64_t* __restrict__ positions, const float* __restrict__ r1,
     const float* __restrict__ r2, const uint16_t* __restrict__ gate, int64_t gate_stride, int gate_per_channel, int H, int G,
-    int d, int dv, int block, int window, float scale, float* __restrict__ part_acc, float* __restrict__ part_ml,
-    int64_t total_rows, const float* __restrict__ sink, int64_t out_stride) {
+    int d, int dv, int block, int window, int keep, float scale, float* __restrict__ part_acc, float* __restrict__ part_ml,
+    int64_t total_rows, const float* __restrict__ sink, int64_t out_stride, float out_scale) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   // Workgroups go to the 8 XCDs in turn (x fastest), each XCD with an L2 of its own.  Where the plane of
   // workgroups divides by 8, XCD k takes the k-th eighth of the (head group, tile) pairs in head-major order:
@@ -223,19 +297,27 @@ __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
   }
   // the pages of a tile are looked up one tile ahead: the table's trip to memory then runs beside the
   // current tile's K/V loads instead of in front of the next tile's
-  const int64_t first = ((lo0 >> 5) << 5) + 32 * z;
+  // 32-key tiles in walking order: those that hold kept first keys and lie before the window's first tile, then
+  // the window's; tile number i starts at key 32 i, or (past the kept ones) 32 (i + skip)
+  const int64_t wt0 = lo0 >> 5, kt = (keep + 31) >> 5, nk = kt < wt0 ? kt : wt0;
+  const int64_t skip = wt0 - nk;
+  const int64_t walk_end = (p_last >> 5) - skip;           // last tile number
+  auto tile_base = [&](int64_t i) { return (i < nk ? i : i + skip) << 5; };
   int32_t pg[2] = {0, 0};
 #pragma unroll
-  for (int half = 0; half < 2; ++half)
-    if (first + 16 * half <= p_last) pg[half] = MI355_LD(int32_t, block_tables, bt + (first + 16 * half) / kPageB);
-  for (int64_t base = first; base <= p_last; base += 32 * nz) {
+  for (int half = 0; half < 2; ++half) {
+    const int64_t kb = tile_base(z) + 16 * half;
+    if (z <= walk_end && kb <= p_last) pg[half] = MI355_LD(int32_t, block_tables, bt + kb / kPageB);
+  }
+  for (int64_t it = z; it <= walk_end; it += nz) {
+    const int64_t base = tile_base(it);
     uint4 kf[2][DS];
     uint2 vf[2][CB];
     int32_t npg[2] = {0, 0};
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
-      const int64_t nb = base + 32 * nz + 16 * half;
-      if (nb <= p_last) npg[half] = MI355_LD(int32_t, block_tables, bt + nb / kPageB);
+      const int64_t nb = tile_base(it + nz) + 16 * half;
+      if (it + nz <= walk_end && nb <= p_last) npg[half] = MI355_LD(int32_t, block_tables, bt + nb / kPageB);
     }
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
@@ -272,7 +354,7 @@ __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int64_t key = base + 16 * half + 4 * kk + r;
-        vis[half][r] = valid && key <= my_p && key >= my_lo;
+        vis[half][r] = valid && key <= my_p && (key >= my_lo || key < keep);
         dist[half][r] = PEN && vis[half][r] ? static_cast<float>(my_p - key) : 0.f;
       }
     }
@@ -375,14 +457,14 @@ __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
       }
       continue;
     }
-    float f = 1.0f / lt;
+    float f = out_scale / lt;
     if (sink != nullptr) {
       // the extra term of the denominator, base 2 like the maxima: numerator and denominator are both
       // relative to m[i], so the accumulators only need the ratio
       const float sk = MI355_LD(float, sink, sink + h) * kLog2eB;
       const float mn = fmaxf(m[i], sk);
       const float cm = __builtin_amdgcn_exp2f(m[i] - mn);
-      f = cm / (lt * cm + __builtin_amdgcn_exp2f(sk - mn));
+      f = out_scale * cm / (lt * cm + __builtin_amdgcn_exp2f(sk - mn));
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -410,7 +492,7 @@ __global__ __launch_bounds__(256) void bias_attn_merge_kernel(uint16_t* __restri
                                                               const float* __restrict__ part_ml,
                                                               const uint16_t* __restrict__ gate, int64_t gate_stride,
                                                               int gate_per_channel, int64_t rows, int H, int dv, int splits,
-                                                              const float* __restrict__ sink, int64_t out_stride) {
+                                                              const float* __restrict__ sink, int64_t out_stride, float out_scale) {
   const int64_t pairs = rows * H, total = pairs * dv;
   for (int64_t i = blockIdx.x * static_cast<int64_t>(blockDim.x) + threadIdx.x; i < total;
        i += static_cast<int64_t>(gridDim.x) * blockDim.x) {
@@ -434,7 +516,7 @@ __global__ __launch_bounds__(256) void bias_attn_merge_kernel(uint16_t* __restri
       num *= cm;
       den = den * cm + __builtin_amdgcn_exp2f(sk - mn);
     }
-    float v = num / den;
+    float v = num / den * out_scale;
     if (gate != nullptr)
       v /= 1.0f + expf(-T::to_f(MI355_LD(uint16_t, gate, gate + row * gate_stride + (gate_per_channel ? h * dv + c : h))));
     MI355_ST(uint16_t, out, out + row * out_stride + static_cast<int64_t>(h) * dv + c, T::from_f(v));
@@ -473,12 +555,41 @@ extern "C" int32_t mi355_qk_norm_kv_write(void* q, int64_t q_stride, const void*
   return check_launch("qk_norm_kv_write");
 }
 
+extern "C" int32_t mi355_row_norm_rope_kv_write(void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
+                                                int64_t v_stride, const float* q_weight, const float* k_weight,
+                                                const float* cos_sin, int64_t max_pos, const int64_t* positions,
+                                                const int64_t* slot_mapping, void* k_cache, void* v_cache,
+                                                int64_t num_tokens, int32_t num_heads, int32_t num_kv_heads,
+                                                int32_t head_dim, int32_t v_dim, int32_t rot_dims, float eps, int32_t dtype,
+                                                void* stream) {
+  MI355_REQUIRE(q && k && v && q_weight && k_weight && positions && slot_mapping && k_cache && v_cache, MI355_ERR_INVALID,
+                "row_norm_rope_kv_write: null pointer");
+  MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && num_kv_heads > 0 && head_dim > 0 && v_dim > 0 && rot_dims >= 0 &&
+                    rot_dims <= head_dim && rot_dims % 2 == 0 && (rot_dims == 0 || (cos_sin && max_pos > 0)),
+                MI355_ERR_INVALID, "row_norm_rope_kv_write: sizes");
+  MI355_REQUIRE(q_stride >= static_cast<int64_t>(num_heads) * head_dim &&
+                    k_stride >= static_cast<int64_t>(num_kv_heads) * head_dim &&
+                    v_stride >= static_cast<int64_t>(num_kv_heads) * v_dim,
+                MI355_ERR_INVALID, "row_norm_rope_kv_write: row strides shorter than the rows");
+  REQ_DTYPE(dtype);
+  if (num_tokens == 0) return MI355_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((row_norm_rope_kv_write_kernel<TT>), dim3(num_tokens), dim3(256), 0, s,
+                                                  static_cast<Elem<TT>::S*>(q), q_stride,
+                                                  static_cast<const Elem<TT>::S*>(k), k_stride,
+                                                  static_cast<const Elem<TT>::S*>(v), v_stride, q_weight, k_weight, cos_sin,
+                                                  max_pos, positions, slot_mapping, static_cast<Elem<TT>::S*>(k_cache),
+                                                  static_cast<Elem<TT>::S*>(v_cache), num_heads, num_kv_heads, head_dim,
+                                                  v_dim, rot_dims, eps));
+  return check_launch("row_norm_rope_kv_write");
+}
+
 template <typename TT>
 static void launch_bias_attn(hipStream_t s, void* out, const void* q, int64_t q_stride, const void* k_cache,
                              const void* v_cache, const int32_t* block_tables, int32_t max_blocks, const int32_t* tok_seq,
                              const int64_t* positions, const float* r1, const float* r2, const void* gate,
                              int64_t gate_stride, int gate_per_channel, int64_t T, int H, int G, int d, int dv, int block,
-                             int window, float scale, const float* sink, int64_t out_stride) {
+                             int window, int keep, float scale, const float* sink, int64_t out_stride, float out_scale) {
   typedef typename Elem<TT>::S E;
   const dim3 grid(static_cast<unsigned>(T), static_cast<unsigned>(H));
   const size_t lds = (static_cast<size_t>(d) + 64) * sizeof(float);
@@ -486,11 +597,12 @@ static void launch_bias_attn(hipStream_t s, void* out, const void* q, int64_t q_
   hipLaunchKernelGGL((softmax_bias_attn_kernel<TT, N>), grid, dim3(64), lds, s, static_cast<E*>(out),              \
                      static_cast<const E*>(q), q_stride, static_cast<const E*>(k_cache),                           \
                      static_cast<const E*>(v_cache), block_tables, max_blocks, tok_seq, positions, r1, r2,         \
-                     static_cast<const E*>(gate), gate_stride, gate_per_channel, H, G, d, dv, block, window, scale, \
-                     sink, out_stride)
+                     static_cast<const E*>(gate), gate_stride, gate_per_channel, H, G, d, dv, block, window, keep, \
+                     scale, sink, out_stride, out_scale)
   if (dv <= 64) MI355_BATTN(1);
   else if (dv <= 128) MI355_BATTN(2);
-  else MI355_BATTN(4);
+  else if (dv <= 256) MI355_BATTN(4);
+  else MI355_BATTN(8);
 #undef MI355_BATTN
 }
 
@@ -504,17 +616,17 @@ extern "C" int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_s
                                            const float* r2, const void* gate, int64_t gate_stride,
                                            int32_t gate_per_channel, int64_t num_tokens, int32_t num_heads,
                                            int32_t num_kv_heads, int32_t head_dim, int32_t v_dim, int32_t block,
-                                           int32_t window, float scale, const int32_t* tiles, int32_t num_tiles,
-                                           float* workspace, int32_t num_splits, const float* sink, int64_t out_stride,
-                                           int32_t dtype, void* stream) {
+                                           int32_t window, int32_t keep, float scale, const int32_t* tiles,
+                                           int32_t num_tiles, float* workspace, int32_t num_splits, const float* sink,
+                                           int64_t out_stride, float out_scale, int32_t dtype, void* stream) {
   MI355_REQUIRE(out && q && k_cache && v_cache && block_tables && tok_seq && positions, MI355_ERR_INVALID,
                 "softmax_bias_attn: null pointer");
   MI355_REQUIRE((r1 == nullptr) == (r2 == nullptr), MI355_ERR_INVALID, "softmax_bias_attn: r1 and r2 go together");
   MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && num_kv_heads > 0 && num_heads % num_kv_heads == 0 &&
-                    head_dim > 0 && v_dim > 0 && max_blocks > 0 && block >= 0 && window >= 0,
+                    head_dim > 0 && v_dim > 0 && max_blocks > 0 && block >= 0 && window >= 0 && keep >= 0 && (keep == 0 || block == 0),
                 MI355_ERR_INVALID, "softmax_bias_attn: sizes");
-  MI355_REQUIRE(v_dim <= 256 && head_dim <= 8192 && num_heads <= 65535, MI355_ERR_UNSUPPORTED,
-                "softmax_bias_attn: v_dim %d (at most 256), head_dim %d", v_dim, head_dim);
+  MI355_REQUIRE(v_dim <= 512 && head_dim <= 8192 && num_heads <= 65535, MI355_ERR_UNSUPPORTED,
+                "softmax_bias_attn: v_dim %d (at most 512), head_dim %d", v_dim, head_dim);
   MI355_REQUIRE(gate == nullptr || gate_stride >= (gate_per_channel ? static_cast<int64_t>(num_heads) * v_dim : num_heads),
                 MI355_ERR_INVALID, "softmax_bias_attn: gate rows shorter than the gate");
   MI355_REQUIRE(out_stride >= static_cast<int64_t>(num_heads) * v_dim, MI355_ERR_INVALID,
@@ -548,8 +660,8 @@ extern "C" int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_s
                      static_cast<uint16_t*>(out), static_cast<const uint16_t*>(q), q_stride,                        \
                      static_cast<const uint16_t*>(k_cache), static_cast<const uint16_t*>(v_cache), block_tables,    \
                      max_blocks, tiles, num_tiles, positions, r1, r2, static_cast<const uint16_t*>(gate),           \
-                     gate_stride, gate_per_channel, num_heads, num_kv_heads, head_dim, v_dim, block, window, scale, \
-                     part_acc, part_ml, num_tokens, sink, out_stride)
+                     gate_stride, gate_per_channel, num_heads, num_kv_heads, head_dim, v_dim, block, window, keep,  \
+                     scale, part_acc, part_ml, num_tokens, sink, out_stride, out_scale)
 #define MI355_BMFMA_HB(TT)                                                                                          \
   do {                                                                                                              \
     if (hb == 4) MI355_BMFMA(TT, 4);                                                                                \
@@ -562,7 +674,7 @@ extern "C" int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_s
                          dim3(static_cast<unsigned>((total + 255) / 256 > 4096 ? 4096 : (total + 255) / 256)),      \
                          dim3(256), 0, s, static_cast<uint16_t*>(out), part_acc, part_ml,                           \
                          static_cast<const uint16_t*>(gate), gate_stride, gate_per_channel, num_tokens, num_heads,  \
-                         v_dim, num_splits, sink, out_stride);                                                      \
+                         v_dim, num_splits, sink, out_stride, out_scale);                                                      \
     }                                                                                                               \
   } while (0)
     if (dtype == MI355_BF16) MI355_BMFMA_HB(BF16); else MI355_BMFMA_HB(F16);
@@ -574,6 +686,6 @@ extern "C" int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_s
   MI355_DISPATCH_DTYPE3(dtype, launch_bias_attn<TT>(s, out, q, q_stride, k_cache, v_cache, block_tables, max_blocks,
                                                    tok_seq, positions, r1, r2, gate, gate_stride, gate_per_channel,
                                                    num_tokens, num_heads, num_kv_heads, head_dim, v_dim, block, window,
-                                                   scale, sink, out_stride));
+                                                   keep, scale, sink, out_stride, out_scale));
   return check_launch("softmax_bias_attn");
 }

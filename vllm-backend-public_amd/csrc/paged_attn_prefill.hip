@@ -32,8 +32,10 @@
 // EXT (a second set of instantiations; the plain ones compile as before): attention inside chunks of
 // positions -- a column at position p sees the keys from (p / chunk) * chunk on, the walk starts at the
 // chunk of the tile's first query and columns of a tile that straddles a chunk edge mask for themselves;
-// one more term exp(sink[head]) in the softmax denominator that carries no value; and the output times
-// the sigmoid of one gate number per (token, head).
+// or a sliding window (keys after p - window) beside the first `keep` keys of the sequence: the walk takes
+// the barrier intervals that hold kept keys and lie before the window's first interval, then the window's;
+// value sizes that differ from the key size (64 / 128 either way); one more term exp(sink[head]) in the softmax denominator that carries no value; and the output times
+// the sigmoid of one gate number per (token, head), and times a constant.
 #include "common.h"
 
 #include <math.h>
@@ -54,15 +56,16 @@ __device__ __forceinline__ float max3(float a, float b, float c) {
 
 // Second launch bound: waves per SIMD the register allocation must leave room for.  Two workgroups
 // per CU overlap each other's dependent chains (LDS reads -> MFMAs -> exp2 -> MFMAs -> barrier).
-template <typename T, int D, int NQ, bool EXT>
+template <typename T, int D, int DV, int NQ, bool EXT>
 __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_prefill_kernel(
     uint16_t* __restrict__ out, int64_t out_stride, const uint16_t* __restrict__ q, int64_t q_stride,
     const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache, int num_blocks,
     const int32_t* __restrict__ block_tables, int max_blocks, const int32_t* __restrict__ cu_seqlens,
     const int32_t* __restrict__ context_lens, int num_heads, int num_kv_heads, float scale_log2e, int qt,
-    int chunk, const float* __restrict__ sink, const uint16_t* __restrict__ gate, int64_t gate_stride) {
+    int chunk, int window, int keep, const float* __restrict__ sink, const uint16_t* __restrict__ gate, int64_t gate_stride,
+    float out_scale) {
   constexpr int KS = D / 32;
-  constexpr int NT = D / 16;
+  constexpr int NT = DV / 16;
   constexpr int BS = MI355_BLOCK_SIZE;
   // K image of a step: [tile a/b][k-step][h = lane >> 4][c' = (lane & 15) ^ (2h + (k-step & 1))][16 B].
   // Reads (`ds_read_b128`: 16 lanes per LDS cycle, a bank per dword of 256 B) want the lanes of a
@@ -72,11 +75,11 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
   // slots of a block among the lanes that read it: both sides are conflict-free.
   constexpr int KFRAG = 1024;
   constexpr int KBYTES = 2 * KS * KFRAG;
-  constexpr int VBYTES = NT * 1024;              // V image: [16-row tile of head_dim][lane][16 B]
+  constexpr int VBYTES = NT * 1024;              // V image: [16-row tile of v_dim][lane][16 B]
   constexpr int BUF = KBYTES + VBYTES;
-  constexpr int PIECES = 8 * D;                  // 16-byte pieces per step: two K pages + two V pages
-  constexpr int PPT = PIECES / kPrefillThreads;  // per thread: 4 (D = 128) or 2 (D = 64)
-  static_assert(PIECES % kPrefillThreads == 0, "whole pieces per thread");
+  constexpr int KPT = 4 * D / kPrefillThreads;   // 16-byte pieces of a step's two K pages per thread: 2 (D = 128) or 1 (64)
+  constexpr int PPT = KPT + 4 * DV / kPrefillThreads;   // and with those of its two V pages
+  static_assert(4 * D % kPrefillThreads == 0 && 4 * DV % kPrefillThreads == 0, "whole pieces per thread");
   // HS 32-token images per barrier interval, two such sets (one computed on, one being staged):
   // half as many workgroup barriers per key as with one image per interval
   constexpr int HS = 2;
@@ -121,7 +124,9 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
     col_head[t] = kvh * group + p % group;
     col_ok[t] = (p < qt * group) && (col_q[t] < q_len);
     col_pos[t] = col_ok[t] ? pos0 + col_q[t] : -1;
-    col_lo[t] = (EXT && chunk > 0 && col_ok[t]) ? (col_pos[t] / chunk) * chunk : 0;      // first key the column sees
+    col_lo[t] = 0;                               // first key the column sees (past the kept ones)
+    if (EXT && chunk > 0 && col_ok[t]) col_lo[t] = (col_pos[t] / chunk) * chunk;
+    if (EXT && window > 0 && col_ok[t]) col_lo[t] = max(col_lo[t], col_pos[t] - window + 1);
     const uint16_t* qp = q + (q_begin + (col_ok[t] ? col_q[t] : 0)) * q_stride +
                          static_cast<int64_t>(col_ok[t] ? col_head[t] : 0) * D + 8 * h;
 #pragma unroll
@@ -145,7 +150,13 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
   }
   const int t_lo_max = __builtin_amdgcn_readfirstlane(lomax);
   // the walk starts at the chunk of the tile's first query, on a boundary of the barrier interval (HS steps)
-  const int s0 = (EXT && chunk > 0) ? ((pos0 + q0) / chunk) * chunk / 64 * 2 : 0;
+  int walk_lo = 0;                                                // first key of the walk past the kept ones
+  if (EXT && chunk > 0) walk_lo = (pos0 + q0) / chunk * chunk;
+  if (EXT && window > 0) walk_lo = max(walk_lo, pos0 + q0 - window + 1);
+  // barrier intervals (HS steps) in walking order: interval i is at step HS * i for the nk intervals that hold kept
+  // keys and lie before the walk's first, at HS * (i + skip) behind them.  Keys between are not visited.
+  const int nk = EXT ? min((keep + 63) / 64, walk_lo / 64) : 0;
+  const int skip = HS * (walk_lo / 64 - nk);                      // in steps
   const int t_end_wg = pos0 + min(q0 + qt, q_len);              // the tile's last query sees keys [0, t_end_wg)
 
   const int32_t* bt = block_tables + static_cast<int64_t>(seq) * max_blocks;
@@ -154,12 +165,12 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
   // ---- staging: thread tid copies pieces g = j*256 + tid of a step (j < PPT/2: the two K pages,
   // the rest: the two V pages).  Source addresses walk a page front to back (coalesced);
   // destinations are in fragment order.
-  int src_page[PPT], dst_off[PPT], v_tok[PPT / 2];               // v_tok: token offset of a V piece inside the step
+  int src_page[PPT], dst_off[PPT], v_tok[PPT - KPT];              // v_tok: token offset of a V piece inside the step
   int64_t src_off[PPT];                                          // element offset inside the (block, kv head) page
 #pragma unroll
   for (int j = 0; j < PPT; ++j) {
     const int g = j * kPrefillThreads + tid;
-    if (j < PPT / 2) {                                           // K: [page][row 0..15][16-byte slot 0..D/8)
+    if (j < KPT) {                                               // K: [page][row 0..15][16-byte slot 0..D/8)
       const int pg = g / (2 * D), rem = g % (2 * D);
       const int r = rem / (D / 8), sl = rem % (D / 8);
       const int ks = sl >> 2, hh = sl & 3;
@@ -168,13 +179,13 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
       src_page[j] = pg;
       src_off[j] = r * D + sl * 8;
       dst_off[j] = (tile * KS + ks) * KFRAG + hh * 256 + (cc ^ (2 * hh + (ks & 1))) * 16;
-    } else {                                                     // V: [page][head_dim row][half of the 16 tokens]
-      const int g2 = g - PIECES / 2;
-      const int pg = g2 / (2 * D), rem = g2 % (2 * D);
+    } else {                                                     // V: [page][v_dim row][half of the 16 tokens]
+      const int g2 = g - KPT * kPrefillThreads;
+      const int pg = g2 / (2 * DV), rem = g2 % (2 * DV);
       const int dr = rem >> 1, half = rem & 1;
       src_page[j] = pg;
       src_off[j] = dr * BS + half * 8;
-      v_tok[j - PPT / 2] = pg * BS + half * 8;
+      v_tok[j - KPT] = pg * BS + half * 8;
       dst_off[j] = KBYTES + ((dr >> 4) * 64 + (pg * 2 + half) * 16 + (dr & 15)) * 16;
     }
   }
@@ -187,9 +198,9 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
     blk[1] = min(max(blk[1], 0), num_blocks - 1);
 #pragma unroll
     for (int j = 0; j < NP; ++j) {
-      const int64_t page = (static_cast<int64_t>(blk[src_page[j]]) * num_kv_heads + kvh) * (BS * D);
-      const uint16_t* src = (j < PPT / 2 ? k_cache : v_cache) + page + src_off[j];
-      regs[j] = MI355_LD(pvec, j < PPT / 2 ? k_cache : v_cache, src);
+      const int64_t page = (static_cast<int64_t>(blk[src_page[j]]) * num_kv_heads + kvh) * (BS * (j < KPT ? D : DV));
+      const uint16_t* src = (j < KPT ? k_cache : v_cache) + page + src_off[j];
+      regs[j] = MI355_LD(pvec, j < KPT ? k_cache : v_cache, src);
     }
   };
   // In the image that reaches the tile's end the V columns of tokens beyond its last query may be
@@ -197,11 +208,11 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
   // accumulator is live across the branch, rather than in the MFMA loop.
   auto stage_store = [&](const pvec (&regs)[PPT], int image, int tb) {   // image = interval parity * HS + half-step
 #pragma unroll
-    for (int j = 0; j < PPT / 2; ++j) *reinterpret_cast<pvec*>(&lds[image * BUF + dst_off[j]]) = regs[j];
+    for (int j = 0; j < KPT; ++j) *reinterpret_cast<pvec*>(&lds[image * BUF + dst_off[j]]) = regs[j];
     if (tb + 32 > t_end_wg) {                                      // workgroup-uniform
 #pragma unroll
-      for (int j = PPT / 2; j < PPT; ++j) {
-        const int tok = tb + v_tok[j - PPT / 2];                   // first of the piece's 8 tokens
+      for (int j = KPT; j < PPT; ++j) {
+        const int tok = tb + v_tok[j - KPT];                   // first of the piece's 8 tokens
         pvec v = regs[j];
 #pragma unroll
         for (int w = 0; w < 4; ++w)
@@ -210,11 +221,12 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
       }
     } else {
 #pragma unroll
-      for (int j = PPT / 2; j < PPT; ++j) *reinterpret_cast<pvec*>(&lds[image * BUF + dst_off[j]]) = regs[j];
+      for (int j = KPT; j < PPT; ++j) *reinterpret_cast<pvec*>(&lds[image * BUF + dst_off[j]]) = regs[j];
     }
   };
 
-  const int steps = (t_end_wg + 31) / 32;
+  const int steps = (t_end_wg + 31) / 32 - (EXT ? skip : 0);      // of the walk
+  auto key_step = [&](int s) { return EXT && s >= HS * nk ? s + skip : s; };      // the 32-key step of the sequence at walk step s
   const int tok_h = 8 * h;
 
   // S^T = K . Q^T of one step for all column tiles (a K fragment is read from LDS once and used NQ
@@ -252,8 +264,8 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
       for (int t = 0; t < NQ; ++t) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          sa[t][j] = (tok0 + j >= col_lo[t]) ? sa[t][j] : -INFINITY;
-          sb[t][j] = (tok0 + 4 + j >= col_lo[t]) ? sb[t][j] : -INFINITY;
+          sa[t][j] = (tok0 + j >= col_lo[t] || tok0 + j < keep) ? sa[t][j] : -INFINITY;
+          sb[t][j] = (tok0 + 4 + j >= col_lo[t] || tok0 + 4 + j < keep) ? sb[t][j] : -INFINITY;
         }
       }
     }
@@ -343,25 +355,25 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
 #pragma unroll
     for (int hs = 0; hs < HS; ++hs) {          // images beyond the last step re-read the last pages (clamped), unused
       pvec r0[PPT];
-      stage_load(r0, (s0 + hs) * 32);
-      stage_store(r0, hs, (s0 + hs) * 32);
+      stage_load(r0, key_step(hs) * 32);
+      stage_store(r0, hs, key_step(hs) * 32);
     }
   }
   __syncthreads();
-  for (int s = s0; s < steps; s += HS) {
+  for (int s = 0; s < steps; s += HS) {
     const bool more = s + HS < steps;
-    const int par = ((s - s0) / HS) & 1;
+    const int par = (s / HS) & 1;
     pvec nxt[HS][PPT];
     if (more) {                                                  // workgroup-uniform branch
 #pragma unroll
-      for (int hs = 0; hs < HS; ++hs) stage_load(nxt[hs], (s + HS + hs) * 32);
+      for (int hs = 0; hs < HS; ++hs) stage_load(nxt[hs], key_step(s + HS + hs) * 32);
     }
 #pragma unroll
     for (int hs = 0; hs < HS; ++hs)
-      if (s + hs < steps) half_step(s + hs, par * HS + hs);      // workgroup-uniform
+      if (s + hs < steps) half_step(key_step(s + hs), par * HS + hs);      // workgroup-uniform
     if (more) {
 #pragma unroll
-      for (int hs = 0; hs < HS; ++hs) stage_store(nxt[hs], (par ^ 1) * HS + hs, (s + HS + hs) * 32);
+      for (int hs = 0; hs < HS; ++hs) stage_store(nxt[hs], (par ^ 1) * HS + hs, key_step(s + HS + hs) * 32);
       __syncthreads();
     }
   }
@@ -375,9 +387,10 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
     if (EXT && sink != nullptr)          // the value-less term, against the column's reference (a valid column has seen a key)
       lt += __builtin_amdgcn_exp2f(MI355_LD(float, sink, sink + col_head[t]) * 1.4426950408889634f - m_ref[t]);
     float inv = lt > 0.f ? 1.0f / lt : 0.f;
+    if (EXT) inv *= out_scale;
     if (EXT && gate != nullptr)
       inv /= 1.0f + expf(-T::to_f(MI355_LD(uint16_t, gate, gate + (q_begin + col_q[t]) * gate_stride + col_head[t])));
-    uint16_t* op = out + (q_begin + col_q[t]) * out_stride + static_cast<int64_t>(col_head[t]) * D + 4 * h;
+    uint16_t* op = out + (q_begin + col_q[t]) * out_stride + static_cast<int64_t>(col_head[t]) * DV + 4 * h;
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
       // lane (pair c, h) holds d = 16n + 4h + r, r = 0..3: one 8-byte store
@@ -392,8 +405,8 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
 
 }  // namespace mi355
 
-static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chunk, const float* sink, const void* gate,
-                                          int64_t gate_stride, void* out, int64_t out_stride, const void* q, int64_t q_stride,
+static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chunk, int32_t window, int32_t keep, const float* sink,
+                                          const void* gate, int64_t gate_stride, float out_scale, int32_t v_dim, void* out, int64_t out_stride, const void* q, int64_t q_stride,
                                             const void* k_cache, const void* v_cache, int32_t num_blocks,
                                             const int32_t* block_tables, int32_t max_blocks_per_seq,
                                             const int32_t* cu_seqlens, const int32_t* context_lens,
@@ -412,10 +425,10 @@ static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chu
   const int group = num_heads / num_kv_heads;
   MI355_REQUIRE(group <= 16 && num_kv_heads <= 65535, MI355_ERR_UNSUPPORTED,
                 "%s: at most 16 query heads per kv head (got %d)", name, group);
-  MI355_REQUIRE(head_dim == 64 || head_dim == 128, MI355_ERR_UNSUPPORTED,
-                "%s: head_dim %d not supported (64 or 128)", name, head_dim);
+  MI355_REQUIRE((head_dim == 64 || head_dim == 128) && (v_dim == head_dim || (ext && (v_dim == 64 || v_dim == 128))),
+                MI355_ERR_UNSUPPORTED, "%s: head_dim %d / v_dim %d not supported (64 or 128)", name, head_dim, v_dim);
   const int64_t width = static_cast<int64_t>(num_heads) * head_dim;
-  MI355_REQUIRE(q_stride >= width && q_stride % 8 == 0 && out_stride >= width && out_stride % 8 == 0,
+  MI355_REQUIRE(q_stride >= width && q_stride % 8 == 0 && out_stride >= static_cast<int64_t>(num_heads) * v_dim && out_stride % 8 == 0,
                 MI355_ERR_INVALID, "%s: q_stride/out_stride invalid", name);
   MI355_REQUIRE(aligned16(out) && aligned16(q) && aligned16(k_cache) && aligned16(v_cache),
                 MI355_ERR_INVALID, "%s: pointers must be 16-byte aligned", name);
@@ -435,17 +448,18 @@ static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chu
   const int qt = 64 * nq / group;                      // queries per workgroup (>= 4: group <= 16)
   dim3 grid((max_q_len + qt - 1) / qt, num_kv_heads, num_seqs), block(kPrefillThreads);
   hipStream_t s = static_cast<hipStream_t>(stream);
-#define MI355_PRE_E(TT, DD, NN, EE)                                                                     \
-  hipLaunchKernelGGL((paged_attn_prefill_kernel<TT, DD, NN, EE>), grid, block, 0, s,                    \
+#define MI355_PRE_E(TT, DD, DV, NN, EE)                                                                 \
+  hipLaunchKernelGGL((paged_attn_prefill_kernel<TT, DD, DV, NN, EE>), grid, block, 0, s,                    \
                      static_cast<uint16_t*>(out), out_stride, static_cast<const uint16_t*>(q), q_stride, \
                      static_cast<const uint16_t*>(k_cache), static_cast<const uint16_t*>(v_cache),      \
                      num_blocks, block_tables, max_blocks_per_seq, cu_seqlens, context_lens, num_heads, \
-                     num_kv_heads, scale * 1.4426950408889634f, qt, chunk, sink,                        \
-                     static_cast<const uint16_t*>(gate), gate_stride)
+                     num_kv_heads, scale * 1.4426950408889634f, qt, chunk, window, keep, sink,          \
+                     static_cast<const uint16_t*>(gate), gate_stride, out_scale)
 #define MI355_PRE(TT, DD, NN)                                                                           \
   do {                                                                                                  \
-    if (ext) MI355_PRE_E(TT, DD, NN, true);                                                             \
-    else MI355_PRE_E(TT, DD, NN, false);                                                                \
+    if (ext && v_dim == 64) MI355_PRE_E(TT, DD, 64, NN, true);                                          \
+    else if (ext) MI355_PRE_E(TT, DD, 128, NN, true);                                                   \
+    else MI355_PRE_E(TT, DD, DD, NN, false);                                                            \
   } while (0)
 #define MI355_PRE_NQ(TT, DD)                \
   switch (nq) {                             \
@@ -470,7 +484,7 @@ extern "C" int32_t mi355_paged_attn_prefill(void* out, int64_t out_stride, const
                                             int32_t num_seqs, int32_t max_q_len, int32_t num_heads,
                                             int32_t num_kv_heads, int32_t head_dim, float scale,
                                             int32_t dtype, void* stream) {
-  return launch_paged_attn_prefill("mi355_paged_attn_prefill", false, 0, nullptr, nullptr, 0, out, out_stride, q, q_stride, k_cache,
+  return launch_paged_attn_prefill("mi355_paged_attn_prefill", false, 0, 0, 0, nullptr, nullptr, 0, 1.0f, head_dim, out, out_stride, q, q_stride, k_cache,
                                    v_cache, num_blocks, block_tables, max_blocks_per_seq, cu_seqlens, context_lens, num_seqs,
                                    max_q_len, num_heads, num_kv_heads, head_dim, scale, dtype, stream);
 }
@@ -480,12 +494,15 @@ extern "C" int32_t mi355_paged_attn_prefill_ext(void* out, int64_t out_stride, c
                                                 const int32_t* block_tables, int32_t max_blocks_per_seq,
                                                 const int32_t* cu_seqlens, const int32_t* context_lens,
                                                 int32_t num_seqs, int32_t max_q_len, int32_t num_heads,
-                                                int32_t num_kv_heads, int32_t head_dim, float scale, int32_t chunk,
-                                                const float* sink, const void* gate, int64_t gate_stride,
-                                                int32_t dtype, void* stream) {
+                                                int32_t num_kv_heads, int32_t head_dim, int32_t v_dim, float scale,
+                                                int32_t chunk, int32_t window, int32_t keep, const float* sink,
+                                                const void* gate, int64_t gate_stride, float out_scale, int32_t dtype,
+                                                void* stream) {
+  MI355_REQUIRE(window >= 0 && keep >= 0 && (keep == 0 || chunk == 0), MI355_ERR_INVALID,
+                "mi355_paged_attn_prefill_ext: window %d, keep %d (not with chunks)", window, keep);
   MI355_REQUIRE(chunk >= 0 && (gate == nullptr || gate_stride >= num_heads), MI355_ERR_INVALID,
                 "mi355_paged_attn_prefill_ext: chunk %d, gate rows shorter than the heads", chunk);
-  return launch_paged_attn_prefill("mi355_paged_attn_prefill_ext", true, chunk, sink, gate, gate_stride, out, out_stride, q,
+  return launch_paged_attn_prefill("mi355_paged_attn_prefill_ext", true, chunk, window, keep, sink, gate, gate_stride, out_scale, v_dim, out, out_stride, q,
                                    q_stride, k_cache, v_cache, num_blocks, block_tables, max_blocks_per_seq, cu_seqlens,
                                    context_lens, num_seqs, max_q_len, num_heads, num_kv_heads, head_dim, scale, dtype, stream);
 }

@@ -1,5 +1,5 @@
 // Pointwise and normalisation kernels for decoders that keep the residual stream in fp32:
-//   embed_scale_f32          resid = embed[id] * scale
+//   embed_scale_f32          resid = embed[id] * scale          (optionally once more as activation rows)
 //   embed_scale_pos_f32      resid = embed[id] * scale + pos_table[position]      (learned positions)
 //   resid_add_f32            resid += other (fp32 rows) + rows (activation rows) + vec (one row, broadcast)
 //   add_rms_norm_f32         resid += add; out = resid / rms(resid) * w      (w: one number or a vector)
@@ -7,6 +7,11 @@
 //   gelu_tanh_and_mul        out = gelu_tanh(gate) * up for rows holding gate | up
 //   gated_head_rms_norm      out = o / rms(o) * w * act(gate) per (token, head) row of an fp32 tensor
 //   softcap                  z = cap * tanh(z / cap)
+//   norm_resid_f32           resid += y / rms(y * y_scale) * y_scale * w, and the new residual once more as activation
+//                            rows (norms on a sub-layer's output; the sub-layers read the residual itself)
+//   token_gate_rows          out = gelu_tanh(z) * table[id, column offset ..]: a gate on a per-layer part of a token's row
+//   token_side_f32           the whole per-layer token input for few rows: gate projection, gate, projection back, norm,
+//                            residual add and activation copy in one launch
 //   group_rms_norm_f32       out = gn(x) * w: an RMS norm over each of `groups` equal consecutive parts of an
 //                            fp32 row, to activation rows or (in place or not) to fp32 rows
 //   gated_norm_resid_f32     resid += mult * gn(y * sigmoid(g + b)) * w: a sub-layer's result, gated element by
@@ -22,11 +27,15 @@ namespace mi355 {
 template <typename T>
 __global__ __launch_bounds__(256) void embed_scale_f32_kernel(float* __restrict__ out,
                                                               const typename Elem<T>::S* __restrict__ embed,
-                                                              const int64_t* __restrict__ ids, int W, float scale) {
+                                                              const int64_t* __restrict__ ids, int W, float scale,
+                                                              typename Elem<T>::S* __restrict__ act) {
   const int64_t t = blockIdx.x;
   const int64_t id = MI355_LD(int64_t, ids, ids + t);
-  for (int c = threadIdx.x; c < W; c += blockDim.x)
-    MI355_ST(float, out, out + t * W + c, MI355_LDF(T, embed, embed + id * W + c) * scale);
+  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+    const float v = MI355_LDF(T, embed, embed + id * W + c) * scale;
+    MI355_ST(float, out, out + t * W + c, v);
+    if (act != nullptr) MI355_STF(T, act, act + t * W + c, v);
+  }
 }
 
 template <typename T>
@@ -164,7 +173,7 @@ __global__ __launch_bounds__(256) void gated_head_rms_norm_kernel(typename Elem<
                                                                   const typename Elem<T>::S* __restrict__ gate,
                                                                   int64_t gate_stride, const float* __restrict__ w,
                                                                   int w_heads, int64_t rows, int H, int dv, float eps,
-                                                                  int act) {
+                                                                  int act, int64_t out_stride) {
   const int64_t row = blockIdx.x * static_cast<int64_t>(blockDim.x >> 6) + (threadIdx.x >> 6);
   if (row >= rows) return;
   const int lane = threadIdx.x & 63;
@@ -182,7 +191,231 @@ __global__ __launch_bounds__(256) void gated_head_rms_norm_kernel(typename Elem<
     const float g = MI355_LDF(T, gate, gate + t * gate_stride + static_cast<int64_t>(h) * dv + c);
     const float s = 1.0f / (1.0f + expf(-g));
     const float a = act == 0 ? g * s : s;
-    MI355_STF(T, out, out + row * dv + c, v * r * MI355_LD(float, w, w + (w_heads > 1 ? h * dv : 0) + c) * a);
+    MI355_STF(T, out, out + t * out_stride + static_cast<int64_t>(h) * dv + c,
+              v * r * MI355_LD(float, w, w + (w_heads > 1 ? h * dv : 0) + c) * a);
+  }
+}
+
+// one workgroup per row, for rows of many columns (a norm over all heads at once)
+template <typename T>
+__global__ __launch_bounds__(256) void gated_wide_rms_norm_kernel(typename Elem<T>::S* __restrict__ out,
+                                                                  const float* __restrict__ o,
+                                                                  const typename Elem<T>::S* __restrict__ gate,
+                                                                  int64_t gate_stride, const float* __restrict__ w, int n,
+                                                                  float eps, int act, int64_t out_stride) {
+  __shared__ float scratch[32];
+  const int64_t t = blockIdx.x;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < n; c += blockDim.x) {
+    const float v = MI355_LD(float, o, o + t * n + c);
+    ss += v * v;
+  }
+  const float r = 1.0f / sqrtf(block_sum32(ss, scratch) / static_cast<float>(n) + eps);
+  for (int c = threadIdx.x; c < n; c += blockDim.x) {
+    const float g = MI355_LDF(T, gate, gate + t * gate_stride + c);
+    const float s = 1.0f / (1.0f + expf(-g));
+    MI355_STF(T, out, out + t * out_stride + c, MI355_LD(float, o, o + t * n + c) * r * MI355_LD(float, w, w + c) * (act == 0 ? g * s : s));
+  }
+}
+
+// 16-bit rows of a multiple of 8 columns, up to 2048 * NV columns: 8 columns per thread and turn, o read once
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void gated_wide_rms_norm_vec_kernel(uint16_t* __restrict__ out, const float* __restrict__ o,
+                                                                      const uint16_t* __restrict__ gate, int64_t gate_stride,
+                                                                      const float* __restrict__ w, int n, float eps, int act,
+                                                                      int64_t out_stride) {
+  __shared__ float scratch[32];
+  const int64_t t = blockIdx.x;
+  float v[NV][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + 256 * i) * 8;
+    float4 a = make_float4(0.f, 0.f, 0.f, 0.f), b = a;
+    if (c < n) {
+      a = MI355_LD(float4, o, o + t * n + c);
+      b = MI355_LD(float4, o, o + t * n + c + 4);
+    }
+    v[i][0] = a.x, v[i][1] = a.y, v[i][2] = a.z, v[i][3] = a.w, v[i][4] = b.x, v[i][5] = b.y, v[i][6] = b.z, v[i][7] = b.w;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss += v[i][j] * v[i][j];
+  }
+  const float r = 1.0f / sqrtf(block_sum32(ss, scratch) / static_cast<float>(n) + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + 256 * i) * 8;
+    if (c >= n) continue;
+    float g[8], wv[8];
+    unpack8<T>(MI355_LD(uint4, gate, gate + t * gate_stride + c), g);
+    const float4 a = MI355_LD(float4, w, w + c), b = MI355_LD(float4, w, w + c + 4);
+    wv[0] = a.x, wv[1] = a.y, wv[2] = a.z, wv[3] = a.w, wv[4] = b.x, wv[5] = b.y, wv[6] = b.z, wv[7] = b.w;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float s = 1.0f / (1.0f + expf(-g[j]));
+      g[j] = v[i][j] * r * wv[j] * (act == 0 ? g[j] * s : s);
+    }
+    MI355_ST(uint4, out, out + t * out_stride + c, pack8<T>(g));
+  }
+}
+
+// one workgroup per row; y is read once where the row fits (8 columns per thread and turn), the activation
+// copy leaves in the same pass as the residual
+template <typename T>
+__global__ __launch_bounds__(256) void norm_resid_f32_kernel(float* __restrict__ resid, typename Elem<T>::S* __restrict__ act,
+                                                             const typename Elem<T>::S* __restrict__ y,
+                                                             const float* __restrict__ w, int W, float eps, float y_scale) {
+  __shared__ float scratch[32];
+  const int64_t t = blockIdx.x;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+    const float v = MI355_LDF(T, y, y + t * W + c) * y_scale;
+    ss += v * v;
+  }
+  const float r = y_scale / sqrtf(block_sum32(ss, scratch) / static_cast<float>(W) + eps);
+  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+    const float v = MI355_LD(float, resid, resid + t * W + c) + MI355_LDF(T, y, y + t * W + c) * r * MI355_LD(float, w, w + c);
+    MI355_ST(float, resid, resid + t * W + c, v);
+    if (act != nullptr) MI355_STF(T, act, act + t * W + c, v);
+  }
+}
+
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void norm_resid_f32_vec_kernel(float* __restrict__ resid, uint16_t* __restrict__ act,
+                                                                 const uint16_t* __restrict__ y, const float* __restrict__ w,
+                                                                 int W, float eps, float y_scale) {
+  __shared__ float scratch[32];
+  const int64_t t = blockIdx.x;
+  float v[NV][8], x[NV][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + 256 * i) * 8;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[i][j] = x[i][j] = 0.f;
+    if (c < W) {
+      unpack8<T>(MI355_LD(uint4, y, y + t * W + c), v[i]);
+      const float4 a = MI355_LD(float4, resid, resid + t * W + c), b = MI355_LD(float4, resid, resid + t * W + c + 4);
+      x[i][0] = a.x, x[i][1] = a.y, x[i][2] = a.z, x[i][3] = a.w, x[i][4] = b.x, x[i][5] = b.y, x[i][6] = b.z, x[i][7] = b.w;
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      v[i][j] *= y_scale;
+      ss += v[i][j] * v[i][j];
+    }
+  }
+  const float r = 1.0f / sqrtf(block_sum32(ss, scratch) / static_cast<float>(W) + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + 256 * i) * 8;
+    if (c >= W) continue;
+    const float4 a = MI355_LD(float4, w, w + c), b = MI355_LD(float4, w, w + c + 4);
+    const float wv[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[i][j] += v[i][j] * r * wv[j];
+    MI355_ST(float4, resid, resid + t * W + c, make_float4(x[i][0], x[i][1], x[i][2], x[i][3]));
+    MI355_ST(float4, resid, resid + t * W + c + 4, make_float4(x[i][4], x[i][5], x[i][6], x[i][7]));
+    if (act != nullptr) MI355_ST(uint4, act, act + t * W + c, pack8<T>(x[i]));
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void token_gate_rows_kernel(typename Elem<T>::S* __restrict__ out,
+                                                              const typename Elem<T>::S* __restrict__ z, int64_t z_stride,
+                                                              const typename Elem<T>::S* __restrict__ table,
+                                                              int64_t table_stride, int64_t offset,
+                                                              const int64_t* __restrict__ ids, int64_t vocab, int64_t rows,
+                                                              int n) {
+  const int64_t total = rows * n;
+  for (int64_t i = blockIdx.x * static_cast<int64_t>(blockDim.x) + threadIdx.x; i < total;
+       i += static_cast<int64_t>(gridDim.x) * blockDim.x) {
+    const int64_t t = i / n;
+    const int c = static_cast<int>(i % n);
+    int64_t id = MI355_LD(int64_t, ids, ids + t);
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    const float e = MI355_LDF(T, table, table + id * table_stride + offset + c);
+    MI355_STF(T, out, out + i, gelu_tanh_f(MI355_LDF(T, z, z + t * z_stride + c)) * e);
+  }
+}
+
+// One workgroup per row: n gate products over the residual row (one wave each in turn), the gate against the
+// token's part of the table, W products of n terms back, their norm, the residual add and the activation
+// copy.  fp32 throughout; LDS: the residual row [W], the gated numbers [n], the products [W].
+template <typename T>
+__global__ __launch_bounds__(512) void token_side_f32_kernel(float* __restrict__ resid, typename Elem<T>::S* __restrict__ act,
+                                                             const typename Elem<T>::S* __restrict__ gate_w,
+                                                             const typename Elem<T>::S* __restrict__ proj_w,
+                                                             const float* __restrict__ norm,
+                                                             const typename Elem<T>::S* __restrict__ table,
+                                                             int64_t table_stride, int64_t offset,
+                                                             const int64_t* __restrict__ ids, int64_t vocab, int W, int n,
+                                                             float eps, int vec) {
+  extern __shared__ float lds[];
+  __shared__ float scratch[32];
+  float* xs = lds;                                        // [W]
+  float* gs = xs + W;                                     // [n]
+  const int64_t t = blockIdx.x;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  for (int c = threadIdx.x; c < W; c += blockDim.x) xs[c] = MI355_LD(float, resid, resid + t * W + c);
+  int64_t id = MI355_LD(int64_t, ids, ids + t);
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  __syncthreads();
+  for (int j = wave; j < n; j += nw) {
+    const typename Elem<T>::S* wr = gate_w + static_cast<int64_t>(j) * W;
+    float z = 0.f;
+    if constexpr (sizeof(typename Elem<T>::S) == 2) {
+      if (vec) {
+        for (int c = lane * 8; c < W; c += 512) {
+          float f[8];
+          unpack8<T>(MI355_LD(uint4, gate_w, wr + c), f);
+#pragma unroll
+          for (int u = 0; u < 8; ++u) z += f[u] * xs[c + u];
+        }
+      } else {
+        for (int c = lane; c < W; c += 64) z += MI355_LDF(T, gate_w, wr + c) * xs[c];
+      }
+    } else {
+      for (int c = lane; c < W; c += 64) z += MI355_LDF(T, gate_w, wr + c) * xs[c];
+    }
+    z = wave_sum(z);
+    if (lane == 0) gs[j] = gelu_tanh_f(z) * MI355_LDF(T, table, table + id * table_stride + offset + j);
+  }
+  __syncthreads();
+  constexpr int PER = 16;                                 // products held per thread: up to 8192 columns
+  float y[PER];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = threadIdx.x + i * static_cast<int>(blockDim.x);
+    y[i] = 0.f;
+    if (c < W) {
+      const typename Elem<T>::S* pr = proj_w + static_cast<int64_t>(c) * n;
+      float a = 0.f;
+      if constexpr (sizeof(typename Elem<T>::S) == 2) {
+        if (vec) {
+          for (int j = 0; j < n; j += 8) {
+            float f[8];
+            unpack8<T>(MI355_LD(uint4, proj_w, pr + j), f);
+#pragma unroll
+            for (int u = 0; u < 8; ++u) a += f[u] * gs[j + u];
+          }
+        } else {
+          for (int j = 0; j < n; ++j) a += MI355_LDF(T, proj_w, pr + j) * gs[j];
+        }
+      } else {
+        for (int j = 0; j < n; ++j) a += MI355_LDF(T, proj_w, pr + j) * gs[j];
+      }
+      y[i] = a;
+      ss += a * a;
+    }
+  }
+  const float r = 1.0f / sqrtf(block_sum32(ss, scratch) / static_cast<float>(W) + eps);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = threadIdx.x + i * static_cast<int>(blockDim.x);
+    if (c >= W) continue;
+    const float v = xs[c] + y[i] * r * MI355_LD(float, norm, norm + c);
+    MI355_ST(float, resid, resid + t * W + c, v);
+    if (act != nullptr) MI355_STF(T, act, act + t * W + c, v);
   }
 }
 
@@ -368,7 +601,7 @@ using namespace mi355;
 
 #define REQ_DTYPE(dtype) MI355_REQUIRE((dtype) >= MI355_BF16 && (dtype) <= MI355_F32, MI355_ERR_UNSUPPORTED, "dtype code %d", (dtype))
 
-extern "C" int32_t mi355_embed_scale_f32(float* out, const void* embed, const int64_t* ids, int64_t num_tokens,
+extern "C" int32_t mi355_embed_scale_f32(float* out, void* act_out, const void* embed, const int64_t* ids, int64_t num_tokens,
                                          int32_t width, int64_t vocab, float scale, int32_t dtype, void* stream) {
   MI355_REQUIRE(out && embed && ids, MI355_ERR_INVALID, "embed_scale_f32: null pointer");
   MI355_REQUIRE(num_tokens >= 0 && width > 0 && vocab > 0, MI355_ERR_INVALID, "embed_scale_f32: sizes");
@@ -376,7 +609,8 @@ extern "C" int32_t mi355_embed_scale_f32(float* out, const void* embed, const in
   if (num_tokens == 0) return MI355_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
   MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((embed_scale_f32_kernel<TT>), dim3(num_tokens), dim3(256), 0, s, out,
-                                                  static_cast<const Elem<TT>::S*>(embed), ids, width, scale));
+                                                  static_cast<const Elem<TT>::S*>(embed), ids, width, scale,
+                                                  static_cast<Elem<TT>::S*>(act_out)));
   return check_launch("embed_scale_f32");
 }
 
@@ -516,13 +750,13 @@ extern "C" int32_t mi355_gelu_tanh_and_mul(void* out, const void* x, int64_t x_s
   return check_launch("gelu_tanh_and_mul");
 }
 
-extern "C" int32_t mi355_gated_head_rms_norm(void* out, const float* o, const void* gate, int64_t gate_stride,
-                                             const float* weight, int32_t weight_heads, int64_t num_tokens,
-                                             int32_t num_heads, int32_t head_dim, float eps, int32_t activation,
-                                             int32_t dtype, void* stream) {
+extern "C" int32_t mi355_gated_head_rms_norm(void* out, int64_t out_stride, const float* o, const void* gate,
+                                             int64_t gate_stride, const float* weight, int32_t weight_heads,
+                                             int64_t num_tokens, int32_t num_heads, int32_t head_dim, float eps,
+                                             int32_t activation, int32_t dtype, void* stream) {
   MI355_REQUIRE(out && o && gate && weight, MI355_ERR_INVALID, "gated_head_rms_norm: null pointer");
-  MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && head_dim > 0 &&
-                    gate_stride >= static_cast<int64_t>(num_heads) * head_dim,
+  const int64_t width = static_cast<int64_t>(num_heads) * head_dim;
+  MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && head_dim > 0 && gate_stride >= width && out_stride >= width,
                 MI355_ERR_INVALID, "gated_head_rms_norm: sizes");
   MI355_REQUIRE(activation == 0 || activation == 1, MI355_ERR_INVALID,
                 "gated_head_rms_norm: activation is 0 (silu) or 1 (sigmoid)");
@@ -532,11 +766,101 @@ extern "C" int32_t mi355_gated_head_rms_norm(void* out, const float* o, const vo
   const int64_t rows = num_tokens * num_heads;
   if (rows == 0) return MI355_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
+  if (num_heads == 1 && head_dim >= 512) {
+    if (dtype != MI355_F32 && head_dim % 8 == 0 && head_dim <= 8192 && gate_stride % 8 == 0 && out_stride % 8 == 0 &&
+        aligned16(out) && aligned16(o) && aligned16(gate) && aligned16(weight)) {
+#define MI355_WIDE(TT, NV)                                                                                                  \
+  hipLaunchKernelGGL((gated_wide_rms_norm_vec_kernel<TT, NV>), dim3(num_tokens), dim3(256), 0, s, static_cast<uint16_t*>(out), \
+                     o, static_cast<const uint16_t*>(gate), gate_stride, weight, head_dim, eps, activation, out_stride)
+#define MI355_WIDE_NV(TT)                      \
+  do {                                         \
+    if (head_dim <= 2048) MI355_WIDE(TT, 1);   \
+    else if (head_dim <= 4096) MI355_WIDE(TT, 2); \
+    else MI355_WIDE(TT, 4);                    \
+  } while (0)
+      if (dtype == MI355_BF16) MI355_WIDE_NV(BF16); else MI355_WIDE_NV(F16);
+#undef MI355_WIDE_NV
+#undef MI355_WIDE
+      return check_launch("gated_head_rms_norm");
+    }
+    MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((gated_wide_rms_norm_kernel<TT>), dim3(num_tokens), dim3(256), 0, s,
+                                                    static_cast<Elem<TT>::S*>(out), o,
+                                                    static_cast<const Elem<TT>::S*>(gate), gate_stride, weight, head_dim, eps,
+                                                    activation, out_stride));
+    return check_launch("gated_head_rms_norm");
+  }
   MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((gated_head_rms_norm_kernel<TT>), dim3((rows + 3) / 4), dim3(256), 0, s,
                                                   static_cast<Elem<TT>::S*>(out), o,
                                                   static_cast<const Elem<TT>::S*>(gate), gate_stride, weight,
-                                                  weight_heads, rows, num_heads, head_dim, eps, activation));
+                                                  weight_heads, rows, num_heads, head_dim, eps, activation, out_stride));
   return check_launch("gated_head_rms_norm");
+}
+
+extern "C" int32_t mi355_norm_resid_f32(float* resid, void* act_out, const void* y, const float* weight, int64_t num_tokens,
+                                        int32_t width, float eps, float y_scale, int32_t dtype, void* stream) {
+  MI355_REQUIRE(resid && y && weight, MI355_ERR_INVALID, "norm_resid_f32: null pointer");
+  MI355_REQUIRE(num_tokens >= 0 && width > 0, MI355_ERR_INVALID, "norm_resid_f32: sizes");
+  REQ_DTYPE(dtype);
+  if (num_tokens == 0) return MI355_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (dtype != MI355_F32 && width % 8 == 0 && width <= 8192 && aligned16(resid) && aligned16(y) && aligned16(weight) &&
+      aligned16(act_out)) {
+#define MI355_NR(TT, NV)                                                                                               \
+  hipLaunchKernelGGL((norm_resid_f32_vec_kernel<TT, NV>), dim3(num_tokens), dim3(256), 0, s, resid,                    \
+                     static_cast<uint16_t*>(act_out), static_cast<const uint16_t*>(y), weight, width, eps, y_scale)
+#define MI355_NR_NV(TT)                      \
+  do {                                       \
+    if (width <= 2048) MI355_NR(TT, 1);      \
+    else if (width <= 4096) MI355_NR(TT, 2); \
+    else MI355_NR(TT, 4);                    \
+  } while (0)
+    if (dtype == MI355_BF16) MI355_NR_NV(BF16); else MI355_NR_NV(F16);
+#undef MI355_NR_NV
+#undef MI355_NR
+    return check_launch("norm_resid_f32");
+  }
+  MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((norm_resid_f32_kernel<TT>), dim3(num_tokens), dim3(256), 0, s, resid,
+                                                  static_cast<Elem<TT>::S*>(act_out), static_cast<const Elem<TT>::S*>(y),
+                                                  weight, width, eps, y_scale));
+  return check_launch("norm_resid_f32");
+}
+
+extern "C" int32_t mi355_token_gate_rows(void* out, const void* z, int64_t z_stride, const void* table, int64_t table_stride,
+                                         int64_t offset, const int64_t* ids, int64_t vocab, int64_t num_tokens, int32_t n,
+                                         int32_t dtype, void* stream) {
+  MI355_REQUIRE(out && z && table && ids, MI355_ERR_INVALID, "token_gate_rows: null pointer");
+  MI355_REQUIRE(num_tokens >= 0 && n > 0 && z_stride >= n && offset >= 0 && table_stride >= offset + n && vocab > 0,
+                MI355_ERR_INVALID, "token_gate_rows: sizes");
+  REQ_DTYPE(dtype);
+  if (num_tokens == 0) return MI355_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((token_gate_rows_kernel<TT>), stride_grid(num_tokens * n), dim3(256), 0, s,
+                                                  static_cast<Elem<TT>::S*>(out), static_cast<const Elem<TT>::S*>(z), z_stride,
+                                                  static_cast<const Elem<TT>::S*>(table), table_stride, offset, ids, vocab,
+                                                  num_tokens, n));
+  return check_launch("token_gate_rows");
+}
+
+extern "C" int32_t mi355_token_side_f32(float* resid, void* act_out, const void* gate_w, const void* proj_w, const float* norm,
+                                        const void* table, int64_t table_stride, int64_t offset, const int64_t* ids,
+                                        int64_t vocab, int64_t num_tokens, int32_t width, int32_t n, float eps, int32_t dtype,
+                                        void* stream) {
+  MI355_REQUIRE(resid && gate_w && proj_w && norm && table && ids, MI355_ERR_INVALID, "token_side_f32: null pointer");
+  MI355_REQUIRE(num_tokens >= 0 && n > 0 && width > 0 && offset >= 0 && table_stride >= offset + n && vocab > 0,
+                MI355_ERR_INVALID, "token_side_f32: sizes");
+  MI355_REQUIRE(width <= 8192 && n <= 4096, MI355_ERR_UNSUPPORTED, "token_side_f32: width %d (at most 8192), %d numbers (4096)",
+                width, n);
+  REQ_DTYPE(dtype);
+  if (num_tokens == 0) return MI355_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const int vec = dtype != MI355_F32 && width % 8 == 0 && n % 8 == 0 && aligned16(gate_w) && aligned16(proj_w);
+  const size_t lds = sizeof(float) * (static_cast<size_t>(width) + n);
+  MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((token_side_f32_kernel<TT>), dim3(num_tokens), dim3(512), lds, s, resid,
+                                                  static_cast<Elem<TT>::S*>(act_out), static_cast<const Elem<TT>::S*>(gate_w),
+                                                  static_cast<const Elem<TT>::S*>(proj_w), norm,
+                                                  static_cast<const Elem<TT>::S*>(table), table_stride, offset, ids, vocab,
+                                                  width, n, eps, vec));
+  return check_launch("token_side_f32");
 }
 
 extern "C" int32_t mi355_softcap(void* z, int64_t numel, float cap, int32_t dtype, void* stream) {

@@ -50,8 +50,8 @@ def _load() -> ctypes.CDLL:
         "mi355_paged_attn_decode_static": (I32, [P, P, I64, P, P, I32, P, I32, P, I32, I32, I32, I32, F, I32, I32, P]),
         "mi355_paged_attn_prefill": (I32, [P, I64, P, I64, P, P, I32, P, I32, P, P, I32, I32, I32, I32, I32,
                                            F, I32, P]),
-        "mi355_paged_attn_prefill_ext": (I32, [P, I64, P, I64, P, P, I32, P, I32, P, P, I32, I32, I32, I32, I32,
-                                               F, I32, P, P, I64, I32, P]),
+        "mi355_paged_attn_prefill_ext": (I32, [P, I64, P, I64, P, P, I32, P, I32, P, P, I32, I32, I32, I32, I32, I32,
+                                               F, I32, I32, I32, P, P, I64, F, I32, P]),
         "mi355_silu_and_mul": (I32, [P, P, I64, I64, I32, I32, P]),
         "mi355_sum_slabs": (I32, [P, I64, P, I32, P, I32, I32, I32, P]),
         "mi355_silu_and_mul_slabs": (I32, [P, I64, P, I32, I32, I32, I32, P]),
@@ -98,13 +98,13 @@ def _load() -> ctypes.CDLL:
         "mi355_allreduce_oneshot_status_async": (I32, [P, P, P]),
         "mi355_allreduce_oneshot_destroy": (I32, [P]),
         "mi355_linear_decode": (I32, [P, I64, P, I64, P, P, I32, I32, I32, I32, I32, P]),
-        "mi355_embed_scale_f32": (I32, [P, P, P, I64, I32, I64, F, I32, P]),
+        "mi355_embed_scale_f32": (I32, [P, P, P, P, I64, I32, I64, F, I32, P]),
         "mi355_embed_scale_pos_f32": (I32, [P, P, P, P, P, I64, I32, I64, I64, F, I32, P]),
         "mi355_resid_add_f32": (I32, [P, P, P, P, I64, I32, I32, P]),
         "mi355_add_rms_norm_f32": (I32, [P, P, P, P, I32, I64, I32, F, I32, P]),
         "mi355_rms_norm_mix_f32": (I32, [P, P, P, P, P, I64, I32, F, F, I32, P]),
         "mi355_gelu_tanh_and_mul": (I32, [P, P, I64, I64, I32, I32, P]),
-        "mi355_gated_head_rms_norm": (I32, [P, P, P, I64, P, I32, I64, I32, I32, F, I32, I32, P]),
+        "mi355_gated_head_rms_norm": (I32, [P, I64, P, P, I64, P, I32, I64, I32, I32, F, I32, I32, P]),
         "mi355_softcap": (I32, [P, I64, F, I32, P]),
         "mi355_rope_partial_kv_write": (I32, [P, I64, P, I64, P, I64, P, I32, P, P, P, P, I64, I32, I32, I32, I32, I32,
                                               I32, P]),
@@ -142,7 +142,20 @@ def _load() -> ctypes.CDLL:
         "mi355_qk_norm_kv_write": (I32, [P, I64, P, I64, P, I64, P, P, P, P, P, I64, I32, I32, I32, I32, F, I32, P]),
         "mi355_softmax_bias_attn_workspace": (I64, [I64, I32, I32, I32]),
         "mi355_softmax_bias_attn": (I32, [P, P, I64, P, P, P, I32, P, P, P, P, P, I64, I32, I64, I32, I32, I32, I32, I32,
-                                          I32, F, P, I32, P, I32, P, I64, I32, P]),
+                                          I32, I32, F, P, I32, P, I32, P, I64, F, I32, P]),
+        "mi355_row_norm_rope_kv_write": (I32, [P, I64, P, I64, P, I64, P, P, P, I64, P, P, P, P, I64, I32, I32, I32, I32,
+                                               I32, F, I32, P]),
+        "mi355_norm_resid_f32": (I32, [P, P, P, P, I64, I32, F, F, I32, P]),
+        "mi355_token_gate_rows": (I32, [P, P, I64, P, I64, I64, P, I64, I64, I32, I32, P]),
+        "mi355_token_side_f32": (I32, [P, P, P, P, P, P, I64, I64, P, I64, I64, I32, I32, F, I32, P]),
+        "mi355_linear_attn_state_floats": (I64, [I32, I32, I32]),
+        "mi355_linear_attn_tile_rows": (I32, [I32, I32]),
+        "mi355_mlstm_gates": (I32, [P, P, P, P, P, P, F, P, P, P, P, P, I32, I32, I32, I64, P]),
+        "mi355_linear_attn_chunks": (I32, [P, P, I64, P, I64, P, I64, F, P, P, P, P, P, P, P, P, P, P, P, I32, I32, I32, I32,
+                                           I32, I32, I64, P, I64, I32, P]),
+        "mi355_decay_attn_step": (I32, [P, P, I64, P, I64, P, I64, P, P, P, P, P, I32, I32, I32, I32, I32, P]),
+        "mi355_mlstm_step": (I32, [P, I64, P, I64, P, I64, P, I64, F, P, I64, P, P, I32, F, P, I64, P, F, P, P, P, P, P,
+                                   I32, I32, I32, I32, I32, P]),
         "mi355_mingru_scan": (I32, [P, P, I64, I32, I32, I32, P, P, P, P, P, P, I32, I64, I32, I32, P, I32, I32, P]),
         "mi355_mingru_scan_workspace": (I64, [I32, I32, I32]),
     }
@@ -186,7 +199,9 @@ EXPORTS = ("mi355_abi_version", "mi355_last_error", "mi355_target_arch",
            "mi355_moe_gate_up_rows", "mi355_moe_down_rows", "mi355_moe_silu_and_mul", "mi355_moe_combine",
            "mi355_embed_bigram_pos_f32", "mi355_prev_token_update", "mi355_relu_squared", "mi355_qk_norm_kv_write",
            "mi355_softmax_bias_attn_workspace", "mi355_softmax_bias_attn", "mi355_mingru_scan",
-           "mi355_mingru_scan_workspace")
+           "mi355_mingru_scan_workspace", "mi355_row_norm_rope_kv_write", "mi355_norm_resid_f32", "mi355_token_gate_rows",
+           "mi355_token_side_f32", "mi355_linear_attn_state_floats", "mi355_linear_attn_tile_rows", "mi355_mlstm_gates",
+           "mi355_linear_attn_chunks", "mi355_decay_attn_step", "mi355_mlstm_step")
 
 
 def check(status: int) -> None:

@@ -14,7 +14,8 @@ import os
 from dataclasses import dataclass, field
 from typing import Any, Optional
 
-SUPPORTED_ARCHS = ("LlamaForCausalLM", "Qwen2ForCausalLM", "MistralForCausalLM", "OPTForCausalLM", "Lozupel", "Tativik", "Tafisun", "Bemulorn")
+SUPPORTED_ARCHS = ("LlamaForCausalLM", "Qwen2ForCausalLM", "MistralForCausalLM", "OPTForCausalLM", "Lozupel", "Tativik", "Tafisun", "Bemulorn",
+                   "Rigazen")
 
 # Well-known geometries, used when --model names one of them and no local
 # config.json exists (synthetic-weight benchmarking; there is no network).
@@ -159,7 +160,9 @@ class BlockAttnSpec:
     longer contexts by rot_scaling; bias: q, k and v projections carry biases; sink: the softmax
     denominator holds one more term exp(sink) that carries no value; gate_per_head: the gate is one
     number per head; kv_from: the layer has no key / value projections and attends to the pages of
-    that earlier layer."""
+    that earlier layer; window > 0: the last `window` keys only, and beside them the sequence's first
+    `keep_first` keys; row_norm: queries and keys get an RMS norm over the whole projection (all heads at
+    once) with a weight of that size, ahead of the rotation."""
     heads: int
     kv_heads: int
     dim: int
@@ -176,6 +179,9 @@ class BlockAttnSpec:
     sink: Optional[float] = None
     gate_per_head: bool = False
     kv_from: Optional[int] = None
+    window: int = 0
+    keep_first: int = 0
+    row_norm: bool = False
 
 
 @dataclass(frozen=True)
@@ -212,6 +218,26 @@ class MinGRUSpec:
 
 
 @dataclass
+class DecayAttnSpec:
+    """Linear attention with a constant decay per head: S <- decay[h] S + k v^T, o = S^T q, with a silu on q,
+    k and v; the heads' outputs normed together and gated."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+
+
+@dataclass
+class MatrixMemorySpec:
+    """Matrix memory with exponential gates (mLSTM): input and forget gates from logits capped at gate_cap by a
+    tanh, a running maximum of the exponents, a normalizer state; the output normed per head and gated."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+
+@dataclass
 class BigramSpec:
     """A second embedding table indexed by a hash of the previous and the current token:
     row (prev * mul_prev + cur * mul_cur) mod buckets; the first token of a sequence takes row `buckets`."""
@@ -223,7 +249,9 @@ class BigramSpec:
 @dataclass
 class HybridLayerSpec:
     # "delta": one DeltaSpec; "parallel": window attention beside a delta mixer;
-    # "general_delta": one GeneralDeltaSpec; "latent_attention": one LatentAttnSpec
+    # "general_delta": one GeneralDeltaSpec; "latent_attention": one LatentAttnSpec;
+    # "attention": one BlockAttnSpec; "mingru": one MinGRUSpec; "mlstm": one MatrixMemorySpec;
+    # "attention_decay": a BlockAttnSpec beside a DecayAttnSpec, left_scale * one + right_scale * the other
     kind: str
     delta: DeltaSpec = None
     attn: Optional[WindowAttnSpec] = None
@@ -237,6 +265,10 @@ class HybridLayerSpec:
                                             # or "limited": g' sigmoid(1.702 g') (u' + 1), g' = min(g, ff_limit),
                                             # u' = clamp(u, -ff_limit, ff_limit)
     ff_limit: Optional[float] = None
+    lin: Optional[DecayAttnSpec] = None
+    mem: Optional[MatrixMemorySpec] = None
+    left_scale: float = 1.0
+    right_scale: float = 1.0
 
 
 @dataclass
@@ -254,7 +286,9 @@ class HybridSpec:
     # "pre": x += sublayer(norm(x)), norms with one learned number.  "sandwich": the embedding is
     # normed, and x += residual_mult * norm_b(sublayer(h) * sigmoid(Wg h + bg)) with h = norm(x);
     # every such norm is an RMS norm in norm_groups equal parts with a weight vector.  "parallel":
-    # x += mixer(h) + ff(h) with h = norm(x): one norm per layer, both sub-layers read it
+    # x += mixer(h) + ff(h) with h = norm(x): one norm per layer, both sub-layers read it.  "post":
+    # x += norm(sublayer(x)): the sub-layers read the residual itself, norm weights are stored around zero,
+    # the head is the embedding table
     arrangement: str = "pre"
     norm_groups: int = 1
     residual_mult: float = 1.0
@@ -263,6 +297,8 @@ class HybridSpec:
     sinusoid_base: float = 0.0              # > 0: sin / cos of pos * base^(-2i / width) in entries 2i / 2i + 1 is added
     learned_positions: bool = False         # a learned vector per position is added to the scaled embedding
     logit_scale: float = 1.0                # the logits are multiplied by this
+    token_side: int = 0                     # > 0: after a layer's feed-forward, x += norm(proj(gelu(gate x) * e)) with e the
+                                            # layer's token_side numbers of a second token table
 
     def runs(self):
         """[(layer index, pass number or None)] in execution order: one cache / state each."""
@@ -273,6 +309,45 @@ class HybridSpec:
         for t in range(self.loop_times):
             out += [(i, t) for i in range(self.loop_start, self.loop_stop)]
         return out + [(i, None) for i in range(self.loop_stop, n)]
+
+    @classmethod
+    def from_rigazen(cls, d: dict) -> "HybridSpec":
+        layers = []
+        for i, spec in enumerate(d["layers"]):
+            m, mlp = spec["mixer"], spec.get("mlp")
+            kw = {}
+            if mlp is not None:
+                if mlp.get("kind", "dense") != "dense":
+                    raise ValueError(f"feed-forward kind {mlp.get('kind')!r} is not supported (dense)")
+                kw.update(ff=int(mlp["ff"]), ff_act="relu2")
+            if spec["type"] == "mlstm":
+                mem = MatrixMemorySpec(int(m["heads"]), int(m["dim"]), int(m["vdim"]), float(m["gate_cap"]))
+                if mem.heads < 1 or not mem.gate_cap > 0:
+                    raise ValueError(f"layer {i}: {mem.heads} heads, gate cap {mem.gate_cap}")
+                layers.append(HybridLayerSpec("mlstm", mem=mem, **kw))
+            elif spec["type"] == "parallel":
+                a, r = m["left"], m["right"]
+                mask, rot = a.get("mask") or {}, a.get("rot") or {}
+                battn = BlockAttnSpec(heads=int(a["heads"]), kv_heads=int(a["kv_heads"]), dim=int(a["dim"]), vdim=int(a["vdim"]),
+                                      block=0, scale=float(a["scale"]), values_are_keys=False, qk_norm=False, penalty=False,
+                                      rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 10000.0)), bias=True,
+                                      window=int(mask.get("size") or 0), keep_first=int(mask.get("keep_first") or 0),
+                                      row_norm=True)
+                if battn.heads < 1 or battn.kv_heads < 1 or battn.heads % battn.kv_heads:
+                    raise ValueError(f"layer {i}: kv_heads {battn.kv_heads} must divide heads {battn.heads}")
+                if battn.rot_dims > battn.dim or battn.rot_dims % 2 or battn.window < 0 or battn.keep_first < 0:
+                    raise ValueError(f"layer {i}: {battn.rot_dims} rotated coordinates of {battn.dim}, window {battn.window}, "
+                                     f"{battn.keep_first} kept")
+                lin = DecayAttnSpec(int(r["heads"]), int(r["dim"]), int(r["vdim"]), tuple(float(x) for x in r["decay"]))
+                if lin.heads < 1 or len(lin.decay) != lin.heads or min(lin.decay) < 0:
+                    raise ValueError(f"layer {i}: decays {lin.decay} of {lin.heads} heads")
+                layers.append(HybridLayerSpec("attention_decay", battn=battn, lin=lin, left_scale=float(m.get("left_scale", 1.0)),
+                                              right_scale=float(m.get("right_scale", 1.0)), **kw))
+            else:
+                raise ValueError(f"layer type {spec['type']!r} is not supported (mlstm, parallel)")
+        return cls(layers=layers, arrangement="post", norm_vector=True,
+                   embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+                   token_side=int((d.get("token_side") or {}).get("dim", 0)))
 
     @classmethod
     def from_bemulorn(cls, d: dict) -> "HybridSpec":
@@ -503,6 +578,19 @@ class ModelConfig:
                    eos_token_id=d.get("eos_token_id"), family="hybrid", hybrid=spec)
 
     @classmethod
+    def _from_rigazen_dict(cls, d: dict) -> "ModelConfig":
+        spec = HybridSpec.from_rigazen(d)
+        att = [L.battn for L in spec.layers if L.battn is not None]
+        mixers = [m for L in spec.layers for m in (L.battn, L.lin, L.mem) if m is not None]
+        return cls(architecture="Rigazen", vocab_size=int(d["vocab"]), hidden_size=int(d["width"]),
+                   intermediate_size=max([L.ff or 0 for L in spec.layers] + [0]), num_hidden_layers=len(spec.layers),
+                   num_attention_heads=max(m.heads for m in mixers), num_key_value_heads=max([a.kv_heads for a in att] + [1]),
+                   head_dim=max(m.dim for m in mixers), rope_theta=0.0, rope_scaling=None,
+                   rms_norm_eps=float(d["norm"]["eps"]), max_position_embeddings=int(d.get("max_positions", 1 << 17)),
+                   tie_word_embeddings=True, attention_bias=True, bos_token_id=d.get("bos_token_id"),
+                   eos_token_id=d.get("eos_token_id"), family="hybrid", hybrid=spec)
+
+    @classmethod
     def _from_tativik_dict(cls, d: dict) -> "ModelConfig":
         spec = HybridSpec.from_tativik(d)
         if int(d["width"]) % spec.norm_groups:
@@ -551,9 +639,10 @@ class ModelConfig:
             cfg = cls._from_opt_dict(d)
             cfg.torch_dtype = stored
             return cfg
-        if arch in ("Lozupel", "Tativik", "Tafisun", "Bemulorn"):
+        if arch in ("Lozupel", "Tativik", "Tafisun", "Bemulorn", "Rigazen"):
             cfg = {"Lozupel": cls._from_lozupel_dict, "Tativik": cls._from_tativik_dict,
-                   "Tafisun": cls._from_tafisun_dict, "Bemulorn": cls._from_bemulorn_dict}[arch](d)
+                   "Tafisun": cls._from_tafisun_dict, "Bemulorn": cls._from_bemulorn_dict,
+                   "Rigazen": cls._from_rigazen_dict}[arch](d)
             cfg.torch_dtype = stored or "bfloat16"
             return cfg
         nh = d["num_attention_heads"]

@@ -1,5 +1,5 @@
 """One model step on one GPU for hybrid decoders (config.HybridSpec): every layer names its sequence
-mixer and may carry a feed-forward.  Two arrangements share this runner:
+mixer and may carry a feed-forward.  Four arrangements share this runner:
   * "pre" (the Lozupel design): a gated delta rule (a linear recurrence with a matrix state per
     head), or a sliding-window attention with sigmoid weights beside such a recurrence, and a dense
     gated feed-forward; a span of layers can run several times with shared weights;
@@ -18,7 +18,12 @@ mixer and may carry a feed-forward.  Two arrangements share this runner:
     of every head (frequencies blended for long contexts), a value-less term in the softmax
     denominator, one gate per head and key / value pages that a later layer may share; the
     feed-forward is a limited gated unit or a mixture whose weights are a softmax over the chosen
-    logits, plus an ungated shared expert.
+    logits, plus an ungated shared expert;
+  * "post" (the Rigazen design): the sub-layers read the residual itself and the norms sit on their outputs,
+    x += norm(mixer(x)), x += norm(ff(x)), then x += norm of a gated per-layer part of the token's own row of
+    a second table; the mixer is a softmax attention with a sliding window beside kept first tokens and a
+    linear attention with constant decays side by side, or a matrix memory with exponential gates
+    (csrc/linear_attn.hip); the head is the embedding table.
 
 What differs from ModelRunner's decoders, and where it lives:
   * the residual stream is float32 (csrc/resid32.hip: norms with one learned number or a vector,
@@ -49,11 +54,16 @@ from .model_runner import ModelRunner, batch_buckets
 from .weights import ModelWeights
 
 
-def rotary_table(rot_dims: int, base: float, max_pos: int, device, scaling=None) -> torch.Tensor:
+def rotary_table(rot_dims: int, base: float, max_pos: int, device, scaling=None, exact: bool = False) -> torch.Tensor:
     """float32 [max_pos, rot_dims] = cos | sin of pos * base^(-2i / rot_dims), i < rot_dims / 2.
     scaling (config.RotaryScaling): its blended frequencies instead, cos and sin times its factor.
-    Angles are formed in float32 from float32 frequencies."""
+    Angles are formed in float32 from float32 frequencies; exact: in float64 (no scaling), so that far
+    positions keep the angle's digits."""
     half = rot_dims // 2
+    if exact and scaling is None:
+        inv = float(base) ** (-2.0 * torch.arange(half, dtype=torch.float64, device=device) / max(rot_dims, 1))
+        ang = torch.arange(max_pos, dtype=torch.float64, device=device)[:, None] * inv[None, :]
+        return torch.cat([ang.cos(), ang.sin()], dim=1).to(torch.float32).contiguous()
     mult = 1.0
     if scaling is None:
         inv = float(base) ** (-2.0 * torch.arange(half, dtype=torch.float32, device=device) / rot_dims)
@@ -67,10 +77,11 @@ def rotary_table(rot_dims: int, base: float, max_pos: int, device, scaling=None)
 class StepBatch:
     """Device-side description of one packed step (see csrc/seqmix.hip)."""
     __slots__ = ("ids", "positions", "slot_mapping", "block_tables", "cu_seqlens", "tok_seq", "state_slots",
-                 "num_tokens", "num_seqs", "tiles", "long_chunks", "pair_tiles", "context_lens", "max_q_len")
+                 "num_tokens", "num_seqs", "tiles", "long_chunks", "pair_tiles", "context_lens", "max_q_len", "row_tiles")
 
     def __init__(self, ids, positions, slot_mapping, block_tables, cu_seqlens, tok_seq, state_slots, tiles=None,
-                 long_chunks=False, pair_tiles=None, context_lens=None, max_q_len=0):
+                 long_chunks=False, pair_tiles=None, context_lens=None, max_q_len=0, row_tiles=None):
+        self.row_tiles = row_tiles                    # rows -> ops.RowTiles of the step, or None (captured decode steps)
         # every chunk's length of context after the step (int32, on the device) and the longest chunk: what the
         # LDS-staged prompt attention walks by; None: not known to this step (captured decode steps)
         self.context_lens, self.max_q_len = context_lens, int(max_q_len)
@@ -231,6 +242,66 @@ class RotaryBlockAttention:
                                               s.kv_heads, s.dim, s.scale, chunk=s.block, sink=lw.sink, gate=col("g"), out=out)
         return ops.softmax_bias_attn(q, kc, vc, b.block_tables, b.tok_seq, b.positions, None, None, col("g"), s.heads, s.scale,
                                      block=s.block, tiles=b.tiles, num_splits=r.block_key_splits(b, s), sink=lw.sink, out=out)
+
+
+class AttentionBesideDecay:
+    """A softmax attention over the paged K/V of one layer run (sliding window beside the sequence's first
+    tokens; queries and keys normed over their whole rows, then rotated) and a linear attention with
+    constant decays on its state slots, both on the same projections.  The two write side by side into the
+    row that the layer's one output matrix multiplies, each times its scale."""
+
+    STEP_MAX = 4                     # chunks of up to this many tokens go token by token
+
+    def __init__(self, spec, lw, runner, cache_index: int, state_index: int):
+        self.a, self.d, self.scale = spec.battn, spec.lin, spec.left_scale
+        self.lw, self.r, self.ci, self.si = lw, runner, cache_index, state_index
+        self.tile_rows = ops.linear_attn_tile_rows(self.d.dim, self.d.vdim)
+
+    def __call__(self, proj: torch.Tensor, resid: torch.Tensor, b: StepBatch) -> torch.Tensor:
+        a, d, lw, r = self.a, self.d, self.lw, self.r
+        col = lambda n: proj[:, lw.seg[n][0]: lw.seg[n][0] + lw.seg[n][1]]     # noqa: E731
+        n1, at, K = a.heads * a.vdim, lw.out_w.shape[1] - d.heads * d.vdim, lw.out_w.shape[1]
+        row = (torch.zeros if at != n1 else torch.empty)(proj.shape[0], K, dtype=proj.dtype, device=proj.device)
+        q, kc, vc = col("lq"), r.k_cache[self.ci], r.v_cache[self.ci]
+        ops.row_norm_rope_kv_write(q, col("lk"), col("lv"), lw.q_norm, lw.k_norm, r.rotary(a.rot_dims, a.rot_base, exact=True),
+                                   b.positions, b.slot_mapping, kc, vc, a.heads, a.kv_heads, a.dim, a.vdim, r.eps)
+        if b.long_chunks and b.context_lens is not None and ops.chunk_attn_prefill_ok(q.dtype, a.heads, a.kv_heads, a.dim, a.vdim) \
+                and proj.stride(0) % 8 == 0 and K % 8 == 0:
+            ops.paged_attn_prefill_ext(q, kc, vc, b.block_tables, b.cu_seqlens, b.context_lens, b.max_q_len, a.heads, a.kv_heads,
+                                       a.dim, a.scale, window=a.window, keep=a.keep_first, out_scale=self.scale, out=row[:, :n1])
+        else:
+            ops.softmax_bias_attn(q, kc, vc, b.block_tables, b.tok_seq, b.positions, None, None, None, a.heads, a.scale,
+                                  window=a.window, keep=a.keep_first, out_scale=self.scale, tiles=b.tiles,
+                                  num_splits=r.block_key_splits(b, a), out=row[:, :n1])
+        tiles = b.row_tiles(self.tile_rows) if b.row_tiles is not None and b.max_q_len > self.STEP_MAX else None
+        o = ops.decay_attn(col("q"), col("k"), col("v"), lw.log_decay, r.rec_state[self.si], b.cu_seqlens, b.positions,
+                           b.state_slots, d.heads, d.dim, d.vdim, tiles=tiles)
+        ops.gated_head_rms_norm(o.view(o.shape[0], 1, -1), col("g"), lw.head_norm, r.eps, ops.ACT_SIGMOID, out=row[:, at:])
+        return row
+
+
+class MatrixMemory:
+    """Matrix memory with exponential gates on one layer run's state slots, normed per head and gated.  The
+    gates read the float32 residual."""
+
+    STEP_MAX = 4
+
+    def __init__(self, spec, lw, runner, state_index: int):
+        self.s, self.lw, self.r, self.si = spec, lw, runner, state_index
+        self.tile_rows = ops.linear_attn_tile_rows(spec.dim, spec.vdim)
+
+    def __call__(self, proj: torch.Tensor, resid: torch.Tensor, b: StepBatch) -> torch.Tensor:
+        s, lw, r = self.s, self.lw, self.r
+        col = lambda n: proj[:, lw.seg[n][0]: lw.seg[n][0] + lw.seg[n][1]]     # noqa: E731
+        state, m_state = r.rec_state[self.si], r.max_state[self.si]
+        if b.row_tiles is None or b.max_q_len <= self.STEP_MAX:
+            return ops.mlstm_step(col("q"), col("k"), col("v"), s.dim ** -0.5, resid, lw.gate_w, lw.gate_b, s.gate_cap, col("g"),
+                                  lw.head_norm, r.eps, state, m_state, b.cu_seqlens, b.positions, b.state_slots, s.heads, s.dim,
+                                  s.vdim)
+        o = ops.mlstm_chunks(col("q"), col("k"), col("v"), s.dim ** -0.5, torch.mm(resid, lw.gate_w32.t()), lw.gate_b, s.gate_cap,
+                             state, m_state, b.cu_seqlens, b.positions, b.state_slots, s.heads, s.dim, s.vdim,
+                             b.row_tiles(self.tile_rows))
+        return ops.gated_head_rms_norm(o, col("g"), lw.head_norm, r.eps, ops.ACT_SIGMOID)
 
 
 class MinGRUMixer:
@@ -410,6 +481,24 @@ class HybridRunner(ModelRunner):
             self.mixers.append(RotaryBlockAttention(A, lw, self, pages_of[li if A.kv_from is None else A.kv_from],
                                                     A.kv_from is None))
             self.ffs.append(MoEFeedForward(L.moe, lw, self) if L.moe is not None else None)
+        self.max_state = {}                             # index into rec_state -> running maxima of a matrix memory [slots + 1, heads]
+        for li, _ in self.runs if spec.arrangement == "post" else ():
+            L, lw = spec.layers[li], weights.layers[li]
+            D = L.mem if L.mem is not None else L.lin
+            if ops.linear_attn_tile_rows(D.dim, D.vdim) == 0:
+                raise ValueError(f"layer {li}: linear attention heads of {D.dim} x {D.vdim} are too large")
+            self.rec_state.append(torch.zeros(self.num_state_slots + 1, D.heads,
+                                              ops.linear_attn_state_floats(D.dim, D.vdim, L.mem is not None),
+                                              dtype=torch.float32, device=dev))
+            si = len(self.rec_state) - 1
+            if L.mem is not None:
+                self.max_state[si] = torch.zeros(self.num_state_slots + 1, D.heads, dtype=torch.float32, device=dev)
+                self.mixers.append(MatrixMemory(D, lw, self, si))
+                continue
+            A = L.battn
+            self.k_cache.append(torch.zeros(self.num_blocks, A.kv_heads, BLOCK_SIZE, A.dim, dtype=dtype, device=dev))
+            self.v_cache.append(torch.zeros(self.num_blocks, A.kv_heads, A.vdim, BLOCK_SIZE, dtype=dtype, device=dev))
+            self.mixers.append(AttentionBesideDecay(L, lw, self, len(self.k_cache) - 1, si))
         for li, _ in self.runs if spec.arrangement == "pre" else ():
             L, lw = spec.layers[li], weights.layers[li]
             self.ffs.append(MoEFeedForward(L.moe, lw, self) if L.moe is not None else
@@ -451,7 +540,8 @@ class HybridRunner(ModelRunner):
         # the samplers want 16-byte aligned logit rows: the head is padded with zero rows to a multiple
         # of 8 and the logits are the first V columns of what it yields
         self.Vp = -(-self.V // 8) * 8
-        self._forward = {"sandwich": self._forward_sandwich, "parallel": self._forward_parallel}.get(spec.arrangement,
+        self._forward = {"sandwich": self._forward_sandwich, "parallel": self._forward_parallel,
+                         "post": self._forward_post}.get(spec.arrangement,
                                                                                                      self._forward_pre)
         self.head_w = weights.lm_head
         if self.Vp != self.V:
@@ -472,13 +562,14 @@ class HybridRunner(ModelRunner):
         self._attn_partial = torch.empty(max(self.MAX_KEY_SPLITS * B * widest, 4), dtype=torch.float32, device=dev)
         self.layer_trace = None                       # a list: _forward appends the residual after every layer run
         self._pair_tiles = {}                         # of the step at hand: heads -> device tiles
+        self._row_tiles = {}                          # of the step at hand: rows -> ops.RowTiles
         self._dec_pairs = {}                          # of a decode step of max_num_seqs rows: heads -> device tiles
 
     # ------------------------------------------------------------------ #
-    def rotary(self, rot_dims: int, base: float, scaling=None) -> torch.Tensor:
-        key = (rot_dims, base, scaling)
+    def rotary(self, rot_dims: int, base: float, scaling=None, exact: bool = False) -> torch.Tensor:
+        key = (rot_dims, base, scaling, exact)
         if key not in self._rotary:
-            self._rotary[key] = rotary_table(rot_dims, base, self.max_blocks * BLOCK_SIZE, self.device, scaling)
+            self._rotary[key] = rotary_table(rot_dims, base, self.max_blocks * BLOCK_SIZE, self.device, scaling, exact)
         return self._rotary[key]
 
     def _decode_pair_tiles(self, heads: int) -> torch.Tensor:
@@ -493,6 +584,11 @@ class HybridRunner(ModelRunner):
         if heads not in self._pair_tiles:
             self._pair_tiles[heads] = torch.from_numpy(ops.pair_tiles(self._step_cu, heads)).to(self.device, non_blocking=True)
         return self._pair_tiles[heads]
+
+    def _chunk_row_tiles(self, rows: int) -> ops.RowTiles:
+        if rows not in self._row_tiles:
+            self._row_tiles[rows] = ops.RowTiles(self._step_cu, rows, self.device)
+        return self._row_tiles[rows]
 
     MAX_KEY_SPLITS = 16
 
@@ -518,6 +614,8 @@ class HybridRunner(ModelRunner):
         hb = 4 if rep % 4 == 0 else 3 if rep % 3 == 0 else 2 if rep % 2 == 0 else 1
         waves = int(b.tiles.shape[0]) * a.kv_heads * (rep // hb)
         span = a.block if a.block > 0 else self.max_model_len
+        if a.window > 0:
+            span = min(span, a.window + a.keep_first)
         # about a wave per SIMD: every further split costs its fp32 partial sums and their merge (measured: a
         # 2048-token prompt of 16 heads 203 / 117 / 130 / 161 us with 1 / 2 / 4 / 8 splits, 32 decoded rows
         # 148 / 83 / 51 / 36 / 43 us with 1 / 2 / 4 / 8 / 16)
@@ -529,7 +627,7 @@ class HybridRunner(ModelRunner):
         return sum(t[0].numel() * t.element_size() for t in pages)
 
     def state_bytes_per_slot(self) -> int:
-        return sum(t[0].numel() * t.element_size() for t in self.conv_state + self.rec_state) \
+        return sum(t[0].numel() * t.element_size() for t in self.conv_state + self.rec_state + list(self.max_state.values())) \
             + (4 if self.prev_tokens is not None else 0)
 
     def _init_tiled_copies(self, want: Optional[bool]) -> None:
@@ -700,10 +798,39 @@ class HybridRunner(ModelRunner):
                 self.layer_trace.append(resid.clone())
         return resid
 
+    SIDE_FUSED_ROWS = 64             # steps of up to this many rows take the per-layer token input in one launch
+
+    def _forward_post(self, b: StepBatch) -> torch.Tensor:
+        """All layers of the post arrangement over one packed batch; returns the float32 residual stream
+        [tokens, width].  Beside the residual its copy in the activation type is kept up to date by the
+        launches that add to the residual: the products read it."""
+        w, spec, eps, n = self.w, self.spec, self.eps, self.spec.token_side
+        T = b.num_tokens
+        act = None if self.dtype == torch.float32 else torch.empty(T, self.H, dtype=self.dtype, device=self.device)
+        resid = ops.embed_scale_f32(w.embed, b.ids, spec.embed_scale, act_out=act)
+        x = resid if act is None else act
+        for ri, (li, _) in enumerate(self.runs):
+            L, lw = spec.layers[li], w.layers[li]
+            row = self.mixers[ri](self.linear(x, lw.in_w, bias=lw.in_b), resid, b)
+            ops.norm_resid_f32(resid, self.linear(row, lw.out_w), lw.norm1, eps, act_out=act)
+            if L.ff:
+                y = self.linear(ops.relu_squared(self.linear(x, lw.up_w)), lw.down_w)
+                ops.norm_resid_f32(resid, y, lw.norm2, eps, act_out=act)
+            if n and T <= self.SIDE_FUSED_ROWS and self.H <= 8192 and n <= 4096:
+                ops.token_side_f32(resid, lw.side_gate_w, lw.side_proj_w, lw.side_norm, w.side_embed, li * n, b.ids, eps, act_out=act)
+            elif n:
+                g = ops.token_gate_rows(self.linear(x, lw.side_gate_w), w.side_embed, li * n, b.ids)
+                ops.norm_resid_f32(resid, self.linear(g, lw.side_proj_w), lw.side_norm, eps, act_out=act)
+            if self.layer_trace is not None:
+                self.layer_trace.append(resid.clone())
+        return resid
+
     def _logits(self, resid: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Final norm, head and soft cap over the given residual rows."""
         if self.spec.arrangement == "sandwich":
             h = ops.group_rms_norm_f32(resid, self.w.final_norm, self.spec.norm_groups, self.eps, dtype=self.dtype)
+        elif self.spec.arrangement == "post":
+            h = ops.group_rms_norm_f32(resid, self.w.final_norm, 1, self.eps, dtype=self.dtype)
         else:
             h = ops.add_rms_norm_f32(resid, self.w.final_norm, self.eps)
         z = self.linear(h, self.head_w, out=out)
@@ -733,7 +860,7 @@ class HybridRunner(ModelRunner):
         self._step_state_slots = np.asarray(state_slots, dtype=np.int32)
         # rows go to the matrix cores in tiles of up to 16 rows of one chunk
         self._step_tiles = ops.query_tiles(cu_seqlens)
-        self._step_cu, self._pair_tiles = np.asarray(cu_seqlens, dtype=np.int64), {}
+        self._step_cu, self._pair_tiles, self._row_tiles = np.asarray(cu_seqlens, dtype=np.int64), {}, {}
         self._step_long = int(max_q_len) > 1
         if logit_rows is None:
             return super().run_prefill(token_ids, positions, slot_mapping, block_tables, cu_seqlens, context_lens,
@@ -761,7 +888,7 @@ class HybridRunner(ModelRunner):
         return self._forward(StepBatch(token_ids, positions, slot_mapping, block_tables.contiguous(), cu_seqlens,
                                        tok_seq, slots, tiles, self._step_long, pair_tiles=self._chunk_pair_tiles,
                                        context_lens=None if context_lens is None else context_lens.to(torch.int32).contiguous(),
-                                       max_q_len=max_q_len))
+                                       max_q_len=max_q_len, row_tiles=self._chunk_row_tiles))
 
     def prefill(self, token_ids: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Tensor,
                 block_tables: torch.Tensor, cu_seqlens: torch.Tensor, context_lens: torch.Tensor,

@@ -289,38 +289,49 @@ def paged_attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Te
 
 
 def chunk_attn_prefill_ok(dtype: torch.dtype, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int) -> bool:
-    """Whether paged_attn_prefill_ext covers these sizes (16-bit storage, equal key and value sizes of 64 or 128,
+    """Whether paged_attn_prefill_ext covers these sizes (16-bit storage, key and value sizes of 64 or 128,
     at most 16 query heads to a kv head)."""
-    return dtype in (torch.bfloat16, torch.float16) and head_dim == v_dim and head_dim in (64, 128) \
+    return dtype in (torch.bfloat16, torch.float16) and v_dim in (64, 128) and head_dim in (64, 128) \
         and num_heads % num_kv_heads == 0 and num_heads // num_kv_heads <= 16
 
 
 def paged_attn_prefill_ext(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
                            cu_seqlens: torch.Tensor, context_lens: torch.Tensor, max_q_len: int, num_heads: int,
                            num_kv_heads: int, head_dim: int, scale: float, chunk: int = 0, sink: torch.Tensor | None = None,
-                           gate: torch.Tensor | None = None, out: torch.Tensor | None = None):
+                           gate: torch.Tensor | None = None, out: torch.Tensor | None = None, window: int = 0,
+                           keep: int = 0, out_scale: float = 1.0):
     """paged_attn_prefill (K/V steps staged through LDS for a workgroup's query tile) for attention inside
     chunks of `chunk` positions counted from position 0 (0: plain causal), with one more value-less term
     exp(sink[h]) in the softmax denominator (float32 [heads]) and the output times sigmoid(gate[t, h])
-    (gate [tokens, heads], a column slice is fine).  q and out may be column slices on 16-byte boundaries."""
+    (gate [tokens, heads], a column slice is fine).  window > 0: the last `window` keys only, and (chunk 0) the
+    first `keep` keys of the sequence.  The output is multiplied by out_scale.  q and out may be column
+    slices on 16-byte boundaries; the value size (V pages [blocks, kv_heads, v_dim, 16]) may differ from
+    the key size."""
     dt = _dt16(q, "q")
     T = q.shape[0]
-    nb = _check_cache(q, k_cache, v_cache, block_tables, num_kv_heads, head_dim)
+    nb, dv = k_cache.shape[0], v_cache.shape[2]
+    for t, n, shape in ((k_cache, "k_cache", (nb, num_kv_heads, BLOCK_SIZE, head_dim)),
+                        (v_cache, "v_cache", (nb, num_kv_heads, dv, BLOCK_SIZE))):
+        _same(t, q, n)
+        if tuple(t.shape) != shape or not t.is_contiguous():
+            raise ValueError(f"{n} must be contiguous {shape}")
+    if block_tables.dim() != 2 or block_tables.dtype != torch.int32 or not block_tables.is_contiguous():
+        raise ValueError("block_tables must be contiguous int32 [sequences, max_blocks]")
     S = block_tables.shape[0]
     for t, n, cnt in ((cu_seqlens, "cu_seqlens", S + 1), (context_lens, "context_lens", S)):
         _dev(t, n)
         if t.dtype != torch.int32 or t.numel() != cnt or not t.is_contiguous():
             raise ValueError(f"{n} must be contiguous int32 [{cnt}]")
     if out is None:
-        out = torch.empty((T, num_heads * head_dim), dtype=q.dtype, device=q.device)
-    if out.dtype != q.dtype or tuple(out.shape) != (T, num_heads * head_dim):
-        raise ValueError("out must be [tokens, heads * head_dim] in the dtype of q")
+        out = torch.empty((T, num_heads * dv), dtype=q.dtype, device=q.device)
+    if out.dtype != q.dtype or tuple(out.shape) != (T, num_heads * dv):
+        raise ValueError("out must be [tokens, heads * v_dim] in the dtype of q")
     check(lib.mi355_paged_attn_prefill_ext(
         out.data_ptr(), _rows(out, "out"), q.data_ptr(), _cols(q, "q", num_heads * head_dim), k_cache.data_ptr(),
         v_cache.data_ptr(), nb, block_tables.data_ptr(), block_tables.shape[1], cu_seqlens.data_ptr(), context_lens.data_ptr(),
-        S, int(max_q_len), num_heads, num_kv_heads, head_dim, float(scale), int(chunk),
+        S, int(max_q_len), num_heads, num_kv_heads, head_dim, dv, float(scale), int(chunk), int(window), int(keep),
         None if sink is None else _f32(sink, "sink", num_heads), None if gate is None else _same(gate, q, "gate"),
-        0 if gate is None else _cols(gate, "gate", num_heads), dt, _stream()))
+        0 if gate is None else _cols(gate, "gate", num_heads), float(out_scale), dt, _stream()))
     return out
 
 
@@ -987,15 +998,26 @@ def _same(t: torch.Tensor, ref: torch.Tensor, name: str) -> int:
     return t.data_ptr()
 
 
-def embed_scale_f32(embed: torch.Tensor, ids: torch.Tensor, scale: float, out: torch.Tensor | None = None):
-    """out[t] = embed[ids[t]] * scale as float32 rows."""
+def _act_rows(act: torch.Tensor | None, dtype: torch.dtype, T: int, W: int):
+    """Pointer of an optional activation copy of residual rows."""
+    if act is None:
+        return None
+    _dev(act, "act_out")
+    if act.dtype != dtype or tuple(act.shape) != (T, W) or not act.is_contiguous():
+        raise ValueError(f"act_out must be contiguous [{T}, {W}] in {dtype}")
+    return act.data_ptr()
+
+
+def embed_scale_f32(embed: torch.Tensor, ids: torch.Tensor, scale: float, out: torch.Tensor | None = None,
+                    act_out: torch.Tensor | None = None):
+    """out[t] = embed[ids[t]] * scale as float32 rows; act_out: the same rows in embed's dtype as well."""
     dt = _dt3(embed, "embed")
     if embed.dim() != 2 or not embed.is_contiguous():
         raise ValueError("embed must be contiguous [vocab, width]")
     T, W = ids.numel(), embed.shape[1]
     if out is None:
         out = torch.empty(T, W, dtype=torch.float32, device=embed.device)
-    check(lib.mi355_embed_scale_f32(_f32(out, "out", T * W), embed.data_ptr(), _idx(ids, "ids", torch.int64), T, W,
+    check(lib.mi355_embed_scale_f32(_f32(out, "out", T * W), _act_rows(act_out, embed.dtype, T, W), embed.data_ptr(), _idx(ids, "ids", torch.int64), T, W,
                                     embed.shape[0], float(scale), dt, _stream()))
     return out
 
@@ -1088,7 +1110,7 @@ def gated_head_rms_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tenso
                         out: torch.Tensor | None = None):
     """o float32 [tokens, heads, dim]; gate [tokens, >= heads * dim] (a column slice is fine);
     weight float32 [dim] (shared by the heads) or [heads * dim].  Returns o / rms(o) * weight * act(gate)
-    as [tokens, heads * dim] in gate's dtype."""
+    as [tokens, heads * dim] in gate's dtype (out: a column slice is fine)."""
     T, H, D = o.shape
     wh = H if weight.numel() == H * D and H > 1 else 1
     dt = _dt3(gate, "gate")
@@ -1096,7 +1118,9 @@ def gated_head_rms_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tenso
         raise ValueError("gate must be [tokens, heads * dim] with a contiguous last dim")
     if out is None:
         out = torch.empty(T, H * D, dtype=gate.dtype, device=o.device)
-    check(lib.mi355_gated_head_rms_norm(out.data_ptr(), _f32(o, "o"), gate.data_ptr(), gate.stride(0) if T > 1 else H * D,
+    if out.dtype != gate.dtype:
+        raise TypeError("out must be in the dtype of gate")
+    check(lib.mi355_gated_head_rms_norm(out.data_ptr(), _cols(out, "out", H * D), _f32(o, "o"), gate.data_ptr(), gate.stride(0) if T > 1 else H * D,
                                         _f32(weight, "weight", wh * D), wh, T, H, D, float(eps), int(activation), dt,
                                         _stream()))
     return out
@@ -1182,15 +1206,15 @@ def sigmoid_window_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.T
     return out
 
 
-def query_tiles(cu_seqlens) -> "np.ndarray":
-    """(chunk, first packed row, rows <= 16) for every 16-row tile of a packed batch, from the host
-    copy of cu_seqlens: the work list of the matrix-core window attention."""
+def query_tiles(cu_seqlens, rows: int = 16) -> "np.ndarray":
+    """(chunk, first packed row, number of rows <= rows) for every tile of `rows` rows of a packed batch, from
+    the host copy of cu_seqlens: the work list of the matrix-core attentions and of the tiled linear attention."""
     import numpy as np
     cu = np.asarray(cu_seqlens, dtype=np.int64)
     out = []
     for s in range(len(cu) - 1):
-        for a in range(int(cu[s]), int(cu[s + 1]), 16):
-            out.append((s, a, min(16, int(cu[s + 1]) - a)))
+        for a in range(int(cu[s]), int(cu[s + 1]), rows):
+            out.append((s, a, min(rows, int(cu[s + 1]) - a)))
     return np.asarray(out, dtype=np.int32).reshape(-1, 3)
 
 
@@ -1673,10 +1697,11 @@ def softmax_bias_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
                       tok_seq: torch.Tensor, positions: torch.Tensor, r1: torch.Tensor | None, r2: torch.Tensor | None,
                       gate: torch.Tensor | None, num_heads: int, scale: float, block: int = 0, window: int = 0,
                       tiles: torch.Tensor | None = None, num_splits: int = 0, sink: torch.Tensor | None = None,
-                      out: torch.Tensor | None = None):
+                      out: torch.Tensor | None = None, keep: int = 0, out_scale: float = 1.0):
     """Softmax attention over the paged K/V [blocks, kv_heads, 16, dim] / [blocks, kv_heads, vdim, 16] with
     the score q.k * scale - r1[h] ln(1 + r2[h] * distance); a row at position p sees the keys j <= p of
-    its block of `block` positions (0: all) and, window > 0, the last `window` of them.  gate
+    its block of `block` positions (0: all) and, window > 0, the last `window` of them and (block 0) the
+    sequence's first `keep`.  The output is multiplied by out_scale.  gate
     [tokens, heads] or [tokens, heads * vdim]: the output is multiplied by its sigmoid.  tiles
     (query_tiles) selects the matrix-core form where the sizes allow; num_splits > 1 spreads a
     tile's keys over that many workgroups.  sink (float32 [heads]): the softmax denominator holds one
@@ -1707,10 +1732,10 @@ def softmax_bias_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
         _idx(block_tables, "block_tables", torch.int32), block_tables.shape[1], _idx(tok_seq, "tok_seq", torch.int32, T),
         _idx(positions, "positions", torch.int64, T), None if r1 is None else _f32(r1, "r1", num_heads),
         None if r2 is None else _f32(r2, "r2", num_heads), None if gate is None else _same(gate, q, "gate"), gs, per_channel,
-        T, num_heads, G, d, dv, int(block), int(window), float(scale),
+        T, num_heads, G, d, dv, int(block), int(window), int(keep), float(scale),
         None if tiles is None else _idx(tiles, "tiles", torch.int32), 0 if tiles is None else tiles.shape[0],
         None if ws is None else ws.data_ptr(), n, None if sink is None else _f32(sink, "sink", num_heads),
-        _cols(out, "out", num_heads * dv), dt, _stream()))
+        _cols(out, "out", num_heads * dv), float(out_scale), dt, _stream()))
     return out
 
 
@@ -1741,3 +1766,179 @@ def mingru_scan(proj: torch.Tensor, z_off: int, x_off: int, g_off: int, channels
         _idx(state_slots, "state_slots", torch.int32, S), S, T, int(channels), int(bool(long_chunks)),
         None if ws is None else ws.data_ptr(), num_parts, dt, _stream()))
     return out
+
+
+# ---- norms on the sub-layers' outputs, per-layer token inputs, linear attention with scalar decays
+def norm_resid_f32(resid: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, y_scale: float = 1.0,
+                   act_out: torch.Tensor | None = None):
+    """resid (float32, in place) += rms(y * y_scale) * weight (float32 [width]); act_out: the new residual in
+    y's dtype."""
+    T, W = resid.shape
+    dt = _dt3(y, "y")
+    if tuple(y.shape) != (T, W) or not y.is_contiguous():
+        raise ValueError("y must be contiguous, shaped like resid")
+    check(lib.mi355_norm_resid_f32(_f32(resid, "resid"), _act_rows(act_out, y.dtype, T, W), y.data_ptr(),
+                                   _f32(weight, "weight", W), T, W, float(eps), float(y_scale), dt, _stream()))
+    return resid
+
+
+def token_gate_rows(z: torch.Tensor, table: torch.Tensor, offset: int, ids: torch.Tensor):
+    """gelu_tanh(z[t]) * table[ids[t], offset : offset + n] for z [tokens, n] (a column slice is fine)."""
+    dt = _dt3(z, "z")
+    T, n = z.shape
+    if table.dim() != 2 or table.stride(1) != 1 or table.shape[1] < offset + n:
+        raise ValueError("table must be [vocab, columns] with contiguous rows that hold the columns asked for")
+    out = torch.empty(T, n, dtype=z.dtype, device=z.device)
+    check(lib.mi355_token_gate_rows(out.data_ptr(), z.data_ptr(), _cols(z, "z", n), _same(table, z, "table"), table.stride(0),
+                                    int(offset), _idx(ids, "ids", torch.int64, T), table.shape[0], T, n, dt, _stream()))
+    return out
+
+
+def token_side_f32(resid: torch.Tensor, gate_w: torch.Tensor, proj_w: torch.Tensor, norm: torch.Tensor, table: torch.Tensor,
+                   offset: int, ids: torch.Tensor, eps: float, act_out: torch.Tensor | None = None):
+    """resid (float32, in place) += rms(proj_w (gelu_tanh(gate_w resid) * table[ids, offset : offset + n])) * norm in
+    one launch, a workgroup per row: for steps of few rows.  act_out: the new residual in gate_w's dtype."""
+    T, W = resid.shape
+    dt = _dt3(gate_w, "gate_w")
+    n = gate_w.shape[0]
+    if tuple(gate_w.shape) != (n, W) or tuple(proj_w.shape) != (W, n) or not gate_w.is_contiguous() or not proj_w.is_contiguous():
+        raise ValueError("gate_w must be contiguous [n, width] and proj_w [width, n]")
+    if table.dim() != 2 or table.stride(1) != 1 or table.shape[1] < offset + n:
+        raise ValueError("table must be [vocab, columns] with contiguous rows that hold the columns asked for")
+    check(lib.mi355_token_side_f32(_f32(resid, "resid"), _act_rows(act_out, gate_w.dtype, T, W), gate_w.data_ptr(),
+                                   _same(proj_w, gate_w, "proj_w"), _f32(norm, "norm", W), _same(table, gate_w, "table"),
+                                   table.stride(0), int(offset), _idx(ids, "ids", torch.int64, T), table.shape[0], T, W, n,
+                                   float(eps), dt, _stream()))
+    return resid
+
+
+def row_norm_rope_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, q_weight: torch.Tensor, k_weight: torch.Tensor,
+                           cos_sin: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Tensor, k_cache: torch.Tensor,
+                           v_cache: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, eps: float):
+    """q [tokens, heads * dim] is RMS-normed as one row, weighted (float32 [heads * dim]) and rotated in place by
+    the float32 table cos_sin [max_pos, rot_dims]; k likewise into the K pages, v as given into the V pages.
+    q / k / v may be column slices."""
+    dt = _dt3(q, "q")
+    T, rot = q.shape[0], cos_sin.shape[1]
+    for t, n, shape in ((k_cache, "k_cache", (num_kv_heads, BLOCK_SIZE, head_dim)), (v_cache, "v_cache", (num_kv_heads, v_dim, BLOCK_SIZE))):
+        if tuple(t.shape[1:]) != shape or not t.is_contiguous():
+            raise ValueError(f"{n} must be contiguous [blocks, {', '.join(map(str, shape))}]")
+    check(lib.mi355_row_norm_rope_kv_write(
+        q.data_ptr(), _cols(q, "q", num_heads * head_dim), _same(k, q, "k"), _cols(k, "k", num_kv_heads * head_dim),
+        _same(v, q, "v"), _cols(v, "v", num_kv_heads * v_dim), _f32(q_weight, "q_weight", num_heads * head_dim),
+        _f32(k_weight, "k_weight", num_kv_heads * head_dim), _f32(cos_sin, "cos_sin") if rot else None, cos_sin.shape[0],
+        _idx(positions, "positions", torch.int64, T), _idx(slot_mapping, "slot_mapping", torch.int64, T),
+        _same(k_cache, q, "k_cache"), _same(v_cache, q, "v_cache"), T, num_heads, num_kv_heads, head_dim, v_dim, rot, float(eps),
+        dt, _stream()))
+
+
+def linear_attn_state_floats(dim: int, vdim: int, normalizer: bool) -> int:
+    """float32 numbers of one head's state: S [dim, vdim], then (normalizer) n [dim], padded to a multiple of 4."""
+    return int(lib.mi355_linear_attn_state_floats(int(dim), int(vdim), int(normalizer)))
+
+
+def linear_attn_tile_rows(dim: int, vdim: int) -> int:
+    """Rows of a tile of the tiled linear attention for heads of these sizes; 0: too large."""
+    return int(lib.mi355_linear_attn_tile_rows(int(dim), int(vdim)))
+
+
+class RowTiles:
+    """Tiles of up to `rows` rows of every chunk of a packed batch, and every chunk's first tile: int32 tensors
+    on the device, made from the host copy of cu_seqlens."""
+
+    def __init__(self, cu_seqlens, rows: int, device):
+        import numpy as np
+        cu = np.asarray(cu_seqlens, dtype=np.int64)
+        t = query_tiles(cu, rows)
+        start = np.concatenate([[0], np.cumsum(-(-(cu[1:] - cu[:-1]) // rows))]).astype(np.int32)
+        self.rows, self.count = int(rows), int(t.shape[0])
+        self.tiles = torch.from_numpy(t).to(device, non_blocking=True)
+        self.start = torch.from_numpy(start).to(device, non_blocking=True)
+
+
+def _linear_attn_state(state: torch.Tensor, H: int, dim: int, vdim: int, normalizer: bool) -> int:
+    n = linear_attn_state_floats(dim, vdim, normalizer)
+    if state.dim() != 3 or tuple(state.shape[1:]) != (H, n):
+        raise ValueError(f"state must be float32 [slots, {H}, {n}]")
+    return _f32(state, "state")
+
+
+def decay_attn(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, log_decay: torch.Tensor, state: torch.Tensor,
+               cu_seqlens: torch.Tensor, positions: torch.Tensor, state_slots: torch.Tensor, num_heads: int, dim: int, vdim: int,
+               tiles: RowTiles | None = None):
+    """Linear attention with a constant decay per head: S <- exp(log_decay[h]) S + k v^T, o = S^T q, where q, k
+    [tokens, heads * dim] and v [tokens, heads * vdim] go through silu (column slices are fine); log_decay
+    float64 [heads].  state float32 [slots, heads, linear_attn_state_floats(dim, vdim, False)].  tiles: the
+    tiled form for chunks of many tokens; None: token by token.  Returns o float32 [tokens, heads, vdim]."""
+    dt = _dt3(q, "q")
+    T, S = q.shape[0], cu_seqlens.numel() - 1
+    if log_decay.dtype != torch.float64 or log_decay.numel() != num_heads or not log_decay.is_contiguous() or not log_decay.is_cuda:
+        raise ValueError("log_decay must be a contiguous float64 [heads] tensor on the GPU")
+    o = torch.empty(T, num_heads, vdim, dtype=torch.float32, device=q.device)
+    rows = (q.data_ptr(), _cols(q, "q", num_heads * dim), _same(k, q, "k"), _cols(k, "k", num_heads * dim),
+            _same(v, q, "v"), _cols(v, "v", num_heads * vdim))
+    chunk = (_idx(cu_seqlens, "cu_seqlens", torch.int32), _idx(positions, "positions", torch.int64, T),
+             _idx(state_slots, "state_slots", torch.int32, S))
+    sp = _linear_attn_state(state, num_heads, dim, vdim, False)
+    if tiles is None:
+        check(lib.mi355_decay_attn_step(o.data_ptr(), *rows, log_decay.data_ptr(), sp, *chunk, S, num_heads, dim, vdim, dt, _stream()))
+        return o
+    ws = torch.empty(tiles.count * num_heads * state.shape[2], dtype=torch.float32, device=q.device)
+    check(lib.mi355_linear_attn_chunks(o.data_ptr(), *rows, 1.0, log_decay.data_ptr(), None, None, None, None, sp, *chunk,
+                                       tiles.tiles.data_ptr(), tiles.start.data_ptr(), tiles.count, tiles.rows, S, num_heads,
+                                       dim, vdim, T, ws.data_ptr(), ws.numel(), dt, _stream()))
+    return o
+
+
+def mlstm_step(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, q_scale: float, x: torch.Tensor, gate_w: torch.Tensor,
+               gate_b: torch.Tensor, cap: float, g: torch.Tensor, norm: torch.Tensor, eps: float, state: torch.Tensor,
+               m_state: torch.Tensor, cu_seqlens: torch.Tensor, positions: torch.Tensor, state_slots: torch.Tensor, num_heads: int,
+               dim: int, vdim: int, out: torch.Tensor | None = None):
+    """The matrix memory with exponential gates for chunks of a few tokens, one launch: gate products over the
+    float32 rows x [tokens, width] (gate_w [2 heads, width] input gates first, gate_b float32 [2 heads]), the
+    recurrence on state / m_state (float32 [slots, heads]), the norm per head (norm float32 [heads * vdim]) and
+    the sigmoid of g [tokens, heads * vdim].  Returns [tokens, heads * vdim] in q's dtype."""
+    dt = _dt3(q, "q")
+    T, S, W = q.shape[0], cu_seqlens.numel() - 1, x.shape[1]
+    if tuple(gate_w.shape) != (2 * num_heads, W) or not gate_w.is_contiguous() or x.dtype != torch.float32:
+        raise ValueError("gate_w must be contiguous [2 heads, width] and x float32 [tokens, width]")
+    if tuple(m_state.shape[1:]) != (num_heads,):
+        raise ValueError("m_state must be float32 [slots, heads]")
+    if out is None:
+        out = torch.empty(T, num_heads * vdim, dtype=q.dtype, device=q.device)
+    check(lib.mi355_mlstm_step(
+        _same(out, q, "out"), _cols(out, "out", num_heads * vdim), q.data_ptr(), _cols(q, "q", num_heads * dim), _same(k, q, "k"),
+        _cols(k, "k", num_heads * dim), _same(v, q, "v"), _cols(v, "v", num_heads * vdim), float(q_scale), x.data_ptr(),
+        _cols(x, "x", W), _same(gate_w, q, "gate_w"), _f32(gate_b, "gate_b", 2 * num_heads), W, float(cap), _same(g, q, "g"),
+        _cols(g, "g", num_heads * vdim), _f32(norm, "norm", num_heads * vdim), float(eps),
+        _linear_attn_state(state, num_heads, dim, vdim, True), _f32(m_state, "m_state"),
+        _idx(cu_seqlens, "cu_seqlens", torch.int32), _idx(positions, "positions", torch.int64, T),
+        _idx(state_slots, "state_slots", torch.int32, S), S, num_heads, dim, vdim, dt, _stream()))
+    return out
+
+
+def mlstm_chunks(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, q_scale: float, z: torch.Tensor, gate_b: torch.Tensor, cap: float,
+                 state: torch.Tensor, m_state: torch.Tensor, cu_seqlens: torch.Tensor, positions: torch.Tensor,
+                 state_slots: torch.Tensor, num_heads: int, dim: int, vdim: int, tiles: RowTiles):
+    """The matrix memory for chunks of many tokens, by tiles; z float32 [tokens, 2 heads]: the gate products
+    without their biases.  Returns o float32 [tokens, heads, vdim] ahead of the norm and the output gate."""
+    dt = _dt3(q, "q")
+    T, S, H, dev = q.shape[0], cu_seqlens.numel() - 1, num_heads, q.device
+    chunk = (_idx(cu_seqlens, "cu_seqlens", torch.int32), _idx(positions, "positions", torch.int64, T),
+             _idx(state_slots, "state_slots", torch.int32, S))
+    if tuple(m_state.shape[1:]) != (H,):
+        raise ValueError("m_state must be float32 [slots, heads]")
+    ga, gm = torch.empty(2, H, T, dtype=torch.float32, device=dev)
+    gf = torch.empty(H, T, dtype=torch.float64, device=dev)
+    tm = torch.empty(tiles.count, H, dtype=torch.float32, device=dev)
+    sp = _linear_attn_state(state, H, dim, vdim, True)
+    check(lib.mi355_mlstm_gates(ga.data_ptr(), gf.data_ptr(), gm.data_ptr(), tm.data_ptr(), _f32(z, "z", T * 2 * H),
+                                _f32(gate_b, "gate_b", 2 * H), float(cap), _f32(m_state, "m_state"), *chunk,
+                                tiles.start.data_ptr(), S, H, tiles.rows, T, _stream()))
+    o = torch.empty(T, H, vdim, dtype=torch.float32, device=dev)
+    ws = torch.empty(tiles.count * H * state.shape[2], dtype=torch.float32, device=dev)
+    check(lib.mi355_linear_attn_chunks(o.data_ptr(), q.data_ptr(), _cols(q, "q", H * dim), _same(k, q, "k"), _cols(k, "k", H * dim),
+                                       _same(v, q, "v"), _cols(v, "v", H * vdim), float(q_scale), None, ga.data_ptr(), gf.data_ptr(),
+                                       gm.data_ptr(), tm.data_ptr(), sp, *chunk, tiles.tiles.data_ptr(), tiles.start.data_ptr(),
+                                       tiles.count, tiles.rows, S, H, dim, vdim, T, ws.data_ptr(), ws.numel(), dt, _stream()))
+    return o

@@ -208,6 +208,40 @@ class ParallelLayerWeights:
 
 
 @dataclass
+class PostNormLayerWeights:
+    """One layer of a hybrid decoder in the "post" arrangement (the sub-layers read the residual itself, norms
+    sit on their outputs).  Everything of the mixer that reads the residual in the activation type is ONE
+    matrix in_w with one bias row in_b (None if no segment has one); segments `seg`:
+      attention_decay:  lq | lk | lv of the attention, then q | k | v | g of the linear attention
+      mlstm:            q | k | v | g
+    and what leads back is one matrix out_w over the row [attention heads | linear attention heads] (the
+    first part padded to a 16-byte boundary) or [heads].  gate_w / gate_b: input, then forget gates of the
+    matrix memory [2 heads, width].  Norm weights are float32; norm1, norm2 hold one plus the stored weight, the
+    linear attention's norm is multiplied by the layer's right_scale."""
+    norm1: torch.Tensor
+    in_w: torch.Tensor
+    in_b: Optional[torch.Tensor]
+    seg: dict
+    out_w: torch.Tensor
+    head_norm: torch.Tensor                     # f32 [heads * vdim] of the linear attention or the matrix memory
+    q_norm: Optional[torch.Tensor] = None       # f32 [heads * dim]
+    k_norm: Optional[torch.Tensor] = None       # f32 [kv_heads * dim]
+    log_decay: Optional[torch.Tensor] = None    # f64 [heads]
+    gate_w: Optional[torch.Tensor] = None       # [2 heads, width]
+    gate_w32: Optional[torch.Tensor] = None     # the same in float32 (many rows: one library product)
+    gate_b: Optional[torch.Tensor] = None       # f32 [2 heads]
+    norm2: Optional[torch.Tensor] = None
+    up_w: Optional[torch.Tensor] = None         # [ff, width]
+    down_w: Optional[torch.Tensor] = None       # [width, ff]
+    side_gate_w: Optional[torch.Tensor] = None  # [token_side, width]
+    side_proj_w: Optional[torch.Tensor] = None  # [width, token_side]
+    side_norm: Optional[torch.Tensor] = None    # f32 [width]
+
+    def tensors(self):
+        return [t for t in vars(self).values() if isinstance(t, torch.Tensor)]
+
+
+@dataclass
 class ModelWeights:
     embed: torch.Tensor
     layers: list = field(default_factory=list)
@@ -219,18 +253,19 @@ class ModelWeights:
     loop_step: Optional[torch.Tensor] = None     # hybrid decoders with a loop: [passes, width]
     embed_norm: Optional[torch.Tensor] = None    # hybrid decoders that norm the embedding: f32 [width]
     bigram: Optional[torch.Tensor] = None        # hashed previous-token embedding: [buckets + 1, width]
+    side_embed: Optional[torch.Tensor] = None    # per-layer token numbers: [vocab, layers * token_side]
 
     def nbytes(self) -> int:
         total = self.embed.numel() * self.embed.element_size()
         if self.lm_head.untyped_storage().data_ptr() != self.embed.untyped_storage().data_ptr():
             total += self.lm_head.numel() * self.lm_head.element_size()
         total += self.final_norm.numel() * self.final_norm.element_size()
-        for t in (self.pos_embed, self.final_norm_b, self.loop_step, self.embed_norm, self.bigram):
+        for t in (self.pos_embed, self.final_norm_b, self.loop_step, self.embed_norm, self.bigram, self.side_embed):
             if t is not None:
                 total += t.numel() * t.element_size()
         for lw in self.layers:
             ts = lw.tensors() if isinstance(lw, (OPTLayerWeights, HybridLayerWeights, SandwichLayerWeights, MixerLayerWeights,
-                                                 ParallelLayerWeights)) else \
+                                                 ParallelLayerWeights, PostNormLayerWeights)) else \
                 (lw.qkv_w, lw.qkv_b, lw.o_w, lw.gate_up_w, lw.down_w, lw.input_norm, lw.post_norm)
             for t in ts:
                 if t is not None:
@@ -390,6 +425,8 @@ def _hybrid_from_getter(cfg: ModelConfig, get, dtype, device, tp_size: int, num_
         return _tafisun_from_getter(cfg, get, dtype, device)
     if spec.arrangement == "parallel":
         return _bemulorn_from_getter(cfg, get, dtype, device)
+    if spec.arrangement == "post":
+        return _rigazen_from_getter(cfg, get, dtype, device)
 
     def put(t, dt=dtype):
         return t.to(dt).contiguous().to(device)
@@ -670,6 +707,121 @@ def _bemulorn_from_getter(cfg: ModelConfig, get, dtype, device) -> ModelWeights:
     return w
 
 
+def _rigazen_from_getter(cfg: ModelConfig, get, dtype, device) -> ModelWeights:
+    """Rigazen checkpoints: 'embed' (also the head), 'side.embed', 'final.norm', and per layer i
+    'l<i>.norm1|norm2', 'l<i>.mix.*' (parallel: left.q|k|v with '.b', left.q|k '.norm', left.o, and
+    right.q|k|v|g|o|norm; mlstm: q k v g o norm, i and f with '.b'), 'l<i>.mlp.up|down',
+    'l<i>.side.gate|proj|norm'.  Linear weights are [out, in]."""
+    import math
+    spec, W = cfg.hybrid, cfg.hidden_size
+
+    def put(t, dt=dtype):
+        return t.to(dt).contiguous().to(device)
+
+    def f32(t):
+        return put(t.reshape(-1), torch.float32)
+
+    def expect(name, shape):
+        t = get(name)
+        if tuple(t.shape) != tuple(shape):
+            raise ValueError(f"{name}: shape {tuple(t.shape)}, expected {tuple(shape)}")
+        return t
+
+    def one_plus(name):
+        return f32(expect(name, (W,)).float() + 1.0)
+
+    n = spec.token_side
+    w = ModelWeights(embed=put(expect("embed", (cfg.vocab_size, W))))
+    if n:
+        w.side_embed = put(expect("side.embed", (cfg.vocab_size, len(spec.layers) * n)))
+    for i, L in enumerate(spec.layers):
+        p, m = f"l{i}.", f"l{i}.mix."
+        kw = {}
+        if L.kind == "attention_decay":
+            A, D, a, r = L.battn, L.lin, m + "left.", m + "right."
+            Dv = D.heads * D.vdim
+            left = [("l" + c, expect(a + c, (rows, W))) for c, rows in (("q", A.heads * A.dim), ("k", A.kv_heads * A.dim),
+                                                                        ("v", A.kv_heads * A.vdim))]
+            right = [(c, expect(r + c, (rows, W))) for c, rows in (("q", D.heads * D.dim), ("k", D.heads * D.dim), ("v", Dv), ("g", Dv))]
+            in_w, seg = _fuse_segments(left + right, W, put)
+            b = torch.zeros(in_w.shape[0], dtype=torch.float32)
+            for c in "qkv":
+                at, rows = seg["l" + c]
+                b[at: at + rows] = expect(a + c + ".b", (rows,)).float()
+            at = -(-A.heads * A.vdim // 8) * 8                # the second part starts on a 16-byte boundary
+            o1, o2 = expect(a + "o", (W, A.heads * A.vdim)), expect(r + "o", (W, Dv))
+            out_w = torch.zeros(W, at + Dv, dtype=o1.dtype)
+            out_w[:, : A.heads * A.vdim], out_w[:, at:] = o1, o2
+            logs = [math.log(x) if x > 0 else -1e30 for x in D.decay]
+            kw.update(in_b=put(b), out_w=put(out_w), q_norm=f32(expect(a + "q.norm", (A.heads * A.dim,))),
+                      k_norm=f32(expect(a + "k.norm", (A.kv_heads * A.dim,))),
+                      head_norm=f32(expect(r + "norm", (Dv,)).float() * L.right_scale),
+                      log_decay=torch.tensor(logs, dtype=torch.float64, device=device))
+        else:
+            M = L.mem
+            Hd, Hv = M.heads * M.dim, M.heads * M.vdim
+            in_w, seg = _fuse_segments([(c, expect(m + c, (rows, W))) for c, rows in (("q", Hd), ("k", Hd), ("v", Hv), ("g", Hv))], W, put)
+            gates = torch.cat([expect(m + "i", (M.heads, W)), expect(m + "f", (M.heads, W))], dim=0)
+            kw.update(in_b=None, out_w=put(expect(m + "o", (W, Hv))), head_norm=f32(expect(m + "norm", (Hv,))), gate_w=put(gates),
+                      gate_w32=put(gates, torch.float32),
+                      gate_b=f32(torch.cat([expect(m + "i.b", (M.heads,)), expect(m + "f.b", (M.heads,))])))
+        if L.ff:
+            kw.update(norm2=one_plus(p + "norm2"), up_w=put(expect(p + "mlp.up", (L.ff, W))),
+                      down_w=put(expect(p + "mlp.down", (W, L.ff))))
+        if n:
+            kw.update(side_gate_w=put(expect(p + "side.gate", (n, W))), side_proj_w=put(expect(p + "side.proj", (W, n))),
+                      side_norm=f32(expect(p + "side.norm", (W,))))
+        w.layers.append(PostNormLayerWeights(norm1=one_plus(p + "norm1"), in_w=in_w, seg=seg, **kw))
+    w.final_norm = one_plus("final.norm")
+    w.lm_head = w.embed
+    return w
+
+
+def rigazen_synthetic_state(cfg: ModelConfig, seed: int = 0, device="cpu", dtype=torch.float32) -> dict:
+    """Seeded random tensors under a Rigazen checkpoint's names (benchmarks and tests: nothing can be
+    downloaded)."""
+    spec, W = cfg.hybrid, cfg.hidden_size
+    gen = torch.Generator(device=device).manual_seed(seed)
+
+    def mat(*shape, s=1.0):
+        return torch.empty(shape, dtype=dtype, device=device).normal_(0.0, s, generator=gen)
+
+    def near(value, *shape, s=0.1):
+        return torch.full(shape, float(value), dtype=dtype, device=device) + mat(*shape, s=s)
+
+    n = spec.token_side
+    st = {"embed": mat(cfg.vocab_size, W, s=W ** -0.5), "final.norm": mat(W, s=0.1)}
+    if n:
+        st["side.embed"] = mat(cfg.vocab_size, len(spec.layers) * n)
+    for i, L in enumerate(spec.layers):
+        p, m = f"l{i}.", f"l{i}.mix."
+        st[p + "norm1"] = mat(W, s=0.1)
+        if L.kind == "attention_decay":
+            A, D, a, r = L.battn, L.lin, m + "left.", m + "right."
+            for c, rows in (("q", A.heads * A.dim), ("k", A.kv_heads * A.dim), ("v", A.kv_heads * A.vdim)):
+                st[a + c], st[a + c + ".b"] = mat(rows, W, s=W ** -0.5), mat(rows, s=0.2)
+            st[a + "q.norm"], st[a + "k.norm"] = near(1.0, A.heads * A.dim), near(1.0, A.kv_heads * A.dim)
+            st[a + "o"] = mat(W, A.heads * A.vdim, s=(A.heads * A.vdim) ** -0.5)
+            Hv = D.heads * D.vdim
+            for c, rows in (("q", D.heads * D.dim), ("k", D.heads * D.dim), ("v", Hv), ("g", Hv)):
+                st[r + c] = mat(rows, W, s=W ** -0.5)
+            st[r + "norm"], st[r + "o"] = near(1.0, Hv), mat(W, Hv, s=Hv ** -0.5)
+        else:
+            M = L.mem
+            Hv = M.heads * M.vdim
+            for c, rows in (("q", M.heads * M.dim), ("k", M.heads * M.dim), ("v", Hv), ("g", Hv), ("i", M.heads), ("f", M.heads)):
+                st[m + c] = mat(rows, W, s=W ** -0.5)
+            st[m + "i.b"], st[m + "f.b"] = mat(M.heads, s=0.5), near(3.0, M.heads, s=1.0)
+            st[m + "norm"], st[m + "o"] = near(1.0, Hv), mat(W, Hv, s=Hv ** -0.5)
+        if L.ff:
+            st[p + "norm2"] = mat(W, s=0.1)
+            st[p + "mlp.up"], st[p + "mlp.down"] = mat(L.ff, W, s=W ** -0.5), mat(W, L.ff, s=L.ff ** -0.5)
+        if n:
+            st[p + "side.gate"], st[p + "side.proj"] = mat(n, W, s=W ** -0.5), mat(W, n, s=n ** -0.5)
+            st[p + "side.norm"] = near(0.5, W)
+    return st
+
+
 def bemulorn_synthetic_state(cfg: ModelConfig, seed: int = 0, device="cpu", dtype=torch.float32) -> dict:
     """Seeded random tensors under a Bemulorn checkpoint's names (benchmarks and tests: nothing can be
     downloaded)."""
@@ -814,6 +966,8 @@ def hybrid_synthetic_state(cfg: ModelConfig, seed: int = 0, std: float = 0.02, r
         return tafisun_synthetic_state(cfg, seed=seed, device=device, dtype=dtype)
     if spec.arrangement == "parallel":
         return bemulorn_synthetic_state(cfg, seed=seed, device=device, dtype=dtype)
+    if spec.arrangement == "post":
+        return rigazen_synthetic_state(cfg, seed=seed, device=device, dtype=dtype)
     gen = torch.Generator(device=device).manual_seed(seed)
 
     def mat(*shape, s=std):
