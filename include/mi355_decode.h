@@ -1119,7 +1119,7 @@ int64_t mi355_mingru_scan_workspace(int32_t num_seqs, int32_t channels, int32_t 
  *   linear_attn_chunks    both recurrences over chunks of any length by such tiles (tiles: chunk, first row, rows;
  *                         tile_start [chunks + 1]): log_decay for the constant decay (silu on q, k, v), null and the
  *                         four arrays of mlstm_gates otherwise.  o fp32 [tokens, heads, v_dim] (not normed or gated).
- *                         workspace: tiles * heads * linear_attn_state_floats floats
+ *                         workspace: tiles * heads * (linear_attn_state_floats + 1) floats
  *   linear_attn_tile_rows  rows of a tile that fit (64, 32 or 16); 0: heads too large
  */
 int32_t mi355_norm_resid_f32(float* resid, void* act_out, const void* y, const float* weight,

@@ -75,24 +75,29 @@ __device__ __forceinline__ void stage_rows(float* dst, int ld, const typename El
   }
 }
 
-// ---- 1: a, F, m of every row.  One wave per (chunk, head); lane = row of the tile.
-// ga / gm [H][T] float, gf [H][T] double, mstart [tiles][H].
-__global__ __launch_bounds__(64) void mlstm_gates_kernel(float* __restrict__ ga, double* __restrict__ gf, float* __restrict__ gm,
-                                                         float* __restrict__ mstart, const float* __restrict__ z,
-                                                         const float* __restrict__ bias, float cap, float* __restrict__ m_state,
-                                                         const int32_t* __restrict__ cu_seqlens,
-                                                         const int64_t* __restrict__ positions,
-                                                         const int32_t* __restrict__ state_slots,
-                                                         const int32_t* __restrict__ tile_start, int H, int C, int64_t T) {
-  const int s = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+// ---- 1: a, F, m of every row.  One workgroup per (chunk, head): its 16 waves scan a tile each (lane = row), then
+// m at the tiles' starts follows from the tiles' ends, wave by wave.  ga / gm [H][T] float, gf [H][T] double,
+// mstart [tiles][H].
+__global__ __launch_bounds__(1024) void mlstm_gates_kernel(float* __restrict__ ga, double* __restrict__ gf, float* __restrict__ gm,
+                                                           float* __restrict__ mstart, const float* __restrict__ z,
+                                                           const float* __restrict__ bias, float cap, float* __restrict__ m_state,
+                                                           const int32_t* __restrict__ cu_seqlens,
+                                                           const int64_t* __restrict__ positions,
+                                                           const int32_t* __restrict__ state_slots,
+                                                           const int32_t* __restrict__ tile_start, int H, int C, int64_t T) {
+  constexpr int NW = 16;
+  __shared__ double ends[2][NW];                          // F and M of the tiles' last rows
+  const int s = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int64_t cs = MI355_LD(int32_t, cu_seqlens, cu_seqlens + s);
   const int64_t n = MI355_LD(int32_t, cu_seqlens, cu_seqlens + s + 1) - cs;
-  if (n <= 0) return;
+  if (n <= 0) return;                                     // (the whole workgroup)
   const int64_t slot = MI355_LD(int32_t, state_slots, state_slots + s);
   const int64_t tile0 = MI355_LD(int32_t, tile_start, tile_start + s);
   float m0 = MI355_LD(int64_t, positions, positions + cs) == 0 ? 0.f : MI355_LD(float, m_state, m_state + slot * H + h);
   const float bi = MI355_LD(float, bias, bias + h), bf = MI355_LD(float, bias, bias + H + h);
-  for (int64_t r0 = 0, ti = 0; r0 < n; r0 += C, ++ti) {
+  const int64_t num = (n + C - 1) / C;
+  for (int64_t g = 0; g < num; g += NW) {
+    const int64_t r0 = (g + wave) * C;
     const bool live = lane < C && r0 + lane < n;
     const int64_t t = cs + r0 + lane;
     float a = 0.f;
@@ -111,17 +116,22 @@ __global__ __launch_bounds__(64) void mlstm_gates_kernel(float* __restrict__ ga,
         F += Fp;
       }
     }
-    const float m = static_cast<float>(fmax(M, F + static_cast<double>(m0)));
+    if (lane == 63) ends[0][wave] = F, ends[1][wave] = M; // (rows past the tile's last add nothing to either)
+    __syncthreads();
+    float mine = m0;                                      // m ahead of this wave's tile
+    for (int w = 0; w < NW; ++w) {
+      if (w == wave) mine = m0;
+      m0 = static_cast<float>(fmax(ends[1][w], ends[0][w] + static_cast<double>(m0)));
+    }
     if (live) {
       MI355_ST(float, ga, ga + h * T + t, a);
       MI355_ST(double, gf, gf + h * T + t, F);
-      MI355_ST(float, gm, gm + h * T + t, m);
+      MI355_ST(float, gm, gm + h * T + t, static_cast<float>(fmax(M, F + static_cast<double>(mine))));
     }
-    if (lane == 0) MI355_ST(float, mstart, mstart + (tile0 + ti) * H + h, m0);
-    const int last = static_cast<int>(n - r0 < C ? n - r0 : C) - 1;
-    m0 = __shfl(m, last, 64);
+    if (lane == 0 && g + wave < num) MI355_ST(float, mstart, mstart + (tile0 + g + wave) * H + h, mine);
+    __syncthreads();                                      // the ends are read before the next turn writes them
   }
-  if (lane == 0) MI355_ST(float, m_state, m_state + slot * H + h, m0);
+  if (threadIdx.x == 0) MI355_ST(float, m_state, m_state + slot * H + h, m0);
 }
 
 // ---- 2: sum_j e^(F_end - F_j + a_j - m_end) k_j v_j^T of every tile and head
@@ -130,7 +140,8 @@ __global__ __launch_bounds__(256) void la_states_kernel(
     float* __restrict__ ws, const typename Elem<T>::S* __restrict__ k, int64_t k_stride,
     const typename Elem<T>::S* __restrict__ v, int64_t v_stride, const double* __restrict__ log_decay,
     const float* __restrict__ ga, const double* __restrict__ gf, const float* __restrict__ gm,
-    const int32_t* __restrict__ tiles, LaDims D, int64_t total_rows, int vec) {
+    const float* __restrict__ mstart, const int32_t* __restrict__ tiles, LaDims D, int64_t total_rows, int64_t num_tiles,
+    int vec) {
   extern __shared__ float lds[];
   const int tile = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int d = D.d, dv = D.dv, dp = (d + 15) & ~15, dvp = (dv + 15) & ~15;
@@ -151,6 +162,18 @@ __global__ __launch_bounds__(256) void la_states_kernel(
     } else {
       wr[i] = expf(static_cast<float>((n - 1 - i) * MI355_LD(double, log_decay, log_decay + h)));
     }
+  }
+  if (tid == 0) {                                         // the factor on the tile's incoming state, for la_scan
+    float f;
+    if (MEM) {
+      const int64_t end = h * total_rows + row0 + n - 1;
+      f = expf(static_cast<float>(MI355_LD(double, gf, gf + end) +
+                                  static_cast<double>(MI355_LD(float, mstart, mstart + static_cast<int64_t>(tile) * D.H + h)) -
+                                  static_cast<double>(MI355_LD(float, gm, gm + end))));
+    } else {
+      f = expf(static_cast<float>(n * MI355_LD(double, log_decay, log_decay + h)));
+    }
+    MI355_ST(float, ws, ws + num_tiles * D.H * D.us + static_cast<int64_t>(tile) * D.H + h, f);
   }
   __syncthreads();
   stage_rows<T>(Ks, kl, k, k + row0 * k_stride + static_cast<int64_t>(h) * d, k_stride, n, np, d, dp, !MEM, 1.0f, wr, vec);
@@ -197,15 +220,11 @@ __global__ __launch_bounds__(256) void la_states_kernel(
 }
 
 // ---- 3: tile by tile, elementwise: ws[tile] becomes the state at the tile's start
-template <bool MEM>
 __global__ __launch_bounds__(256) void la_scan_kernel(float* __restrict__ ws, float* __restrict__ state,
-                                                      const double* __restrict__ log_decay, const double* __restrict__ gf,
-                                                      const float* __restrict__ gm, const float* __restrict__ mstart,
                                                       const int32_t* __restrict__ cu_seqlens,
                                                       const int64_t* __restrict__ positions,
                                                       const int32_t* __restrict__ state_slots,
-                                                      const int32_t* __restrict__ tiles,
-                                                      const int32_t* __restrict__ tile_start, LaDims D, int64_t total_rows) {
+                                                      const int32_t* __restrict__ tile_start, LaDims D, int64_t num_tiles) {
   const int h = blockIdx.y, s = blockIdx.z;
   const int t0 = MI355_LD(int32_t, tile_start, tile_start + s), t1 = MI355_LD(int32_t, tile_start, tile_start + s + 1);
   if (t0 >= t1) return;
@@ -218,31 +237,24 @@ __global__ __launch_bounds__(256) void la_scan_kernel(float* __restrict__ ws, fl
   if (MI355_LD(int64_t, positions, positions + cs) != 0) S = MI355_LD(float4, state, sp);
   const int64_t step = static_cast<int64_t>(D.H) * D.us;
   float* w = ws + (static_cast<int64_t>(t0) * D.H + h) * D.us + 4 * e4;
+  const float* fac = ws + num_tiles * step + static_cast<int64_t>(t0) * D.H + h;
   constexpr int PF = 8;
-  for (int t = t0; t < t1; t += PF) {
+  for (int t = 0; t < t1 - t0; t += PF) {
     float4 u[PF];
     float f[PF];
 #pragma unroll
     for (int j = 0; j < PF; ++j) {
       u[j] = make_float4(0.f, 0.f, 0.f, 0.f);
       f[j] = 1.f;
-      if (t + j < t1) {
-        u[j] = MI355_LD(float4, ws, w + (t - t0 + j) * step);
-        const int n = MI355_LD(int32_t, tiles, tiles + 3 * (t + j) + 2);
-        if (MEM) {
-          const int64_t end = h * total_rows + MI355_LD(int32_t, tiles, tiles + 3 * (t + j) + 1) + n - 1;
-          f[j] = expf(static_cast<float>(MI355_LD(double, gf, gf + end) +
-                                         static_cast<double>(MI355_LD(float, mstart, mstart + static_cast<int64_t>(t + j) * D.H + h)) -
-                                         static_cast<double>(MI355_LD(float, gm, gm + end))));
-        } else {
-          f[j] = expf(static_cast<float>(n * MI355_LD(double, log_decay, log_decay + h)));
-        }
+      if (t + j < t1 - t0) {
+        u[j] = MI355_LD(float4, ws, w + (t + j) * step);
+        f[j] = MI355_LD(float, ws, fac + static_cast<int64_t>(t + j) * D.H);
       }
     }
 #pragma unroll
     for (int j = 0; j < PF; ++j) {
-      if (t + j < t1) {
-        MI355_ST(float4, ws, w + (t - t0 + j) * step, S);
+      if (t + j < t1 - t0) {
+        MI355_ST(float4, ws, w + (t + j) * step, S);
         S.x = f[j] * S.x + u[j].x, S.y = f[j] * S.y + u[j].y, S.z = f[j] * S.z + u[j].z, S.w = f[j] * S.w + u[j].w;
       }
     }
@@ -328,14 +340,21 @@ __global__ __launch_bounds__(512) void la_out_kernel(
   const float* S = ws + (static_cast<int64_t>(tile) * D.H + h) * D.us;
   __syncthreads();
   if (MEM) {
-    // n . q: the rows' sums of P, and the state's part; one wave per row in turn
-    for (int i = wave; i < n; i += nw) {
-      float sum = 0.f;
-      for (int j = lane; j <= i; j += 64) sum += Ps[i * pl + j];
-      float nq = 0.f;
-      for (int c = lane; c < d; c += 64) nq += MI355_LD(float, ws, S + static_cast<int64_t>(d) * dv + c) * Qs[i * ql + c];
-      sum = wave_sum(sum + er[i] * nq);
-      if (lane == 0) dr[i] = 1.0f / (fmaxf(fabsf(sum), expf(-mr[i])) + 1e-6f);
+    for (int c = tid; c < d; c += blockDim.x) Ks[c] = MI355_LD(float, ws, S + static_cast<int64_t>(d) * dv + c);
+    __syncthreads();
+  }
+  if (MEM) {
+    // n . q: the rows' sums of P, and the state's part; 8 adjacent lanes per row (n lies over the keys, which are done with)
+    for (int i = tid >> 3; i < np; i += blockDim.x >> 3) {
+      const int u = tid & 7;
+      float sum = 0.f, nq = 0.f;
+      for (int j = u; j < np && j <= i; j += 8) sum += Ps[i * pl + j];
+      for (int c = u; c < d; c += 8) nq += Ks[c] * Qs[i * ql + c];
+      sum += er[i] * nq;
+      sum += __shfl_xor(sum, 1, 64);
+      sum += __shfl_xor(sum, 2, 64);
+      sum += __shfl_xor(sum, 4, 64);
+      if (u == 0) dr[i] = 1.0f / (fmaxf(fabsf(sum), expf(-mr[i])) + 1e-6f);
     }
     __syncthreads();
   }
@@ -346,15 +365,39 @@ __global__ __launch_bounds__(512) void la_out_kernel(
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
     const float* qa = Qs + (bi * 16 + li) * ql + kk;
-#pragma unroll 4
-    for (int c = 0; c < dp; c += 4) {
-      const float a = qa[c];
+    // the incoming state's part: 16 rows of it at a time, the next 16 on their way meanwhile.  Rows and columns past
+    // the head read its last ones: the former meet zeros of Q, the latter are not stored.
+    const float* sc[4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int col = (n0 + j) * 16 + li;
-        const float b = (c + kk < d && col < dv) ? MI355_LD(float, ws, S + static_cast<int64_t>(c + kk) * dv + col) : 0.f;
-        acc[j] = mfma_f32(a, b, acc[j]);
+    for (int j = 0; j < 4; ++j) {
+      const int col = (n0 + j) * 16 + li;
+      sc[j] = S + (col < dv ? col : dv - 1);
+    }
+    float b[4][4], bn[4][4];
+    auto fetch = [&](float (&x)[4][4], int c) {
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int row = c + 4 * u + kk;
+        const int64_t at = static_cast<int64_t>(row < d ? row : d - 1) * dv;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) x[u][j] = MI355_LD(float, ws, sc[j] + at);
       }
+    };
+    auto work = [&](const float (&x)[4][4], int c) {
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const float a = qa[c + 4 * u];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[j] = mfma_f32(a, x[u][j], acc[j]);
+      }
+    };
+    fetch(b, 0);
+    for (int c = 0; c < dp; c += 32) {
+      if (c + 16 < dp) fetch(bn, c + 16);
+      work(b, c);
+      if (c + 16 >= dp) break;
+      if (c + 32 < dp) fetch(b, c + 32);
+      work(bn, c + 16);
     }
 #pragma unroll
     for (int j = 0; j < 4; ++j)
@@ -428,8 +471,25 @@ __global__ __launch_bounds__(256) void la_step_kernel(
   if (MEM && !fresh) m = MI355_LD(float, M.m_state, M.m_state + slot * D.H + h);
   const float dec = MEM ? 0.f : expf(static_cast<float>(MI355_LD(double, log_decay, log_decay + h)));
   const int tx = tid % cg, ty = tid / cg;
+  constexpr int PF = 16;
+  float S[PF][VW];
+  // rows i0, i0 + rg, ... of column group c of the state
+  auto fetch = [&](int i0, int c) {
+#pragma unroll
+    for (int u = 0; u < PF; ++u) {
+      const int i = i0 + u * rg;
+      if constexpr (VW == 4) {
+        float4 x4 = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (i < d && !fresh) x4 = MI355_LD(float4, state, sp + static_cast<int64_t>(i) * dv + c * 4);
+        S[u][0] = x4.x, S[u][1] = x4.y, S[u][2] = x4.z, S[u][3] = x4.w;
+      } else {
+        S[u][0] = i < d && !fresh ? MI355_LD(float, state, sp + static_cast<int64_t>(i) * dv + c) : 0.f;
+      }
+    }
+  };
   for (int64_t t = cs; t < cs + n; ++t) {
     __syncthreads();                                      // the previous token's reads of LDS are done
+    if (ty < rg) fetch(ty, tx);                           // the first rows travel while the gates are worked out
     for (int i = tid; i < d; i += 256) {
       const float qv = MI355_LDF(T, q, q + t * q_stride + static_cast<int64_t>(h) * d + i);
       const float kv = MI355_LDF(T, k, k + t * k_stride + static_cast<int64_t>(h) * d + i);
@@ -482,20 +542,8 @@ __global__ __launch_bounds__(256) void la_step_kernel(
         }
       }
       if (live) {
-        constexpr int PF = 8;
         for (int i0 = ty; i0 < d; i0 += PF * rg) {
-          float S[PF][VW];
-#pragma unroll
-          for (int u = 0; u < PF; ++u) {
-            const int i = i0 + u * rg;
-            if constexpr (VW == 4) {
-              float4 x4 = make_float4(0.f, 0.f, 0.f, 0.f);
-              if (i < d && !fresh) x4 = MI355_LD(float4, state, sp + static_cast<int64_t>(i) * dv + c * 4);
-              S[u][0] = x4.x, S[u][1] = x4.y, S[u][2] = x4.z, S[u][3] = x4.w;
-            } else {
-              S[u][0] = i < d && !fresh ? MI355_LD(float, state, sp + static_cast<int64_t>(i) * dv + c) : 0.f;
-            }
-          }
+          if (c0 > 0 || i0 > ty) fetch(i0, c);
 #pragma unroll
           for (int u = 0; u < PF; ++u) {
             const int i = i0 + u * rg;
@@ -582,7 +630,7 @@ extern "C" int32_t mi355_mlstm_gates(float* log_in, double* log_decay_sum, float
   MI355_REQUIRE(num_seqs >= 0 && num_heads > 0 && num_heads <= 65535 && tile_rows > 0 && tile_rows <= 64 && num_tokens >= 0 && cap > 0.f,
                 MI355_ERR_INVALID, "mlstm_gates: sizes");
   if (num_seqs == 0 || num_tokens == 0) return MI355_OK;
-  hipLaunchKernelGGL(mlstm_gates_kernel, dim3(num_seqs, num_heads), dim3(64), 0, static_cast<hipStream_t>(stream), log_in,
+  hipLaunchKernelGGL(mlstm_gates_kernel, dim3(num_seqs, num_heads), dim3(1024), 0, static_cast<hipStream_t>(stream), log_in,
                      log_decay_sum, running_max, tile_max, z, bias, cap, m_state, cu_seqlens, positions, state_slots,
                      tile_start, num_heads, tile_rows, num_tokens);
   return check_launch("mlstm_gates");
@@ -613,7 +661,7 @@ extern "C" int32_t mi355_linear_attn_chunks(float* o, const void* q, int64_t q_s
                     la_states_lds(tile_rows, head_dim, v_dim) <= kLdsBytes,
                 MI355_ERR_UNSUPPORTED, "linear_attn_chunks: tiles of %d rows of heads of %d / %d do not fit the LDS", tile_rows,
                 head_dim, v_dim);
-  MI355_REQUIRE(workspace_floats >= static_cast<int64_t>(num_tiles) * num_heads * D.us && aligned16(workspace) && aligned16(state),
+  MI355_REQUIRE(workspace_floats >= static_cast<int64_t>(num_tiles) * num_heads * (D.us + 1) && aligned16(workspace) && aligned16(state),
                 MI355_ERR_INVALID, "linear_attn_chunks: workspace of %lld floats", static_cast<long long>(workspace_floats));
   if (num_seqs == 0 || num_tiles == 0 || num_tokens == 0) return MI355_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
@@ -630,10 +678,10 @@ extern "C" int32_t mi355_linear_attn_chunks(float* o, const void* q, int64_t q_s
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(la_out_kernel<TT, MM>), hipFuncAttributeMaxDynamicSharedMemorySize, \
                               static_cast<int>(lds_out));                                                                      \
     hipLaunchKernelGGL((la_states_kernel<TT, MM>), grid, dim3(256), lds_states, s, workspace, static_cast<const E*>(k), k_stride, \
-                       static_cast<const E*>(v), v_stride, log_decay, log_in, log_decay_sum, running_max, tiles, D,            \
-                       num_tokens, vec);                                                                                       \
-    hipLaunchKernelGGL((la_scan_kernel<MM>), sgrid, dim3(256), 0, s, workspace, state, log_decay, log_decay_sum, running_max,   \
-                       tile_max, cu_seqlens, positions, state_slots, tiles, tile_start, D, num_tokens);                        \
+                       static_cast<const E*>(v), v_stride, log_decay, log_in, log_decay_sum, running_max, tile_max, tiles, D,  \
+                       num_tokens, static_cast<int64_t>(num_tiles), vec);                                                      \
+    hipLaunchKernelGGL(la_scan_kernel, sgrid, dim3(256), 0, s, workspace, state, cu_seqlens, positions, state_slots,           \
+                       tile_start, D, static_cast<int64_t>(num_tiles));                                                        \
     hipLaunchKernelGGL((la_out_kernel<TT, MM>), grid, dim3(512), lds_out, s, o, workspace, static_cast<const E*>(q), q_stride, \
                        static_cast<const E*>(k), k_stride, static_cast<const E*>(v), v_stride, q_scale, log_decay, log_in,     \
                        log_decay_sum, running_max, tile_max, tiles, D, num_tokens, vec);                                       \

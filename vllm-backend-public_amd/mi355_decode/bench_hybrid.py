@@ -76,6 +76,23 @@ def bemulorn_config(width: int, layers: int, vocab: int = 32000, max_positions: 
             "embedding": {"scale": 2.0}, "logit_scale": 0.5, "layers": ls}
 
 
+def rigazen_config(width: int, layers: int, vocab: int = 32000) -> dict:
+    """Alternating parallel / mlstm layers: 128-wide attention heads, four query heads to a key head, a window of
+    1024 beside 4 kept tokens, all of a head rotated; beside it a linear attention of half as many 128 x 128
+    heads with constant decays; matrix memories of as many 128 x 128 heads as the width holds; a relu^2 feed-forward of
+    3 * width (as many weights as a gated one of 2 * width) and width / 32 numbers per token and layer."""
+    nh = width // 128
+    left = {"heads": nh, "kv_heads": max(nh // 4, 1), "dim": 128, "vdim": 128, "mask": {"size": 1024, "keep_first": 4},
+            "rot": {"dims": 128, "base": 1.0e6}, "scale": 128 ** -0.5}
+    hl = max(nh // 2, 1)
+    right = {"heads": hl, "dim": 128, "vdim": 128, "decay": [float(np.exp(-(2.0 ** (-8.0 * (h + 1) / hl)))) for h in range(hl)]}
+    ls = [{"type": "parallel" if i % 2 == 0 else "mlstm",
+           "mixer": {"left": left, "right": right, "left_scale": 0.7, "right_scale": 0.7} if i % 2 == 0 else
+           {"heads": nh, "dim": 128, "vdim": 128, "gate_cap": 15.0}, "mlp": {"kind": "dense", "ff": 3 * width}} for i in range(layers)]
+    return {"architecture": "Rigazen", "embedding": {"scale": float(width) ** 0.5}, "width": width, "vocab": vocab,
+            "norm": {"eps": 1e-6}, "token_side": {"dim": max(width // 32, 8)}, "layers": ls}
+
+
 def lozupel_config(width: int, layers: int, vocab: int = 32000, loop: bool = True) -> dict:
     """Alternating parallel / delta layers with 128-wide heads, a 1024-token window, a feed-forward in
     every layer; the middle of the stack loops twice."""
@@ -725,4 +742,162 @@ def compare_bemulorn(widths, layers: int, batch: int, prompt_len: int, steps: in
                                  "prefill_ratio": round(b["prefill_tok_s"] / ll["prefill_tok_s"], 3),
                                  "decode_ratio": round(b["decode_tok_s"] / ll["decode_tok_s"], 3)})
         result["kernels"][str(width)] = bemulorn_kernel_table(width, prompt_len, batch)
+    return result
+
+
+def rigazen_kernel_table(width: int, prompt_len: int, batch: int) -> list:
+    """The Rigazen design's kernels at the prefill and the decode shape, each against its own roofline, beside
+    the like kernel of the closest existing model (the Lozupel design) at the same shape."""
+    from .hybrid_runner import HybridRunner, rotary_table
+    dev, bf = "cuda", torch.bfloat16
+    g = torch.Generator(device=dev).manual_seed(0)
+    rnd = lambda *s, dt=bf: torch.randn(*s, device=dev, dtype=torch.float32, generator=g).to(dt)  # noqa: E731
+    rows = []
+
+    def row(kernel, shape, t, bound, work, like=None, like_t=None, like_work=None, like_bound=None):
+        peak = {"hbm": HBM, "mfma": MFMA, "valu": VALU}
+        r = {"kernel": kernel, "shape": shape, "us": round(t * 1e6, 2), "bound": bound,
+             "frac_of_roofline": round(work / peak[bound] / t, 4)}
+        if like is not None:
+            r.update(like=like, like_us=round(like_t * 1e6, 2), like_frac=round(like_work / peak[like_bound or bound] / like_t, 4))
+            r["distance_ratio"] = round(r["like_frac"] / max(r["frac_of_roofline"], 1e-9), 2)
+        rows.append(r)
+
+    P, W, V = prompt_len, width, 32000
+    H, G, d, window, keep = W // 128, max(W // 512, 1), 128, 1024, 4
+    pages = (P + BLOCK_SIZE) // BLOCK_SIZE + 1
+    nb = pages * batch
+    kc, vct = rnd(nb, G, BLOCK_SIZE, d), rnd(nb, G, d, BLOCK_SIZE)
+    bt = torch.arange(nb, dtype=torch.int32, device=dev).view(batch, pages)
+    embed = rnd(V, W)
+    cs = rotary_table(d, 1.0e6, pages * BLOCK_SIZE, dev, exact=True)
+    temp, bias = torch.ones(H, device=dev), torch.full((H,), -2.0, device=dev)
+    wq, wk = torch.ones(H * d, device=dev), torch.ones(G * d, device=dev)
+    for T, S, tag in ((P, 1, "prefill"), (batch, batch, "decode")):
+        shape = f"{tag} {T} rows x {W}"
+        per = T // S
+        cu_h = np.arange(0, T + 1, per)
+        cu = torch.from_numpy(cu_h.astype(np.int32)).to(dev)
+        pos = (torch.arange(T, device=dev) % per + (0 if S == 1 else P - 1)).to(torch.int64)
+        seq = (torch.arange(T, device=dev) // per).to(torch.int32)
+        slots = torch.arange(S, dtype=torch.int32, device=dev)
+        ids = torch.randint(0, V, (T,), device=dev, generator=g)
+        # ---- embedding, norm of a sub-layer's output, feed-forward activation
+        resid, act, y, w32, wv, w1 = rnd(T, W, dt=torch.float32), rnd(T, W), rnd(T, W), rnd(W, dt=torch.float32), rnd(W), rnd(1)
+        row("embed_scale_f32 (with activation copy)", shape, _time(lambda: ops.embed_scale_f32(embed, ids, 2.0, act_out=act)), "hbm",
+            T * W * 8, "embed_scale_f32", _time(lambda: ops.embed_scale_f32(embed, ids, 2.0)), T * W * 6)
+        row("norm_resid_f32", shape, _time(lambda: ops.norm_resid_f32(resid, y, w32, 1e-6, act_out=act)), "hbm", T * W * 12,
+            "add_rms_norm_f32", _time(lambda: ops.add_rms_norm_f32(resid, wv, 1e-6, add=y, out=act)), T * W * 12)
+        F = 3 * W
+        up, gu, hid = rnd(T, F), rnd(T, 2 * F), torch.empty(T, F, device=dev, dtype=bf)
+        row("relu_squared", f"{tag} {T} rows x {F}", _time(lambda: ops.relu_squared(up)), "hbm", T * F * 4,
+            "gelu_tanh_and_mul", _time(lambda: ops.gelu_tanh_and_mul(gu, out=hid)), T * F * 6)
+        # ---- the per-layer token input
+        n = max(W // 32, 8)
+        gw, pw, table, z = rnd(n, W) * W ** -0.5, rnd(W, n) * n ** -0.5, rnd(V, 4 * n), rnd(T, n)
+        if S == 1:
+            gu2 = rnd(T, 2 * n)
+            row("token_gate_rows", f"{tag} {T} rows x {n}", _time(lambda: ops.token_gate_rows(z, table, n, ids)), "hbm", T * n * 6,
+                "gelu_tanh_and_mul", _time(lambda: ops.gelu_tanh_and_mul(gu2)), T * n * 6)
+        else:                                       # (as the runner: one launch while the two matrices are small)
+            fused = T <= HybridRunner.SIDE_FUSED_ROWS and n * W <= HybridRunner.SIDE_FUSED_WEIGHTS
+            lin = ops.linear_decode
+            t_n = _time((lambda: ops.token_side_f32(resid, gw, pw, w32, table, n, ids, 1e-6, act_out=act)) if fused else
+                        lambda: ops.norm_resid_f32(resid, lin(ops.token_gate_rows(lin(act, gw), table, n, ids), pw), w32, 1e-6, act_out=act))
+            gu2 = rnd(T, 2 * n)
+            t_l = _time(lambda: ops.add_rms_norm_f32(resid, wv, 1e-6, add=lin(ops.gelu_tanh_and_mul(gu2), pw), out=act)) \
+                + _time(lambda: lin(y, gw))
+            row("token_side_f32 (one launch)" if fused else "token input (product, gate, product, norm)", f"{tag} {T} rows x {W} / {n}", t_n,
+                "hbm", 2 * n * W * 2 + T * W * 10, "two linear_decode, gelu_tanh_and_mul, add_rms_norm_f32", t_l,
+                2 * n * W * 2 + T * W * 12)
+        # ---- attention
+        proj = rnd(T, (H + 2 * G) * d)
+        q, k, v_ = proj[:, : H * d], proj[:, H * d: (H + G) * d], proj[:, (H + G) * d:]
+        gh = rnd(T, H)
+        wslots = (torch.arange(T, device=dev) if S == 1 else torch.arange(T, device=dev) * pages * BLOCK_SIZE + P - 1).to(torch.int64)
+        row("row_norm_rope_kv_write", f"{tag} {T} rows, {H}/{G} heads x {d}",
+            _time(lambda: ops.row_norm_rope_kv_write(q, k, v_, wq, wk, cs, pos, wslots, kc, vct, H, G, d, d, 1e-6)), "hbm",
+            T * (2 * H * d + 4 * G * d) * 2, "rope_partial_kv_write",
+            _time(lambda: ops.rope_partial_kv_write(q, k, v_, cs, pos, wslots, kc, vct, H, G, d, d)), T * (2 * H * d + 4 * G * d) * 2)
+        b_t = bt[:1] if S == 1 else bt
+        tiles = torch.from_numpy(ops.query_tiles(cu_h)).to(dev)
+        rep = H // G
+        hb = 4 if rep % 4 == 0 else 3 if rep % 3 == 0 else 2 if rep % 2 == 0 else 1
+        nsb = max(min(16, window // 64, 1024 // max(int(tiles.shape[0]) * G * (rep // hb), 1)), 1)
+        nsw = max(min(16, 2048 // max(int(tiles.shape[0]) * G * max(rep // 4, 1), 1)), 1)
+        part = torch.empty(nsw * T * H * d, device=dev)
+        o, qc = torch.empty(T, H * d, device=dev, dtype=bf), q.contiguous()
+        t_t = _time(lambda: ops.softmax_bias_attn(q, kc, vct, b_t, seq, pos, None, None, None, H, d ** -0.5, window=window, keep=keep,
+                                                  tiles=tiles, num_splits=nsb if nsb > 1 else 0, out=o), 5)
+        t_l = _time(lambda: ops.sigmoid_window_attn(q, kc, vct, b_t, seq, pos, temp, bias, gh, H, window, d ** -0.5, out=o, tiles=tiles,
+                                                    partial=part, num_splits=nsw), 5)
+        nkeys = sum(min(i + 1, window) for i in range(P)) if S == 1 else T * min(P, window)
+        vis = nkeys + sum(min(keep, max(i + 1 - window, 0)) for i in range(P)) if S == 1 else T * min(P, window + keep)
+        if S == 1:
+            ctx = torch.tensor([P], dtype=torch.int32, device=dev)
+            t_s = _time(lambda: ops.paged_attn_prefill_ext(q, kc, vct, b_t, cu, ctx, P, H, G, d, d ** -0.5, window=window, keep=keep,
+                                                           out=o), 5)
+            t_c = _time(lambda: ops.paged_attn_prefill(qc, kc, vct, b_t, cu, ctx, P, H, G, d, d ** -0.5, out=o), 5)
+            ashape = f"prefill {P} tokens, window {window} + {keep}, {H}/{G} heads x {d}"
+            row("paged_attn_prefill_ext", ashape, t_s, "mfma", 2.0 * vis * H * 2 * d, "sigmoid_window_attn", t_l, 2.0 * nkeys * H * 2 * d)
+            row("paged_attn_prefill_ext", ashape, t_s, "mfma", 2.0 * vis * H * 2 * d, "paged_attn_prefill (causal softmax)", t_c,
+                2.0 * (P * (P + 1) // 2) * H * 2 * d)
+            row("softmax_bias_attn, tile form (other head sizes)", ashape, t_t, "mfma", 2.0 * vis * H * 2 * d, "sigmoid_window_attn",
+                t_l, 2.0 * nkeys * H * 2 * d)
+        else:
+            row("softmax_bias_attn", f"decode {T} rows at context {P}, window {window} + {keep}", t_t, "hbm", vis * G * 2 * d * 2,
+                "sigmoid_window_attn", t_l, nkeys * G * 2 * d * 2)
+        # ---- the recurrences, 128 x 128 heads all three
+        Hd, Gd = W // 128, max(W // 256, 1)
+        Cd = 2 * Gd * d + Hd * d
+        xd, beta, dec = rnd(T, Cd), rnd(T, Hd), rnd(T, Hd)
+        a_log, dtb = torch.zeros(Hd, device=dev), torch.zeros(Hd, device=dev)
+        std, od = torch.zeros(S + 1, Hd, d, d, device=dev), torch.empty(T, Hd, d, device=dev)
+        t_l = _time(lambda: ops.gated_delta_rule(xd, 0, Gd * d, 2 * Gd * d, beta, dec, a_log, dtb, std, cu, pos, slots, Hd, Gd, d, d,
+                                                 out=od, long_chunks=S == 1), 5)
+        x4 = rnd(T, 4 * Hd * d)
+        c = [x4[:, i * Hd * d: (i + 1) * Hd * d] for i in range(4)]
+        ld = torch.full((Hd,), -0.05, dtype=torch.float64, device=dev)
+        st = torch.zeros(S + 1, Hd, ops.linear_attn_state_floats(d, d, False), device=dev)
+        rt = ops.RowTiles(cu_h, ops.linear_attn_tile_rows(d, d), dev) if S == 1 else None
+        t_n = _time(lambda: ops.decay_attn(c[0], c[1], c[2], ld, st, cu, pos, slots, Hd, d, d, tiles=rt), 5)
+        rshape, lshape = f"{tag} {T} rows, {Hd} heads x {d} x {d}", f"gated_delta_rule, {Hd} heads x {d} x {d}"
+        if S == 1:
+            row("decay_attn", rshape, t_n, "valu", 5.0 * T * Hd * d * d, lshape, t_l, 6.0 * T * Hd * d * d)
+        else:
+            row("decay_attn", rshape, t_n, "hbm", S * Hd * d * d * 8, lshape, t_l, S * Hd * d * d * 8)
+        sm, mm = torch.zeros(S + 1, Hd, ops.linear_attn_state_floats(d, d, True), device=dev), torch.zeros(S + 1, Hd, device=dev)
+        gb, hn = torch.cat([torch.zeros(Hd), torch.full((Hd,), 3.0)]).to(dev), torch.ones(Hd * d, device=dev)
+        gtw = rnd(2 * Hd, W) * W ** -0.5
+        if S == 1:
+            gtw32 = gtw.float()
+            row("gate product of the matrix memory (float32)", f"{tag} {T} rows x {W} -> {2 * Hd}",
+                _time(lambda: torch.mm(resid, gtw32.t()), 5), "valu", 4.0 * T * Hd * W)
+            zz = torch.mm(resid, gtw32.t())
+            t_n = _time(lambda: ops.mlstm_chunks(c[0], c[1], c[2], d ** -0.5, zz, gb, 15.0, sm, mm, cu, pos, slots, Hd, d, d, rt), 5)
+            row("mlstm_chunks", rshape, t_n, "valu", 5.0 * T * Hd * d * d, lshape, t_l, 6.0 * T * Hd * d * d)
+        else:
+            t_n = _time(lambda: ops.mlstm_step(c[0], c[1], c[2], d ** -0.5, resid, gtw, gb, 15.0, c[3], hn, 1e-6, sm, mm, cu, pos, slots,
+                                               Hd, d, d), 5)
+            row("mlstm_step (with gates, norm, output gate)", rshape, t_n, "hbm", S * Hd * d * d * 8, lshape, t_l, S * Hd * d * d * 8)
+        row("gated_head_rms_norm (all heads at once)", f"{tag} {T} rows x {Hd * d}",
+            _time(lambda: ops.gated_head_rms_norm(od.view(T, 1, -1), c[3], hn, 1e-6, ops.ACT_SIGMOID)), "hbm", T * Hd * d * 8,
+            "gated_head_rms_norm (per head)", _time(lambda: ops.gated_head_rms_norm(od, c[3], hn[:d], 1e-6, ops.ACT_SIGMOID)), T * Hd * d * 8)
+    return rows
+
+
+def compare_rigazen(widths, layers: int, batch: int, prompt_len: int, steps: int, warmup: int) -> dict:
+    """The Rigazen design beside the closest existing model, the "pre" arrangement (Lozupel: a windowed
+    attention beside a recurrence, recurrent layers with a matrix state, dense feed-forwards), at equal width,
+    depth and feed-forward weights."""
+    result = {"metric": "rigazen_vs_lozupel_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic",
+              "config": {"layers": layers, "batch": batch, "prompt_len": prompt_len, "decode_steps": steps},
+              "models": [], "kernels": {}}
+    for width in widths:
+        t = through_engine(ModelConfig.from_dict(rigazen_config(width, layers)), batch, prompt_len, steps, warmup)
+        z = through_engine(ModelConfig.from_dict(lozupel_config(width, layers, loop=False)), batch, prompt_len, steps, warmup)
+        result["models"].append({"width": width, "layers": layers, "rigazen": t, "lozupel": z,
+                                 "prefill_ratio": round(t["prefill_tok_s"] / z["prefill_tok_s"], 3),
+                                 "decode_ratio": round(t["decode_tok_s"] / z["decode_tok_s"], 3)})
+        result["kernels"][str(width)] = rigazen_kernel_table(width, prompt_len, batch)
     return result

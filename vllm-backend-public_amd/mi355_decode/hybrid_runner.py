@@ -798,7 +798,9 @@ class HybridRunner(ModelRunner):
                 self.layer_trace.append(resid.clone())
         return resid
 
-    SIDE_FUSED_ROWS = 64             # steps of up to this many rows take the per-layer token input in one launch
+    # steps of up to this many rows take the per-layer token input in one launch, if its two matrices are small
+    # (every row's workgroup reads both: measured 28 us for 32 rows of 2 x 2048 x 64, 93 us for 2 x 4096 x 128)
+    SIDE_FUSED_ROWS, SIDE_FUSED_WEIGHTS = 64, 1 << 17
 
     def _forward_post(self, b: StepBatch) -> torch.Tensor:
         """All layers of the post arrangement over one packed batch; returns the float32 residual stream
@@ -816,7 +818,7 @@ class HybridRunner(ModelRunner):
             if L.ff:
                 y = self.linear(ops.relu_squared(self.linear(x, lw.up_w)), lw.down_w)
                 ops.norm_resid_f32(resid, y, lw.norm2, eps, act_out=act)
-            if n and T <= self.SIDE_FUSED_ROWS and self.H <= 8192 and n <= 4096:
+            if n and T <= self.SIDE_FUSED_ROWS and self.H * n <= self.SIDE_FUSED_WEIGHTS and self.H <= 8192 and n <= 4096:
                 ops.token_side_f32(resid, lw.side_gate_w, lw.side_proj_w, lw.side_norm, w.side_embed, li * n, b.ids, eps, act_out=act)
             elif n:
                 g = ops.token_gate_rows(self.linear(x, lw.side_gate_w), w.side_embed, li * n, b.ids)

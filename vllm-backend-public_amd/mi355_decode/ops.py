@@ -1883,7 +1883,7 @@ def decay_attn(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, log_decay: tor
     if tiles is None:
         check(lib.mi355_decay_attn_step(o.data_ptr(), *rows, log_decay.data_ptr(), sp, *chunk, S, num_heads, dim, vdim, dt, _stream()))
         return o
-    ws = torch.empty(tiles.count * num_heads * state.shape[2], dtype=torch.float32, device=q.device)
+    ws = torch.empty(tiles.count * num_heads * (state.shape[2] + 1), dtype=torch.float32, device=q.device)
     check(lib.mi355_linear_attn_chunks(o.data_ptr(), *rows, 1.0, log_decay.data_ptr(), None, None, None, None, sp, *chunk,
                                        tiles.tiles.data_ptr(), tiles.start.data_ptr(), tiles.count, tiles.rows, S, num_heads,
                                        dim, vdim, T, ws.data_ptr(), ws.numel(), dt, _stream()))
@@ -1936,7 +1936,7 @@ def mlstm_chunks(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, q_scale: flo
                                 _f32(gate_b, "gate_b", 2 * H), float(cap), _f32(m_state, "m_state"), *chunk,
                                 tiles.start.data_ptr(), S, H, tiles.rows, T, _stream()))
     o = torch.empty(T, H, vdim, dtype=torch.float32, device=dev)
-    ws = torch.empty(tiles.count * H * state.shape[2], dtype=torch.float32, device=dev)
+    ws = torch.empty(tiles.count * H * (state.shape[2] + 1), dtype=torch.float32, device=dev)
     check(lib.mi355_linear_attn_chunks(o.data_ptr(), q.data_ptr(), _cols(q, "q", H * dim), _same(k, q, "k"), _cols(k, "k", H * dim),
                                        _same(v, q, "v"), _cols(v, "v", H * vdim), float(q_scale), None, ga.data_ptr(), gf.data_ptr(),
                                        gm.data_ptr(), tm.data_ptr(), sp, *chunk, tiles.tiles.data_ptr(), tiles.start.data_ptr(),
