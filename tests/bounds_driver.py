@@ -293,6 +293,64 @@ def parallel_layer_generation():
     return out
 
 
+def post_norm_generation():
+    """A hybrid decoder of the Rigazen design (norms on the outputs, windowed attention with kept tokens
+    beside a constant-decay linear attention, a matrix memory, per-layer token inputs): the same schedule
+    as above, in bfloat16 and in float32."""
+    from mi355_decode import weights as W
+    from mi355_decode.config import EngineArgs, ModelConfig
+    from mi355_decode.llm import build_engine
+    from mi355_decode.sampling_params import SamplingParams
+    left = {"heads": 8, "kv_heads": 2, "dim": 64, "vdim": 128, "mask": {"size": 40, "keep_first": 5}, "scale": 0.2,
+            "rot": {"dims": 32, "base": 10000.0}}
+    right = {"heads": 3, "dim": 32, "vdim": 40, "decay": [0.5, 0.99, 1.0]}
+    odd = dict(left, heads=3, kv_heads=1, dim=40, vdim=9, mask=None, rot=None)
+    cfg = ModelConfig.from_dict({
+        "architecture": "Rigazen", "width": 128, "vocab": 300, "norm": {"eps": 1e-6}, "embedding": {"scale": 10.0},
+        "token_side": {"dim": 24},
+        "layers": [{"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.5, "right_scale": 1.5},
+                    "mlp": {"kind": "dense", "ff": 192}},
+                   {"type": "mlstm", "mixer": {"heads": 3, "dim": 40, "vdim": 24, "gate_cap": 8.0}, "mlp": {"kind": "dense", "ff": 100}},
+                   {"type": "parallel", "mixer": {"left": odd, "right": dict(right, dim=21, vdim=7), "left_scale": 1.0, "right_scale": 1.0},
+                    "mlp": None},
+                   {"type": "mlstm", "mixer": {"heads": 2, "dim": 13, "vdim": 9, "gate_cap": 4.0}, "mlp": None}]})
+    state = W.hybrid_synthetic_state(cfg, seed=3)
+    rng = np.random.default_rng(1)
+    out = []
+    for dtype in ("bfloat16", "float32"):
+        bounds.clear()
+        eng = build_engine(EngineArgs(model="kept", dtype=dtype, max_num_seqs=4, max_model_len=256,
+                                      num_gpu_blocks_override=48, gpu_memory_utilization=0.0, max_num_batched_tokens=1 << 20),
+                           state_dict=state, model_config=cfg)
+
+        def run(tag):
+            toks = {r: rng.integers(0, 300, n).tolist() for r, n in (("a", 150), ("b", 37), ("c", 2))}
+            eng.forced_step([(tag + "a", toks["a"][:100], [99]), (tag + "c", toks["c"][:1], [0])])
+            eng.forced_step([(tag + "a", toks["a"][100:102], [1]), (tag + "b", toks["b"][:33], []), (tag + "c", toks["c"][1:], [0])],
+                            [tag + "c"])
+            for i in range(4):
+                eng.forced_step([(tag + "a", toks["a"][102 + i:103 + i], [0]), (tag + "b", toks["b"][33 + i:34 + i], [0])])
+            eng.forced_step([(tag + "a", toks["a"][106:], [])], [tag + "a", tag + "b"])
+            for i, n in enumerate((5, 70, 17)):
+                eng.add_request(f"{tag}g{i}", rng.integers(0, 300, n).tolist(),
+                                SamplingParams(max_tokens=10, temperature=0.0 if i else 0.8, seed=i, ignore_eos=True))
+            n = 0
+            while eng.has_unfinished():
+                n += sum(len(o.new_token_ids) for o in eng.step())
+            return n
+
+        run("warm")
+        n = bounds.sync_allocations(granularity="segment")
+        toks = run("checked")
+        rep = bounds.report()
+        assert rep is None or rep["refused"] == 0, (dtype, rep)
+        out.append(f"{dtype}:{toks} tokens:{n} segments:{rep['unknown_base'] if rep else 0} accesses with an unlisted base")
+        del eng
+        gc.collect()
+        torch.cuda.empty_cache()
+    return out
+
+
 def sampler_rows():
     """The sampling launch on exactly sized logits (no slack behind the last row), every kind of
     row in one call: greedy, whole-vocabulary draw, top-k / top-p cuts, an all-tied row (the list
@@ -333,4 +391,5 @@ if __name__ == "__main__":
     res["sandwich"] = sandwich_generation()
     res["block_mixers"] = block_mixer_generation()
     res["parallel_layers"] = parallel_layer_generation()
+    res["post_norms"] = post_norm_generation()
     print(json.dumps(res))
