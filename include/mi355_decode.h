@@ -1109,8 +1109,8 @@ int64_t mi355_mingru_scan_workspace(int32_t num_seqs, int32_t channels, int32_t 
  *                         (fp32 [slots, heads, linear_attn_state_floats]) updated in place, zeros for a chunk that
  *                         starts at position 0
  *   mlstm_step            a = cap tanh((gate_w[h] x + b[h]) / cap), f = log sigmoid(cap tanh((gate_w[H + h] x +
- *                         b[H + h]) / cap)); m' = max(f + m, a); S <- e^(f + m - m') S + e^(a - m') k v^T, n likewise
- *                         with k alone; o = S^T q / (max(|n . q|, e^-m') + 1e-6), q times q_scale; out = o / rms(o) *
+ *                         b[H + h]) / cap)); m' = max(f + m, a); S <- e^(f + m - m') S + e^(a - m') k v^T, n the same
+ *                         sum over the keys; o = S^T q / (max(|n . q|, e^-m') + 1e-6), q times q_scale; out = o / rms(o) *
  *                         norm[h] * sigmoid(g) in `dtype`.  State: S, then n; m_state [slots, heads]
  *   mlstm_gates           for chunks of many tokens, from z [tokens, 2 heads] (the gate products without biases), by
  *                         tiles of up to tile_rows rows of a chunk: log_in = a, log_decay_sum = f summed from the

@@ -3,7 +3,7 @@
 //
 //   constant decay    S <- decay[h] S + k v^T,  o = S^T q         q, k, v through silu
 //   matrix memory     a = cap tanh((zi + bi) / cap),  b = log sigmoid(cap tanh((zf + bf) / cap))
-//                     m' = max(b + m, a);  S <- e^(b + m - m') S + e^(a - m') k v^T;  n likewise with k alone
+//                     m' = max(b + m, a);  S <- e^(b + m - m') S + e^(a - m') k v^T;  n the same sum over the keys
 //                     o = S^T q / (max(|n . q|, e^-m') + 1e-6)         q times a constant
 //
 // State, per slot and head: S [d, dv], then (matrix memory) n [d], padded to a multiple of 4 floats;
@@ -471,7 +471,7 @@ __global__ __launch_bounds__(256) void la_step_kernel(
   if (MEM && !fresh) m = MI355_LD(float, M.m_state, M.m_state + slot * D.H + h);
   const float dec = MEM ? 0.f : expf(static_cast<float>(MI355_LD(double, log_decay, log_decay + h)));
   const int tx = tid % cg, ty = tid / cg;
-  constexpr int PF = 16;
+  constexpr int PF = 8;
   float S[PF][VW];
   // rows i0, i0 + rg, ... of column group c of the state
   auto fetch = [&](int i0, int c) {
