@@ -298,7 +298,8 @@ int32_t mi355_paged_attn_prefill(void* out, int64_t out_stride, const void* q,
  * sink (fp32 [num_heads], may be null): one more term exp(sink[h]) in the softmax denominator,
  * without a value; gate (dtype, rows gate_stride apart, may be null): the output of (token, head) is
  * multiplied by sigmoid(gate[token, head]).  window > 0: the keys j > p - window only, and (chunk 0)
- * the first `keep` keys of the sequence.  The output is multiplied by out_scale.  K pages
+ * the first `keep` keys of the sequence.  The output is multiplied by out_scale.  softcap > 0: scores are
+ * softcap * tanh(q.k * scale / softcap).  K pages
  * [blocks, kv_heads, 16, head_dim], V pages [blocks, kv_heads, v_dim, 16], head_dim and v_dim each 64 or 128.
  */
 int32_t mi355_paged_attn_prefill_ext(void* out, int64_t out_stride, const void* q, int64_t q_stride,
@@ -308,7 +309,7 @@ int32_t mi355_paged_attn_prefill_ext(void* out, int64_t out_stride, const void* 
                                      int32_t num_seqs, int32_t max_q_len, int32_t num_heads,
                                      int32_t num_kv_heads, int32_t head_dim, int32_t v_dim, float scale,
                                      int32_t chunk, int32_t window, int32_t keep, const float* sink,
-                                     const void* gate, int64_t gate_stride, float out_scale,
+                                     const void* gate, int64_t gate_stride, float out_scale, float softcap,
                                      int32_t dtype, void* stream);
 
 /*
@@ -782,6 +783,13 @@ int32_t mi355_resid_add_f32(float* resid, const float* other, const void* rows, 
 int32_t mi355_add_rms_norm_f32(void* out, float* resid, const void* add, const void* weight,
                                int32_t weight_numel, int64_t num_tokens, int32_t width, float eps,
                                int32_t dtype, void* stream);
+/* resid += add, then out = (resid - mean) / sqrt(variance + eps) * weight (dtype, width numbers; out null: the add
+ * alone).  inv not null: add holds a mixture's rows in expert order and token t's addend is
+ * row_weight * sum_k add[inv[t * top + k]]. */
+int32_t mi355_add_layer_norm_f32(void* out, float* resid, const void* add, const int32_t* inv,
+                                 int32_t top, float row_weight, const void* weight,
+                                 int64_t num_tokens, int32_t width, float eps, int32_t dtype,
+                                 void* stream);
 int32_t mi355_rms_norm_mix_f32(float* resid, const void* xa, const void* wa, const void* xb,
                                const void* wb, int64_t num_tokens, int32_t width, float eps,
                                float alpha, int32_t dtype, void* stream);
@@ -915,7 +923,7 @@ int32_t mi355_tanh_rows(void* out, const void* x, int64_t x_stride, int64_t num_
  * rotated key part [rot] shared by all heads: cache [blocks, 16, rank + rot].
  *   latent_kv_write      x [tokens, rank + rot] (a column slice is fine): c = x[:rank] / rms * norm_weight,
  *                        the last rot columns rotated (first rot_dims of them, coordinate i with
- *                        i + rot_dims / 2, table cos_sin [max_pos, rot_dims] = cos | sin), into the
+ *                        i + rot_dims / 2, or neighbours 2i, 2i + 1 if `interleaved`, table cos_sin [max_pos, rot_dims] = cos | sin), into the
  *                        row's page slot; rows with slot < 0 store nothing.  cache_t (may be null):
  *                        a second, channel-major copy of the latent, [blocks, rank, 16]
  *   latent_window_attn   out[t, h] = sigmoid(gate[t, h]) * sum_j p_j c_j over the keys j of the row's
@@ -926,13 +934,15 @@ int32_t mi355_tanh_rows(void* out, const void* x, int64_t x_stride, int64_t num_
  *                        space, rank numbers at q_latent + t * q_latent_stride + h * q_latent_head_stride
  *                        (token-major or head-major); q [tokens, heads * q_head_width] holds the part to
  *                        rotate at q_rot_offset of every head.  out: rank numbers per (t, h), strides
- *                        likewise; the caller applies the value up-projection.  gate may be null.
+ *                        likewise; the caller applies the value up-projection.  gate and sink (an ordinary
+ *                        softmax then) may be null.
  */
 int32_t mi355_latent_kv_write(void* cache, void* cache_t, const void* x, int64_t x_stride,
                               const float* norm_weight,
                               const float* cos_sin, int32_t max_pos, const int64_t* positions,
                               const int64_t* slot_mapping, int64_t num_tokens, int32_t rank,
-                              int32_t rot, int32_t rot_dims, float eps, int32_t dtype, void* stream);
+                              int32_t rot, int32_t rot_dims, int32_t interleaved, float eps,
+                              int32_t dtype, void* stream);
 /*
  * The matrix-core form of latent_window_attn (16-bit storage, rank a multiple of 16 up to 512,
  * rank + rot a multiple of 8 up to 640), same result.
@@ -949,7 +959,7 @@ int32_t mi355_latent_q_pack(void* q_packed, const void* q_latent, int64_t q_late
                             int32_t q_head_width, int32_t q_rot_offset, const float* cos_sin,
                             int32_t max_pos, const int64_t* positions, int64_t num_tokens,
                             int32_t num_heads, int32_t rank, int32_t rot, int32_t rot_dims,
-                            int32_t dtype, void* stream);
+                            int32_t interleaved, int32_t dtype, void* stream);
 int32_t mi355_latent_window_attn_tiles(void* out, int64_t out_stride, int64_t out_head_stride,
                                        const void* q_packed, const void* cache, const void* cache_t,
                                        const int32_t* block_tables, int32_t max_blocks,
@@ -967,7 +977,7 @@ int32_t mi355_latent_window_attn(void* out, int64_t out_stride, int64_t out_head
                                  const float* sink, const void* gate, int64_t gate_stride,
                                  const float* cos_sin, int32_t max_pos, int64_t num_tokens,
                                  int32_t num_heads, int32_t rank, int32_t rot, int32_t rot_dims,
-                                 int32_t window, float scale, int32_t dtype, void* stream);
+                                 int32_t interleaved, int32_t window, float scale, int32_t dtype, void* stream);
 
 /*
  * Mixture-of-experts feed-forward.  A routed row is (token t, choice k), number t * top + k.
@@ -982,6 +992,9 @@ int32_t mi355_latent_window_attn(void* out, int64_t out_stride, int64_t out_head
  *                     alone, times weight_scale
  *   moe_sort          routed rows by expert: offsets [experts + 1], perm[position] = row,
  *                     inv[row] = position
+ *   moe_table_sort    a mixture without a router: tables [layers][vocab, top] name the experts of every token
+ *                     id; for every layer offsets [experts + 1], perm and inv as moe_sort, and tile_start
+ *                     [experts + 1], the first tile of tile_rows rows of every expert (stacked by layer)
  *   moe_gather_rows   xs[position] = x[perm[position] / top] for num_rows positions (pad_to 0); with
  *                     pad_to > 0, num_rows = experts * pad_to and xs[e * pad_to + j] is the j-th row of
  *                     expert e, zeros past its count (one batched product over all experts then)
@@ -989,6 +1002,8 @@ int32_t mi355_latent_window_attn(void* out, int64_t out_stride, int64_t out_head
  *                     a(g, u) = silu(g) * u (act 0), or with g = min(g, limit), u = clamp(u, -limit,
  *                     limit): g * sigmoid(1.702 g) * (u + 1) (act 1)
  *   moe_down_rows     y[position] = Wd[e] act[position]; w_down [experts, width, ff]
+ *   moe_linear_rows   y[position] = a(W[e] x[perm[position] / top]) (perm null: x[position]); w [experts,
+ *                     out_width, in_width]; a: identity, or relu2: max(., 0)^2
  *   moe_silu_and_mul  out = a(x[:, :ff], x[:, ff:])
  *   gated_act_rows    out[r, :ff] = a(gate[r, :ff], up[r, :ff]): gate and up rows in_stride apart, out
  *                     rows out_stride apart (column slices of wider buffers)
@@ -1011,6 +1026,13 @@ int32_t mi355_moe_gate_up_rows(void* act, const void* x, const void* w_gate_up, 
                                int32_t ff, int32_t act_fn, float limit, int32_t dtype, void* stream);
 int32_t mi355_moe_down_rows(void* y, const void* act, const void* w_down, const int32_t* offsets,
                             int32_t experts, int32_t width, int32_t ff, int32_t dtype, void* stream);
+int32_t mi355_moe_linear_rows(void* y, const void* x, const void* w, const int32_t* offsets,
+                              const int32_t* perm, int32_t top, int32_t relu2, int32_t experts,
+                              int32_t out_width, int32_t in_width, int32_t dtype, void* stream);
+int32_t mi355_moe_table_sort(int32_t* offsets, int32_t* tile_start, int32_t* perm, int32_t* inv,
+                             const int32_t* tables, const int64_t* ids, int64_t num_tokens,
+                             int64_t vocab, int32_t layers, int32_t experts, int32_t top,
+                             int32_t tile_rows, void* stream);
 int32_t mi355_moe_silu_and_mul(void* out, const void* x, int64_t num_rows, int32_t ff, int32_t act_fn,
                                float limit, int32_t dtype, void* stream);
 int32_t mi355_gated_act_rows(void* out, int64_t out_stride, const void* gate, const void* up,
@@ -1036,10 +1058,12 @@ int32_t mi355_moe_combine(void* out, const void* y, const int32_t* inv, const fl
  *   row_norm_rope_kv_write  q <- rotate(rms(q row) * q_weight) in place, the RMS norm over all heads of the row at
  *                         once (weights fp32 [heads * head_dim]); K pages <- the same of the k row; V pages <- v;
  *                         rotation of the first rot_dims coordinates of every head, pairs (i, i + rot_dims / 2), by
- *                         cos_sin fp32 [max_pos, rot_dims] = cos | sin
+ *                         cos_sin fp32 [max_pos, rot_dims] = cos | sin.  temp_every > 0: q is also multiplied by
+ *                         1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
  *   softmax_bias_attn     out[t,h] = sigmoid(gate) * sum_j softmax_j(q.k_j * scale - r1[h] ln(1 + r2[h]
  *                         (p - j))) v_j over the keys j <= p with j >= (p / block) * block (block 0: all)
- *                         and, window > 0, j > p - window or (block 0) j < keep; times out_scale.  gate: one number per head or
+ *                         and, window > 0, j > p - window or (block 0) j < keep; times out_scale.  softcap > 0
+ *                         (r1, r2 null): the score is softcap * tanh(q.k_j * scale / softcap).  gate: one number per head or
  *                         (gate_per_channel) per output channel; r1 / r2 null: no penalty.  sink (fp32
  *                         [heads], may be null): one more term exp(sink[h]) in the softmax denominator,
  *                         without a value.  Output rows are out_stride elements apart.  tiles as for
@@ -1073,8 +1097,8 @@ int32_t mi355_row_norm_rope_kv_write(void* q, int64_t q_stride, const void* k, i
                                      const int64_t* positions, const int64_t* slot_mapping,
                                      void* k_cache, void* v_cache, int64_t num_tokens,
                                      int32_t num_heads, int32_t num_kv_heads, int32_t head_dim,
-                                     int32_t v_dim, int32_t rot_dims, float eps, int32_t dtype,
-                                     void* stream);
+                                     int32_t v_dim, int32_t rot_dims, float eps, float temp_coef,
+                                     double temp_every, int32_t dtype, void* stream);
 int64_t mi355_softmax_bias_attn_workspace(int64_t num_tokens, int32_t num_heads, int32_t v_dim,
                                           int32_t num_splits);
 int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_stride, const void* k_cache,
@@ -1085,8 +1109,8 @@ int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_stride, cons
                                 int32_t num_kv_heads, int32_t head_dim, int32_t v_dim, int32_t block,
                                 int32_t window, int32_t keep, float scale, const int32_t* tiles,
                                 int32_t num_tiles, float* workspace, int32_t num_splits,
-                                const float* sink, int64_t out_stride, float out_scale, int32_t dtype,
-                                void* stream);
+                                const float* sink, int64_t out_stride, float out_scale, float softcap,
+                                int32_t dtype, void* stream);
 int32_t mi355_mingru_scan(void* out, const void* proj, int64_t stride, int32_t z_off, int32_t x_off,
                           int32_t g_off, const float* z_bias, const float* x_bias, float* state,
                           const int32_t* cu_seqlens, const int64_t* positions,

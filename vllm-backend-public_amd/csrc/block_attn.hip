@@ -7,10 +7,12 @@
 //                         passes k again)
 //   row_norm_rope_kv_write   q <- rotate(rms(q row) * wq), in place, the norm over all heads of the row at once; K pages <-
 //                         the same of the k row; V pages <- v.  Rotation of the first rot coordinates of every head by a
-//                         fp32 table (pairs i, i + rot / 2)
+//                         fp32 table (pairs i, i + rot / 2).  temp_every > 0: q is also multiplied by
+//                         1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
 //   softmax_bias_attn     out[t,h] = gate[t,h,:] * sum_j softmax_j(q.k_j * scale - r1[h] ln(1 + r2[h] (p - j))) v_j
 //                         over the keys j <= p of p's block: lo = (p / block) * block (block 0: lo = 0), and
-//                         with a window also j > p - window or (keep first) j < keep.  Blocks are counted from
+//                         with a window also j > p - window or (keep first) j < keep.  softcap > 0: the score
+//                         is softcap * tanh(q.k_j * scale / softcap) instead (no penalty).  Blocks are counted from
 //                         position 0 of the sequence.  The output is multiplied by out_scale.  gate: sigmoid of one number per head or per output channel.
 //                         sink (fp32, one score per head, may be null): the softmax denominator holds one
 //                         more term exp(sink[h]) that carries no value.  Output rows are out_stride apart
@@ -73,11 +75,13 @@ __global__ __launch_bounds__(256) void row_norm_rope_kv_write_kernel(
     const typename Elem<T>::S* __restrict__ v, int64_t v_stride, const float* __restrict__ wq, const float* __restrict__ wk,
     const float* __restrict__ cos_sin, int64_t max_pos, const int64_t* __restrict__ positions,
     const int64_t* __restrict__ slot_mapping, typename Elem<T>::S* __restrict__ k_cache,
-    typename Elem<T>::S* __restrict__ v_cache, int H, int G, int d, int dv, int rot, float eps) {
+    typename Elem<T>::S* __restrict__ v_cache, int H, int G, int d, int dv, int rot, float eps, float temp_coef, double temp_every) {
   typedef typename Elem<T>::S E;
   __shared__ float scratch[32];
   const int64_t t = blockIdx.x;
   int64_t p = MI355_LD(int64_t, positions, positions + t);
+  float temp = 1.0f;
+  if (temp_every > 0.0) temp += temp_coef * logf(static_cast<float>(floor(static_cast<double>(p + 1) / temp_every)) + 1.0f);
   p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
   const int64_t slot = MI355_LD(int64_t, slot_mapping, slot_mapping + t);
   const int64_t page = slot / kPageB, off = slot % kPageB;
@@ -94,7 +98,7 @@ __global__ __launch_bounds__(256) void row_norm_rope_kv_write_kernel(
     const float x = MI355_LDF(T, k, kr + i);
     sk += x * x;
   }
-  const float rq = 1.0f / sqrtf(block_sum32(sq, scratch) / static_cast<float>(H * d) + eps);
+  const float rq = temp / sqrtf(block_sum32(sq, scratch) / static_cast<float>(H * d) + eps);
   const float rk = 1.0f / sqrtf(block_sum32(sk, scratch) / static_cast<float>(G * d) + eps);
   for (int i = threadIdx.x; i < (slot < 0 ? H : H + G) * units; i += blockDim.x) {
     const int hh = i / units, u = i - hh * units;
@@ -147,7 +151,8 @@ __global__ __launch_bounds__(64) void softmax_bias_attn_kernel(
     const int32_t* __restrict__ block_tables, int max_blocks, const int32_t* __restrict__ tok_seq,
     const int64_t* __restrict__ positions, const float* __restrict__ r1, const float* __restrict__ r2,
     const typename Elem<T>::S* __restrict__ gate, int64_t gate_stride, int gate_per_channel, int H, int G, int d, int dv,
-    int block, int window, int keep, float scale, const float* __restrict__ sink, int64_t out_stride, float out_scale) {
+    int block, int window, int keep, float scale, const float* __restrict__ sink, int64_t out_stride, float out_scale,
+    float softcap) {
   extern __shared__ float lds[];                        // q [d] | w [64]
   float* qs = lds;
   float* ws = lds + d;
@@ -180,6 +185,7 @@ __global__ __launch_bounds__(64) void softmax_bias_attn_kernel(
       float dot = 0.f;
       for (int i = 0; i < d; ++i) dot += qs[i] * MI355_LDF(T, k_cache, kr + i);
       s = dot * scale - a1 * log1pf(a2 * static_cast<float>(p - j));
+      if (softcap > 0.f) s = softcap * tanhf(s / softcap);
     }
     float tm = s;
 #pragma unroll
@@ -227,7 +233,7 @@ __global__ __launch_bounds__(64) void softmax_bias_attn_kernel(
   }
 }
 
-// The matrix-core form for 16-bit storage, d a multiple of 32, dv a multiple of 16.  One wave per
+// The matrix-core form for 16-bit storage, d a multiple of 8, dv a multiple of 16.  One wave per
 // (tile of up to 16 consecutive rows of one chunk, HB query heads of one kv head): K and V fragments
 // are loaded once for the HB heads.  Keys go 32 at a time (two pages).  Scores are computed
 // transposed, S^T = K Q^T: a lane then holds, for its query (lane % 16), the scores of keys
@@ -238,15 +244,16 @@ __global__ __launch_bounds__(64) void softmax_bias_attn_kernel(
 // gridDim.z > 1: the 32-key tiles are dealt out to the z workgroups in turn, each leaves its
 // accumulators, maxima and sums in fp32 scratch, and bias_attn_merge_kernel joins them.
 // DS / CB: fragment counts the registers are sized for (2 / 4 for heads of up to 64 channels, else
-// 4 / 8); PEN: the distance penalty is computed (off: no logarithm per score).
-template <typename T, int HB, int DS, int CB, bool PEN>
+// 4 / 8); MODE: 0 the plain score, 1 with the distance penalty, 2 with the soft cap.
+template <typename T, int HB, int DS, int CB, int MODE>
 __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
     uint16_t* __restrict__ out, const uint16_t* __restrict__ q, int64_t q_stride, const uint16_t* __restrict__ k_cache,
     const uint16_t* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tiles, int num_tiles, const int64_t* __restrict__ positions, const float* __restrict__ r1,
     const float* __restrict__ r2, const uint16_t* __restrict__ gate, int64_t gate_stride, int gate_per_channel, int H, int G,
     int d, int dv, int block, int window, int keep, float scale, float* __restrict__ part_acc, float* __restrict__ part_ml,
-    int64_t total_rows, const float* __restrict__ sink, int64_t out_stride, float out_scale) {
+    int64_t total_rows, const float* __restrict__ sink, int64_t out_stride, float out_scale, float softcap) {
+  constexpr bool PEN = MODE == 1, CAP = MODE == 2;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   // Workgroups go to the 8 XCDs in turn (x fastest), each XCD with an L2 of its own.  Where the plane of
   // workgroups divides by 8, XCD k takes the k-th eighth of the (head group, tile) pairs in head-major order:
@@ -270,7 +277,7 @@ __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
   const int nrows = MI355_LD(int32_t, tiles, tiles + 3 * tile + 2);
   const int64_t p0 = MI355_LD(int64_t, positions, positions + row0);
   const int32_t* bt = block_tables + static_cast<int64_t>(seq) * max_blocks;
-  const int ds = d >> 5, cbs = dv >> 4;
+  const int ds = (d + 31) >> 5, cbs = dv >> 4;            // (d a multiple of 8: the last fragment may be part zeros)
   const int64_t p_last = p0 + nrows - 1;
   const int64_t lo0 = first_visible(p0, block, window);
   const bool valid = li < nrows;
@@ -280,12 +287,14 @@ __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
   float a1[HB], a2[HB], m[HB], l[HB];
   f32x4 acc[HB][CB];
   const float scale2 = scale * kLog2eB;
+  // soft cap, base 2: cap tanh(x / cap) log2(e) = cap2 - 2 cap2 / (1 + 2^(x 2 log2(e) / cap)), x = q.k scale
+  const float cap2 = CAP ? softcap * kLog2eB : 0.f, capx = CAP ? 2.0f * scale2 / softcap : 0.f;
 #pragma unroll
   for (int i = 0; i < HB; ++i) {
 #pragma unroll
     for (int s = 0; s < DS; ++s) {
       qf[i][s] = make_uint4(0, 0, 0, 0);
-      if (s < ds && valid)
+      if (valid && 32 * s + 8 * kk < d)
         qf[i][s] = MI355_LD(uint4, q, q + (row0 + li) * q_stride + static_cast<int64_t>(h0 + i) * d + 32 * s + 8 * kk);
     }
     a1[i] = PEN ? MI355_LD(float, r1, r1 + h0 + i) : 0.f;               // ln(x) r1 = log2(x) r1 ln 2, times log2 e again: r1
@@ -328,7 +337,7 @@ __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
       const uint16_t* vr = v_cache + ((page * G + g) * dv + li) * kPageB + 4 * kk;
 #pragma unroll
       for (int s = 0; s < DS; ++s)
-        kf[half][s] = (have && s < ds) ? MI355_LD(uint4, k_cache, kr + 32 * s) : make_uint4(0, 0, 0, 0);
+        kf[half][s] = (have && 32 * s + 8 * kk < d) ? MI355_LD(uint4, k_cache, kr + 32 * s) : make_uint4(0, 0, 0, 0);
 #pragma unroll
       for (int c = 0; c < CB; ++c)
         vf[half][c] = (have && c < cbs) ? MI355_LD(uint2, v_cache, vr + 16 * c * kPageB) : make_uint2(0, 0);
@@ -375,6 +384,7 @@ __global__ __launch_bounds__(256) void softmax_bias_attn_mfma_kernel(
         for (int r = 0; r < 4; ++r) {
           // base 2 throughout: q.k scale log2(e) - r1 log2(1 + r2 dist)
           sc[half][r] = sacc[r] * scale2;
+          if (CAP) sc[half][r] = cap2 - 2.0f * cap2 * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sacc[r] * capx));
           if (PEN) sc[half][r] -= a1[i] * __builtin_amdgcn_logf(1.0f + a2[i] * dist[half][r]);
           if (vis[half][r]) tmax = fmaxf(tmax, sc[half][r]);
         }
@@ -560,8 +570,8 @@ extern "C" int32_t mi355_row_norm_rope_kv_write(void* q, int64_t q_stride, const
                                                 const float* cos_sin, int64_t max_pos, const int64_t* positions,
                                                 const int64_t* slot_mapping, void* k_cache, void* v_cache,
                                                 int64_t num_tokens, int32_t num_heads, int32_t num_kv_heads,
-                                                int32_t head_dim, int32_t v_dim, int32_t rot_dims, float eps, int32_t dtype,
-                                                void* stream) {
+                                                int32_t head_dim, int32_t v_dim, int32_t rot_dims, float eps, float temp_coef,
+                                                double temp_every, int32_t dtype, void* stream) {
   MI355_REQUIRE(q && k && v && q_weight && k_weight && positions && slot_mapping && k_cache && v_cache, MI355_ERR_INVALID,
                 "row_norm_rope_kv_write: null pointer");
   MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && num_kv_heads > 0 && head_dim > 0 && v_dim > 0 && rot_dims >= 0 &&
@@ -580,7 +590,7 @@ extern "C" int32_t mi355_row_norm_rope_kv_write(void* q, int64_t q_stride, const
                                                   static_cast<const Elem<TT>::S*>(v), v_stride, q_weight, k_weight, cos_sin,
                                                   max_pos, positions, slot_mapping, static_cast<Elem<TT>::S*>(k_cache),
                                                   static_cast<Elem<TT>::S*>(v_cache), num_heads, num_kv_heads, head_dim,
-                                                  v_dim, rot_dims, eps));
+                                                  v_dim, rot_dims, eps, temp_coef, temp_every));
   return check_launch("row_norm_rope_kv_write");
 }
 
@@ -589,7 +599,7 @@ static void launch_bias_attn(hipStream_t s, void* out, const void* q, int64_t q_
                              const void* v_cache, const int32_t* block_tables, int32_t max_blocks, const int32_t* tok_seq,
                              const int64_t* positions, const float* r1, const float* r2, const void* gate,
                              int64_t gate_stride, int gate_per_channel, int64_t T, int H, int G, int d, int dv, int block,
-                             int window, int keep, float scale, const float* sink, int64_t out_stride, float out_scale) {
+                             int window, int keep, float scale, const float* sink, int64_t out_stride, float out_scale, float softcap) {
   typedef typename Elem<TT>::S E;
   const dim3 grid(static_cast<unsigned>(T), static_cast<unsigned>(H));
   const size_t lds = (static_cast<size_t>(d) + 64) * sizeof(float);
@@ -598,7 +608,7 @@ static void launch_bias_attn(hipStream_t s, void* out, const void* q, int64_t q_
                      static_cast<const E*>(q), q_stride, static_cast<const E*>(k_cache),                           \
                      static_cast<const E*>(v_cache), block_tables, max_blocks, tok_seq, positions, r1, r2,         \
                      static_cast<const E*>(gate), gate_stride, gate_per_channel, H, G, d, dv, block, window, keep, \
-                     scale, sink, out_stride, out_scale)
+                     scale, sink, out_stride, out_scale, softcap)
   if (dv <= 64) MI355_BATTN(1);
   else if (dv <= 128) MI355_BATTN(2);
   else if (dv <= 256) MI355_BATTN(4);
@@ -618,7 +628,9 @@ extern "C" int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_s
                                            int32_t num_kv_heads, int32_t head_dim, int32_t v_dim, int32_t block,
                                            int32_t window, int32_t keep, float scale, const int32_t* tiles,
                                            int32_t num_tiles, float* workspace, int32_t num_splits, const float* sink,
-                                           int64_t out_stride, float out_scale, int32_t dtype, void* stream) {
+                                           int64_t out_stride, float out_scale, float softcap, int32_t dtype, void* stream) {
+  MI355_REQUIRE(softcap >= 0.f && (softcap == 0.f || r1 == nullptr), MI355_ERR_INVALID,
+                "softmax_bias_attn: a soft cap (%g) does not go with a penalty", softcap);
   MI355_REQUIRE(out && q && k_cache && v_cache && block_tables && tok_seq && positions, MI355_ERR_INVALID,
                 "softmax_bias_attn: null pointer");
   MI355_REQUIRE((r1 == nullptr) == (r2 == nullptr), MI355_ERR_INVALID, "softmax_bias_attn: r1 and r2 go together");
@@ -634,7 +646,7 @@ extern "C" int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_s
   REQ_DTYPE(dtype);
   if (num_tokens == 0) return MI355_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (tiles != nullptr && num_tiles > 0 && dtype != MI355_F32 && head_dim % 32 == 0 && head_dim <= 128 &&
+  if (tiles != nullptr && num_tiles > 0 && dtype != MI355_F32 && head_dim % 8 == 0 && head_dim <= 128 &&
       v_dim % 16 == 0 && v_dim <= 128 && q_stride % 8 == 0 && aligned16(q) && aligned16(k_cache) && aligned16(v_cache)) {
     const int rep = num_heads / num_kv_heads;
     const bool split = workspace != nullptr && num_splits > 1;
@@ -650,18 +662,20 @@ extern "C" int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_s
     float* part_ml = split ? workspace + static_cast<int64_t>(num_splits) * pairs * v_dim : nullptr;
 #define MI355_BMFMA(TT, HB)                                                                                         \
   do {                                                                                                              \
-    if (small && r1 != nullptr) MI355_BMFMA_K(TT, HB, 2, 4, true);                                                  \
-    else if (small) MI355_BMFMA_K(TT, HB, 2, 4, false);                                                             \
-    else if (r1 != nullptr) MI355_BMFMA_K(TT, HB, 4, 8, true);                                                      \
-    else MI355_BMFMA_K(TT, HB, 4, 8, false);                                                                        \
+    if (small && r1 != nullptr) MI355_BMFMA_K(TT, HB, 2, 4, 1);                                                     \
+    else if (small && softcap > 0.f) MI355_BMFMA_K(TT, HB, 2, 4, 2);                                                \
+    else if (small) MI355_BMFMA_K(TT, HB, 2, 4, 0);                                                                 \
+    else if (r1 != nullptr) MI355_BMFMA_K(TT, HB, 4, 8, 1);                                                         \
+    else if (softcap > 0.f) MI355_BMFMA_K(TT, HB, 4, 8, 2);                                                         \
+    else MI355_BMFMA_K(TT, HB, 4, 8, 0);                                                                            \
   } while (0)
-#define MI355_BMFMA_K(TT, HB, DS, CB, PEN)                                                                          \
-  hipLaunchKernelGGL((softmax_bias_attn_mfma_kernel<TT, HB, DS, CB, PEN>), grid, block_dim, 0, s,                   \
+#define MI355_BMFMA_K(TT, HB, DS, CB, MODE)                                                                          \
+  hipLaunchKernelGGL((softmax_bias_attn_mfma_kernel<TT, HB, DS, CB, MODE>), grid, block_dim, 0, s,                  \
                      static_cast<uint16_t*>(out), static_cast<const uint16_t*>(q), q_stride,                        \
                      static_cast<const uint16_t*>(k_cache), static_cast<const uint16_t*>(v_cache), block_tables,    \
                      max_blocks, tiles, num_tiles, positions, r1, r2, static_cast<const uint16_t*>(gate),           \
                      gate_stride, gate_per_channel, num_heads, num_kv_heads, head_dim, v_dim, block, window, keep,  \
-                     scale, part_acc, part_ml, num_tokens, sink, out_stride, out_scale)
+                     scale, part_acc, part_ml, num_tokens, sink, out_stride, out_scale, softcap)
 #define MI355_BMFMA_HB(TT)                                                                                          \
   do {                                                                                                              \
     if (hb == 4) MI355_BMFMA(TT, 4);                                                                                \
@@ -686,6 +700,6 @@ extern "C" int32_t mi355_softmax_bias_attn(void* out, const void* q, int64_t q_s
   MI355_DISPATCH_DTYPE3(dtype, launch_bias_attn<TT>(s, out, q, q_stride, k_cache, v_cache, block_tables, max_blocks,
                                                    tok_seq, positions, r1, r2, gate, gate_stride, gate_per_channel,
                                                    num_tokens, num_heads, num_kv_heads, head_dim, v_dim, block, window,
-                                                   keep, scale, sink, out_stride, out_scale));
+                                                   keep, scale, sink, out_stride, out_scale, softcap));
   return check_launch("softmax_bias_attn");
 }

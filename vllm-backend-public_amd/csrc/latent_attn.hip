@@ -13,6 +13,8 @@
 //                        result is multiplied by sigmoid(gate[i, h])
 //   latent_q_pack        the query as the matrix-core form reads it: [absorbed part | rotated part] per
 //                        (row, head), contiguous
+// Without a sink (null) the softmax is the ordinary one; a window longer than the sequence is plain causal.
+// Rotation pairs coordinates j, j + dims/2 or (interleaved) neighbours.
 // Scores, weights, the softmax and its running sums, norms and angles are fp32.
 //
 // The matrix-core form (16-bit storage, rank a multiple of 16, rank + rot of 8).  All heads of a row
@@ -31,12 +33,19 @@ namespace mi355 {
 
 constexpr int kPageL = MI355_BLOCK_SIZE;
 
-// rotate coordinate j of a vector of `rot` coordinates whose first `dims` are rotated (pairs j, j + dims/2)
+// rotate coordinate j of a vector of `rot` coordinates whose first `dims` are rotated: pairs j, j + dims/2, or
+// (interleaved) neighbours 2i, 2i + 1
 template <typename T>
 __device__ __forceinline__ float rotated_at(const typename Elem<T>::S* base, const typename Elem<T>::S* v, int j, int dims,
-                                            const float* table, const float* cs) {
+                                            int interleaved, const float* table, const float* cs) {
   const int half = dims >> 1;
   if (j >= dims) return MI355_LDF(T, base, v + j);
+  if (interleaved) {
+    const int i = j >> 1;
+    const float c = MI355_LD(float, table, cs + i), s = MI355_LD(float, table, cs + half + i);
+    const float x = MI355_LDF(T, base, v + j), y = MI355_LDF(T, base, v + (j ^ 1));
+    return (j & 1) ? x * c + y * s : x * c - y * s;
+  }
   if (j < half) {
     const float c = MI355_LD(float, table, cs + j), s = MI355_LD(float, table, cs + half + j);
     return MI355_LDF(T, base, v + j) * c - MI355_LDF(T, base, v + j + half) * s;
@@ -54,7 +63,7 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(typename Elem<T>::
                                                               const float* __restrict__ cos_sin, int max_pos,
                                                               const int64_t* __restrict__ positions,
                                                               const int64_t* __restrict__ slot_mapping, int rank, int rot,
-                                                              int dims, float eps) {
+                                                              int dims, int interleaved, float eps) {
   __shared__ float scratch[32];
   const int64_t t = blockIdx.x;
   const int64_t slot = MI355_LD(int64_t, slot_mapping, slot_mapping + t);
@@ -78,7 +87,7 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(typename Elem<T>::
   }
   const float* cs = cos_sin + p * dims;
   for (int j = threadIdx.x; j < rot; j += blockDim.x)
-    MI355_STF(T, cache, dst + rank + j, rotated_at<T>(x, row + rank, j, dims, cos_sin, cs));
+    MI355_STF(T, cache, dst + rank + j, rotated_at<T>(x, row + rank, j, dims, interleaved, cos_sin, cs));
 }
 
 __device__ __forceinline__ float wave_max(float v) {
@@ -98,7 +107,7 @@ __global__ __launch_bounds__(64) void latent_window_attn_kernel(
     const typename Elem<T>::S* __restrict__ cache, const int32_t* __restrict__ block_tables, int max_blocks,
     const int32_t* __restrict__ tok_seq, const int64_t* __restrict__ positions, const float* __restrict__ sink,
     const typename Elem<T>::S* __restrict__ gate, int64_t gate_stride, const float* __restrict__ cos_sin, int max_pos,
-    int H, int rank, int rot, int dims, int window, float scale) {
+    int H, int rank, int rot, int dims, int interleaved, int window, float scale) {
   extern __shared__ float lds[];                        // query [rank + rot] | weights [64]
   float* qs = lds;
   float* ws = lds + rank + rot;
@@ -113,9 +122,10 @@ __global__ __launch_bounds__(64) void latent_window_attn_kernel(
     const int64_t pc = p >= max_pos ? max_pos - 1 : p;
     const float* cs = cos_sin + pc * dims;
     const typename Elem<T>::S* qr = q + t * q_stride + static_cast<int64_t>(h) * q_head + q_rot_off;
-    for (int j = lane; j < rot; j += 64) qs[rank + j] = rotated_at<T>(q, qr, j, dims, cos_sin, cs);
+    for (int j = lane; j < rot; j += 64) qs[rank + j] = rotated_at<T>(q, qr, j, dims, interleaved, cos_sin, cs);
   }
-  float m = MI355_LD(float, sink, sink + h), l = 1.0f;  // the sink: one term exp(sink - m), no key, no value
+  // the sink: one term exp(sink - m), no key, no value
+  float m = sink != nullptr ? MI355_LD(float, sink, sink + h) : -__builtin_inff(), l = sink != nullptr ? 1.0f : 0.f;
   float acc[CPL];
 #pragma unroll
   for (int i = 0; i < CPL; ++i) acc[i] = 0.f;
@@ -171,7 +181,7 @@ __global__ __launch_bounds__(64) void latent_q_pack_kernel(typename Elem<T>::S* 
                                                            int64_t q_stride, int q_head, int q_rot_off,
                                                            const float* __restrict__ cos_sin, int max_pos,
                                                            const int64_t* __restrict__ positions, int H, int rank, int rot,
-                                                           int dims) {
+                                                           int dims, int interleaved) {
   const int64_t t = blockIdx.x;
   const int h = blockIdx.y, lane = threadIdx.x;
   typename Elem<T>::S* dst = qe + (t * H + h) * (rank + rot);
@@ -181,7 +191,7 @@ __global__ __launch_bounds__(64) void latent_q_pack_kernel(typename Elem<T>::S* 
   p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
   const float* cs = cos_sin + p * dims;
   const typename Elem<T>::S* qr = q + t * q_stride + static_cast<int64_t>(h) * q_head + q_rot_off;
-  for (int j = lane; j < rot; j += 64) MI355_STF(T, qe, dst + rank + j, rotated_at<T>(q, qr, j, dims, cos_sin, cs));
+  for (int j = lane; j < rot; j += 64) MI355_STF(T, qe, dst + rank + j, rotated_at<T>(q, qr, j, dims, interleaved, cos_sin, cs));
 }
 
 constexpr float kLog2e = 1.4426950408889634f;
@@ -222,8 +232,9 @@ __global__ __launch_bounds__(256) void latent_window_attn_mfma_kernel(
   for (int c = 0; c < CB; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
   // running maximum (base-2 exponent) and this lane's share of the running sum of its query; without
   // splits the sink opens both: one term 2^(sink - m) = 1, held by the first of the query's four lanes
-  float m = split ? -1.0e30f : MI355_LD(float, sink, sink + my_h) * kLog2e;
-  float l = (!split && kk == 0) ? 1.0f : 0.f;
+  const bool open = !split && sink != nullptr;
+  float m = open ? MI355_LD(float, sink, sink + my_h) * kLog2e : -1.0e30f;
+  float l = (open && kk == 0) ? 1.0f : 0.f;
   int64_t lo = p_first - window + 1;
   if (lo < 0) lo = 0;
   for (int64_t base = ((lo >> 5) << 5) + 32 * z; base <= p_last; base += 32 * nz) {
@@ -364,10 +375,10 @@ __global__ __launch_bounds__(256) void latent_attn_reduce_kernel(uint16_t* __res
     const int c = static_cast<int>(i % rank);
     const int64_t row = pair / H;
     const int h = static_cast<int>(pair % H);
-    const float s2 = MI355_LD(float, sink, sink + h) * kLog2e;
+    const float s2 = sink != nullptr ? MI355_LD(float, sink, sink + h) * kLog2e : -1.0e30f;
     float M = s2;
     for (int z = 0; z < splits; ++z) M = fmaxf(M, MI355_LD(float, part_ml, part_ml + (z * total_pairs + pair) * 2));
-    float den = __builtin_amdgcn_exp2f(s2 - M), num = 0.f;
+    float den = sink != nullptr ? __builtin_amdgcn_exp2f(s2 - M) : 0.f, num = 0.f;
     for (int z = 0; z < splits; ++z) {
       const float* ml = part_ml + (z * total_pairs + pair) * 2;
       const float e = __builtin_amdgcn_exp2f(MI355_LD(float, part_ml, ml) - M);
@@ -389,7 +400,7 @@ using namespace mi355;
 extern "C" int32_t mi355_latent_kv_write(void* cache, void* cache_t, const void* x, int64_t x_stride, const float* norm_weight,
                                          const float* cos_sin, int32_t max_pos, const int64_t* positions,
                                          const int64_t* slot_mapping, int64_t num_tokens, int32_t rank, int32_t rot,
-                                         int32_t rot_dims, float eps, int32_t dtype, void* stream) {
+                                         int32_t rot_dims, int32_t interleaved, float eps, int32_t dtype, void* stream) {
   MI355_REQUIRE(cache && x && norm_weight && cos_sin && positions && slot_mapping, MI355_ERR_INVALID,
                 "latent_kv_write: null pointer");
   MI355_REQUIRE(num_tokens >= 0 && rank > 0 && rot >= 0 && max_pos > 0 && x_stride >= rank + rot, MI355_ERR_INVALID,
@@ -402,7 +413,7 @@ extern "C" int32_t mi355_latent_kv_write(void* cache, void* cache_t, const void*
   MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((latent_kv_write_kernel<TT>), dim3(num_tokens), dim3(256), 0, s,
                                                   static_cast<Elem<TT>::S*>(cache), static_cast<Elem<TT>::S*>(cache_t),
                                                   static_cast<const Elem<TT>::S*>(x), x_stride, norm_weight, cos_sin,
-                                                  max_pos, positions, slot_mapping, rank, rot, rot_dims, eps));
+                                                  max_pos, positions, slot_mapping, rank, rot, rot_dims, interleaved, eps));
   return check_launch("latent_kv_write");
 }
 
@@ -412,7 +423,7 @@ static void launch_latent_attn(hipStream_t s, void* out, int64_t out_stride, int
                                int q_head, int q_rot_off, const void* cache, const int32_t* block_tables, int max_blocks,
                                const int32_t* tok_seq, const int64_t* positions, const float* sink, const void* gate,
                                int64_t gate_stride, const float* cos_sin, int max_pos, int64_t T, int H, int rank, int rot,
-                               int dims, int window, float scale) {
+                               int dims, int interleaved, int window, float scale) {
   typedef typename Elem<TT>::S E;
   const dim3 grid(static_cast<unsigned>(T), static_cast<unsigned>(H));
   const size_t lds = (static_cast<size_t>(rank) + rot + 64) * sizeof(float);
@@ -421,7 +432,7 @@ static void launch_latent_attn(hipStream_t s, void* out, int64_t out_stride, int
                      out_head_stride, static_cast<const E*>(ql), ql_stride, ql_head_stride,                         \
                      static_cast<const E*>(q), q_stride, q_head, q_rot_off,                                         \
                      static_cast<const E*>(cache), block_tables, max_blocks, tok_seq, positions, sink,              \
-                     static_cast<const E*>(gate), gate_stride, cos_sin, max_pos, H, rank, rot, dims, window, scale)
+                     static_cast<const E*>(gate), gate_stride, cos_sin, max_pos, H, rank, rot, dims, interleaved, window, scale)
   if (rank <= 64) MI355_LATTN(1);
   else if (rank <= 128) MI355_LATTN(2);
   else if (rank <= 256) MI355_LATTN(4);
@@ -436,8 +447,9 @@ extern "C" int32_t mi355_latent_window_attn(void* out, int64_t out_stride, int64
                                             const int32_t* tok_seq, const int64_t* positions, const float* sink,
                                             const void* gate, int64_t gate_stride, const float* cos_sin, int32_t max_pos,
                                             int64_t num_tokens, int32_t num_heads, int32_t rank, int32_t rot,
-                                            int32_t rot_dims, int32_t window, float scale, int32_t dtype, void* stream) {
-  MI355_REQUIRE(out && q_latent && q && cache && block_tables && tok_seq && positions && sink && cos_sin,
+                                            int32_t rot_dims, int32_t interleaved, int32_t window, float scale, int32_t dtype,
+                                            void* stream) {
+  MI355_REQUIRE(out && q_latent && q && cache && block_tables && tok_seq && positions && cos_sin,
                 MI355_ERR_INVALID, "latent_window_attn: null pointer");
   MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && num_heads <= 65535 && rank > 0 && rot >= 0 && max_blocks > 0 &&
                     window > 0 && max_pos > 0 && q_rot_offset >= 0 && q_head_width >= q_rot_offset + rot,
@@ -455,7 +467,7 @@ extern "C" int32_t mi355_latent_window_attn(void* out, int64_t out_stride, int64
                                                      q_latent_head_stride, q, q_stride, q_head_width,
                                                      q_rot_offset, cache, block_tables, max_blocks, tok_seq, positions,
                                                      sink, gate, gate_stride, cos_sin, max_pos, num_tokens, num_heads,
-                                                     rank, rot, rot_dims, window, scale));
+                                                     rank, rot, rot_dims, interleaved, window, scale));
   return check_launch("latent_window_attn");
 }
 
@@ -463,7 +475,7 @@ extern "C" int32_t mi355_latent_q_pack(void* q_packed, const void* q_latent, int
                                        int64_t q_latent_head_stride, const void* q, int64_t q_stride, int32_t q_head_width,
                                        int32_t q_rot_offset, const float* cos_sin, int32_t max_pos,
                                        const int64_t* positions, int64_t num_tokens, int32_t num_heads, int32_t rank,
-                                       int32_t rot, int32_t rot_dims, int32_t dtype, void* stream) {
+                                       int32_t rot, int32_t rot_dims, int32_t interleaved, int32_t dtype, void* stream) {
   MI355_REQUIRE(q_packed && q_latent && q && cos_sin && positions, MI355_ERR_INVALID, "latent_q_pack: null pointer");
   MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && num_heads <= 65535 && rank > 0 && rot >= 0 && max_pos > 0 &&
                     q_rot_offset >= 0 && q_head_width >= q_rot_offset + rot && q_latent_stride >= rank &&
@@ -480,7 +492,7 @@ extern "C" int32_t mi355_latent_q_pack(void* q_packed, const void* q_latent, int
                                                   static_cast<const Elem<TT>::S*>(q_latent), q_latent_stride,
                                                   q_latent_head_stride, static_cast<const Elem<TT>::S*>(q), q_stride,
                                                   q_head_width, q_rot_offset, cos_sin, max_pos, positions, num_heads, rank,
-                                                  rot, rot_dims));
+                                                  rot, rot_dims, interleaved));
   return check_launch("latent_q_pack");
 }
 
@@ -491,7 +503,7 @@ extern "C" int32_t mi355_latent_window_attn_tiles(void* out, int64_t out_stride,
                                                   const void* gate, int64_t gate_stride, int64_t num_tokens,
                                                   int32_t num_heads, int32_t rank, int32_t rot, int32_t window, float scale,
                                                   float* partial, int32_t num_splits, int32_t dtype, void* stream) {
-  MI355_REQUIRE(out && q_packed && cache && cache_t && block_tables && tiles && positions && sink, MI355_ERR_INVALID,
+  MI355_REQUIRE(out && q_packed && cache && cache_t && block_tables && tiles && positions, MI355_ERR_INVALID,
                 "latent_window_attn_tiles: null pointer");
   MI355_REQUIRE(num_tokens >= 0 && num_tiles >= 0 && num_heads > 0 && rank > 0 && rot >= 0 && max_blocks > 0 && window > 0 &&
                     out_stride >= rank && out_head_stride >= rank,

@@ -7,11 +7,16 @@
 //                       best), and weighted by the score without correction, times a constant
 //   moe_sort            rows (token, choice) ordered by expert: offsets[E + 1], perm[position] = row,
 //                       inv[row] = position
+//   moe_table_sort      the same for a mixture without a router: a table [vocab, top] names the experts of every
+//                       token id, so a step's row orders of all its layers are made by one launch ahead of the layers;
+//                       also tile_start[E + 1], the first tile of `tile_rows` rows of every expert
 //   moe_gather_rows     xs[position] = x[perm[position] / top]; or every expert's rows padded to a common count
 //   moe_gate_up_rows    a[position] = silu(Wg[e] x) * (Wu[e] x) for every routed row, one wave per
 //                       (expert, hidden unit) walking that expert's rows: an expert's weights leave HBM once
 //   moe_down_rows       y[position] = Wd[e] a[position], the same way; both on the matrix cores where the
 //                       sizes allow (16-bit storage, widths multiples of 32 / 16)
+//   moe_linear_rows     y[position] = a(W[e] x[perm[position] / top]) (perm null: x[position]) with a the identity or
+//                       relu^2: the two products of an expert without a gate, on the kernels of moe_down_rows
 //   moe_silu_and_mul    a = silu(gu[:, :F]) * gu[:, F:] (any storage type)
 //   moe_combine         out[t] = sum_k weight[t, k] * y[inv[t * top + k]]; a chosen id at or past `num_real`
 //                       is an identity expert and stands for x[t]; a shared expert's rows join, times the
@@ -224,6 +229,45 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(int32_t* __restrict__ of
   }
 }
 
+// one workgroup per layer
+__global__ __launch_bounds__(1024) void moe_table_sort_kernel(int32_t* __restrict__ offsets, int32_t* __restrict__ tile_start,
+                                                              int32_t* __restrict__ perm, int32_t* __restrict__ inv,
+                                                              const int32_t* __restrict__ tables,
+                                                              const int64_t* __restrict__ ids, int64_t num_tokens,
+                                                              int64_t vocab, int E, int top, int tile_rows) {
+  extern __shared__ int32_t sm[];                       // counts, then next free positions [E]
+  const int64_t rows = num_tokens * top, layer = blockIdx.x;
+  const int32_t* table = tables + layer * vocab * top;
+  auto expert = [&](int64_t r) {
+    int64_t id = MI355_LD(int64_t, ids, ids + r / top);
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    const int e = MI355_LD(int32_t, tables, table + id * top + r % top);
+    return e < 0 ? 0 : (e >= E ? E - 1 : e);
+  };
+  for (int e = threadIdx.x; e < E; e += blockDim.x) sm[e] = 0;
+  __syncthreads();
+  for (int64_t r = threadIdx.x; r < rows; r += blockDim.x) atomicAdd(&sm[expert(r)], 1);
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    int32_t at = 0, tile = 0;
+    for (int e = 0; e <= E; ++e) {
+      MI355_ST(int32_t, offsets, offsets + layer * (E + 1) + e, at);
+      MI355_ST(int32_t, tile_start, tile_start + layer * (E + 1) + e, tile);
+      if (e == E) break;
+      const int32_t n = sm[e];
+      sm[e] = at;
+      at += n;
+      tile += (n + tile_rows - 1) / tile_rows;
+    }
+  }
+  __syncthreads();
+  for (int64_t r = threadIdx.x; r < rows; r += blockDim.x) {
+    const int32_t at = atomicAdd(&sm[expert(r)], 1);
+    MI355_ST(int32_t, perm, perm + layer * rows + at, static_cast<int32_t>(r));
+    MI355_ST(int32_t, inv, inv + layer * rows + r, at);
+  }
+}
+
 // cap 0: xs[position] for every routed row.  cap > 0: every expert's rows padded to cap, xs[e * cap + j]
 // = the j-th row of expert e, zeros past its count (grid: experts * cap rows)
 template <typename T>
@@ -339,11 +383,22 @@ __global__ __launch_bounds__(256) void moe_gate_up_rows_kernel(typename Elem<T>:
   }
 }
 
+// the row of the input that position p of the expert order reads
+__device__ __forceinline__ int64_t input_row(const int32_t* perm, int top, int p) {
+  return perm != nullptr ? MI355_LD(int32_t, perm, perm + p) / top : p;
+}
+
+__device__ __forceinline__ float relu2_f(float v) {
+  v = fmaxf(v, 0.f);
+  return v * v;
+}
+
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void moe_down_rows_kernel(typename Elem<T>::S* __restrict__ y,
                                                             const typename Elem<T>::S* __restrict__ a,
                                                             const typename Elem<T>::S* __restrict__ w_down,
-                                                            const int32_t* __restrict__ offsets, int W, int F) {
+                                                            const int32_t* __restrict__ offsets,
+                                                            const int32_t* __restrict__ perm, int top, int relu2, int W, int F) {
   typedef typename Elem<T>::S E;
   const int e = blockIdx.y, lane = threadIdx.x & 63;
   const int c = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
@@ -353,12 +408,13 @@ __global__ __launch_bounds__(256) void moe_down_rows_kernel(typename Elem<T>::S*
   for (int p0 = lo; p0 < hi; p0 += kRowBlock) {
     const E* ar[kRowBlock];
 #pragma unroll
-    for (int r = 0; r < kRowBlock; ++r) ar[r] = a + static_cast<int64_t>(p0 + r < hi ? p0 + r : p0) * F;
+    for (int r = 0; r < kRowBlock; ++r) ar[r] = a + input_row(perm, top, p0 + r < hi ? p0 + r : p0) * F;
     float s[kRowBlock];
     RowsDot<T, VEC>::run(w_down, wd, a, ar, F, lane, s);
 #pragma unroll
     for (int r = 0; r < kRowBlock; ++r)
-      if (lane == r && p0 + r < hi) MI355_STF(T, y, y + static_cast<int64_t>(p0 + r) * W + c, s[r]);
+      if (lane == r && p0 + r < hi)
+        MI355_STF(T, y, y + static_cast<int64_t>(p0 + r) * W + c, relu2 ? relu2_f(elem_to_f<T>(elem_from_f<T>(s[r]))) : s[r]);
   }
 }
 
@@ -400,21 +456,25 @@ __global__ __launch_bounds__(256) void moe_gate_up_mfma_kernel(uint16_t* __restr
 template <typename T>
 __global__ __launch_bounds__(256) void moe_down_mfma_kernel(uint16_t* __restrict__ y, const uint16_t* __restrict__ a,
                                                             const uint16_t* __restrict__ w_down,
-                                                            const int32_t* __restrict__ offsets, int W, int F) {
+                                                            const int32_t* __restrict__ offsets,
+                                                            const int32_t* __restrict__ perm, int top, int relu2, int W, int F) {
   const int e = blockIdx.y, lane = threadIdx.x & 63, li = lane & 15, kk = lane >> 4;
   const int c0 = (blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6)) * 16;
   if (c0 >= W) return;
   const int lo = MI355_LD(int32_t, offsets, offsets + e), hi = MI355_LD(int32_t, offsets, offsets + e + 1);
   const uint16_t* wd = w_down + (static_cast<int64_t>(e) * W + c0 + li) * F + 8 * kk;
   for (int p0 = lo; p0 < hi; p0 += 16) {
-    const uint16_t* ar = a + static_cast<int64_t>(p0 + li < hi ? p0 + li : p0) * F + 8 * kk;
+    const uint16_t* ar = a + input_row(perm, top, p0 + li < hi ? p0 + li : p0) * F + 8 * kk;
     f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f}, acc2 = f32x4{0.f, 0.f, 0.f, 0.f};     // two chains of products in turn
     for (int s = 0; s < F; s += 64) {
       acc = T::mfma(MI355_LD(uint4, w_down, wd + s), MI355_LD(uint4, a, ar + s), acc);
       if (s + 32 < F) acc2 = T::mfma(MI355_LD(uint4, w_down, wd + s + 32), MI355_LD(uint4, a, ar + s + 32), acc2);
     }
 #pragma unroll
-    for (int r = 0; r < 4; ++r) acc[r] += acc2[r];
+    for (int r = 0; r < 4; ++r) {
+      acc[r] += acc2[r];
+      if (relu2) acc[r] = relu2_f(round_f<T>(acc[r]));        // (of the product as a 16-bit buffer would hold it)
+    }
     if (p0 + li < hi)
       MI355_ST(uint2, y, y + static_cast<int64_t>(p0 + li) * W + c0 + 4 * kk,
                make_uint2(T::pack2(acc[0], acc[1]), T::pack2(acc[2], acc[3])));
@@ -602,33 +662,62 @@ extern "C" int32_t mi355_moe_gate_up_rows(void* act, const void* x, const void* 
   return check_launch("moe_gate_up_rows");
 }
 
-extern "C" int32_t mi355_moe_down_rows(void* y, const void* act, const void* w_down, const int32_t* offsets,
-                                       int32_t experts, int32_t width, int32_t ff, int32_t dtype, void* stream) {
-  MI355_REQUIRE(y && act && w_down && offsets, MI355_ERR_INVALID, "moe_down_rows: null pointer");
-  MI355_REQUIRE(experts > 0 && experts <= 65535 && width > 0 && ff > 0, MI355_ERR_INVALID, "moe_down_rows: sizes");
+static int32_t launch_moe_linear_rows(const char* name, void* y, const void* x, const void* w, const int32_t* offsets,
+                                      const int32_t* perm, int32_t top, int32_t relu2, int32_t experts, int32_t out_width,
+                                      int32_t in_width, int32_t dtype, void* stream) {
+  MI355_REQUIRE(y && x && w && offsets, MI355_ERR_INVALID, "%s: null pointer", name);
+  MI355_REQUIRE(experts > 0 && experts <= 65535 && out_width > 0 && in_width > 0 && top > 0, MI355_ERR_INVALID, "%s: sizes", name);
   REQ_DTYPE(dtype);
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const dim3 grid(static_cast<unsigned>((width + 3) / 4), static_cast<unsigned>(experts));
-  if (dtype != MI355_F32 && ff % 32 == 0 && width % 16 == 0 && aligned16(act) && aligned16(w_down) && aligned16(y)) {
-    const dim3 mgrid(static_cast<unsigned>((width / 16 + 3) / 4), static_cast<unsigned>(experts));
+  const dim3 grid(static_cast<unsigned>((out_width + 3) / 4), static_cast<unsigned>(experts));
+  if (dtype != MI355_F32 && in_width % 32 == 0 && out_width % 16 == 0 && aligned16(x) && aligned16(w) && aligned16(y)) {
+    const dim3 mgrid(static_cast<unsigned>((out_width / 16 + 3) / 4), static_cast<unsigned>(experts));
     if (dtype == MI355_BF16)
       hipLaunchKernelGGL((moe_down_mfma_kernel<BF16>), mgrid, dim3(256), 0, s, static_cast<uint16_t*>(y),
-                         static_cast<const uint16_t*>(act), static_cast<const uint16_t*>(w_down), offsets, width, ff);
+                         static_cast<const uint16_t*>(x), static_cast<const uint16_t*>(w), offsets, perm, top, relu2, out_width,
+                         in_width);
     else
       hipLaunchKernelGGL((moe_down_mfma_kernel<F16>), mgrid, dim3(256), 0, s, static_cast<uint16_t*>(y),
-                         static_cast<const uint16_t*>(act), static_cast<const uint16_t*>(w_down), offsets, width, ff);
-    return check_launch("moe_down_rows (matrix cores)");
+                         static_cast<const uint16_t*>(x), static_cast<const uint16_t*>(w), offsets, perm, top, relu2, out_width,
+                         in_width);
+    return check_launch(name);
   }
-  const bool vec = dtype != MI355_F32 && ff % 8 == 0 && aligned16(act) && aligned16(w_down);
+  const bool vec = dtype != MI355_F32 && in_width % 8 == 0 && aligned16(x) && aligned16(w);
   MI355_DISPATCH_DTYPE3(dtype, {
     if (vec)
       hipLaunchKernelGGL((moe_down_rows_kernel<TT, true>), grid, dim3(256), 0, s, static_cast<Elem<TT>::S*>(y),
-                         static_cast<const Elem<TT>::S*>(act), static_cast<const Elem<TT>::S*>(w_down), offsets, width, ff);
+                         static_cast<const Elem<TT>::S*>(x), static_cast<const Elem<TT>::S*>(w), offsets, perm, top, relu2,
+                         out_width, in_width);
     else
       hipLaunchKernelGGL((moe_down_rows_kernel<TT, false>), grid, dim3(256), 0, s, static_cast<Elem<TT>::S*>(y),
-                         static_cast<const Elem<TT>::S*>(act), static_cast<const Elem<TT>::S*>(w_down), offsets, width, ff);
+                         static_cast<const Elem<TT>::S*>(x), static_cast<const Elem<TT>::S*>(w), offsets, perm, top, relu2,
+                         out_width, in_width);
   });
-  return check_launch("moe_down_rows");
+  return check_launch(name);
+}
+
+extern "C" int32_t mi355_moe_down_rows(void* y, const void* act, const void* w_down, const int32_t* offsets,
+                                       int32_t experts, int32_t width, int32_t ff, int32_t dtype, void* stream) {
+  return launch_moe_linear_rows("moe_down_rows", y, act, w_down, offsets, nullptr, 1, 0, experts, width, ff, dtype, stream);
+}
+
+extern "C" int32_t mi355_moe_linear_rows(void* y, const void* x, const void* w, const int32_t* offsets, const int32_t* perm,
+                                         int32_t top, int32_t relu2, int32_t experts, int32_t out_width, int32_t in_width,
+                                         int32_t dtype, void* stream) {
+  return launch_moe_linear_rows("moe_linear_rows", y, x, w, offsets, perm, top, relu2, experts, out_width, in_width, dtype, stream);
+}
+
+extern "C" int32_t mi355_moe_table_sort(int32_t* offsets, int32_t* tile_start, int32_t* perm, int32_t* inv, const int32_t* tables,
+                                        const int64_t* ids, int64_t num_tokens, int64_t vocab, int32_t layers, int32_t experts,
+                                        int32_t top, int32_t tile_rows, void* stream) {
+  MI355_REQUIRE(offsets && tile_start && perm && inv && tables && ids, MI355_ERR_INVALID, "moe_table_sort: null pointer");
+  MI355_REQUIRE(num_tokens >= 0 && vocab > 0 && layers > 0 && experts > 0 && experts <= 8192 && top > 0 && top <= experts &&
+                    tile_rows > 0 && num_tokens * top <= 0x7FFFFFFF,
+                MI355_ERR_INVALID, "moe_table_sort: %d layers, %d of %d experts", layers, top, experts);
+  hipLaunchKernelGGL(moe_table_sort_kernel, dim3(layers), dim3(1024), static_cast<size_t>(experts) * sizeof(int32_t),
+                     static_cast<hipStream_t>(stream), offsets, tile_start, perm, inv, tables, ids, num_tokens, vocab, experts, top,
+                     tile_rows);
+  return check_launch("moe_table_sort");
 }
 
 extern "C" int32_t mi355_moe_silu_and_mul(void* out, const void* x, int64_t num_rows, int32_t ff, int32_t act, float limit,

@@ -35,7 +35,8 @@
 // or a sliding window (keys after p - window) beside the first `keep` keys of the sequence: the walk takes
 // the barrier intervals that hold kept keys and lie before the window's first interval, then the window's;
 // value sizes that differ from the key size (64 / 128 either way); one more term exp(sink[head]) in the softmax denominator that carries no value; and the output times
-// the sigmoid of one gate number per (token, head), and times a constant.
+// the sigmoid of one gate number per (token, head), and times a constant; a soft cap on the scores (cap_x > 0),
+// cap * tanh(q.k scale / cap).
 #include "common.h"
 
 #include <math.h>
@@ -63,7 +64,7 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
     const int32_t* __restrict__ block_tables, int max_blocks, const int32_t* __restrict__ cu_seqlens,
     const int32_t* __restrict__ context_lens, int num_heads, int num_kv_heads, float scale_log2e, int qt,
     int chunk, int window, int keep, const float* __restrict__ sink, const uint16_t* __restrict__ gate, int64_t gate_stride,
-    float out_scale) {
+    float out_scale, float cap_x) {
   constexpr int KS = D / 32;
   constexpr int NT = DV / 16;
   constexpr int BS = MI355_BLOCK_SIZE;
@@ -248,6 +249,18 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
       }
     }
     __builtin_amdgcn_s_setprio(0);
+    // soft cap: the scores become tanh(q.k scale / cap) = 1 - 2 / (1 + 2^(cap_x q.k)), cap_x = 2 log2(e) scale / cap;
+    // scale_log2e is then cap log2(e)
+    if (EXT && cap_x > 0.f) {
+#pragma unroll
+      for (int t = 0; t < NQ; ++t) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          sa[t][j] = 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sa[t][j] * cap_x));
+          sb[t][j] = 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sb[t][j] * cap_x));
+        }
+      }
+    }
     const int tok0 = s * 32 + tok_h;
     if (s * 32 + 32 > t_min + 1) {         // wave-uniform: on or beyond the diagonal for some column
 #pragma unroll
@@ -406,7 +419,7 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
 }  // namespace mi355
 
 static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chunk, int32_t window, int32_t keep, const float* sink,
-                                          const void* gate, int64_t gate_stride, float out_scale, int32_t v_dim, void* out, int64_t out_stride, const void* q, int64_t q_stride,
+                                          const void* gate, int64_t gate_stride, float out_scale, float softcap, int32_t v_dim, void* out, int64_t out_stride, const void* q, int64_t q_stride,
                                             const void* k_cache, const void* v_cache, int32_t num_blocks,
                                             const int32_t* block_tables, int32_t max_blocks_per_seq,
                                             const int32_t* cu_seqlens, const int32_t* context_lens,
@@ -453,8 +466,9 @@ static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chu
                      static_cast<uint16_t*>(out), out_stride, static_cast<const uint16_t*>(q), q_stride, \
                      static_cast<const uint16_t*>(k_cache), static_cast<const uint16_t*>(v_cache),      \
                      num_blocks, block_tables, max_blocks_per_seq, cu_seqlens, context_lens, num_heads, \
-                     num_kv_heads, scale * 1.4426950408889634f, qt, chunk, window, keep, sink,          \
-                     static_cast<const uint16_t*>(gate), gate_stride, out_scale)
+                     num_kv_heads, (softcap > 0.f ? softcap : scale) * 1.4426950408889634f, qt, chunk, window,  \
+                     keep, sink, static_cast<const uint16_t*>(gate), gate_stride, out_scale,            \
+                     softcap > 0.f ? 2.0f * 1.4426950408889634f * scale / softcap : 0.f)
 #define MI355_PRE(TT, DD, NN)                                                                           \
   do {                                                                                                  \
     if (ext && v_dim == 64) MI355_PRE_E(TT, DD, 64, NN, true);                                          \
@@ -484,7 +498,7 @@ extern "C" int32_t mi355_paged_attn_prefill(void* out, int64_t out_stride, const
                                             int32_t num_seqs, int32_t max_q_len, int32_t num_heads,
                                             int32_t num_kv_heads, int32_t head_dim, float scale,
                                             int32_t dtype, void* stream) {
-  return launch_paged_attn_prefill("mi355_paged_attn_prefill", false, 0, 0, 0, nullptr, nullptr, 0, 1.0f, head_dim, out, out_stride, q, q_stride, k_cache,
+  return launch_paged_attn_prefill("mi355_paged_attn_prefill", false, 0, 0, 0, nullptr, nullptr, 0, 1.0f, 0.f, head_dim, out, out_stride, q, q_stride, k_cache,
                                    v_cache, num_blocks, block_tables, max_blocks_per_seq, cu_seqlens, context_lens, num_seqs,
                                    max_q_len, num_heads, num_kv_heads, head_dim, scale, dtype, stream);
 }
@@ -496,13 +510,14 @@ extern "C" int32_t mi355_paged_attn_prefill_ext(void* out, int64_t out_stride, c
                                                 int32_t num_seqs, int32_t max_q_len, int32_t num_heads,
                                                 int32_t num_kv_heads, int32_t head_dim, int32_t v_dim, float scale,
                                                 int32_t chunk, int32_t window, int32_t keep, const float* sink,
-                                                const void* gate, int64_t gate_stride, float out_scale, int32_t dtype,
-                                                void* stream) {
+                                                const void* gate, int64_t gate_stride, float out_scale, float softcap,
+                                                int32_t dtype, void* stream) {
+  MI355_REQUIRE(softcap >= 0.f && (softcap == 0.f || scale > 0.f), MI355_ERR_INVALID, "mi355_paged_attn_prefill_ext: soft cap %g", softcap);
   MI355_REQUIRE(window >= 0 && keep >= 0 && (keep == 0 || chunk == 0), MI355_ERR_INVALID,
                 "mi355_paged_attn_prefill_ext: window %d, keep %d (not with chunks)", window, keep);
   MI355_REQUIRE(chunk >= 0 && (gate == nullptr || gate_stride >= num_heads), MI355_ERR_INVALID,
                 "mi355_paged_attn_prefill_ext: chunk %d, gate rows shorter than the heads", chunk);
-  return launch_paged_attn_prefill("mi355_paged_attn_prefill_ext", true, chunk, window, keep, sink, gate, gate_stride, out_scale, v_dim, out, out_stride, q,
+  return launch_paged_attn_prefill("mi355_paged_attn_prefill_ext", true, chunk, window, keep, sink, gate, gate_stride, out_scale, softcap, v_dim, out, out_stride, q,
                                    q_stride, k_cache, v_cache, num_blocks, block_tables, max_blocks_per_seq, cu_seqlens,
                                    context_lens, num_seqs, max_q_len, num_heads, num_kv_heads, head_dim, scale, dtype, stream);
 }

@@ -3,6 +3,8 @@
 //   embed_scale_pos_f32      resid = embed[id] * scale + pos_table[position]      (learned positions)
 //   resid_add_f32            resid += other (fp32 rows) + rows (activation rows) + vec (one row, broadcast)
 //   add_rms_norm_f32         resid += add; out = resid / rms(resid) * w      (w: one number or a vector)
+//   add_layer_norm_f32       resid += add; out = (resid - mean) / sqrt(variance + eps) * w.  The addend may be the rows of a
+//                            mixture of experts still in expert order: token t's is row_weight * sum_k add[inv[t * top + k]]
 //   rms_norm_mix_f32         resid += alpha * (xa / rms(xa) * wa + xb / rms(xb) * wb)
 //   gelu_tanh_and_mul        out = gelu_tanh(gate) * up for rows holding gate | up
 //   gated_head_rms_norm      out = o / rms(o) * w * act(gate) per (token, head) row of an fp32 tensor
@@ -92,6 +94,117 @@ __global__ __launch_bounds__(256) void add_rms_norm_f32_kernel(typename Elem<T>:
     const float v = MI355_LD(float, resid, resid + t * W + c);      // own writes of this thread: same c
     const float g = weight_numel == 1 ? g1 : MI355_LDF(T, weight, weight + c);
     MI355_STF(T, out, out + t * W + c, v * r * g);
+  }
+}
+
+// what add_layer_norm_f32 adds to column c of row t (see the head of this file)
+template <typename T>
+__device__ __forceinline__ float sublayer_out(const typename Elem<T>::S* add, const int32_t* inv, int top, float row_weight,
+                                              int64_t t, int W, int c) {
+  if (inv == nullptr) return MI355_LDF(T, add, add + t * W + c);
+  float s = 0.f;
+  for (int k = 0; k < top; ++k) s += MI355_LDF(T, add, add + static_cast<int64_t>(MI355_LD(int32_t, inv, inv + t * top + k)) * W + c);
+  return s * row_weight;
+}
+
+// one workgroup per row; the sum is stored first and read back by the thread that stored it
+template <typename T>
+__global__ __launch_bounds__(256) void add_layer_norm_f32_kernel(typename Elem<T>::S* __restrict__ out,
+                                                                 float* __restrict__ resid,
+                                                                 const typename Elem<T>::S* __restrict__ add,
+                                                                 const int32_t* __restrict__ inv, int top, float row_weight,
+                                                                 const typename Elem<T>::S* __restrict__ weight, int W,
+                                                                 float eps) {
+  __shared__ float scratch[32];
+  const int64_t t = blockIdx.x;
+  float sum = 0.f;
+  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+    float v = MI355_LD(float, resid, resid + t * W + c);
+    if (add != nullptr) {
+      v += sublayer_out<T>(add, inv, top, row_weight, t, W, c);
+      MI355_ST(float, resid, resid + t * W + c, v);
+    }
+    sum += v;
+  }
+  if (out == nullptr) return;                           // (the add alone)
+  const float mean = block_sum32(sum, scratch) / static_cast<float>(W);
+  float sq = 0.f;
+  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+    const float v = MI355_LD(float, resid, resid + t * W + c) - mean;
+    sq += v * v;
+  }
+  const float r = 1.0f / sqrtf(block_sum32(sq, scratch) / static_cast<float>(W) + eps);
+  for (int c = threadIdx.x; c < W; c += blockDim.x)
+    MI355_STF(T, out, out + t * W + c, (MI355_LD(float, resid, resid + t * W + c) - mean) * r * MI355_LDF(T, weight, weight + c));
+}
+
+// 16-bit rows of a multiple of 8 columns, up to 2048 * NV: the row stays in registers between the passes
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void add_layer_norm_f32_vec_kernel(uint16_t* __restrict__ out, float* __restrict__ resid,
+                                                                     const uint16_t* __restrict__ add,
+                                                                     const int32_t* __restrict__ inv, int top,
+                                                                     float row_weight, const uint16_t* __restrict__ weight,
+                                                                     int W, float eps) {
+  __shared__ float scratch[32];
+  const int64_t t = blockIdx.x;
+  float v[NV][8];
+  uint4 wv[NV];
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + 256 * i) * 8;
+    const bool have = c < W;
+    float4 a = make_float4(0.f, 0.f, 0.f, 0.f), b = a;
+    wv[i] = make_uint4(0, 0, 0, 0);
+    float y[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (have) {
+      a = MI355_LD(float4, resid, resid + t * W + c);
+      b = MI355_LD(float4, resid, resid + t * W + c + 4);
+      if (out != nullptr) wv[i] = MI355_LD(uint4, weight, weight + c);
+      if (add != nullptr && inv == nullptr) {
+        unpack8<T>(MI355_LD(uint4, add, add + t * W + c), y);
+      } else if (add != nullptr) {
+        for (int k = 0; k < top; ++k) {
+          float f[8];
+          unpack8<T>(MI355_LD(uint4, add, add + static_cast<int64_t>(MI355_LD(int32_t, inv, inv + t * top + k)) * W + c), f);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) y[j] += f[j];
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) y[j] *= row_weight;
+      }
+    }
+    v[i][0] = a.x + y[0], v[i][1] = a.y + y[1], v[i][2] = a.z + y[2], v[i][3] = a.w + y[3];
+    v[i][4] = b.x + y[4], v[i][5] = b.y + y[5], v[i][6] = b.z + y[6], v[i][7] = b.w + y[7];
+    if (have && add != nullptr) {
+      MI355_ST(float4, resid, resid + t * W + c, make_float4(v[i][0], v[i][1], v[i][2], v[i][3]));
+      MI355_ST(float4, resid, resid + t * W + c + 4, make_float4(v[i][4], v[i][5], v[i][6], v[i][7]));
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) sum += v[i][j];
+  }
+  if (out == nullptr) return;
+  const float mean = block_sum32(sum, scratch) / static_cast<float>(W);
+  float sq = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    if ((threadIdx.x + 256 * i) * 8 >= static_cast<unsigned>(W)) continue;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      v[i][j] -= mean;
+      sq += v[i][j] * v[i][j];
+    }
+  }
+  const float r = 1.0f / sqrtf(block_sum32(sq, scratch) / static_cast<float>(W) + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (threadIdx.x + 256 * i) * 8;
+    if (c >= W) continue;
+    float f[8];
+    unpack8<T>(wv[i], f);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) f[j] *= v[i][j] * r;
+    MI355_ST(uint4, out, out + t * W + c, pack8<T>(f));
   }
 }
 
@@ -708,6 +821,40 @@ extern "C" int32_t mi355_add_rms_norm_f32(void* out, float* resid, const void* a
                                                   static_cast<const Elem<TT>::S*>(add),
                                                   static_cast<const Elem<TT>::S*>(weight), weight_numel, width, eps));
   return check_launch("add_rms_norm_f32");
+}
+
+extern "C" int32_t mi355_add_layer_norm_f32(void* out, float* resid, const void* add, const int32_t* inv, int32_t top,
+                                            float row_weight, const void* weight, int64_t num_tokens, int32_t width,
+                                            float eps, int32_t dtype, void* stream) {
+  MI355_REQUIRE(resid && (out == nullptr || weight != nullptr), MI355_ERR_INVALID, "add_layer_norm_f32: null pointer");
+  MI355_REQUIRE(out != nullptr || add != nullptr, MI355_ERR_INVALID, "add_layer_norm_f32: nothing to do");
+  MI355_REQUIRE(inv == nullptr || (add != nullptr && top > 0), MI355_ERR_INVALID, "add_layer_norm_f32: %d rows per token", top);
+  MI355_REQUIRE(num_tokens >= 0 && width > 0, MI355_ERR_INVALID, "add_layer_norm_f32: sizes");
+  REQ_DTYPE(dtype);
+  if (num_tokens == 0) return MI355_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (dtype != MI355_F32 && width % 8 == 0 && width <= 8192 && aligned16(out) && aligned16(resid) && aligned16(add) &&
+      aligned16(weight)) {
+#define MI355_LN(TT, NV)                                                                                                   \
+  hipLaunchKernelGGL((add_layer_norm_f32_vec_kernel<TT, NV>), dim3(num_tokens), dim3(256), 0, s, static_cast<uint16_t*>(out), \
+                     resid, static_cast<const uint16_t*>(add), inv, top, row_weight, static_cast<const uint16_t*>(weight),  \
+                     width, eps)
+#define MI355_LN_NV(TT)                      \
+  do {                                       \
+    if (width <= 2048) MI355_LN(TT, 1);      \
+    else if (width <= 4096) MI355_LN(TT, 2); \
+    else MI355_LN(TT, 4);                    \
+  } while (0)
+    if (dtype == MI355_BF16) MI355_LN_NV(BF16); else MI355_LN_NV(F16);
+#undef MI355_LN_NV
+#undef MI355_LN
+    return check_launch("add_layer_norm_f32");
+  }
+  MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((add_layer_norm_f32_kernel<TT>), dim3(num_tokens), dim3(256), 0, s,
+                                                  static_cast<Elem<TT>::S*>(out), resid,
+                                                  static_cast<const Elem<TT>::S*>(add), inv, top, row_weight,
+                                                  static_cast<const Elem<TT>::S*>(weight), width, eps));
+  return check_launch("add_layer_norm_f32");
 }
 
 extern "C" int32_t mi355_rms_norm_mix_f32(float* resid, const void* xa, const void* wa, const void* xb, const void* wb,

@@ -33,7 +33,7 @@ def _load() -> ctypes.CDLL:
             f"{LIB_PATH} not found: build it with `make -C vllm-backend-public_amd/csrc` "
             "(or __graft_entry__.build()); the engine has no fallback path")
     lib = ctypes.CDLL(LIB_PATH)
-    P, I32, I64, F = c_void_p, c_int32, c_int64, c_float
+    P, I32, I64, F, D = c_void_p, c_int32, c_int64, c_float, ctypes.c_double
     sigs = {
         "mi355_abi_version": (I32, []),
         "mi355_last_error": (c_char_p, []),
@@ -51,7 +51,7 @@ def _load() -> ctypes.CDLL:
         "mi355_paged_attn_prefill": (I32, [P, I64, P, I64, P, P, I32, P, I32, P, P, I32, I32, I32, I32, I32,
                                            F, I32, P]),
         "mi355_paged_attn_prefill_ext": (I32, [P, I64, P, I64, P, P, I32, P, I32, P, P, I32, I32, I32, I32, I32, I32,
-                                               F, I32, I32, I32, P, P, I64, F, I32, P]),
+                                               F, I32, I32, I32, P, P, I64, F, F, I32, P]),
         "mi355_silu_and_mul": (I32, [P, P, I64, I64, I32, I32, P]),
         "mi355_sum_slabs": (I32, [P, I64, P, I32, P, I32, I32, I32, P]),
         "mi355_silu_and_mul_slabs": (I32, [P, I64, P, I32, I32, I32, I32, P]),
@@ -122,17 +122,20 @@ def _load() -> ctypes.CDLL:
         "mi355_gated_norm_resid_f32": (I32, [P, P, P, I64, P, P, I64, I32, I32, F, F, I32, P]),
         "mi355_rms_norm_rows": (I32, [P, P, I64, P, I64, I32, F, I32, P]),
         "mi355_tanh_rows": (I32, [P, P, I64, I64, I32, I32, P]),
-        "mi355_latent_kv_write": (I32, [P, P, P, I64, P, P, I32, P, P, I64, I32, I32, I32, F, I32, P]),
-        "mi355_latent_q_pack": (I32, [P, P, I64, I64, P, I64, I32, I32, P, I32, P, I64, I32, I32, I32, I32, I32, P]),
+        "mi355_latent_kv_write": (I32, [P, P, P, I64, P, P, I32, P, P, I64, I32, I32, I32, I32, F, I32, P]),
+        "mi355_latent_q_pack": (I32, [P, P, I64, I64, P, I64, I32, I32, P, I32, P, I64, I32, I32, I32, I32, I32, I32, P]),
         "mi355_latent_window_attn_tiles": (I32, [P, I64, I64, P, P, P, P, I32, P, I32, P, P, P, I64, I64, I32, I32, I32, I32,
                                                  F, P, I32, I32, P]),
         "mi355_latent_window_attn": (I32, [P, I64, I64, P, I64, I64, P, I64, I32, I32, P, P, I32, P, P, P, P, I64, P, I32,
-                                           I64, I32, I32, I32, I32, I32, F, I32, P]),
+                                           I64, I32, I32, I32, I32, I32, I32, F, I32, P]),
         "mi355_moe_route": (I32, [P, P, P, I64, P, I64, I32, I32, I32, I32, I32, I32, F, P]),
         "mi355_moe_sort": (I32, [P, P, P, P, I64, I32, P]),
         "mi355_moe_gather_rows": (I32, [P, P, P, P, I32, I64, I32, I32, I32, P]),
         "mi355_moe_gate_up_rows": (I32, [P, P, P, P, P, I32, I32, I32, I32, I32, F, I32, P]),
         "mi355_moe_down_rows": (I32, [P, P, P, P, I32, I32, I32, I32, P]),
+        "mi355_moe_linear_rows": (I32, [P, P, P, P, P, I32, I32, I32, I32, I32, I32, P]),
+        "mi355_moe_table_sort": (I32, [P, P, P, P, P, P, I64, I64, I32, I32, I32, I32, P]),
+        "mi355_add_layer_norm_f32": (I32, [P, P, P, P, I32, F, P, I64, I32, F, I32, P]),
         "mi355_moe_silu_and_mul": (I32, [P, P, I64, I32, I32, F, I32, P]),
         "mi355_gated_act_rows": (I32, [P, I64, P, P, I64, I64, I32, I32, F, I32, P]),
         "mi355_moe_combine": (I32, [P, P, P, P, P, P, I32, I64, I32, I32, P, I32, P, P, I64, I32, P]),
@@ -142,9 +145,9 @@ def _load() -> ctypes.CDLL:
         "mi355_qk_norm_kv_write": (I32, [P, I64, P, I64, P, I64, P, P, P, P, P, I64, I32, I32, I32, I32, F, I32, P]),
         "mi355_softmax_bias_attn_workspace": (I64, [I64, I32, I32, I32]),
         "mi355_softmax_bias_attn": (I32, [P, P, I64, P, P, P, I32, P, P, P, P, P, I64, I32, I64, I32, I32, I32, I32, I32,
-                                          I32, I32, F, P, I32, P, I32, P, I64, F, I32, P]),
+                                          I32, I32, F, P, I32, P, I32, P, I64, F, F, I32, P]),
         "mi355_row_norm_rope_kv_write": (I32, [P, I64, P, I64, P, I64, P, P, P, I64, P, P, P, P, I64, I32, I32, I32, I32,
-                                               I32, F, I32, P]),
+                                               I32, F, F, D, I32, P]),
         "mi355_norm_resid_f32": (I32, [P, P, P, P, I64, I32, F, F, I32, P]),
         "mi355_token_gate_rows": (I32, [P, P, I64, P, I64, I64, P, I64, I64, I32, I32, P]),
         "mi355_token_side_f32": (I32, [P, P, P, P, P, P, I64, I64, P, I64, I64, I32, I32, F, I32, P]),
@@ -201,7 +204,8 @@ EXPORTS = ("mi355_abi_version", "mi355_last_error", "mi355_target_arch",
            "mi355_softmax_bias_attn_workspace", "mi355_softmax_bias_attn", "mi355_mingru_scan",
            "mi355_mingru_scan_workspace", "mi355_row_norm_rope_kv_write", "mi355_norm_resid_f32", "mi355_token_gate_rows",
            "mi355_token_side_f32", "mi355_linear_attn_state_floats", "mi355_linear_attn_tile_rows", "mi355_mlstm_gates",
-           "mi355_linear_attn_chunks", "mi355_decay_attn_step", "mi355_mlstm_step")
+           "mi355_linear_attn_chunks", "mi355_decay_attn_step", "mi355_mlstm_step",
+           "mi355_moe_linear_rows", "mi355_moe_table_sort", "mi355_add_layer_norm_f32")
 
 
 def check(status: int) -> None:

@@ -15,7 +15,7 @@ from dataclasses import dataclass, field
 from typing import Any, Optional
 
 SUPPORTED_ARCHS = ("LlamaForCausalLM", "Qwen2ForCausalLM", "MistralForCausalLM", "OPTForCausalLM", "Lozupel", "Tativik", "Tafisun", "Bemulorn",
-                   "Rigazen")
+                   "Rigazen", "Bapavik")
 
 # Well-known geometries, used when --model names one of them and no local
 # config.json exists (synthetic-weight benchmarking; there is no network).
@@ -86,6 +86,9 @@ class GeneralDeltaSpec:
     dim: int
 
 
+NO_WINDOW = 1 << 30                       # a window longer than any sequence
+
+
 @dataclass
 class LatentAttnSpec:
     """Softmax attention through low-rank latents: queries through q_rank, keys and values through
@@ -94,7 +97,11 @@ class LatentAttnSpec:
     vdim; sliding window; a learned sink per head in the softmax denominator; one output gate per
     head.  kv_from: the layer whose cached latent and rotated key this layer reads instead of making
     its own (None: its own).  q_rank 0: not in the configuration, the weights' shape gives it; a
-    configuration without a window gets one longer than any sequence."""
+    configuration without a window gets one longer than any sequence (NO_WINDOW).
+
+    What follows the first design's fields switches its particulars off: q_direct: one full-rank query
+    projection; sink / gate False: an ordinary softmax, no output gate; interleaved: the rotation
+    pairs neighbouring coordinates 2i, 2i + 1 instead of i, i + rot_dims / 2, with angles formed in float64."""
     heads: int
     dim: int
     rot_dim: int
@@ -106,6 +113,10 @@ class LatentAttnSpec:
     rot_base: float
     scale: float
     kv_from: Optional[int] = None
+    q_direct: bool = False
+    sink: bool = True
+    gate: bool = True
+    interleaved: bool = False
 
 
 @dataclass
@@ -120,7 +131,8 @@ class MoESpec:
     ff: int
     # what follows defaults to the first design that used this spec
     score: str = "sigmoid"                  # "sigmoid": each expert by itself; "softmax": over all router outputs;
-                                            # "chosen_softmax": choice by the logits, weights a softmax over the chosen alone
+                                            # "chosen_softmax": choice by the logits, weights a softmax over the chosen alone;
+                                            # "table": no router, a table names every token id's experts, weight 1 / top each
     router_bias: bool = False               # the router logits carry a learned bias
     shared_gated: bool = True               # the shared expert is scaled by a sigmoid of one projected number per token
     group_score: str = "top2"               # a group scores the sum of its two best choice scores, or ("max") its best
@@ -129,6 +141,7 @@ class MoESpec:
                                             # are formed over experts and identity outputs together
     limit: Optional[float] = None           # None: silu(g) * u.  A number: g = min(g, limit), u = clamp(u, -limit, limit),
                                             # g * sigmoid(1.702 g) * (u + 1)
+    gated: bool = True                      # False: an expert is down(relu(up h)^2)
     shared_ff: int = 0                      # width of an expert that every token uses, scaled by a sigmoid of one
     shared_limit: Optional[float] = None    # projected number per token; 0: none
 
@@ -162,7 +175,9 @@ class BlockAttnSpec:
     number per head; kv_from: the layer has no key / value projections and attends to the pages of
     that earlier layer; window > 0: the last `window` keys only, and beside them the sequence's first
     `keep_first` keys; row_norm: queries and keys get an RMS norm over the whole projection (all heads at
-    once) with a weight of that size, ahead of the rotation."""
+    once) with a weight of that size, ahead of the rotation; learned_sink: the term exp(sink) is a learned number
+    per head; softcap > 0: scores become softcap * tanh(score / softcap); temp_every > 0: queries are multiplied
+    by 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1) after their norm."""
     heads: int
     kv_heads: int
     dim: int
@@ -182,6 +197,10 @@ class BlockAttnSpec:
     window: int = 0
     keep_first: int = 0
     row_norm: bool = False
+    learned_sink: bool = False
+    softcap: float = 0.0
+    temp_coef: float = 0.0
+    temp_every: float = 0.0
 
 
 @dataclass(frozen=True)
@@ -276,13 +295,14 @@ class HybridSpec:
     """A decoder whose layers each name their sequence mixer, with an optional weight-shared loop:
     layers loop_start .. loop_stop - 1 run loop_times times in a row (separate cache and state per
     pass); before every pass a learned vector is added to the residual, and before every pass but
-    the first the embedding output too."""
+    the first the embedding output too (neither with loop_plain)."""
     layers: list
     embed_scale: float = 1.0
     logit_softcap: Optional[float] = None
     loop_start: int = 0
     loop_stop: int = 0
     loop_times: int = 0                     # 0: no loop
+    loop_plain: bool = False                # nothing is added between the passes
     # "pre": x += sublayer(norm(x)), norms with one learned number.  "sandwich": the embedding is
     # normed, and x += residual_mult * norm_b(sublayer(h) * sigmoid(Wg h + bg)) with h = norm(x);
     # every such norm is an RMS norm in norm_groups equal parts with a weight vector.  "parallel":
@@ -290,6 +310,7 @@ class HybridSpec:
     # x += norm(sublayer(x)): the sub-layers read the residual itself, norm weights are stored around zero,
     # the head is the embedding table
     arrangement: str = "pre"
+    layer_norm: bool = False                # "pre" arrangement: the norms subtract the mean (a weight per channel, no bias)
     norm_groups: int = 1
     residual_mult: float = 1.0
     norm_vector: bool = False               # "pre" arrangement: norms carry a weight per channel instead of one number
@@ -309,6 +330,53 @@ class HybridSpec:
         for t in range(self.loop_times):
             out += [(i, t) for i in range(self.loop_start, self.loop_stop)]
         return out + [(i, None) for i in range(self.loop_stop, n)]
+
+    @classmethod
+    def from_bapavik(cls, d: dict) -> "HybridSpec":
+        layers = []
+        for i, spec in enumerate(d["layers"]):
+            m, mlp = spec["mixer"], spec.get("mlp")
+            kw = {}
+            if mlp is not None and mlp.get("kind", "dense") == "dense":
+                kw.update(ff=int(mlp["ff"]), ff_act="limited", ff_limit=float(mlp["limit"]))
+            elif mlp is not None and mlp.get("kind") == "moe":
+                r = mlp["router"]
+                moe = MoESpec(experts=int(r["experts"]), top=int(r["top"]), groups=1, keep=1, ff=int(mlp["expert"]["ff"]),
+                              score="table", gated=False)
+                moe.check(f"layer {i}")
+                kw.update(moe=moe)
+            elif mlp is not None:
+                raise ValueError(f"feed-forward kind {mlp.get('kind')!r} is not supported (dense, moe)")
+            if spec["type"] == "attention":
+                t = m.get("q_temp") or {}
+                a = BlockAttnSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]),
+                                  vdim=int(m.get("vdim", m["dim"])), block=0, scale=float(m["scale"]), values_are_keys=False,
+                                  qk_norm=False, penalty=False, row_norm=True, learned_sink=True,
+                                  softcap=float(m.get("softcap") or 0.0), temp_coef=float(t.get("coef", 0.0)),
+                                  temp_every=float(t.get("every", 0.0)))
+                if a.heads < 1 or a.kv_heads < 1 or a.heads % a.kv_heads:
+                    raise ValueError(f"layer {i}: kv_heads {a.kv_heads} must divide heads {a.heads}")
+                if a.softcap < 0 or a.temp_every < 0:
+                    raise ValueError(f"layer {i}: soft cap {a.softcap}, query temperature every {a.temp_every}")
+                layers.append(HybridLayerSpec("attention", battn=a, **kw))
+            elif spec["type"] == "latent_attention":
+                rot = m.get("rot") or {}
+                a = LatentAttnSpec(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                                   kv_rank=int(m["kv_rank"]), q_rank=0, window=NO_WINDOW,
+                                   rot_dims=int(rot.get("dims", m["rot_dim"])), rot_base=float(rot.get("base", 10000.0)),
+                                   scale=float(m["scale"]), q_direct=True, sink=False, gate=False, interleaved=True)
+                if a.heads < 1 or a.rot_dims > a.rot_dim or a.rot_dims % 2:
+                    raise ValueError(f"layer {i}: {a.heads} heads, {a.rot_dims} rotated coordinates of {a.rot_dim}")
+                layers.append(HybridLayerSpec("latent_attention", lattn=a, **kw))
+            else:
+                raise ValueError(f"layer type {spec['type']!r} is not supported (attention, latent_attention)")
+        loop = d.get("loop") or {}
+        out = cls(layers=layers, norm_vector=True, layer_norm=True, loop_plain=True,
+                  embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)), loop_start=int(loop.get("start", 0)),
+                  loop_stop=int(loop.get("stop", 0)), loop_times=int(loop.get("times", 0)))
+        if out.loop_times > 0 and not 0 <= out.loop_start < out.loop_stop <= len(layers):
+            raise ValueError(f"loop {out.loop_start}..{out.loop_stop} does not fit {len(layers)} layers")
+        return out
 
     @classmethod
     def from_rigazen(cls, d: dict) -> "HybridSpec":
@@ -456,7 +524,7 @@ class HybridSpec:
                 rot = m.get("rot") or {}
                 a = LatentAttnSpec(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
                                    kv_rank=int(m["kv_rank"]), q_rank=int(m.get("q_rank") or 0),
-                                   window=int((m.get("mask") or {}).get("size") or 1 << 30),
+                                   window=int((m.get("mask") or {}).get("size") or NO_WINDOW),
                                    rot_dims=int(rot.get("dims", m["rot_dim"])), rot_base=float(rot.get("base", 10000.0)),
                                    scale=float(m["scale"]),
                                    kv_from=(int(m["kv_from"]) if m.get("kv_from") is not None else None))
@@ -591,6 +659,19 @@ class ModelConfig:
                    eos_token_id=d.get("eos_token_id"), family="hybrid", hybrid=spec)
 
     @classmethod
+    def _from_bapavik_dict(cls, d: dict) -> "ModelConfig":
+        spec = HybridSpec.from_bapavik(d)
+        att, lat = [L.battn for L in spec.layers if L.battn is not None], [L.lattn for L in spec.layers if L.lattn is not None]
+        return cls(architecture="Bapavik", vocab_size=int(d["vocab"]), hidden_size=int(d["width"]),
+                   intermediate_size=max([L.ff or 0 for L in spec.layers] + [L.moe.ff for L in spec.layers if L.moe] + [0]),
+                   num_hidden_layers=len(spec.layers), num_attention_heads=max(a.heads for a in att + lat),
+                   num_key_value_heads=max([a.kv_heads for a in att] + [1]),
+                   head_dim=max([a.dim for a in att] + [a.dim + a.rot_dim for a in lat]), rope_theta=0.0, rope_scaling=None,
+                   rms_norm_eps=float(d["norm"]["eps"]), max_position_embeddings=int(d.get("max_positions", 1 << 17)),
+                   tie_word_embeddings=False, attention_bias=False, bos_token_id=d.get("bos_token_id"),
+                   eos_token_id=d.get("eos_token_id"), family="hybrid", hybrid=spec)
+
+    @classmethod
     def _from_tativik_dict(cls, d: dict) -> "ModelConfig":
         spec = HybridSpec.from_tativik(d)
         if int(d["width"]) % spec.norm_groups:
@@ -639,10 +720,10 @@ class ModelConfig:
             cfg = cls._from_opt_dict(d)
             cfg.torch_dtype = stored
             return cfg
-        if arch in ("Lozupel", "Tativik", "Tafisun", "Bemulorn", "Rigazen"):
+        if arch in ("Lozupel", "Tativik", "Tafisun", "Bemulorn", "Rigazen", "Bapavik"):
             cfg = {"Lozupel": cls._from_lozupel_dict, "Tativik": cls._from_tativik_dict,
                    "Tafisun": cls._from_tafisun_dict, "Bemulorn": cls._from_bemulorn_dict,
-                   "Rigazen": cls._from_rigazen_dict}[arch](d)
+                   "Rigazen": cls._from_rigazen_dict, "Bapavik": cls._from_bapavik_dict}[arch](d)
             cfg.torch_dtype = stored or "bfloat16"
             return cfg
         nh = d["num_attention_heads"]

@@ -8,6 +8,11 @@ mixer and may carry a feed-forward.  Four arrangements share this runner:
     (logarithmic distance penalty, keys as values, normed queries and keys, a gate per output channel)
     or by a per-channel gated recurrence; its feed-forward is relu^2 or a softmax-routed mixture with
     identity experts and a shared expert;
+    a fourth (Bapavik) norms with the mean taken off, mixes by a causal softmax attention (norms over all
+    heads of a row, a query temperature that grows with the position, capped scores, a learned value-less
+    term per head) or by an attention through latents (full-rank queries, neighbours rotated, no window),
+    and has a limited gated feed-forward or a mixture whose experts a table names per token id; its loop
+    adds nothing between the passes;
   * "sandwich" (the Tativik design): a general delta rule (decay per key channel, removal along the
     unit key) or a softmax attention through low-rank latents (sliding window, a sink in the
     denominator, latent pages that a later layer may share), then a mixture of experts; every
@@ -77,10 +82,12 @@ def rotary_table(rot_dims: int, base: float, max_pos: int, device, scaling=None,
 class StepBatch:
     """Device-side description of one packed step (see csrc/seqmix.hip)."""
     __slots__ = ("ids", "positions", "slot_mapping", "block_tables", "cu_seqlens", "tok_seq", "state_slots",
-                 "num_tokens", "num_seqs", "tiles", "long_chunks", "pair_tiles", "context_lens", "max_q_len", "row_tiles")
+                 "num_tokens", "num_seqs", "tiles", "long_chunks", "pair_tiles", "context_lens", "max_q_len", "row_tiles",
+                 "routes")
 
     def __init__(self, ids, positions, slot_mapping, block_tables, cu_seqlens, tok_seq, state_slots, tiles=None,
                  long_chunks=False, pair_tiles=None, context_lens=None, max_q_len=0, row_tiles=None):
+        self.routes = {}                              # (experts, top) -> ops.TableRoutes of the step's token ids
         self.row_tiles = row_tiles                    # rows -> ops.RowTiles of the step, or None (captured decode steps)
         # every chunk's length of context after the step (int32, on the device) and the longest chunk: what the
         # LDS-staged prompt attention walks by; None: not known to this step (captured decode steps)
@@ -160,8 +167,9 @@ class GeneralDeltaMixer:
 
 
 class LatentAttention:
-    """Sliding-window softmax attention through low-rank latents over the latent pages of one layer
-    run -- its own (it writes them first) or those of the layer it shares with."""
+    """Softmax attention through low-rank latents (in a sliding window or causal; a sink and an output gate
+    where the design has them) over the latent pages of one layer run -- its own (it writes them first)
+    or those of the layer it shares with."""
 
     def __init__(self, spec, lw, runner, cache_index: int, writes: bool):
         self.s, self.lw, self.r, self.ci, self.writes = spec, lw, runner, cache_index, writes
@@ -169,11 +177,12 @@ class LatentAttention:
     def __call__(self, proj: torch.Tensor, b: StepBatch) -> torch.Tensor:
         s, lw, r = self.s, self.lw, self.r
         col = lambda n: proj[:, lw.seg[n][0]: lw.seg[n][0] + lw.seg[n][1]]     # noqa: E731
-        (cache, cache_t), table = r.latent_cache[self.ci], r.rotary(s.rot_dims, s.rot_base)
+        (cache, cache_t), table = r.latent_cache[self.ci], r.rotary(s.rot_dims, s.rot_base, exact=s.interleaved)
         if self.writes:
             ops.latent_kv_write(col("dkv"), lw.dkv_norm, table, b.positions, b.slot_mapping, cache, s.kv_rank, s.rot_dim,
-                                r.eps, cache_t=cache_t)
-        q = r.linear(ops.rms_norm_rows(col("dq"), lw.dq_norm, r.eps), lw.uq_w)
+                                r.eps, cache_t=cache_t, interleaved=s.interleaved)
+        q = col("q") if s.q_direct else r.linear(ops.rms_norm_rows(col("dq"), lw.dq_norm, r.eps), lw.uq_w)
+        gate = col("g") if s.gate else None
         T, hw = q.shape[0], s.dim + s.rot_dim
         # the unrotated query part of every head into the latent space: the keys then are the cached latents
         ql = torch.bmm(q.view(T, s.heads, hw)[:, :, : s.dim].transpose(0, 1), lw.uk_w)
@@ -182,12 +191,12 @@ class LatentAttention:
             # their windows' keys over several workgroups
             tiles = b.pair_tiles(s.heads)
             n = min(16, max(s.window // 64, 1), max(1024 // max(int(tiles.shape[0]), 1), 1))
-            ol = ops.latent_window_attn_tiles(ops.latent_q_pack(ql, q, hw, s.dim, s.rot_dim, table, b.positions), cache,
-                                              cache_t, b.block_tables, tiles, b.positions, lw.sink, col("g"), s.window,
+            ol = ops.latent_window_attn_tiles(ops.latent_q_pack(ql, q, hw, s.dim, s.rot_dim, table, b.positions, interleaved=s.interleaved), cache,
+                                              cache_t, b.block_tables, tiles, b.positions, lw.sink, gate, s.window,
                                               s.scale, num_splits=n)
         else:
-            ol = ops.latent_window_attn(ql, q, hw, s.dim, cache, b.block_tables, b.tok_seq, b.positions, lw.sink, col("g"),
-                                        table, s.window, s.scale)
+            ol = ops.latent_window_attn(ql, q, hw, s.dim, cache, b.block_tables, b.tok_seq, b.positions, lw.sink, gate,
+                                        table, s.window, s.scale, interleaved=s.interleaved)
         o = torch.bmm(ol, lw.uv_t)                      # [heads, tokens, vdim]
         return r.linear(o.transpose(0, 1).reshape(T, s.heads * s.vdim), lw.o_w)
 
@@ -208,6 +217,31 @@ class BlockAttention:
         ops.qk_norm_kv_write(q, k, k, lw.q_norm, lw.k_norm, b.slot_mapping, kc, vc, s.heads, s.kv_heads, s.dim, s.vdim, r.eps)
         o = ops.softmax_bias_attn(q, kc, vc, b.block_tables, b.tok_seq, b.positions, lw.r1, lw.r2, col("g"), s.heads,
                                   s.scale, block=s.block, tiles=b.tiles, num_splits=r.block_key_splits(b, s))
+        return r.linear(o, lw.o_w)
+
+
+class RowNormAttention:
+    """Causal softmax attention over the paged K/V of one layer run: queries and keys normed over their whole
+    rows, a query temperature by position, capped scores, a learned value-less term per head.  Steps that hold a
+    portion of a prompt take the LDS-staged launch where the sizes allow, all others the tile form."""
+
+    def __init__(self, spec, lw, runner, cache_index: int):
+        self.s, self.lw, self.r, self.ci = spec, lw, runner, cache_index
+
+    def __call__(self, proj: torch.Tensor, b: StepBatch) -> torch.Tensor:
+        s, lw, r = self.s, self.lw, self.r
+        col = lambda n: proj[:, lw.seg[n][0]: lw.seg[n][0] + lw.seg[n][1]]     # noqa: E731
+        q, kc, vc = col("q"), r.k_cache[self.ci], r.v_cache[self.ci]
+        ops.row_norm_rope_kv_write(q, col("k"), col("v"), lw.q_norm, lw.k_norm, r.rotary(0, 1.0, exact=True), b.positions,
+                                   b.slot_mapping, kc, vc, s.heads, s.kv_heads, s.dim, s.vdim, r.eps, temp_coef=s.temp_coef,
+                                   temp_every=s.temp_every)
+        if b.long_chunks and b.context_lens is not None and ops.chunk_attn_prefill_ok(q.dtype, s.heads, s.kv_heads, s.dim, s.vdim) \
+                and proj.stride(0) % 8 == 0:
+            o = ops.paged_attn_prefill_ext(q, kc, vc, b.block_tables, b.cu_seqlens, b.context_lens, b.max_q_len, s.heads,
+                                           s.kv_heads, s.dim, s.scale, sink=lw.sink, softcap=s.softcap)
+        else:
+            o = ops.softmax_bias_attn(q, kc, vc, b.block_tables, b.tok_seq, b.positions, None, None, None, s.heads, s.scale,
+                                      tiles=b.tiles, num_splits=r.block_key_splits(b, s), sink=lw.sink, softcap=s.softcap)
         return r.linear(o, lw.o_w)
 
 
@@ -326,6 +360,42 @@ class ReluSquaredFF:
 
     def __call__(self, h: torch.Tensor) -> torch.Tensor:
         return self.r.linear(ops.relu_squared(self.r.linear(h, self.lw.up_w)), self.lw.down_w)
+
+
+class LimitedFF:
+    """Dense gated feed-forward with limited units: down(g' sigmoid(1.702 g') (u' + 1)), g' = min(g, limit),
+    u' = clamp(u, -limit, limit)."""
+
+    def __init__(self, spec, lw, runner):
+        self.ff, self.limit, self.lw, self.r = spec.ff, spec.ff_limit, lw, runner
+
+    def __call__(self, h: torch.Tensor, b: "StepBatch") -> torch.Tensor:
+        gu = self.r.linear(h, self.lw.gate_up_w)
+        return self.r.linear(ops.gated_act_rows(gu[:, : self.ff], gu[:, self.ff:], self.limit), self.lw.down_w)
+
+
+class ExpertRows:
+    """A mixture's output still in expert order: token t's row is weight * sum_k rows[inv[t * top + k]].  The launch
+    that adds it to the residual sums it on the way in."""
+    __slots__ = ("rows", "inv", "top", "weight")
+
+    def __init__(self, rows, inv, top, weight):
+        self.rows, self.inv, self.top, self.weight = rows, inv, top, weight
+
+
+class TableMoE:
+    """Mixture of experts without a router: the runner has sorted the step's rows by the experts that the layer's
+    table names for their token ids (one launch for all such layers, ahead of the first); an expert is
+    down(relu(up h)^2), every chosen one of weight 1 / top."""
+
+    def __init__(self, spec, lw, slot: int):
+        self.s, self.lw, self.slot = spec, lw, slot     # slot: the layer's place among the stacked tables of its kind
+
+    def __call__(self, h: torch.Tensor, b: "StepBatch") -> ExpertRows:
+        s, lw, rt = self.s, self.lw, b.routes[(self.s.experts, self.s.top)]
+        offsets, perm = rt.offsets[self.slot], rt.perm[self.slot]
+        act = ops.moe_linear_rows(h, lw.up_w, offsets, rt.rows, perm=perm, top=s.top, relu2=True)
+        return ExpertRows(ops.moe_linear_rows(act, lw.down_w, offsets, rt.rows), rt.inv[self.slot], s.top, 1.0 / s.top)
 
 
 class MoEFeedForward:
@@ -449,6 +519,14 @@ class HybridRunner(ModelRunner):
         self.runs = spec.runs()
         self.k_cache, self.v_cache, self.conv_state, self.rec_state, self.mixers = [], [], [], [], []
         self.latent_cache, self.ffs = [], []
+        # mixtures without a router: their tables, stacked by (experts, chosen), and every layer's place in its stack
+        stacks, self._table_at = {}, {}
+        for li, L in enumerate(spec.layers):
+            if L.moe is not None and L.moe.score == "table":
+                stack = stacks.setdefault((L.moe.experts, L.moe.top), [])
+                self._table_at[li] = len(stack)
+                stack.append(weights.layers[li].table)
+        self._tables = {k: torch.stack(v).contiguous() for k, v in stacks.items()}
         latent_of = {}                                  # layer index -> index of its latent pages
         for li, _ in self.runs if spec.arrangement == "sandwich" else ():
             L, lw = spec.layers[li], weights.layers[li]
@@ -460,12 +538,7 @@ class HybridRunner(ModelRunner):
             else:
                 A = L.lattn
                 if A.kv_from is None:
-                    # the latent pages, token-major with the rotated key part; where the matrix-core attention
-                    # covers the sizes, the latent once more, channel-major
-                    self.latent_cache.append((
-                        torch.zeros(self.num_blocks, BLOCK_SIZE, A.kv_rank + A.rot_dim, dtype=dtype, device=dev),
-                        torch.zeros(self.num_blocks, A.kv_rank, BLOCK_SIZE, dtype=dtype, device=dev)
-                        if ops.latent_tiles_ok(dtype, A.kv_rank, A.rot_dim) else None))
+                    self._add_latent_pages(A)
                     latent_of[li] = len(self.latent_cache) - 1
                 self.mixers.append(LatentAttention(A, lw, self, latent_of[li if A.kv_from is None else A.kv_from],
                                                    A.kv_from is None))
@@ -501,13 +574,22 @@ class HybridRunner(ModelRunner):
             self.mixers.append(AttentionBesideDecay(L, lw, self, len(self.k_cache) - 1, si))
         for li, _ in self.runs if spec.arrangement == "pre" else ():
             L, lw = spec.layers[li], weights.layers[li]
-            self.ffs.append(MoEFeedForward(L.moe, lw, self) if L.moe is not None else
-                            ReluSquaredFF(lw, self) if L.ff and L.ff_act == "relu2" else None)
+            if L.moe is not None and L.moe.score == "table":
+                self.ffs.append(TableMoE(L.moe, lw, self._table_at[li]))
+            elif L.ff and L.ff_act == "limited":
+                self.ffs.append(LimitedFF(L, lw, self))
+            else:
+                self.ffs.append(MoEFeedForward(L.moe, lw, self) if L.moe is not None else
+                                ReluSquaredFF(lw, self) if L.ff and L.ff_act == "relu2" else None)
+            if L.kind == "latent_attention":
+                self._add_latent_pages(L.lattn)
+                self.mixers.append(LatentAttention(L.lattn, lw, self, len(self.latent_cache) - 1, True))
+                continue
             if L.kind == "attention":
                 A = L.battn
                 self.k_cache.append(torch.zeros(self.num_blocks, A.kv_heads, BLOCK_SIZE, A.dim, dtype=dtype, device=dev))
                 self.v_cache.append(torch.zeros(self.num_blocks, A.kv_heads, A.vdim, BLOCK_SIZE, dtype=dtype, device=dev))
-                self.mixers.append(BlockAttention(A, lw, self, len(self.k_cache) - 1))
+                self.mixers.append((RowNormAttention if A.row_norm else BlockAttention)(A, lw, self, len(self.k_cache) - 1))
                 continue
             if L.kind == "mingru":
                 self.rec_state.append(torch.zeros(self.num_state_slots + 1, L.gru.width, dtype=torch.float32, device=dev))
@@ -571,6 +653,14 @@ class HybridRunner(ModelRunner):
         if key not in self._rotary:
             self._rotary[key] = rotary_table(rot_dims, base, self.max_blocks * BLOCK_SIZE, self.device, scaling, exact)
         return self._rotary[key]
+
+    def _add_latent_pages(self, a) -> None:
+        """Latent pages of one layer run: token-major with the rotated key part; where the matrix-core attention
+        covers the sizes, the latent once more, channel-major."""
+        self.latent_cache.append((
+            torch.zeros(self.num_blocks, BLOCK_SIZE, a.kv_rank + a.rot_dim, dtype=self.dtype, device=self.device),
+            torch.zeros(self.num_blocks, a.kv_rank, BLOCK_SIZE, dtype=self.dtype, device=self.device)
+            if ops.latent_tiles_ok(self.dtype, a.kv_rank, a.rot_dim) else None))
 
     def _decode_pair_tiles(self, heads: int) -> torch.Tensor:
         """Tiles of (row, head) pairs of a decode step: a row's tiles are adjacent, so the first b rows'
@@ -719,6 +809,20 @@ class HybridRunner(ModelRunner):
                 self.layer_trace.append(resid.clone())
         return resid
 
+    def _norm(self, resid: torch.Tensor, weight: Optional[torch.Tensor], pending=None) -> Optional[torch.Tensor]:
+        """resid += pending (rows, or a mixture's rows in expert order); the design's norm of it in the activation
+        type.  weight None: the add alone."""
+        if isinstance(pending, ExpertRows):
+            if self.spec.layer_norm:
+                return ops.add_layer_norm_f32(resid, weight, self.eps, add=pending.rows, inv=pending.inv, top=pending.top,
+                                              row_weight=pending.weight)
+            wts = torch.full((pending.inv.numel(),), pending.weight, dtype=torch.float32, device=resid.device)
+            pending = ops.moe_combine(pending.rows, pending.inv, wts, resid.shape[0], pending.top)
+        if weight is None:
+            ops.resid_add_f32(resid, rows=pending)
+            return None
+        return (ops.add_layer_norm_f32 if self.spec.layer_norm else ops.add_rms_norm_f32)(resid, weight, self.eps, add=pending)
+
     def _forward_pre(self, b: StepBatch) -> torch.Tensor:
         """All layers over one packed batch; returns the float32 residual stream [tokens, width]."""
         w, spec = self.w, self.spec
@@ -731,15 +835,17 @@ class HybridRunner(ModelRunner):
                 ops.prev_token_update(self.prev_tokens, b.ids, b.cu_seqlens, b.state_slots)
         else:
             resid = ops.embed_scale_f32(w.embed, b.ids, spec.embed_scale)
-        x0 = resid.clone() if spec.loop_times > 1 else None
+        for (experts, _), tables in self._tables.items():   # the expert orders of all layers, by one launch per kind of mixture
+            b.routes[(experts, tables.shape[2])] = ops.TableRoutes(tables, b.ids, experts)
+        x0 = resid.clone() if spec.loop_times > 1 and not spec.loop_plain else None
         pending = None                                 # a sub-layer output not yet added to the residual
         last = len(self.runs) - 1
         for ri, (li, t) in enumerate(self.runs):
             L, lw = spec.layers[li], w.layers[li]
-            if t is not None and li == spec.loop_start:    # a pass begins: + embedding output (not the first) + its step vector
+            if t is not None and li == spec.loop_start and not spec.loop_plain:    # a pass begins: + embedding output (not the first) + its step vector
                 ops.resid_add_f32(resid, other=x0 if t > 0 else None, rows=pending, vec=w.loop_step[t])
                 pending = None
-            h = ops.add_rms_norm_f32(resid, lw.norm1, self.eps, add=pending)    # the add rides in the norm's launch
+            h = self._norm(resid, lw.norm1, pending)       # the add rides in the norm's launch
             pending = None
             proj = self.linear(h, lw.in_w)
             mixer, ff = self.mixers[ri], self.ffs[ri]
@@ -751,13 +857,15 @@ class HybridRunner(ModelRunner):
                                      self.eps, 0.5)
             else:
                 pending = mixer[1](proj, b)
-            if ff is not None:
-                pending = ff(ops.add_rms_norm_f32(resid, lw.norm2, self.eps, add=pending))
+            if isinstance(ff, (LimitedFF, TableMoE)):
+                pending = ff(self._norm(resid, lw.norm2, pending), b)
+            elif ff is not None:
+                pending = ff(self._norm(resid, lw.norm2, pending))
             elif L.ff:
-                h = ops.add_rms_norm_f32(resid, lw.norm2, self.eps, add=pending)
+                h = self._norm(resid, lw.norm2, pending)
                 pending = self.linear(ops.gelu_tanh_and_mul(self.linear(h, lw.gate_up_w)), lw.down_w)
             if pending is not None and (ri == last or self.layer_trace is not None):
-                ops.resid_add_f32(resid, rows=pending)
+                self._norm(resid, None, pending)
                 pending = None
             if self.layer_trace is not None:
                 self.layer_trace.append(resid.clone())
@@ -834,7 +942,7 @@ class HybridRunner(ModelRunner):
         elif self.spec.arrangement == "post":
             h = ops.group_rms_norm_f32(resid, self.w.final_norm, 1, self.eps, dtype=self.dtype)
         else:
-            h = ops.add_rms_norm_f32(resid, self.w.final_norm, self.eps)
+            h = self._norm(resid, self.w.final_norm)
         z = self.linear(h, self.head_w, out=out)
         if self.spec.logit_softcap:
             ops.softcap(z, self.spec.logit_softcap)

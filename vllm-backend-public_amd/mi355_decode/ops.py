@@ -299,12 +299,13 @@ def paged_attn_prefill_ext(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torc
                            cu_seqlens: torch.Tensor, context_lens: torch.Tensor, max_q_len: int, num_heads: int,
                            num_kv_heads: int, head_dim: int, scale: float, chunk: int = 0, sink: torch.Tensor | None = None,
                            gate: torch.Tensor | None = None, out: torch.Tensor | None = None, window: int = 0,
-                           keep: int = 0, out_scale: float = 1.0):
+                           keep: int = 0, out_scale: float = 1.0, softcap: float = 0.0):
     """paged_attn_prefill (K/V steps staged through LDS for a workgroup's query tile) for attention inside
     chunks of `chunk` positions counted from position 0 (0: plain causal), with one more value-less term
     exp(sink[h]) in the softmax denominator (float32 [heads]) and the output times sigmoid(gate[t, h])
     (gate [tokens, heads], a column slice is fine).  window > 0: the last `window` keys only, and (chunk 0) the
-    first `keep` keys of the sequence.  The output is multiplied by out_scale.  q and out may be column
+    first `keep` keys of the sequence.  The output is multiplied by out_scale.  softcap > 0: the scores are
+    softcap * tanh(q.k * scale / softcap).  q and out may be column
     slices on 16-byte boundaries; the value size (V pages [blocks, kv_heads, v_dim, 16]) may differ from
     the key size."""
     dt = _dt16(q, "q")
@@ -331,7 +332,7 @@ def paged_attn_prefill_ext(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torc
         v_cache.data_ptr(), nb, block_tables.data_ptr(), block_tables.shape[1], cu_seqlens.data_ptr(), context_lens.data_ptr(),
         S, int(max_q_len), num_heads, num_kv_heads, head_dim, dv, float(scale), int(chunk), int(window), int(keep),
         None if sink is None else _f32(sink, "sink", num_heads), None if gate is None else _same(gate, q, "gate"),
-        0 if gate is None else _cols(gate, "gate", num_heads), float(out_scale), dt, _stream()))
+        0 if gate is None else _cols(gate, "gate", num_heads), float(out_scale), float(softcap), dt, _stream()))
     return out
 
 
@@ -1077,6 +1078,32 @@ def add_rms_norm_f32(resid: torch.Tensor, weight: torch.Tensor, eps: float, add:
     return out
 
 
+def add_layer_norm_f32(resid: torch.Tensor, weight: torch.Tensor | None, eps: float, add: torch.Tensor | None = None,
+                       inv: torch.Tensor | None = None, top: int = 1, row_weight: float = 1.0,
+                       out: torch.Tensor | None = None):
+    """resid (float32, in place) += add; returns (resid - mean) / sqrt(variance + eps) * weight in the dtype of
+    weight [width]; weight None: the add alone, nothing returned.  inv (int32 [tokens * top]): add holds a
+    mixture's rows in expert order, token t's addend is row_weight * sum_k add[inv[t * top + k]]."""
+    T, W = resid.shape
+    ref = weight if weight is not None else add
+    dt = _dt3(ref, "weight")
+    if weight is not None and (tuple(weight.shape) != (W,) or not weight.is_contiguous()):
+        raise ValueError("weight must be one contiguous row")
+    if weight is not None and out is None:
+        out = torch.empty(T, W, dtype=weight.dtype, device=resid.device)
+    if out is not None and (out.dtype != weight.dtype or not out.is_contiguous() or out.shape != resid.shape):
+        raise ValueError("out must be contiguous, shaped like resid, in the dtype of weight")
+    if add is not None and (add.dtype != ref.dtype or not add.is_contiguous()
+                            or tuple(add.shape) != ((T if inv is None else T * top), W)):
+        raise ValueError("add must be contiguous rows in the dtype of weight, one per token or (inv) per routed row")
+    check(lib.mi355_add_layer_norm_f32(None if out is None else out.data_ptr(), _f32(resid, "resid"),
+                                       None if add is None else add.data_ptr(),
+                                       None if inv is None else _idx(inv, "inv", torch.int32, T * top), int(top),
+                                       float(row_weight), None if weight is None else weight.data_ptr(), T, W, float(eps), dt,
+                                       _stream()))
+    return out
+
+
 def rms_norm_mix_f32(resid: torch.Tensor, xa: torch.Tensor, wa: torch.Tensor, xb: torch.Tensor | None,
                      wb: torch.Tensor | None, eps: float, alpha: float):
     """resid (float32, in place) += alpha * (rmsnorm(xa) * wa + rmsnorm(xb) * wb)."""
@@ -1361,9 +1388,10 @@ def tanh_rows(x: torch.Tensor):
 
 def latent_kv_write(x: torch.Tensor, norm_weight: torch.Tensor, cos_sin: torch.Tensor, positions: torch.Tensor,
                     slot_mapping: torch.Tensor, cache: torch.Tensor, rank: int, rot: int, eps: float,
-                    cache_t: torch.Tensor | None = None):
+                    cache_t: torch.Tensor | None = None, interleaved: bool = False):
     """x [tokens, rank + rot] (a column slice is fine): the first rank columns RMS-normed with norm_weight
-    (float32), the last rot rotated by the table cos_sin [max_pos, rot_dims], both into the row's slot of
+    (float32), the last rot rotated by the table cos_sin [max_pos, rot_dims] (coordinates i, i + rot_dims / 2, or
+    neighbours if interleaved), both into the row's slot of
     cache [blocks, 16, rank + rot]; the latent also into cache_t [blocks, rank, 16] if given."""
     dt = _dt3(x, "x")
     T = x.shape[0]
@@ -1376,7 +1404,7 @@ def latent_kv_write(x: torch.Tensor, norm_weight: torch.Tensor, cos_sin: torch.T
                                     _f32(norm_weight, "norm_weight", rank), _f32(cos_sin, "cos_sin") or x.data_ptr(),
                                     max(cos_sin.shape[0], 1), _idx(positions, "positions", torch.int64, T),
                                     _idx(slot_mapping, "slot_mapping", torch.int64, T), T, rank, rot, cos_sin.shape[1],
-                                    float(eps), dt, _stream()))
+                                    int(bool(interleaved)), float(eps), dt, _stream()))
 
 
 def pair_tiles(cu_seqlens, num_heads: int) -> "np.ndarray":
@@ -1399,7 +1427,7 @@ def latent_tiles_ok(dtype: torch.dtype, rank: int, rot: int) -> bool:
 
 
 def latent_q_pack(q_latent: torch.Tensor, q: torch.Tensor, q_head_width: int, q_rot_offset: int, rot: int,
-                  cos_sin: torch.Tensor, positions: torch.Tensor):
+                  cos_sin: torch.Tensor, positions: torch.Tensor, interleaved: bool = False):
     """[tokens, heads, rank + rot] = q_latent [heads, tokens, rank] | the rotated `rot` columns of q at
     q_rot_offset of every head: the query as latent_window_attn_tiles reads it."""
     dt = _dt3(q, "q")
@@ -1410,13 +1438,13 @@ def latent_q_pack(q_latent: torch.Tensor, q: torch.Tensor, q_head_width: int, q_
     check(lib.mi355_latent_q_pack(out.data_ptr(), _same(q_latent, q, "q_latent"), max(q_latent.stride(1), rank),
                                   max(q_latent.stride(0), rank), q.data_ptr(), _cols(q, "q", H * q_head_width), q_head_width,
                                   q_rot_offset, _f32(cos_sin, "cos_sin") or q.data_ptr(), max(cos_sin.shape[0], 1),
-                                  _idx(positions, "positions", torch.int64, T), T, H, rank, rot, cos_sin.shape[1], dt,
+                                  _idx(positions, "positions", torch.int64, T), T, H, rank, rot, cos_sin.shape[1], int(bool(interleaved)), dt,
                                   _stream()))
     return out
 
 
 def latent_window_attn_tiles(q_packed: torch.Tensor, cache: torch.Tensor, cache_t: torch.Tensor, block_tables: torch.Tensor,
-                             tiles: torch.Tensor, positions: torch.Tensor, sink: torch.Tensor, gate: torch.Tensor | None,
+                             tiles: torch.Tensor, positions: torch.Tensor, sink: torch.Tensor | None, gate: torch.Tensor | None,
                              window: int, scale: float, num_splits: int = 1, out: torch.Tensor | None = None):
     """The matrix-core form of latent_window_attn: q_packed [tokens, heads, rank + rot] (latent_q_pack),
     both copies of the latent pages, tiles from pair_tiles.  Returns [heads, tokens, rank]."""
@@ -1438,7 +1466,7 @@ def latent_window_attn_tiles(q_packed: torch.Tensor, cache: torch.Tensor, cache_
     check(lib.mi355_latent_window_attn_tiles(
         out.data_ptr(), max(out.stride(1), rank), max(out.stride(0), rank), q_packed.data_ptr(),
         _same(cache, q_packed, "cache"), _same(cache_t, q_packed, "cache_t"), block_tables.data_ptr(), block_tables.shape[1],
-        tiles.data_ptr(), tiles.shape[0], _idx(positions, "positions", torch.int64, T), _f32(sink, "sink", H),
+        tiles.data_ptr(), tiles.shape[0], _idx(positions, "positions", torch.int64, T), None if sink is None else _f32(sink, "sink", H),
         None if gate is None else _same(gate, q_packed, "gate"), 0 if gate is None else _cols(gate, "gate", H), T, H, rank,
         dq - rank, int(window), float(scale), None if partial is None else partial.data_ptr(), int(num_splits), dt,
         _stream()))
@@ -1446,10 +1474,10 @@ def latent_window_attn_tiles(q_packed: torch.Tensor, cache: torch.Tensor, cache_
 
 
 def latent_window_attn(q_latent: torch.Tensor, q: torch.Tensor, q_head_width: int, q_rot_offset: int, cache: torch.Tensor,
-                       block_tables: torch.Tensor, tok_seq: torch.Tensor, positions: torch.Tensor, sink: torch.Tensor,
+                       block_tables: torch.Tensor, tok_seq: torch.Tensor, positions: torch.Tensor, sink: torch.Tensor | None,
                        gate: torch.Tensor | None, cos_sin: torch.Tensor, window: int, scale: float,
-                       out: torch.Tensor | None = None):
-    """Sliding-window softmax attention with a sink over latent pages (see latent_kv_write).  q_latent
+                       out: torch.Tensor | None = None, interleaved: bool = False):
+    """Sliding-window softmax attention with a sink (None: an ordinary softmax) over latent pages (see latent_kv_write).  q_latent
     [heads, tokens, rank]: the unrotated query part multiplied into the latent space; q [tokens, heads *
     q_head_width] holds the part to rotate at q_rot_offset of every head.  Returns the gated weighted
     latent [heads, tokens, rank]."""
@@ -1472,10 +1500,10 @@ def latent_window_attn(q_latent: torch.Tensor, q: torch.Tensor, q_head_width: in
         max(q_latent.stride(1), rank), max(q_latent.stride(0), rank), q.data_ptr(), _cols(q, "q", H * q_head_width),
         q_head_width, q_rot_offset, _same(cache, q, "cache"),
         block_tables.data_ptr(), block_tables.shape[1], _idx(tok_seq, "tok_seq", torch.int32, T),
-        _idx(positions, "positions", torch.int64, T), _f32(sink, "sink", H),
+        _idx(positions, "positions", torch.int64, T), None if sink is None else _f32(sink, "sink", H),
         None if gate is None else _same(gate, q, "gate"), 0 if gate is None else _cols(gate, "gate", H),
         _f32(cos_sin, "cos_sin") or q.data_ptr(), max(cos_sin.shape[0], 1), T, H, rank, rot, cos_sin.shape[1],
-        int(window), float(scale), dt, _stream()))
+        int(bool(interleaved)), int(window), float(scale), dt, _stream()))
     return out
 
 
@@ -1561,6 +1589,45 @@ def moe_down_rows(act: torch.Tensor, w_down: torch.Tensor, offsets: torch.Tensor
     check(lib.mi355_moe_down_rows(y.data_ptr(), act.data_ptr(), _same(w_down, act, "w_down"),
                                   _idx(offsets, "offsets", torch.int32, E + 1), E, W, F, dt, _stream()))
     return y
+
+
+def moe_linear_rows(x: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, rows: int, perm: torch.Tensor | None = None,
+                    top: int = 1, relu2: bool = False):
+    """y[position] = W[e] x[perm[position] / top] (perm None: x[position]) for `rows` routed rows in expert order, w
+    [experts, out, in]; relu2: max(., 0)^2 of it."""
+    dt = _dt3(x, "x")
+    E, N, K = w.shape
+    if not x.is_contiguous() or x.shape[1] != K or not w.is_contiguous() or x.shape[0] * (top if perm is not None else 1) != rows:
+        raise ValueError("x must be contiguous [rows or tokens, in], w contiguous [experts, out, in]")
+    y = torch.empty(rows, N, dtype=x.dtype, device=x.device)
+    check(lib.mi355_moe_linear_rows(y.data_ptr(), x.data_ptr(), _same(w, x, "w"), _idx(offsets, "offsets", torch.int32, E + 1),
+                                    None if perm is None else _idx(perm, "perm", torch.int32, rows), int(top),
+                                    int(bool(relu2)), E, N, K, dt, _stream()))
+    return y
+
+
+MOE_TILE_ROWS = 128
+
+
+class TableRoutes:
+    """Row orders of a step for `layers` mixtures whose experts a table [layers, vocab, top] names per token id:
+    offsets and tile_start [layers, experts + 1], perm and inv [layers, tokens * top] (see moe_sort)."""
+
+    def __init__(self, tables: torch.Tensor, ids: torch.Tensor, experts: int):
+        L, V, top = tables.shape
+        if tables.dtype != torch.int32 or not tables.is_contiguous():
+            raise ValueError("tables must be contiguous int32 [layers, vocab, top]")
+        _dev(tables, "tables")
+        T, dev = ids.numel(), ids.device
+        self.top, self.experts, self.rows = int(top), int(experts), T * int(top)
+        buf = torch.empty(2 * L * (experts + 1) + 2 * L * max(self.rows, 1), dtype=torch.int32, device=dev)
+        n = L * (experts + 1)
+        self.offsets, self.tile_start = buf[:n].view(L, -1), buf[n: 2 * n].view(L, -1)
+        m = L * self.rows
+        self.perm, self.inv = buf[2 * n: 2 * n + m].view(L, -1), buf[2 * n + m: 2 * n + 2 * m].view(L, -1)
+        check(lib.mi355_moe_table_sort(self.offsets.data_ptr(), self.tile_start.data_ptr(), self.perm.data_ptr(),
+                                       self.inv.data_ptr(), tables.data_ptr(), _idx(ids, "ids", torch.int64), T, V, L,
+                                       int(experts), int(top), MOE_TILE_ROWS, _stream()))
 
 
 def moe_silu_and_mul(x: torch.Tensor, limit: float | None = None):
@@ -1697,11 +1764,12 @@ def softmax_bias_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
                       tok_seq: torch.Tensor, positions: torch.Tensor, r1: torch.Tensor | None, r2: torch.Tensor | None,
                       gate: torch.Tensor | None, num_heads: int, scale: float, block: int = 0, window: int = 0,
                       tiles: torch.Tensor | None = None, num_splits: int = 0, sink: torch.Tensor | None = None,
-                      out: torch.Tensor | None = None, keep: int = 0, out_scale: float = 1.0):
+                      out: torch.Tensor | None = None, keep: int = 0, out_scale: float = 1.0, softcap: float = 0.0):
     """Softmax attention over the paged K/V [blocks, kv_heads, 16, dim] / [blocks, kv_heads, vdim, 16] with
     the score q.k * scale - r1[h] ln(1 + r2[h] * distance); a row at position p sees the keys j <= p of
     its block of `block` positions (0: all) and, window > 0, the last `window` of them and (block 0) the
-    sequence's first `keep`.  The output is multiplied by out_scale.  gate
+    sequence's first `keep`.  The output is multiplied by out_scale.  softcap > 0 (no penalty): the score is
+    softcap * tanh(q.k * scale / softcap).  gate
     [tokens, heads] or [tokens, heads * vdim]: the output is multiplied by its sigmoid.  tiles
     (query_tiles) selects the matrix-core form where the sizes allow; num_splits > 1 spreads a
     tile's keys over that many workgroups.  sink (float32 [heads]): the softmax denominator holds one
@@ -1735,7 +1803,7 @@ def softmax_bias_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
         T, num_heads, G, d, dv, int(block), int(window), int(keep), float(scale),
         None if tiles is None else _idx(tiles, "tiles", torch.int32), 0 if tiles is None else tiles.shape[0],
         None if ws is None else ws.data_ptr(), n, None if sink is None else _f32(sink, "sink", num_heads),
-        _cols(out, "out", num_heads * dv), float(out_scale), dt, _stream()))
+        _cols(out, "out", num_heads * dv), float(out_scale), float(softcap), dt, _stream()))
     return out
 
 
@@ -1814,9 +1882,11 @@ def token_side_f32(resid: torch.Tensor, gate_w: torch.Tensor, proj_w: torch.Tens
 
 def row_norm_rope_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, q_weight: torch.Tensor, k_weight: torch.Tensor,
                            cos_sin: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Tensor, k_cache: torch.Tensor,
-                           v_cache: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, eps: float):
+                           v_cache: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, eps: float,
+                           temp_coef: float = 0.0, temp_every: float = 0.0):
     """q [tokens, heads * dim] is RMS-normed as one row, weighted (float32 [heads * dim]) and rotated in place by
     the float32 table cos_sin [max_pos, rot_dims]; k likewise into the K pages, v as given into the V pages.
+    temp_every > 0: q is also multiplied by 1 + temp_coef ln(floor((position + 1) / temp_every) + 1).
     q / k / v may be column slices."""
     dt = _dt3(q, "q")
     T, rot = q.shape[0], cos_sin.shape[1]
@@ -1829,7 +1899,7 @@ def row_norm_rope_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, q_
         _f32(k_weight, "k_weight", num_kv_heads * head_dim), _f32(cos_sin, "cos_sin") if rot else None, cos_sin.shape[0],
         _idx(positions, "positions", torch.int64, T), _idx(slot_mapping, "slot_mapping", torch.int64, T),
         _same(k_cache, q, "k_cache"), _same(v_cache, q, "v_cache"), T, num_heads, num_kv_heads, head_dim, v_dim, rot, float(eps),
-        dt, _stream()))
+        float(temp_coef), float(temp_every), dt, _stream()))
 
 
 def linear_attn_state_floats(dim: int, vdim: int, normalizer: bool) -> int:

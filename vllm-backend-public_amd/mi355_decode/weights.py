@@ -146,12 +146,16 @@ class SandwichLayerWeights:
 
 @dataclass
 class MixerLayerWeights:
-    """One layer of a hybrid decoder in the "pre" arrangement whose mixer is a block attention or a
-    per-channel gated recurrence (config.BlockAttnSpec / MinGRUSpec).  Everything that reads the
-    mixer's normed input is ONE matrix in_w (segments `seg`: name -> (first column, width)):
+    """One layer of a hybrid decoder in the "pre" arrangement whose mixer is a block attention, a latent
+    attention or a per-channel gated recurrence (config.BlockAttnSpec / LatentAttnSpec / MinGRUSpec).
+    Everything that reads the mixer's normed input is ONE matrix in_w (segments `seg`: name -> (first
+    column, width)):
       attention:  q | k | g        (g: the output gate, heads * vdim wide; the values are the keys)
+                  q | k | v        (row_norm: norms over all heads, a learned sink)
+      latent_attention:  q | dkv   (q_direct)
       mingru:     z | x | g
-    The feed-forward is dense (up_w, down_w), a mixture of experts (router_w float32 [experts +
+    The feed-forward is dense (up_w, or gate_up_w of a gated one; down_w), a mixture without a router (table,
+    up_w [experts, ff, width], down_w), a mixture of experts (router_w float32 [experts +
     identity (+ 1), width]: the shared expert's gate row rides last in the fp32 router product;
     expert matrices stacked [experts, ...]; the shared expert as one more gate|up and down pair), or
     absent.  Norm weights are in the activation type, per-head numbers and biases float32."""
@@ -159,18 +163,23 @@ class MixerLayerWeights:
     in_w: torch.Tensor
     seg: dict
     o_w: torch.Tensor
-    q_norm: Optional[torch.Tensor] = None   # f32 [dim]
-    k_norm: Optional[torch.Tensor] = None   # f32 [dim]
+    q_norm: Optional[torch.Tensor] = None   # f32 [dim], or [heads * dim] with row_norm
+    k_norm: Optional[torch.Tensor] = None   # f32 [dim], or [kv_heads * dim]
+    sink: Optional[torch.Tensor] = None     # f32 [heads]
+    dkv_norm: Optional[torch.Tensor] = None     # f32 [kv_rank]
+    uk_w: Optional[torch.Tensor] = None     # [heads, dim, kv_rank]
+    uv_t: Optional[torch.Tensor] = None     # [heads, kv_rank, vdim]
     r1: Optional[torch.Tensor] = None       # f32 [heads]
     r2: Optional[torch.Tensor] = None       # f32 [heads]
     z_b: Optional[torch.Tensor] = None      # f32 [width of the recurrence]
     x_b: Optional[torch.Tensor] = None
     norm2: Optional[torch.Tensor] = None
-    up_w: Optional[torch.Tensor] = None     # dense: [ff, width]
+    up_w: Optional[torch.Tensor] = None     # dense: [ff, width]; ungated experts: [experts, ff, width]
     down_w: Optional[torch.Tensor] = None   # dense: [width, ff]; mixture: [experts, width, ff]
+    table: Optional[torch.Tensor] = None    # int32 [vocab, top]: the experts of every token id
     router_w: Optional[torch.Tensor] = None
     correction: Optional[torch.Tensor] = None   # f32 [experts + identity]
-    gate_up_w: Optional[torch.Tensor] = None    # [experts, 2 ff, width]
+    gate_up_w: Optional[torch.Tensor] = None    # [experts, 2 ff, width]; dense gated: [2 ff, width]
     shared_gate_up_w: Optional[torch.Tensor] = None     # [2 shared_ff, width]
     shared_down_w: Optional[torch.Tensor] = None        # [width, shared_ff]
 
@@ -423,6 +432,8 @@ def _hybrid_from_getter(cfg: ModelConfig, get, dtype, device, tp_size: int, num_
         return _sandwich_from_getter(cfg, get, dtype, device)
     if cfg.architecture == "Tafisun":
         return _tafisun_from_getter(cfg, get, dtype, device)
+    if cfg.architecture == "Bapavik":
+        return _bapavik_from_getter(cfg, get, dtype, device)
     if spec.arrangement == "parallel":
         return _bemulorn_from_getter(cfg, get, dtype, device)
     if spec.arrangement == "post":
@@ -640,6 +651,62 @@ def _tafisun_from_getter(cfg: ModelConfig, get, dtype, device) -> ModelWeights:
     return w
 
 
+def _bapavik_from_getter(cfg: ModelConfig, get, dtype, device) -> ModelWeights:
+    """Bapavik checkpoints: 'embed', 'final.norm', 'head', and per layer i 'l<i>.norm1|norm2', 'l<i>.mix.*' (attention:
+    q k v q.norm k.norm sink o; latent_attention: q dkv dkv.norm uk uv o), 'l<i>.mlp.gate|up|down' (dense) or
+    'l<i>.mlp.table' and 'l<i>.mlp.e<j>.up|down' (mixture).  Linear weights are [out, in]."""
+    spec, W = cfg.hybrid, cfg.hidden_size
+
+    def put(t, dt=dtype):
+        return t.to(dt).contiguous().to(device)
+
+    def f32(t):
+        return put(t.reshape(-1), torch.float32)
+
+    def expect(name, shape):
+        t = get(name)
+        if tuple(t.shape) != tuple(shape):
+            raise ValueError(f"{name}: shape {tuple(t.shape)}, expected {tuple(shape)}")
+        return t
+
+    w = ModelWeights(embed=put(expect("embed", (cfg.vocab_size, W))))
+    for i, L in enumerate(spec.layers):
+        p, m, q = f"l{i}.", f"l{i}.mix.", f"l{i}.mlp."
+        kw = {}
+        if L.kind == "attention":
+            A = L.battn
+            in_w, seg = _fuse_segments([(c, expect(m + c, (rows, W))) for c, rows in
+                                        (("q", A.heads * A.dim), ("k", A.kv_heads * A.dim), ("v", A.kv_heads * A.vdim))], W, put)
+            kw.update(q_norm=f32(expect(m + "q.norm", (A.heads * A.dim,))), k_norm=f32(expect(m + "k.norm", (A.kv_heads * A.dim,))),
+                      sink=f32(expect(m + "sink", (A.heads,))))
+        else:
+            A = L.lattn
+            in_w, seg = _fuse_segments([("q", expect(m + "q", (A.heads * (A.dim + A.rot_dim), W))),
+                                        ("dkv", expect(m + "dkv", (A.kv_rank + A.rot_dim, W)))], W, put)
+            uk = expect(m + "uk", (A.heads * A.dim, A.kv_rank)).view(A.heads, A.dim, A.kv_rank)
+            uv = expect(m + "uv", (A.heads * A.vdim, A.kv_rank)).view(A.heads, A.vdim, A.kv_rank)
+            kw.update(dkv_norm=f32(expect(m + "dkv.norm", (A.kv_rank,))), uk_w=put(uk), uv_t=put(uv.transpose(1, 2)))
+        lw = MixerLayerWeights(norm1=put(expect(p + "norm1", (W,))), in_w=in_w, seg=seg,
+                               o_w=put(expect(m + "o", (W, A.heads * A.vdim))), **kw)
+        if L.ff:
+            lw.norm2 = put(expect(p + "norm2", (W,)))
+            lw.gate_up_w = put(torch.cat([expect(q + "gate", (L.ff, W)), expect(q + "up", (L.ff, W))], dim=0))
+            lw.down_w = put(expect(q + "down", (W, L.ff)))
+        elif L.moe is not None:
+            M = L.moe
+            lw.norm2 = put(expect(p + "norm2", (W,)))
+            table = expect(q + "table", (cfg.vocab_size, M.top)).to(torch.int32)
+            if int(table.min()) < 0 or int(table.max()) >= M.experts:
+                raise ValueError(f"{q}table names experts outside 0 .. {M.experts - 1}")
+            lw.table = put(table, torch.int32)
+            lw.up_w = put(torch.stack([expect(f"{q}e{e}.up", (M.ff, W)) for e in range(M.experts)]))
+            lw.down_w = put(torch.stack([expect(f"{q}e{e}.down", (W, M.ff)) for e in range(M.experts)]))
+        w.layers.append(lw)
+    w.final_norm = put(expect("final.norm", (W,)))
+    w.lm_head = put(expect("head", (cfg.vocab_size, W)))
+    return w
+
+
 def _bemulorn_from_getter(cfg: ModelConfig, get, dtype, device) -> ModelWeights:
     """Bemulorn checkpoints: 'embed', 'pos', 'final.norm', 'head', and per layer i 'l<i>.norm1',
     'l<i>.mix.q|k|v' with '.b', 'l<i>.mix.g|o' (no k, v in a layer that reads another layer's pages),
@@ -822,6 +889,47 @@ def rigazen_synthetic_state(cfg: ModelConfig, seed: int = 0, device="cpu", dtype
     return st
 
 
+def bapavik_synthetic_state(cfg: ModelConfig, seed: int = 0, device="cpu", dtype=torch.float32) -> dict:
+    """Seeded random tensors under a Bapavik checkpoint's names (benchmarks and tests: nothing can be
+    downloaded).  Scales keep activations near 1."""
+    spec, W, V = cfg.hybrid, cfg.hidden_size, cfg.vocab_size
+    gen = torch.Generator(device=device).manual_seed(seed)
+
+    def mat(*shape, s=1.0, mean=0.0):
+        return (torch.empty(shape, dtype=torch.float32, device=device).normal_(mean, s, generator=gen)).to(dtype)
+
+    st = {"embed": mat(V, W, s=1.0 / spec.embed_scale), "head": mat(V, W, s=W ** -0.5), "final.norm": mat(W, s=0.1, mean=1.0)}
+    for i, L in enumerate(spec.layers):
+        p, m, f = f"l{i}.", f"l{i}.mix.", f"l{i}.mlp."
+        st[p + "norm1"] = mat(W, s=0.1, mean=1.0)
+        if L.kind == "attention":
+            A = L.battn
+            for n, rows in (("q", A.heads * A.dim), ("k", A.kv_heads * A.dim), ("v", A.kv_heads * A.vdim)):
+                st[m + n] = mat(rows, W, s=W ** -0.5)
+            st[m + "q.norm"], st[m + "k.norm"] = mat(A.heads * A.dim, s=0.1, mean=1.0), mat(A.kv_heads * A.dim, s=0.1, mean=1.0)
+            st[m + "sink"] = mat(A.heads)
+        else:
+            A = L.lattn
+            st[m + "q"], st[m + "dkv"] = mat(A.heads * (A.dim + A.rot_dim), W, s=W ** -0.5), mat(A.kv_rank + A.rot_dim, W, s=W ** -0.5)
+            st[m + "dkv.norm"] = mat(A.kv_rank, s=0.1, mean=1.0)
+            st[m + "uk"] = mat(A.heads * A.dim, A.kv_rank, s=A.kv_rank ** -0.5)
+            st[m + "uv"] = mat(A.heads * A.vdim, A.kv_rank, s=A.kv_rank ** -0.5)
+        st[m + "o"] = mat(W, A.heads * A.vdim, s=(A.heads * A.vdim) ** -0.5)
+        if L.ff or L.moe is not None:
+            st[p + "norm2"] = mat(W, s=0.1, mean=1.0)
+        if L.ff:
+            st[f + "gate"], st[f + "up"] = mat(L.ff, W, s=W ** -0.5), mat(L.ff, W, s=W ** -0.5)
+            st[f + "down"] = mat(W, L.ff, s=L.ff ** -0.5)
+        elif L.moe is not None:
+            M = L.moe
+            # `top` different experts per token id: consecutive ones from a random first
+            first = torch.randint(0, M.experts, (V, 1), device=device, generator=gen)
+            st[f + "table"] = ((first + torch.arange(M.top, device=device)[None, :]) % M.experts).to(torch.int32)
+            for e in range(M.experts):
+                st[f"{f}e{e}.up"], st[f"{f}e{e}.down"] = mat(M.ff, W, s=W ** -0.5), mat(W, M.ff, s=M.ff ** -0.5)
+    return st
+
+
 def bemulorn_synthetic_state(cfg: ModelConfig, seed: int = 0, device="cpu", dtype=torch.float32) -> dict:
     """Seeded random tensors under a Bemulorn checkpoint's names (benchmarks and tests: nothing can be
     downloaded)."""
@@ -964,6 +1072,8 @@ def hybrid_synthetic_state(cfg: ModelConfig, seed: int = 0, std: float = 0.02, r
         return sandwich_synthetic_state(cfg, seed=seed, device=device, dtype=dtype)
     if cfg.architecture == "Tafisun":
         return tafisun_synthetic_state(cfg, seed=seed, device=device, dtype=dtype)
+    if cfg.architecture == "Bapavik":
+        return bapavik_synthetic_state(cfg, seed=seed, device=device, dtype=dtype)
     if spec.arrangement == "parallel":
         return bemulorn_synthetic_state(cfg, seed=seed, device=device, dtype=dtype)
     if spec.arrangement == "post":
