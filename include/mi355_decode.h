@@ -300,7 +300,8 @@ int32_t mi355_paged_attn_prefill(void* out, int64_t out_stride, const void* q,
  * multiplied by sigmoid(gate[token, head]).  window > 0: the keys j > p - window only, and (chunk 0)
  * the first `keep` keys of the sequence.  The output is multiplied by out_scale.  softcap > 0: scores are
  * softcap * tanh(q.k * scale / softcap).  K pages
- * [blocks, kv_heads, 16, head_dim], V pages [blocks, kv_heads, v_dim, 16], head_dim and v_dim each 64 or 128.
+ * [blocks, kv_heads, 16, head_dim], V pages [blocks, kv_heads, v_dim, 16], head_dim 64, 128
+ * or 192, v_dim 64 or 128.
  */
 int32_t mi355_paged_attn_prefill_ext(void* out, int64_t out_stride, const void* q, int64_t q_stride,
                                      const void* k_cache, const void* v_cache, int32_t num_blocks,
@@ -947,6 +948,7 @@ int32_t mi355_latent_kv_write(void* cache, void* cache_t, const void* x, int64_t
  * The matrix-core form of latent_window_attn (16-bit storage, rank a multiple of 16 up to 512,
  * rank + rot a multiple of 8 up to 640), same result.
  *   latent_q_pack              q_packed [tokens, heads, rank + rot] = q_latent | rotated part of q
+ *                              (q_latent null: the rotated part alone is stored)
  *   latent_window_attn_tiles   tiles [num_tiles][3] = (chunk, first pair, pairs <= 16): a pair is
  *                              (packed row, head), number row * heads + head; a tile's pairs are
  *                              consecutive and of one chunk, every pair in exactly one tile.  Reads both
@@ -960,6 +962,11 @@ int32_t mi355_latent_q_pack(void* q_packed, const void* q_latent, int64_t q_late
                             int32_t max_pos, const int64_t* positions, int64_t num_tokens,
                             int32_t num_heads, int32_t rank, int32_t rot, int32_t rot_dims,
                             int32_t interleaved, int32_t dtype, void* stream);
+/* q [tokens, heads * q_head_width]: the first rot_dims columns at q_rot_offset of every head are rotated in place. */
+int32_t mi355_latent_q_rotate(void* q, int64_t q_stride, int32_t q_head_width, int32_t q_rot_offset,
+                              const float* cos_sin, int32_t max_pos, const int64_t* positions,
+                              int64_t num_tokens, int32_t num_heads, int32_t rot_dims,
+                              int32_t interleaved, int32_t dtype, void* stream);
 int32_t mi355_latent_window_attn_tiles(void* out, int64_t out_stride, int64_t out_head_stride,
                                        const void* q_packed, const void* cache, const void* cache_t,
                                        const int32_t* block_tables, int32_t max_blocks,
@@ -991,7 +998,8 @@ int32_t mi355_latent_window_attn(void* out, int64_t out_stride, int64_t out_head
  *                     score is the logit itself and the weights are a softmax over the chosen logits
  *                     alone, times weight_scale
  *   moe_sort          routed rows by expert: offsets [experts + 1], perm[position] = row,
- *                     inv[row] = position
+ *                     inv[row] = position; tile_start [experts + 1] (may be null): the first tile of tile_rows
+ *                     rows of every expert
  *   moe_table_sort    a mixture without a router: tables [layers][vocab, top] name the experts of every token
  *                     id; for every layer offsets [experts + 1], perm and inv as moe_sort, and tile_start
  *                     [experts + 1], the first tile of tile_rows rows of every expert (stacked by layer)
@@ -1017,7 +1025,8 @@ int32_t mi355_moe_route(int32_t* ids, float* weights, const float* logits, int64
                         int32_t groups, int32_t keep, int32_t softmax, int32_t group_max,
                         float weight_scale, void* stream);
 int32_t mi355_moe_sort(int32_t* offsets, int32_t* perm, int32_t* inv, const int32_t* ids,
-                       int64_t num_rows, int32_t experts, void* stream);
+                       int64_t num_rows, int32_t experts, int32_t* tile_start, int32_t tile_rows,
+                       void* stream);
 int32_t mi355_moe_gather_rows(void* xs, const void* x, const int32_t* perm, const int32_t* offsets,
                               int32_t pad_to, int64_t num_rows, int32_t top, int32_t width,
                               int32_t dtype, void* stream);
@@ -1043,6 +1052,26 @@ int32_t mi355_moe_combine(void* out, const void* y, const int32_t* inv, const fl
                           int64_t num_tokens, int32_t top, int32_t width, const void* x,
                           int32_t num_real, const void* shared, const float* shared_gate,
                           int64_t shared_gate_stride, int32_t dtype, void* stream);
+
+/*
+ * Grouped products on the matrix cores (16-bit storage, fp32 accumulation), in_width a multiple of 8, out_width of 4.
+ *   expert_gemm   y[p] = a(W[e] x[perm[p] / top]) (perm null: x[p]) for the positions p of expert e's range of the
+ *                 expert order (offsets, tile_start of 128 rows: see moe_table_sort), w [experts, out_width, in_width],
+ *                 x [x_rows, in_width], y [num_rows, out_width]; a: identity, or relu2: max(., 0)^2.  Positions
+ *                 past offsets[experts] are left alone
+ *   head_gemm     for every head h: y_h[m] = W_h x_h[m], w [heads, out_width, in_width], x_h[m] = x + row * x_stride
+ *                 + h * x_group, row = index[m] (null: m); output n of row m at y + (m / 16) * y_block + (m % 16) *
+ *                 y_stride + h * y_group + n, or (transposed) y + (m / 16) * y_block + h * y_group + n * 16 + m % 16.
+ *                 copy: columns in_width .. in_width + copy of the x row follow the outputs
+ */
+int32_t mi355_expert_gemm(void* y, const void* x, int64_t x_rows, const void* w, const int32_t* offsets,
+                          const int32_t* tile_start, const int32_t* perm, int32_t top, int64_t num_rows,
+                          int32_t experts, int32_t out_width, int32_t in_width, int32_t relu2,
+                          int32_t dtype, void* stream);
+int32_t mi355_head_gemm(void* y, int64_t y_block, int64_t y_stride, int64_t y_group, const void* x,
+                        int64_t x_stride, int64_t x_group, int64_t x_rows, const int32_t* index,
+                        const void* w, int64_t num_rows, int32_t heads, int32_t out_width,
+                        int32_t in_width, int32_t copy, int32_t transposed, int32_t dtype, void* stream);
 
 /*
  * A decoder with a hashed previous-token embedding, sinusoidal positions, softmax attention inside

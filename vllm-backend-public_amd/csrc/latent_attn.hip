@@ -11,8 +11,10 @@
 //   latent_window_attn   p_ij = exp(s_ij) / (exp(sink_h) + sum_{j' in window} exp(s_ij')), keys j with
 //                        0 <= i - j < window; the query's rotated part is rotated on the way in; the
 //                        result is multiplied by sigmoid(gate[i, h])
+//   latent_q_rotate      the rotated part of every head of q, in place: prompts whose keys and values are expanded from
+//                        the latents (group_gemm.hip) attend with the query as projected
 //   latent_q_pack        the query as the matrix-core form reads it: [absorbed part | rotated part] per
-//                        (row, head), contiguous
+//                        (row, head), contiguous (without an absorbed part: the rotated part alone is stored)
 // Without a sink (null) the softmax is the ordinary one; a window longer than the sequence is plain causal.
 // Rotation pairs coordinates j, j + dims/2 or (interleaved) neighbours.
 // Scores, weights, the softmax and its running sums, norms and angles are fp32.
@@ -185,13 +187,37 @@ __global__ __launch_bounds__(64) void latent_q_pack_kernel(typename Elem<T>::S* 
   const int64_t t = blockIdx.x;
   const int h = blockIdx.y, lane = threadIdx.x;
   typename Elem<T>::S* dst = qe + (t * H + h) * (rank + rot);
-  for (int i = lane; i < rank; i += 64)
+  for (int i = lane; ql != nullptr && i < rank; i += 64)
     MI355_ST(typename Elem<T>::S, qe, dst + i, MI355_LD(typename Elem<T>::S, ql, ql + t * ql_stride + h * ql_head_stride + i));
   int64_t p = MI355_LD(int64_t, positions, positions + t);
   p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
   const float* cs = cos_sin + p * dims;
   const typename Elem<T>::S* qr = q + t * q_stride + static_cast<int64_t>(h) * q_head + q_rot_off;
   for (int j = lane; j < rot; j += 64) MI355_STF(T, qe, dst + rank + j, rotated_at<T>(q, qr, j, dims, interleaved, cos_sin, cs));
+}
+
+// the rotated columns of every head of q, in place: a wave per row, a pair of coordinates per lane in turn
+template <typename T>
+__global__ __launch_bounds__(256) void latent_q_rotate_kernel(typename Elem<T>::S* __restrict__ q, int64_t q_stride, int q_head,
+                                                              int q_rot_off, const float* __restrict__ cos_sin, int max_pos,
+                                                              const int64_t* __restrict__ positions, int64_t T_, int H,
+                                                              int dims, int interleaved) {
+  const int64_t t = blockIdx.x * 4ll + (threadIdx.x >> 6);
+  if (t >= T_) return;
+  const int lane = threadIdx.x & 63, half = dims >> 1;
+  int64_t p = MI355_LD(int64_t, positions, positions + t);
+  p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
+  const float* cs = cos_sin + p * dims;
+  for (int i = lane; i < H * half; i += 64) {
+    const int h = i / half, j = i % half;
+    typename Elem<T>::S* v = q + t * q_stride + static_cast<int64_t>(h) * q_head + q_rot_off;
+    typename Elem<T>::S* a = v + (interleaved ? 2 * j : j);
+    typename Elem<T>::S* b = v + (interleaved ? 2 * j + 1 : j + half);
+    const float c = MI355_LD(float, cos_sin, cs + j), s = MI355_LD(float, cos_sin, cs + half + j);
+    const float x = MI355_LDF(T, q, a), y = MI355_LDF(T, q, b);
+    MI355_STF(T, q, a, x * c - y * s);
+    MI355_STF(T, q, b, y * c + x * s);
+  }
 }
 
 constexpr float kLog2e = 1.4426950408889634f;
@@ -476,10 +502,10 @@ extern "C" int32_t mi355_latent_q_pack(void* q_packed, const void* q_latent, int
                                        int32_t q_rot_offset, const float* cos_sin, int32_t max_pos,
                                        const int64_t* positions, int64_t num_tokens, int32_t num_heads, int32_t rank,
                                        int32_t rot, int32_t rot_dims, int32_t interleaved, int32_t dtype, void* stream) {
-  MI355_REQUIRE(q_packed && q_latent && q && cos_sin && positions, MI355_ERR_INVALID, "latent_q_pack: null pointer");
+  MI355_REQUIRE(q_packed && q && cos_sin && positions, MI355_ERR_INVALID, "latent_q_pack: null pointer");
   MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && num_heads <= 65535 && rank > 0 && rot >= 0 && max_pos > 0 &&
-                    q_rot_offset >= 0 && q_head_width >= q_rot_offset + rot && q_latent_stride >= rank &&
-                    q_latent_head_stride >= rank && q_stride >= static_cast<int64_t>(num_heads) * q_head_width,
+                    q_rot_offset >= 0 && q_head_width >= q_rot_offset + rot &&
+                    (q_latent == nullptr || (q_latent_stride >= rank && q_latent_head_stride >= rank)) && q_stride >= static_cast<int64_t>(num_heads) * q_head_width,
                 MI355_ERR_INVALID, "latent_q_pack: sizes");
   MI355_REQUIRE(rot_dims >= 0 && rot_dims <= rot && rot_dims % 2 == 0, MI355_ERR_INVALID,
                 "latent_q_pack: rot_dims %d must be even and at most %d", rot_dims, rot);
@@ -494,6 +520,23 @@ extern "C" int32_t mi355_latent_q_pack(void* q_packed, const void* q_latent, int
                                                   q_head_width, q_rot_offset, cos_sin, max_pos, positions, num_heads, rank,
                                                   rot, rot_dims, interleaved));
   return check_launch("latent_q_pack");
+}
+
+extern "C" int32_t mi355_latent_q_rotate(void* q, int64_t q_stride, int32_t q_head_width, int32_t q_rot_offset, const float* cos_sin,
+                                         int32_t max_pos, const int64_t* positions, int64_t num_tokens, int32_t num_heads,
+                                         int32_t rot_dims, int32_t interleaved, int32_t dtype, void* stream) {
+  MI355_REQUIRE(q && cos_sin && positions, MI355_ERR_INVALID, "latent_q_rotate: null pointer");
+  MI355_REQUIRE(num_tokens >= 0 && num_heads > 0 && max_pos > 0 && rot_dims >= 0 && rot_dims % 2 == 0 && q_rot_offset >= 0 &&
+                    q_head_width >= q_rot_offset + rot_dims && q_stride >= static_cast<int64_t>(num_heads) * q_head_width,
+                MI355_ERR_INVALID, "latent_q_rotate: sizes");
+  REQ_DTYPE(dtype);
+  if (num_tokens == 0 || rot_dims == 0) return MI355_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  MI355_DISPATCH_DTYPE3(dtype, hipLaunchKernelGGL((latent_q_rotate_kernel<TT>), dim3(static_cast<unsigned>((num_tokens + 3) / 4)),
+                                                  dim3(256), 0, s, static_cast<Elem<TT>::S*>(q), q_stride, q_head_width,
+                                                  q_rot_offset, cos_sin, max_pos, positions, num_tokens, num_heads, rot_dims,
+                                                  interleaved));
+  return check_launch("latent_q_rotate");
 }
 
 extern "C" int32_t mi355_latent_window_attn_tiles(void* out, int64_t out_stride, int64_t out_head_stride,

@@ -7,9 +7,9 @@
 //                       best), and weighted by the score without correction, times a constant
 //   moe_sort            rows (token, choice) ordered by expert: offsets[E + 1], perm[position] = row,
 //                       inv[row] = position
+//                       (and tile_start[E + 1], the first tile of tile_rows rows of every expert, if asked for)
 //   moe_table_sort      the same for a mixture without a router: a table [vocab, top] names the experts of every
-//                       token id, so a step's row orders of all its layers are made by one launch ahead of the layers;
-//                       also tile_start[E + 1], the first tile of `tile_rows` rows of every expert
+//                       token id, so a step's row orders of all its layers are made by one launch ahead of the layers
 //   moe_gather_rows     xs[position] = x[perm[position] / top]; or every expert's rows padded to a common count
 //   moe_gate_up_rows    a[position] = silu(Wg[e] x) * (Wu[e] x) for every routed row, one wave per
 //                       (expert, hidden unit) walking that expert's rows: an expert's weights leave HBM once
@@ -201,7 +201,8 @@ __global__ __launch_bounds__(256) void moe_route_wave_kernel(int32_t* __restrict
 // one workgroup: counts, an exclusive prefix, then a position for every row
 __global__ __launch_bounds__(1024) void moe_sort_kernel(int32_t* __restrict__ offsets, int32_t* __restrict__ perm,
                                                         int32_t* __restrict__ inv, const int32_t* __restrict__ ids,
-                                                        int64_t rows, int E) {
+                                                        int64_t rows, int E, int32_t* __restrict__ tile_start,
+                                                        int tile_rows) {
   extern __shared__ int32_t sm[];                       // counts [E] | starts [E + 1]
   int32_t* cnt = sm;
   int32_t* start = sm + E;
@@ -210,12 +211,15 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(int32_t* __restrict__ of
   for (int64_t r = threadIdx.x; r < rows; r += blockDim.x) atomicAdd(&cnt[MI355_LD(int32_t, ids, ids + r)], 1);
   __syncthreads();
   if (threadIdx.x == 0) {
-    int32_t at = 0;
+    int32_t at = 0, tile = 0;
     for (int e = 0; e < E; ++e) {
       start[e] = at;
       at += cnt[e];
+      if (tile_start != nullptr) MI355_ST(int32_t, tile_start, tile_start + e, tile);
+      tile += (cnt[e] + tile_rows - 1) / tile_rows;
     }
     start[E] = at;
+    if (tile_start != nullptr) MI355_ST(int32_t, tile_start, tile_start + E, tile);
   }
   __syncthreads();
   for (int e = threadIdx.x; e <= E; e += blockDim.x) MI355_ST(int32_t, offsets, offsets + e, start[e]);
@@ -603,12 +607,13 @@ extern "C" int32_t mi355_moe_route(int32_t* ids, float* weights, const float* lo
 }
 
 extern "C" int32_t mi355_moe_sort(int32_t* offsets, int32_t* perm, int32_t* inv, const int32_t* ids, int64_t num_rows,
-                                  int32_t experts, void* stream) {
+                                  int32_t experts, int32_t* tile_start, int32_t tile_rows, void* stream) {
   MI355_REQUIRE(offsets && perm && inv && ids, MI355_ERR_INVALID, "moe_sort: null pointer");
-  MI355_REQUIRE(num_rows >= 0 && num_rows <= 0x7FFFFFFF && experts > 0 && experts <= 4096, MI355_ERR_INVALID,
+  MI355_REQUIRE(num_rows >= 0 && num_rows <= 0x7FFFFFFF && experts > 0 && experts <= 4096 && tile_rows > 0, MI355_ERR_INVALID,
                 "moe_sort: sizes");
   hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), (2 * static_cast<size_t>(experts) + 1) * sizeof(int32_t),
-                     static_cast<hipStream_t>(stream), offsets, perm, inv, ids, num_rows, experts);
+                     static_cast<hipStream_t>(stream), offsets, perm, inv, ids, num_rows, experts,
+                     tile_start, tile_rows);
   return check_launch("moe_sort");
 }
 

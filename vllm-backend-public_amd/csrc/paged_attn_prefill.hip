@@ -34,7 +34,7 @@
 // chunk of the tile's first query and columns of a tile that straddles a chunk edge mask for themselves;
 // or a sliding window (keys after p - window) beside the first `keep` keys of the sequence: the walk takes
 // the barrier intervals that hold kept keys and lie before the window's first interval, then the window's;
-// value sizes that differ from the key size (64 / 128 either way); one more term exp(sink[head]) in the softmax denominator that carries no value; and the output times
+// value sizes that differ from the key size (64 / 128; keys of 64, 128 or 192); one more term exp(sink[head]) in the softmax denominator that carries no value; and the output times
 // the sigmoid of one gate number per (token, head), and times a constant; a soft cap on the scores (cap_x > 0),
 // cap * tanh(q.k scale / cap).
 #include "common.h"
@@ -438,7 +438,7 @@ static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chu
   const int group = num_heads / num_kv_heads;
   MI355_REQUIRE(group <= 16 && num_kv_heads <= 65535, MI355_ERR_UNSUPPORTED,
                 "%s: at most 16 query heads per kv head (got %d)", name, group);
-  MI355_REQUIRE((head_dim == 64 || head_dim == 128) && (v_dim == head_dim || (ext && (v_dim == 64 || v_dim == 128))),
+  MI355_REQUIRE((head_dim == 64 || head_dim == 128 || (ext && head_dim == 192)) && (v_dim == head_dim || (ext && (v_dim == 64 || v_dim == 128))),
                 MI355_ERR_UNSUPPORTED, "%s: head_dim %d / v_dim %d not supported (64 or 128)", name, head_dim, v_dim);
   const int64_t width = static_cast<int64_t>(num_heads) * head_dim;
   MI355_REQUIRE(q_stride >= width && q_stride % 8 == 0 && out_stride >= static_cast<int64_t>(num_heads) * v_dim && out_stride % 8 == 0,
@@ -480,11 +480,21 @@ static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chu
     case 1: MI355_PRE(TT, DD, 1); break;    \
     default: MI355_PRE(TT, DD, 2); break;   \
   }
+#define MI355_PRE_192(TT)                                               \
+  do {                                                                  \
+    if (v_dim == 64 && nq == 1) MI355_PRE_E(TT, 192, 64, 1, true);      \
+    else if (v_dim == 64) MI355_PRE_E(TT, 192, 64, 2, true);            \
+    else if (nq == 1) MI355_PRE_E(TT, 192, 128, 1, true);               \
+    else MI355_PRE_E(TT, 192, 128, 2, true);                            \
+  } while (0)
   if (dtype == MI355_BF16) {
-    if (head_dim == 64) { MI355_PRE_NQ(BF16, 64) } else { MI355_PRE_NQ(BF16, 128) }
+    if (head_dim == 192) MI355_PRE_192(BF16);
+    else if (head_dim == 64) { MI355_PRE_NQ(BF16, 64) } else { MI355_PRE_NQ(BF16, 128) }
   } else {
-    if (head_dim == 64) { MI355_PRE_NQ(F16, 64) } else { MI355_PRE_NQ(F16, 128) }
+    if (head_dim == 192) MI355_PRE_192(F16);
+    else if (head_dim == 64) { MI355_PRE_NQ(F16, 64) } else { MI355_PRE_NQ(F16, 128) }
   }
+#undef MI355_PRE_192
 #undef MI355_PRE_NQ
 #undef MI355_PRE
 #undef MI355_PRE_E

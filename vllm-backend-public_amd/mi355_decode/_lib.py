@@ -129,13 +129,16 @@ def _load() -> ctypes.CDLL:
         "mi355_latent_window_attn": (I32, [P, I64, I64, P, I64, I64, P, I64, I32, I32, P, P, I32, P, P, P, P, I64, P, I32,
                                            I64, I32, I32, I32, I32, I32, I32, F, I32, P]),
         "mi355_moe_route": (I32, [P, P, P, I64, P, I64, I32, I32, I32, I32, I32, I32, F, P]),
-        "mi355_moe_sort": (I32, [P, P, P, P, I64, I32, P]),
+        "mi355_moe_sort": (I32, [P, P, P, P, I64, I32, P, I32, P]),
         "mi355_moe_gather_rows": (I32, [P, P, P, P, I32, I64, I32, I32, I32, P]),
         "mi355_moe_gate_up_rows": (I32, [P, P, P, P, P, I32, I32, I32, I32, I32, F, I32, P]),
         "mi355_moe_down_rows": (I32, [P, P, P, P, I32, I32, I32, I32, P]),
         "mi355_moe_linear_rows": (I32, [P, P, P, P, P, I32, I32, I32, I32, I32, I32, P]),
         "mi355_moe_table_sort": (I32, [P, P, P, P, P, P, I64, I64, I32, I32, I32, I32, P]),
         "mi355_add_layer_norm_f32": (I32, [P, P, P, P, I32, F, P, I64, I32, F, I32, P]),
+        "mi355_expert_gemm": (I32, [P, P, I64, P, P, P, P, I32, I64, I32, I32, I32, I32, I32, P]),
+        "mi355_head_gemm": (I32, [P, I64, I64, I64, P, I64, I64, I64, P, P, I64, I32, I32, I32, I32, I32, I32, P]),
+        "mi355_latent_q_rotate": (I32, [P, I64, I32, I32, P, I32, P, I64, I32, I32, I32, I32, P]),
         "mi355_moe_silu_and_mul": (I32, [P, P, I64, I32, I32, F, I32, P]),
         "mi355_gated_act_rows": (I32, [P, I64, P, P, I64, I64, I32, I32, F, I32, P]),
         "mi355_moe_combine": (I32, [P, P, P, P, P, P, I32, I64, I32, I32, P, I32, P, P, I64, I32, P]),
@@ -205,7 +208,8 @@ EXPORTS = ("mi355_abi_version", "mi355_last_error", "mi355_target_arch",
            "mi355_mingru_scan_workspace", "mi355_row_norm_rope_kv_write", "mi355_norm_resid_f32", "mi355_token_gate_rows",
            "mi355_token_side_f32", "mi355_linear_attn_state_floats", "mi355_linear_attn_tile_rows", "mi355_mlstm_gates",
            "mi355_linear_attn_chunks", "mi355_decay_attn_step", "mi355_mlstm_step",
-           "mi355_moe_linear_rows", "mi355_moe_table_sort", "mi355_add_layer_norm_f32")
+           "mi355_moe_linear_rows", "mi355_moe_table_sort", "mi355_add_layer_norm_f32", "mi355_expert_gemm",
+           "mi355_head_gemm", "mi355_latent_q_rotate")
 
 
 def check(status: int) -> None:

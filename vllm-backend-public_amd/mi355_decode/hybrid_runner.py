@@ -54,7 +54,7 @@ import torch
 
 from . import ops
 from ._lib import BLOCK_SIZE
-from .config import ModelConfig
+from .config import NO_WINDOW, ModelConfig
 from .model_runner import ModelRunner, batch_buckets
 from .weights import ModelWeights
 
@@ -83,11 +83,13 @@ class StepBatch:
     """Device-side description of one packed step (see csrc/seqmix.hip)."""
     __slots__ = ("ids", "positions", "slot_mapping", "block_tables", "cu_seqlens", "tok_seq", "state_slots",
                  "num_tokens", "num_seqs", "tiles", "long_chunks", "pair_tiles", "context_lens", "max_q_len", "row_tiles",
-                 "routes")
+                 "routes", "latent_plan")
 
     def __init__(self, ids, positions, slot_mapping, block_tables, cu_seqlens, tok_seq, state_slots, tiles=None,
-                 long_chunks=False, pair_tiles=None, context_lens=None, max_q_len=0, row_tiles=None):
+                 long_chunks=False, pair_tiles=None, context_lens=None, max_q_len=0, row_tiles=None,
+                 latent_plan=None):
         self.routes = {}                              # (experts, top) -> ops.TableRoutes of the step's token ids
+        self.latent_plan = latent_plan                # () -> the step's LatentPlan, or None (captured decode steps)
         self.row_tiles = row_tiles                    # rows -> ops.RowTiles of the step, or None (captured decode steps)
         # every chunk's length of context after the step (int32, on the device) and the longest chunk: what the
         # LDS-staged prompt attention walks by; None: not known to this step (captured decode steps)
@@ -166,13 +168,67 @@ class GeneralDeltaMixer:
         return r.linear(ops.gated_head_rms_norm(o, col("g"), lw.head_norm, r.eps, ops.ACT_SIGMOID), lw.o_w)
 
 
+class LatentPlan:
+    """Which chunks of a step attend with keys and values expanded from their latents, and where those go: chunks of
+    EXPAND_MIN_ROWS rows and more, whose queries are many enough to pay for one product per context token.  Pages
+    of 16 tokens per such chunk, numbered from 0, hold the expanded context for the length of one layer.  The other
+    chunks (decoded tokens, short portions) stay on the latents, as rows of their own.
+
+      index     int32 [16 * pages]: the slot of the latent pages that every expanded row reads
+      tables    int32 [chunks, most pages]: the expanded pages of every chunk
+      ctx       int32 [chunks]: its context after the step, 0 for a chunk that is not expanded
+      short     None, or (rows int64, block tables, chunk of every row, tiles by heads) of the remaining rows"""
+
+    EXPAND_MIN_ROWS = 48
+    MAX_BYTES = 4 << 30                        # of expanded keys and values of one layer
+
+    def __init__(self, cu, ctx, block_tables, device):
+        self.device = device
+        cu, ctx = np.asarray(cu, dtype=np.int64), np.asarray(ctx, dtype=np.int64)
+        lens = cu[1:] - cu[:-1]
+        long = lens >= self.EXPAND_MIN_ROWS
+        pages = np.where(long, -(-ctx // BLOCK_SIZE), 0)
+        self.pages, self.max_q_len = int(pages.sum()), int(lens[long].max()) if long.any() else 0
+        self.fits = bool(long.any())
+        if not self.fits:
+            return
+        bt = np.asarray(block_tables)
+        first = np.cumsum(pages) - pages
+        slots = np.concatenate([bt[s, : pages[s]] for s in np.flatnonzero(long)]).astype(np.int64)
+        index = (slots[:, None] * BLOCK_SIZE + np.arange(BLOCK_SIZE)).reshape(-1).astype(np.int32)
+        tables = np.minimum(first[:, None] + np.arange(max(int(pages.max()), 1))[None, :], max(self.pages - 1, 0)).astype(np.int32)
+        t = lambda a: torch.from_numpy(np.ascontiguousarray(a)).to(device, non_blocking=True)     # noqa: E731
+        self.index, self.tables, self.ctx = t(index), t(tables), t(np.where(long, ctx, 0).astype(np.int32))
+        self.short, self._short_tiles = None, {}
+        if not long.all():
+            ids = np.flatnonzero(~long)
+            rows = np.concatenate([np.arange(cu[s], cu[s + 1]) for s in ids])
+            self._short_cu = np.concatenate([[0], np.cumsum(lens[ids])])
+            seq = np.repeat(np.arange(len(ids)), lens[ids]).astype(np.int32)
+            self.short = (t(rows), t(bt[ids].astype(np.int32)), t(seq))
+
+    def short_tiles(self, heads: int) -> torch.Tensor:
+        if heads not in self._short_tiles:
+            self._short_tiles[heads] = torch.from_numpy(ops.pair_tiles(self._short_cu, heads)).to(self.device, non_blocking=True)
+        return self._short_tiles[heads]
+
+
 class LatentAttention:
     """Softmax attention through low-rank latents (in a sliding window or causal; a sink and an output gate
     where the design has them) over the latent pages of one layer run -- its own (it writes them first)
-    or those of the layer it shares with."""
+    or those of the layer it shares with.
+
+    Two forms.  On the latents: the up-projections of keys and values move to the query and to the result, every
+    head then reads the same latents; decoded tokens and windows.  Expanded (no window, 16-bit, key and value sizes
+    of the LDS-staged prompt attention): the keys and values of a chunk's context are made from its latents into
+    pages that live for this layer, and the chunk attends to them with the queries as projected -- a third of
+    the products per (query, key) pair at a latent four times as wide as a head."""
 
     def __init__(self, spec, lw, runner, cache_index: int, writes: bool):
         self.s, self.lw, self.r, self.ci, self.writes = spec, lw, runner, cache_index, writes
+        self.head_gemm = getattr(lw, "uk_t", None) is not None
+        self.expands = self.head_gemm and spec.window >= NO_WINDOW and writes \
+            and ops.chunk_attn_prefill_ok(runner.dtype, spec.heads, spec.heads, spec.dim + spec.rot_dim, spec.vdim)
 
     def __call__(self, proj: torch.Tensor, b: StepBatch) -> torch.Tensor:
         s, lw, r = self.s, self.lw, self.r
@@ -183,22 +239,63 @@ class LatentAttention:
                                 r.eps, cache_t=cache_t, interleaved=s.interleaved)
         q = col("q") if s.q_direct else r.linear(ops.rms_norm_rows(col("dq"), lw.dq_norm, r.eps), lw.uq_w)
         gate = col("g") if s.gate else None
-        T, hw = q.shape[0], s.dim + s.rot_dim
-        # the unrotated query part of every head into the latent space: the keys then are the cached latents
-        ql = torch.bmm(q.view(T, s.heads, hw)[:, :, : s.dim].transpose(0, 1), lw.uk_w)
-        if cache_t is not None and b.pair_tiles is not None:
+        plan = b.latent_plan() if self.expands and b.long_chunks and b.latent_plan is not None else None
+        if plan is None or not plan.fits or plan.pages * BLOCK_SIZE * s.heads * (s.dim + s.rot_dim + s.vdim) * 2 > plan.MAX_BYTES:
+            return r.linear(self._on_latents(q, gate, b.positions, b.block_tables, b.tok_seq, b.pair_tiles), lw.o_w)
+        return r.linear(self._expanded(q, gate, b, plan), lw.o_w)
+
+    def _expanded(self, q: torch.Tensor, gate: Optional[torch.Tensor], b: StepBatch, plan: LatentPlan) -> torch.Tensor:
+        s, lw, r = self.s, self.lw, self.r
+        (cache, _), table = r.latent_cache[self.ci], r.rotary(s.rot_dims, s.rot_base, exact=s.interleaved)
+        H, D, hw = s.heads, s.dim + s.rot_dim, s.dim + s.rot_dim
+        rest = None
+        if plan.short is not None:
+            rows, bt, seq = plan.short
+            rest = self._on_latents(q.index_select(0, rows), None if gate is None else gate.index_select(0, rows),
+                                    b.positions.index_select(0, rows), bt, seq, plan.short_tiles)
+        ops.latent_q_rotate(q, H, hw, s.dim, table, b.positions, interleaved=s.interleaved)
+        flat, n = cache.view(-1, s.kv_rank + s.rot_dim), plan.pages * BLOCK_SIZE
+        k = torch.empty(plan.pages, H, BLOCK_SIZE, D, dtype=q.dtype, device=q.device)
+        v = torch.empty(plan.pages, H, s.vdim, BLOCK_SIZE, dtype=q.dtype, device=q.device)
+        ops.head_gemm(flat, 0, lw.uk_w, k, H * BLOCK_SIZE * D, D, BLOCK_SIZE * D, n, index=plan.index, copy=s.rot_dim)
+        ops.head_gemm(flat, 0, lw.uv_w, v, H * s.vdim * BLOCK_SIZE, 0, s.vdim * BLOCK_SIZE, n, index=plan.index, transposed=True)
+        o = ops.paged_attn_prefill_ext(q, k, v, plan.tables, b.cu_seqlens, plan.ctx, plan.max_q_len, H, H, D, s.scale,
+                                       sink=lw.sink, gate=gate)
+        if rest is not None:
+            o.index_copy_(0, plan.short[0], rest)
+        return o
+
+    def _on_latents(self, q, gate, positions, block_tables, tok_seq, pair_tiles) -> torch.Tensor:
+        """The concatenated heads [tokens, heads * vdim]."""
+        s, lw, r = self.s, self.lw, self.r
+        (cache, cache_t), table = r.latent_cache[self.ci], r.rotary(s.rot_dims, s.rot_base, exact=s.interleaved)
+        T, H, hw, R, dq = q.shape[0], s.heads, s.dim + s.rot_dim, s.kv_rank, s.kv_rank + s.rot_dim
+        matrix_cores = cache_t is not None and pair_tiles is not None
+        if matrix_cores:
             # the matrix cores: tiles of 16 (row, head) pairs; few tiles (decoded tokens, short prompts) spread
             # their windows' keys over several workgroups
-            tiles = b.pair_tiles(s.heads)
+            tiles = pair_tiles(H)
             n = min(16, max(s.window // 64, 1), max(1024 // max(int(tiles.shape[0]), 1), 1))
-            ol = ops.latent_window_attn_tiles(ops.latent_q_pack(ql, q, hw, s.dim, s.rot_dim, table, b.positions, interleaved=s.interleaved), cache,
-                                              cache_t, b.block_tables, tiles, b.positions, lw.sink, gate, s.window,
-                                              s.scale, num_splits=n)
+        if matrix_cores and self.head_gemm:
+            qe = torch.empty(T, H, dq, dtype=q.dtype, device=q.device)
+            ops.head_gemm(q, hw, lw.uk_t, qe, 16 * H * dq, H * dq, dq, T)
+            ops.latent_q_pack(None, q, hw, s.dim, s.rot_dim, table, positions, interleaved=s.interleaved, out=qe)
+            ol = torch.empty(T, H, R, dtype=q.dtype, device=q.device)
+            ops.latent_window_attn_tiles(qe, cache, cache_t, block_tables, tiles, positions, lw.sink, gate, s.window, s.scale,
+                                         num_splits=n, out=ol.transpose(0, 1))
+            o = torch.empty(T, H * s.vdim, dtype=q.dtype, device=q.device)
+            return ops.head_gemm(ol.view(T, H * R), R, lw.uv_w, o, 16 * H * s.vdim, H * s.vdim, s.vdim, T)
+        # the unrotated query part of every head into the latent space: the keys then are the cached latents
+        ql = torch.bmm(q.view(T, H, hw)[:, :, : s.dim].transpose(0, 1), lw.uk_w)
+        if matrix_cores:
+            ol = ops.latent_window_attn_tiles(ops.latent_q_pack(ql, q, hw, s.dim, s.rot_dim, table, positions, interleaved=s.interleaved),
+                                              cache, cache_t, block_tables, tiles, positions, lw.sink, gate, s.window, s.scale,
+                                              num_splits=n)
         else:
-            ol = ops.latent_window_attn(ql, q, hw, s.dim, cache, b.block_tables, b.tok_seq, b.positions, lw.sink, gate,
-                                        table, s.window, s.scale, interleaved=s.interleaved)
-        o = torch.bmm(ol, lw.uv_t)                      # [heads, tokens, vdim]
-        return r.linear(o.transpose(0, 1).reshape(T, s.heads * s.vdim), lw.o_w)
+            ol = ops.latent_window_attn(ql, q, hw, s.dim, cache, block_tables, tok_seq, positions, lw.sink, gate, table, s.window,
+                                        s.scale, interleaved=s.interleaved)
+        o = torch.bmm(ol, lw.uv_t if lw.uv_t is not None else lw.uv_w.transpose(1, 2).contiguous())      # [heads, tokens, vdim]
+        return o.transpose(0, 1).reshape(T, H * s.vdim)
 
 
 class BlockAttention:
@@ -383,6 +480,10 @@ class ExpertRows:
         self.rows, self.inv, self.top, self.weight = rows, inv, top, weight
 
 
+# from this many rows per expert on, tiles of 128 rows through LDS; below, one pass over each expert's weights
+EXPERT_GEMM_MIN_ROWS = 32
+
+
 class TableMoE:
     """Mixture of experts without a router: the runner has sorted the step's rows by the experts that the layer's
     table names for their token ids (one launch for all such layers, ahead of the first); an expert is
@@ -394,6 +495,11 @@ class TableMoE:
     def __call__(self, h: torch.Tensor, b: "StepBatch") -> ExpertRows:
         s, lw, rt = self.s, self.lw, b.routes[(self.s.experts, self.s.top)]
         offsets, perm = rt.offsets[self.slot], rt.perm[self.slot]
+        if rt.rows >= EXPERT_GEMM_MIN_ROWS * s.experts and ops.expert_gemm_ok(h.dtype, h.shape[1], s.ff):
+            start = rt.tile_start[self.slot]
+            act = ops.expert_gemm(h, lw.up_w, offsets, start, rt.rows, perm=perm, top=s.top, relu2=True)
+            y = ops.expert_gemm(act, lw.down_w, offsets, start, rt.rows)
+            return ExpertRows(y, rt.inv[self.slot], s.top, 1.0 / s.top)
         act = ops.moe_linear_rows(h, lw.up_w, offsets, rt.rows, perm=perm, top=s.top, relu2=True)
         return ExpertRows(ops.moe_linear_rows(act, lw.down_w, offsets, rt.rows), rt.inv[self.slot], s.top, 1.0 / s.top)
 
@@ -402,7 +508,7 @@ class MoEFeedForward:
     """Mixture of experts: fp32 routing, rows sorted by expert, the expert products, the weighted sum
     (which also takes in identity experts and a gated shared expert where the design has them)."""
 
-    GROUPED_MIN_ROWS = 512          # from this many routed rows on, one library GEMM per expert (needs the counts on the host)
+    GROUPED_MIN_ROWS = 512          # from this many routed rows on (and EXPERT_GEMM_MIN_ROWS per expert) products by row tiles
 
     def __init__(self, spec, lw, runner):
         self.s, self.lw, self.r = spec, lw, runner
@@ -440,7 +546,9 @@ class MoEFeedForward:
         ids, wts = ops.moe_route(logits, lw.correction, s.top, s.groups, s.keep, softmax=s.score == "softmax",
                                  group_max=s.group_score == "max", weight_scale=s.weight_scale, experts=s.outputs,
                                  chosen_softmax=s.score == "chosen_softmax")
-        offsets, perm, inv = ops.moe_sort(ids, s.outputs)
+        rows = T * s.top
+        tiled = rows >= max(self.GROUPED_MIN_ROWS, EXPERT_GEMM_MIN_ROWS * E) and ops.expert_gemm_ok(h.dtype, h.shape[1], s.ff)
+        offsets, perm, inv, start = ops.moe_sort(ids, s.outputs, tiles=True)
         extra = {}
         if s.identity:
             extra.update(ids=ids, x=h, num_real=E)
@@ -451,19 +559,14 @@ class MoEFeedForward:
             extra.update(shared=self.r.linear(self._act(gu, s.shared_limit, s.shared_ff), lw.shared_down_w))
             if s.shared_gated:
                 extra.update(shared_gate=logits[:, s.outputs:])
-        rows = T * s.top
-        if rows >= self.GROUPED_MIN_ROWS and not torch.cuda.is_current_stream_capturing():
-            # many rows: library GEMMs per expert.  The experts' row ranges come to the host (one wait); when
-            # the loads are near even, every expert's rows are padded to the largest count and the two products
-            # are one batched GEMM each; otherwise one GEMM per expert on its range of the sorted rows.
+        if tiled:
+            # many rows: one launch per product over all experts' row tiles
+            gu = ops.expert_gemm(h, lw.gate_up_w, offsets, start, rows, perm=perm, top=s.top)
+            y = ops.expert_gemm(self._act(gu, s.limit, s.ff), lw.down_w, offsets, start, rows)
+        elif rows >= self.GROUPED_MIN_ROWS and not torch.cuda.is_current_stream_capturing():
+            # sizes the tiles do not cover (and float32): one library GEMM per expert on its range of the sorted
+            # rows; the ranges come to the host (one wait)
             off = offsets.tolist()
-            cap = -(-max(off[e + 1] - off[e] for e in range(E)) // 16) * 16
-            if 0 < E * cap <= 2 * off[E]:
-                xp = ops.moe_gather_rows(h, perm, rows, s.top, offsets=offsets, pad_to=cap, experts=E)
-                gu = torch.bmm(xp.view(E, cap, -1), lw.gate_up_w.transpose(1, 2)).view(E * cap, 2 * s.ff)
-                y = torch.bmm(self._act(gu, s.limit, s.ff).view(E, cap, s.ff), lw.down_w.transpose(1, 2)).view(E * cap, -1)
-                extra["ids"] = ids
-                return ops.moe_combine(y, inv, wts, T, s.top, offsets=offsets, pad_to=cap, **extra)
             xs = ops.moe_gather_rows(h, perm, rows, s.top)
             gu = torch.empty(rows, 2 * s.ff, dtype=h.dtype, device=h.device)
             for e in range(E):
@@ -645,6 +748,7 @@ class HybridRunner(ModelRunner):
         self.layer_trace = None                       # a list: _forward appends the residual after every layer run
         self._pair_tiles = {}                         # of the step at hand: heads -> device tiles
         self._row_tiles = {}                          # of the step at hand: rows -> ops.RowTiles
+        self._latent_plan = None                      # of the step at hand
         self._dec_pairs = {}                          # of a decode step of max_num_seqs rows: heads -> device tiles
 
     # ------------------------------------------------------------------ #
@@ -679,6 +783,11 @@ class HybridRunner(ModelRunner):
         if rows not in self._row_tiles:
             self._row_tiles[rows] = ops.RowTiles(self._step_cu, rows, self.device)
         return self._row_tiles[rows]
+
+    def _chunk_latent_plan(self) -> LatentPlan:
+        if self._latent_plan is None:
+            self._latent_plan = LatentPlan(self._step_cu, self._step_ctx, self._step_tables, self.device)
+        return self._latent_plan
 
     MAX_KEY_SPLITS = 16
 
@@ -971,6 +1080,7 @@ class HybridRunner(ModelRunner):
         # rows go to the matrix cores in tiles of up to 16 rows of one chunk
         self._step_tiles = ops.query_tiles(cu_seqlens)
         self._step_cu, self._pair_tiles, self._row_tiles = np.asarray(cu_seqlens, dtype=np.int64), {}, {}
+        self._step_ctx, self._step_tables, self._latent_plan = context_lens, block_tables, None
         self._step_long = int(max_q_len) > 1
         if logit_rows is None:
             return super().run_prefill(token_ids, positions, slot_mapping, block_tables, cu_seqlens, context_lens,
@@ -998,7 +1108,7 @@ class HybridRunner(ModelRunner):
         return self._forward(StepBatch(token_ids, positions, slot_mapping, block_tables.contiguous(), cu_seqlens,
                                        tok_seq, slots, tiles, self._step_long, pair_tiles=self._chunk_pair_tiles,
                                        context_lens=None if context_lens is None else context_lens.to(torch.int32).contiguous(),
-                                       max_q_len=max_q_len, row_tiles=self._chunk_row_tiles))
+                                       max_q_len=max_q_len, row_tiles=self._chunk_row_tiles, latent_plan=self._chunk_latent_plan))
 
     def prefill(self, token_ids: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Tensor,
                 block_tables: torch.Tensor, cu_seqlens: torch.Tensor, context_lens: torch.Tensor,

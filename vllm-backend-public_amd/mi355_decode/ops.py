@@ -289,9 +289,9 @@ def paged_attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Te
 
 
 def chunk_attn_prefill_ok(dtype: torch.dtype, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int) -> bool:
-    """Whether paged_attn_prefill_ext covers these sizes (16-bit storage, key and value sizes of 64 or 128,
+    """Whether paged_attn_prefill_ext covers these sizes (16-bit storage, key and value sizes of 64 or 128 (keys of 192 too),
     at most 16 query heads to a kv head)."""
-    return dtype in (torch.bfloat16, torch.float16) and v_dim in (64, 128) and head_dim in (64, 128) \
+    return dtype in (torch.bfloat16, torch.float16) and v_dim in (64, 128) and head_dim in (64, 128, 192) \
         and num_heads % num_kv_heads == 0 and num_heads // num_kv_heads <= 16
 
 
@@ -1426,20 +1426,31 @@ def latent_tiles_ok(dtype: torch.dtype, rank: int, rot: int) -> bool:
         and rank + rot <= 640
 
 
-def latent_q_pack(q_latent: torch.Tensor, q: torch.Tensor, q_head_width: int, q_rot_offset: int, rot: int,
-                  cos_sin: torch.Tensor, positions: torch.Tensor, interleaved: bool = False):
+def latent_q_pack(q_latent: torch.Tensor | None, q: torch.Tensor, q_head_width: int, q_rot_offset: int, rot: int,
+                  cos_sin: torch.Tensor, positions: torch.Tensor, interleaved: bool = False, out: torch.Tensor | None = None):
     """[tokens, heads, rank + rot] = q_latent [heads, tokens, rank] | the rotated `rot` columns of q at
-    q_rot_offset of every head: the query as latent_window_attn_tiles reads it."""
+    q_rot_offset of every head: the query as latent_window_attn_tiles reads it.  q_latent None: `out` [tokens, heads,
+    rank + rot] holds the first part already, the rotated part joins it."""
     dt = _dt3(q, "q")
-    H, T, rank = q_latent.shape
-    if q_latent.stride(2) != 1 or q.shape[0] != T:
-        raise ValueError("q_latent must be [heads, tokens, rank] with a contiguous last dim")
-    out = torch.empty(T, H, rank + rot, dtype=q.dtype, device=q.device)
-    check(lib.mi355_latent_q_pack(out.data_ptr(), _same(q_latent, q, "q_latent"), max(q_latent.stride(1), rank),
-                                  max(q_latent.stride(0), rank), q.data_ptr(), _cols(q, "q", H * q_head_width), q_head_width,
+    if q_latent is None:
+        T, H, rank = out.shape[0], out.shape[1], out.shape[2] - rot
+    else:
+        H, T, rank = q_latent.shape
+        if q_latent.stride(2) != 1:
+            raise ValueError("q_latent must be [heads, tokens, rank] with a contiguous last dim")
+    if q.shape[0] != T:
+        raise ValueError("q has another number of rows")
+    if out is None:
+        out = torch.empty(T, H, rank + rot, dtype=q.dtype, device=q.device)
+    if tuple(out.shape) != (T, H, rank + rot) or not out.is_contiguous():
+        raise ValueError("out must be contiguous [tokens, heads, rank + rot]")
+    check(lib.mi355_latent_q_pack(_same(out, q, "out"), None if q_latent is None else _same(q_latent, q, "q_latent"),
+                                  0 if q_latent is None else max(q_latent.stride(1), rank),
+                                  0 if q_latent is None else max(q_latent.stride(0), rank), q.data_ptr(),
+                                  _cols(q, "q", H * q_head_width), q_head_width,
                                   q_rot_offset, _f32(cos_sin, "cos_sin") or q.data_ptr(), max(cos_sin.shape[0], 1),
-                                  _idx(positions, "positions", torch.int64, T), T, H, rank, rot, cos_sin.shape[1], int(bool(interleaved)), dt,
-                                  _stream()))
+                                  _idx(positions, "positions", torch.int64, T), T, H, rank, rot, cos_sin.shape[1],
+                                  int(bool(interleaved)), dt, _stream()))
     return out
 
 
@@ -1528,16 +1539,18 @@ def moe_route(logits: torch.Tensor, correction: torch.Tensor, top: int, groups: 
     return ids, wts
 
 
-def moe_sort(ids: torch.Tensor, experts: int):
-    """Routed rows by expert: (offsets int32 [experts + 1], perm [rows], inv [rows])."""
+def moe_sort(ids: torch.Tensor, experts: int, tiles: bool = False):
+    """Routed rows by expert: (offsets int32 [experts + 1], perm [rows], inv [rows]) and with `tiles` also
+    tile_start [experts + 1], the first tile of MOE_TILE_ROWS rows of every expert."""
     rows = ids.numel()
     dev = ids.device
     offsets = torch.empty(experts + 1, dtype=torch.int32, device=dev)
     perm = torch.empty(max(rows, 1), dtype=torch.int32, device=dev)
     inv = torch.empty(max(rows, 1), dtype=torch.int32, device=dev)
+    start = torch.empty(experts + 1, dtype=torch.int32, device=dev) if tiles else None
     check(lib.mi355_moe_sort(offsets.data_ptr(), perm.data_ptr(), inv.data_ptr(), _idx(ids, "ids", torch.int32), rows,
-                             int(experts), _stream()))
-    return offsets, perm, inv
+                             int(experts), None if start is None else start.data_ptr(), MOE_TILE_ROWS, _stream()))
+    return (offsets, perm, inv, start) if tiles else (offsets, perm, inv)
 
 
 def moe_gather_rows(x: torch.Tensor, perm: torch.Tensor, rows: int, top: int, offsets: torch.Tensor | None = None,
@@ -1607,6 +1620,59 @@ def moe_linear_rows(x: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, row
 
 
 MOE_TILE_ROWS = 128
+
+
+def expert_gemm_ok(dtype: torch.dtype, in_width: int, out_width: int) -> bool:
+    return dtype in (torch.bfloat16, torch.float16) and in_width % 8 == 0 and out_width % 8 == 0
+
+
+def expert_gemm(x: torch.Tensor, w: torch.Tensor, offsets: torch.Tensor, tile_start: torch.Tensor, rows: int,
+                perm: torch.Tensor | None = None, top: int = 1, relu2: bool = False):
+    """moe_linear_rows for many rows: matrix-core tiles of 128 positions of one expert (tile_start: the first tile
+    of every expert)."""
+    dt = _dt16(x, "x")
+    E, N, K = w.shape
+    if not x.is_contiguous() or x.shape[1] != K or not w.is_contiguous() or (perm is None and x.shape[0] < rows):
+        raise ValueError("x must be contiguous [rows or tokens, in], w contiguous [experts, out, in]")
+    y = torch.empty(rows, N, dtype=x.dtype, device=x.device)
+    check(lib.mi355_expert_gemm(y.data_ptr(), x.data_ptr(), x.shape[0], _same(w, x, "w"), _idx(offsets, "offsets", torch.int32, E + 1),
+                                _idx(tile_start, "tile_start", torch.int32, E + 1),
+                                None if perm is None else _idx(perm, "perm", torch.int32, rows), int(top), rows, E, N, K,
+                                int(bool(relu2)), dt, _stream()))
+    return y
+
+
+def head_gemm(x: torch.Tensor, x_group: int, w: torch.Tensor, out: torch.Tensor, y_block: int, y_stride: int, y_group: int,
+              rows: int, index: torch.Tensor | None = None, copy: int = 0, transposed: bool = False):
+    """Head h of every row: W_h times in_width columns of x (2-D, row stride x.stride(0)) at h * x_group; w [heads, out, in].
+    The outputs of row m go to out's storage at (m / 16) * y_block + (m % 16) * y_stride + h * y_group + n
+    (transposed: (m / 16) * y_block + h * y_group + n * 16 + m % 16).  index (int32): the row of x that row m reads.
+    copy: so many columns behind the in_width ones of x follow the outputs."""
+    dt = _dt16(x, "x")
+    Hn, N, K = w.shape
+    if x.dim() != 2 or x.stride(1) != 1 or not w.is_contiguous() or x.shape[1] < (Hn - 1) * x_group + K + copy:
+        raise ValueError("x must be rows that hold every head's inputs, w contiguous [heads, out, in]")
+    # the furthest output: of the last row, or of the last full block's last row
+    step, tail = (1, (N - 1) * 16) if transposed else (y_stride, N - 1 + copy)
+    last = max(m // 16 * y_block + m % 16 * step for m in (rows - 1, max(rows // 16 * 16 - 1, 0))) + (Hn - 1) * y_group + tail
+    if rows > 0 and (out.dtype != x.dtype or last >= out.numel() or not out.is_contiguous()):
+        raise ValueError("out is smaller than the outputs")
+    check(lib.mi355_head_gemm(_same(out, x, "out"), int(y_block), int(y_stride), int(y_group), x.data_ptr(), x.stride(0), int(x_group),
+                              x.shape[0], None if index is None else _idx(index, "index", torch.int32, rows), _same(w, x, "w"),
+                              int(rows), Hn, N, K, int(copy), int(bool(transposed)), dt, _stream()))
+    return out
+
+
+def latent_q_rotate(q: torch.Tensor, num_heads: int, q_head_width: int, q_rot_offset: int, cos_sin: torch.Tensor,
+                    positions: torch.Tensor, interleaved: bool = False):
+    """q [tokens, heads * q_head_width] (a column slice is fine): the columns at q_rot_offset of every head rotated in
+    place by the table cos_sin [max_pos, rot_dims]."""
+    dt = _dt3(q, "q")
+    T = q.shape[0]
+    check(lib.mi355_latent_q_rotate(q.data_ptr(), _cols(q, "q", num_heads * q_head_width), q_head_width, q_rot_offset,
+                                    _f32(cos_sin, "cos_sin") or q.data_ptr(), max(cos_sin.shape[0], 1),
+                                    _idx(positions, "positions", torch.int64, T), T, num_heads, cos_sin.shape[1],
+                                    int(bool(interleaved)), dt, _stream()))
 
 
 class TableRoutes:

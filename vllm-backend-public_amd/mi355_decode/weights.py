@@ -168,7 +168,9 @@ class MixerLayerWeights:
     sink: Optional[torch.Tensor] = None     # f32 [heads]
     dkv_norm: Optional[torch.Tensor] = None     # f32 [kv_rank]
     uk_w: Optional[torch.Tensor] = None     # [heads, dim, kv_rank]
-    uv_t: Optional[torch.Tensor] = None     # [heads, kv_rank, vdim]
+    uv_t: Optional[torch.Tensor] = None     # [heads, kv_rank, vdim]: where the products per head are the library's
+    uk_t: Optional[torch.Tensor] = None     # [heads, kv_rank, dim] and [heads, vdim, kv_rank]: where they are
+    uv_w: Optional[torch.Tensor] = None     # ops.head_gemm's
     r1: Optional[torch.Tensor] = None       # f32 [heads]
     r2: Optional[torch.Tensor] = None       # f32 [heads]
     z_b: Optional[torch.Tensor] = None      # f32 [width of the recurrence]
@@ -685,7 +687,11 @@ def _bapavik_from_getter(cfg: ModelConfig, get, dtype, device) -> ModelWeights:
                                         ("dkv", expect(m + "dkv", (A.kv_rank + A.rot_dim, W)))], W, put)
             uk = expect(m + "uk", (A.heads * A.dim, A.kv_rank)).view(A.heads, A.dim, A.kv_rank)
             uv = expect(m + "uv", (A.heads * A.vdim, A.kv_rank)).view(A.heads, A.vdim, A.kv_rank)
-            kw.update(dkv_norm=f32(expect(m + "dkv.norm", (A.kv_rank,))), uk_w=put(uk), uv_t=put(uv.transpose(1, 2)))
+            kw.update(dkv_norm=f32(expect(m + "dkv.norm", (A.kv_rank,))), uk_w=put(uk))
+            if dtype != torch.float32 and not any(n % 8 for n in (A.dim, A.rot_dim, A.vdim, A.kv_rank)):
+                kw.update(uk_t=put(uk.transpose(1, 2)), uv_w=put(uv))
+            else:
+                kw.update(uv_t=put(uv.transpose(1, 2)))
         lw = MixerLayerWeights(norm1=put(expect(p + "norm1", (W,))), in_w=in_w, seg=seg,
                                o_w=put(expect(m + "o", (W, A.heads * A.vdim))), **kw)
         if L.ff:
