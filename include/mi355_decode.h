@@ -216,6 +216,18 @@ int32_t mi355_paged_attn_decode(void* out, const void* q, int64_t q_stride,
                                 int64_t workspace_bytes, int32_t dtype,
                                 void* stream);
 
+/* mi355_paged_attn_decode with a soft cap on the scores (softcap > 0: softcap * tanh(q.k * scale / softcap)) and one
+ * more term exp(sink[h]) in the softmax denominator without a value (fp32 [num_heads]; may be null). */
+int32_t mi355_paged_attn_decode_ext(void* out, const void* q, int64_t q_stride,
+                                    const void* k_cache, const void* v_cache,
+                                    int32_t num_blocks, const int32_t* block_tables,
+                                    int32_t max_blocks_per_seq,
+                                    const int32_t* context_lens, int32_t num_seqs,
+                                    int32_t num_heads, int32_t num_kv_heads,
+                                    int32_t head_dim, float scale, const float* sink, float softcap,
+                                    int32_t num_splits, void* workspace, int64_t workspace_bytes,
+                                    int32_t dtype, void* stream);
+
 /*
  * mi355_paged_attn_decode for callers that cannot allocate device memory (code
  * under HIP graph capture, tight serving loops, harnesses that forbid hipMalloc):
@@ -299,7 +311,7 @@ int32_t mi355_paged_attn_prefill(void* out, int64_t out_stride, const void* q,
  * without a value; gate (dtype, rows gate_stride apart, may be null): the output of (token, head) is
  * multiplied by sigmoid(gate[token, head]).  window > 0: the keys j > p - window only, and (chunk 0)
  * the first `keep` keys of the sequence.  The output is multiplied by out_scale.  softcap > 0: scores are
- * softcap * tanh(q.k * scale / softcap).  K pages
+ * softcap * tanh(q.k * scale / softcap).  chunk, window and keep go with neither a soft cap nor keys of 192.  K pages
  * [blocks, kv_heads, 16, head_dim], V pages [blocks, kv_heads, v_dim, 16], head_dim 64, 128
  * or 192, v_dim 64 or 128.
  */

@@ -293,7 +293,10 @@ def _attend_in_cuts(q, k, v, wq, wk, cuts, scale, cap=0.0, sink=None, temp=(0.0,
         qs, ks, vs = buf[:, : H * d], buf[:, H * d: (H + G) * d], buf[:, (H + G) * d: width]
         ops.row_norm_rope_kv_write(qs, ks, vs, wq.cuda(), wk.cuda(), none, pos, slots[at:at + n], kc, vc, H, G, d, dv, 1e-5,
                                    temp_coef=temp[0], temp_every=temp[1])
-        if form == "staged":
+        if form == "staged" and n == 1 and ops.attn_decode_ok(dt, H, G, d, dv):
+            o = ops.paged_attn_decode(qs, kc, vc, bt, torch.tensor([at + 1], dtype=torch.int32, device="cuda"), H, G, d, scale,
+                                      num_splits=max(splits, 1), sink=sk, softcap=cap)
+        elif form == "staged":
             assert ops.chunk_attn_prefill_ok(dt, H, G, d, dv)
             o = ops.paged_attn_prefill_ext(qs, kc, vc, bt, torch.tensor([0, n], dtype=torch.int32, device="cuda"),
                                            torch.tensor([at + n], dtype=torch.int32, device="cuda"), n, H, G, d, scale, sink=sk, softcap=cap)
@@ -373,8 +376,8 @@ def test_capped_attention_staged_through_lds(H, G, d, dv, cap):
     q, k, v = b16(q), b16(k), b16(v)
     kw = dict(cap=cap, sink=sink, temp=(0.4, 20))
     ref = _attend_ref(q, k, v, wq, wk, 0.3, **kw)
-    for cuts in ([2, 3, 1, 30, 2, 16, 36], [90]):
-        _near(_attend_in_cuts(q, k, v, wq, wk, cuts, 0.3, form="staged", **kw), ref, 4e-2)
+    for cuts, splits in (([2, 3, 1, 30, 2, 16, 36], 0), ([90], 0), ([1] * 90, 0), ([50] + [1] * 40, 3)):      # (single tokens: the decode launch)
+        _near(_attend_in_cuts(q, k, v, wq, wk, cuts, 0.3, form="staged", splits=splits, **kw), ref, 4e-2)
     _near(_attend_in_cuts(q, k, v, wq, wk, [90], 0.3, form="staged", cap=cap), _attend_ref(q, k, v, wq, wk, 0.3, cap=cap), 4e-2)
 
 

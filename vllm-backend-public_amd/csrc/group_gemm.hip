@@ -11,7 +11,7 @@
 // copy > 0: columns k .. k + copy of the x row follow the n outputs of every group (a part shared by all heads).
 //
 // One workgroup (4 waves) per BM x BN tile of (rows, outputs).  64-wide K steps of X and W go through registers
-// into LDS, double buffered, one barrier per step.  An LDS row is 128 bytes, eight 16-byte slots; slot s of row r
+// into LDS: two steps on their way in registers, two images in LDS, one barrier per step.  An LDS row is 128 bytes, eight 16-byte slots; slot s of row r
 // sits at s ^ ((r / 2) & 7): the 16 rows of a fragment read then cover 256 bytes without a bank twice.
 #include "common.h"
 
@@ -37,7 +37,7 @@ struct GroupGemmArgs {
 
 // MW: waves along the rows (the other 4 / MW lie along the outputs)
 template <typename T, int BM, int BN, int MW, bool TRANS>
-__global__ __launch_bounds__(256) void group_gemm_kernel(GroupGemmArgs a) {
+__global__ __launch_bounds__(256, 2) void group_gemm_kernel(GroupGemmArgs a) {
   constexpr int NW = 4 / MW, TM = BM / MW / 16, TN = BN / NW / 16;      // a wave's 16 x 16 blocks
   constexpr int XP = BM * 8 / 256, WP = BN * 8 / 256;                   // 16-byte pieces per thread and step
   static_assert(BM * 8 % 256 == 0 && BN * 8 % 256 == 0, "whole pieces per thread");
@@ -96,19 +96,33 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(GroupGemmArgs a) {
     dw[j] = BM * kBK + r * kBK + ((s8 ^ ((r >> 1) & 7)) << 3);
   }
   typedef unsigned int pvec __attribute__((ext_vector_type(4)));
-  pvec rx[XP], rw[WP];
-  auto load = [&](int k0) {
+  pvec rx[2][XP], rw[2][WP];
+  auto load = [&](int set, int k0) {
+    if (k0 + kBK <= a.k) {                                // (uniform)
+#pragma unroll
+      for (int j = 0; j < XP; ++j) rx[set][j] = MI355_LD(pvec, a.x, xp[j] + k0);
+#pragma unroll
+      for (int j = 0; j < WP; ++j) rw[set][j] = MI355_LD(pvec, a.w, wp[j] + k0);
+      return;
+    }
     const bool have = k0 + 8 * s8 < a.k;                 // (k a multiple of 8)
+    const int at = have ? k0 : 0;
 #pragma unroll
-    for (int j = 0; j < XP; ++j) rx[j] = have ? MI355_LD(pvec, a.x, xp[j] + k0) : pvec{0, 0, 0, 0};
+    for (int j = 0; j < XP; ++j) {
+      const pvec v = MI355_LD(pvec, a.x, xp[j] - 8 * s8 + (have ? at + 8 * s8 : 0));
+      rx[set][j] = have ? v : pvec{0, 0, 0, 0};
+    }
 #pragma unroll
-    for (int j = 0; j < WP; ++j) rw[j] = have ? MI355_LD(pvec, a.w, wp[j] + k0) : pvec{0, 0, 0, 0};
+    for (int j = 0; j < WP; ++j) {
+      const pvec v = MI355_LD(pvec, a.w, wp[j] - 8 * s8 + (have ? at + 8 * s8 : 0));
+      rw[set][j] = have ? v : pvec{0, 0, 0, 0};
+    }
   };
-  auto store = [&](int buf) {
+  auto store = [&](int set) {                            // (image = set)
 #pragma unroll
-    for (int j = 0; j < XP; ++j) *reinterpret_cast<pvec*>(&lds[buf][dx[j]]) = rx[j];
+    for (int j = 0; j < XP; ++j) *reinterpret_cast<pvec*>(&lds[set][dx[j]]) = rx[set][j];
 #pragma unroll
-    for (int j = 0; j < WP; ++j) *reinterpret_cast<pvec*>(&lds[buf][dw[j]]) = rw[j];
+    for (int j = 0; j < WP; ++j) *reinterpret_cast<pvec*>(&lds[set][dw[j]]) = rw[set][j];
   };
   const int wm = (wave % MW) * (BM / MW), wn = (wave / MW) * (BN / NW);
   f32x4 acc[TM][TN];
@@ -117,32 +131,37 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(GroupGemmArgs a) {
 #pragma unroll
     for (int j = 0; j < TN; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   const int sw = (li >> 1) & 7;                          // (16-row blocks: the swizzle depends on the row in the block alone)
-  load(0);
+  const int steps = (a.k + kBK - 1) / kBK;
+  load(0, 0);
+  if (steps > 1) load(1, kBK);
   store(0);
   __syncthreads();
-  for (int k0 = 0; k0 < a.k; k0 += kBK) {
-    const int buf = (k0 / kBK) & 1;
-    const bool more = k0 + kBK < a.k;
-    if (more) load(k0 + kBK);
+  // step t computes image t % 2, sends for step t + 2 and stores step t + 1 into the other image
+  auto step = [&](int t, int set) {
+    if (t + 2 < steps) load(set, (t + 2) * kBK);
     __builtin_amdgcn_s_setprio(1);
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
       const int slot = ((4 * ks + kk) ^ sw) << 3;
       uint4 xf[TM], wf[TN];
 #pragma unroll
-      for (int i = 0; i < TM; ++i) xf[i] = *reinterpret_cast<const uint4*>(&lds[buf][(wm + 16 * i + li) * kBK + slot]);
+      for (int i = 0; i < TM; ++i) xf[i] = *reinterpret_cast<const uint4*>(&lds[set][(wm + 16 * i + li) * kBK + slot]);
 #pragma unroll
-      for (int j = 0; j < TN; ++j) wf[j] = *reinterpret_cast<const uint4*>(&lds[buf][BM * kBK + (wn + 16 * j + li) * kBK + slot]);
+      for (int j = 0; j < TN; ++j) wf[j] = *reinterpret_cast<const uint4*>(&lds[set][BM * kBK + (wn + 16 * j + li) * kBK + slot]);
 #pragma unroll
       for (int i = 0; i < TM; ++i)
 #pragma unroll
         for (int j = 0; j < TN; ++j) acc[i][j] = TRANS ? T::mfma(xf[i], wf[j], acc[i][j]) : T::mfma(wf[j], xf[i], acc[i][j]);
     }
     __builtin_amdgcn_s_setprio(0);
-    if (more) {
-      store(buf ^ 1);
+    if (t + 1 < steps) {
+      store(set ^ 1);
       __syncthreads();
     }
+  };
+  for (int t = 0; t < steps; t += 2) {
+    step(t, 0);
+    if (t + 1 < steps) step(t + 1, 1);
   }
 #pragma unroll
   for (int i = 0; i < TM; ++i) {

@@ -37,6 +37,9 @@
 // from registers, whatever the pages held, so nothing waits for that store.  The
 // projection comes either as packed 16-bit rows (FUSE == 1) or as the fp32
 // partial-sum slabs of a K-split GEMM (FUSE == 2: slab sum + bias, rounded, first).
+//
+// EXT (with FUSE == 0): a soft cap on the scores, cap * tanh(q.k scale / cap), and one more term exp(sink[head])
+// in the softmax denominator that carries no value.
 #include "common.h"
 
 #include <math.h>
@@ -82,6 +85,11 @@ struct RopeArgs {             // FUSE != 0
   const uint16_t* cos_sin;    // [max_position][D]: cos | sin halves
   int max_position;
   const int64_t* slots;       // [num_seqs]; < 0 or beyond the pool: not stored
+};
+
+struct ScoreArgs {            // EXT
+  const float* sink;          // [num_heads] or null
+  float cap_x;                // 2 log2(e) scale / cap, 0: no cap (scale_log2e is cap log2(e) otherwise)
 };
 
 // 8 consecutive elements of the projection row of `seq` starting at column `col`: the loads
@@ -157,13 +165,13 @@ __device__ __forceinline__ void rotate8(const float (&x1)[8], const float (&x2)[
   }
 }
 
-template <typename T, int D, int FUSE, int SLABS, bool SPLIT, int kStages, int NW>
+template <typename T, int D, int FUSE, int SLABS, bool SPLIT, int kStages, int NW, bool EXT>
 __global__ __launch_bounds__(64 * NW) void paged_attn_decode_kernel(
     uint16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml,
     const uint16_t* __restrict__ q, int64_t q_stride, uint16_t* k_cache,
     uint16_t* v_cache, int num_blocks, const int32_t* __restrict__ block_tables,
     int max_blocks, const int32_t* __restrict__ context_lens, int num_heads, int num_kv_heads,
-    float scale_log2e, int num_splits, RopeArgs ra) {
+    float scale_log2e, int num_splits, RopeArgs ra, ScoreArgs sx) {
   constexpr int KS = D / 32;  // MFMA k-steps over head_dim for QK^T
   constexpr int NT = D / 16;  // 16-row tiles of head_dim for PV
   constexpr int BS = MI355_BLOCK_SIZE;
@@ -398,6 +406,13 @@ __global__ __launch_bounds__(64 * NW) void paged_attn_decode_kernel(
       sa = T::mfma(kvr.ka[ks], qf[ks], sa);
       sb = T::mfma(kvr.kb[ks], qf[ks], sb);
     }
+    if (EXT && sx.cap_x > 0.f) {                       // the scores become tanh(.) = 1 - 2 / (1 + 2^(cap_x q.k))
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        sa[j] = 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sa[j] * sx.cap_x));
+        sb[j] = 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(sb[j] * sx.cap_x));
+      }
+    }
     // lane (head c, h) now holds tokens tb + 8h + j, j = 0..7 (sa: j<4, sb: j>=4)
     float s[8];
     const int tok0 = tb + 8 * h;
@@ -517,6 +532,8 @@ __global__ __launch_bounds__(64 * NW) void paged_attn_decode_kernel(
       }
     }
     const int head = kvh * group + hh;
+    if (EXT && num_splits == 1 && sx.sink != nullptr && mg != -INFINITY)
+      lsum += exp2f(MI355_LD(float, sx.sink, sx.sink + head) * 1.4426950408889634f - mg);
     if (num_splits == 1) {
       const float v0 = lsum > 0.f ? acc0 / lsum : 0.f, v1 = lsum > 0.f ? acc1 / lsum : 0.f;
       MI355_ST(uint32_t, out, out + (static_cast<int64_t>(seq) * num_heads + head) * D + d,
@@ -539,7 +556,8 @@ template <typename T, int D>
 __global__ __launch_bounds__(D) void paged_attn_merge_kernel(uint16_t* __restrict__ out,
                                                              const float* __restrict__ part_o,
                                                              const float* __restrict__ part_ml,
-                                                             int num_splits) {
+                                                             int num_splits, const float* __restrict__ sink,
+                                                             int num_heads) {
   const int64_t row = blockIdx.x;  // seq * num_heads + head
   const int d = threadIdx.x;
   const float* ml = part_ml + row * num_splits * 2;
@@ -553,15 +571,18 @@ __global__ __launch_bounds__(D) void paged_attn_merge_kernel(uint16_t* __restric
       lsum += f * MI355_LD(float, part_o, ml + 2 * s + 1);
     }
   }
+  if (sink != nullptr && mg != -INFINITY)              // the value-less term joins once
+    lsum += exp2f(MI355_LD(float, sink, sink + row % num_heads) * 1.4426950408889634f - mg);
   MI355_ST(uint16_t, out, out + row * D + d, T::from_f(lsum > 0.f ? acc / lsum : 0.f));
 }
 
-template <typename T, int D, int FUSE, int SLABS = 0>
+template <typename T, int D, int FUSE, int SLABS = 0, bool EXT = false>
 static int32_t launch_decode(void* out, const void* q, int64_t q_stride, void* k_cache,
                              void* v_cache, int32_t num_blocks, const int32_t* block_tables,
                              int32_t max_blocks, const int32_t* context_lens, int32_t num_seqs,
                              int32_t num_heads, int32_t num_kv_heads, float scale, int32_t num_splits,
-                             void* workspace, hipStream_t s, const RopeArgs& ra) {
+                             void* workspace, hipStream_t s, const RopeArgs& ra, const ScoreArgs& sx = ScoreArgs{},
+                             float score_scale = 0.f) {
   float* part_o = nullptr;
   float* part_ml = nullptr;
   if (num_splits > 1) {
@@ -584,10 +605,11 @@ static int32_t launch_decode(void* out, const void* q, int64_t q_stride, void* k
   if (forced == 41 || forced == 42 || (forced == 11 && one_wave_fits)) form = forced;
   dim3 grid(num_seqs, num_kv_heads, num_splits), block(form / 10 == 1 ? 64 : kDecodeThreads);
 #define MI355_PAD_LAUNCH(SPLIT_, STG_, NW_)                                                                        \
-  hipLaunchKernelGGL((paged_attn_decode_kernel<T, D, FUSE, SLABS, SPLIT_, STG_, NW_>), grid, block, 0, s,          \
+  hipLaunchKernelGGL((paged_attn_decode_kernel<T, D, FUSE, SLABS, SPLIT_, STG_, NW_, EXT>), grid, block, 0, s,          \
                      static_cast<uint16_t*>(out), part_o, part_ml, static_cast<const uint16_t*>(q), q_stride,      \
                      static_cast<uint16_t*>(k_cache), static_cast<uint16_t*>(v_cache), num_blocks, block_tables,   \
-                     max_blocks, context_lens, num_heads, num_kv_heads, scale * 1.4426950408889634f, num_splits, ra)
+                     max_blocks, context_lens, num_heads, num_kv_heads,                                            \
+                     (EXT ? score_scale : scale) * 1.4426950408889634f, num_splits, ra, sx)
 #define MI355_PAD_FORMS(SPLIT_)                                     \
   switch (form) {                                                   \
     case 41: MI355_PAD_LAUNCH(SPLIT_, 1, 4); break;                 \
@@ -604,7 +626,7 @@ static int32_t launch_decode(void* out, const void* q, int64_t q_stride, void* k
   int32_t rc = check_launch("mi355_paged_attn_decode");
   if (rc != MI355_OK || num_splits == 1) return rc;
   hipLaunchKernelGGL((paged_attn_merge_kernel<T, D>), dim3(num_seqs * num_heads), dim3(D), 0, s,
-                     static_cast<uint16_t*>(out), part_o, part_ml, num_splits);
+                     static_cast<uint16_t*>(out), part_o, part_ml, num_splits, EXT ? sx.sink : nullptr, num_heads);
   return check_launch("mi355_paged_attn_decode(merge)");
 }
 
@@ -629,7 +651,8 @@ static int32_t decode_entry(const char* name, void* out, const void* q, int64_t 
                             int32_t max_blocks_per_seq, const int32_t* context_lens, int32_t num_seqs,
                             int32_t num_heads, int32_t num_kv_heads, int32_t head_dim, float scale,
                             int32_t num_splits, void* workspace, int64_t workspace_bytes, int32_t dtype,
-                            void* stream, int fuse, const RopeArgs& ra) {
+                            void* stream, int fuse, const RopeArgs& ra, bool ext = false, const float* sink = nullptr,
+                            float softcap = 0.f) {
   MI355_REQUIRE(out && k_cache && v_cache && block_tables && context_lens && (q || fuse == 2), MI355_ERR_INVALID,
                 "%s: null pointer", name);
   MI355_REQUIRE(num_seqs >= 0 && num_blocks > 0 && max_blocks_per_seq > 0, MI355_ERR_INVALID,
@@ -675,8 +698,14 @@ static int32_t decode_entry(const char* name, void* out, const void* q, int64_t 
   return launch_decode<TT, DD, FF, SS>(out, q, q_stride, k_cache, v_cache, num_blocks, block_tables,      \
                                        max_blocks_per_seq, context_lens, num_seqs, num_heads, num_kv_heads, \
                                        scale, num_splits, workspace, s, ra)
+#define MI355_DEC_E(TT, DD)                                                                                  \
+  return launch_decode<TT, DD, 0, 0, true>(out, q, q_stride, k_cache, v_cache, num_blocks, block_tables,      \
+                                           max_blocks_per_seq, context_lens, num_seqs, num_heads, num_kv_heads, \
+                                           scale, num_splits, workspace, s, ra, sx, softcap > 0.f ? softcap : scale)
+  const ScoreArgs sx{sink, softcap > 0.f ? 2.0f * 1.4426950408889634f * scale / softcap : 0.f};
 #define MI355_DEC_F(TT, DD)                                 \
   do {                                                      \
+    if (ext) MI355_DEC_E(TT, DD);                           \
     if (fuse == 0) MI355_DEC(TT, DD, 0, 0);                 \
     if (fuse == 1) MI355_DEC(TT, DD, 1, 0);                 \
     if (ra.num_slabs == 1) MI355_DEC(TT, DD, 2, 1);         \
@@ -691,6 +720,7 @@ static int32_t decode_entry(const char* name, void* out, const void* q, int64_t 
   if (head_dim == 64) MI355_DEC_F(F16, 64);
   MI355_DEC_F(F16, 128);
 #undef MI355_DEC_F
+#undef MI355_DEC_E
 #undef MI355_DEC
 }
 
@@ -708,6 +738,19 @@ extern "C" int32_t mi355_paged_attn_decode(void* out, const void* q, int64_t q_s
                              const_cast<void*>(v_cache), num_blocks, block_tables, max_blocks_per_seq, context_lens,
                              num_seqs, num_heads, num_kv_heads, head_dim, scale, num_splits, workspace,
                              workspace_bytes, dtype, stream, 0, mi355::RopeArgs{});
+}
+
+extern "C" int32_t mi355_paged_attn_decode_ext(void* out, const void* q, int64_t q_stride, const void* k_cache,
+                                               const void* v_cache, int32_t num_blocks, const int32_t* block_tables,
+                                               int32_t max_blocks_per_seq, const int32_t* context_lens, int32_t num_seqs,
+                                               int32_t num_heads, int32_t num_kv_heads, int32_t head_dim, float scale,
+                                               const float* sink, float softcap, int32_t num_splits, void* workspace,
+                                               int64_t workspace_bytes, int32_t dtype, void* stream) {
+  MI355_REQUIRE(softcap >= 0.f && (softcap == 0.f || scale > 0.f), MI355_ERR_INVALID, "mi355_paged_attn_decode_ext: soft cap %g", softcap);
+  return mi355::decode_entry("mi355_paged_attn_decode_ext", out, q, q_stride, const_cast<void*>(k_cache),
+                             const_cast<void*>(v_cache), num_blocks, block_tables, max_blocks_per_seq, context_lens,
+                             num_seqs, num_heads, num_kv_heads, head_dim, scale, num_splits, workspace,
+                             workspace_bytes, dtype, stream, 0, mi355::RopeArgs{}, true, sink, softcap);
 }
 
 // ---- the entry point that allocates nothing.  The split-KV partials (fp32 accumulators and

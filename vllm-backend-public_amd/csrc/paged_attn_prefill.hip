@@ -29,14 +29,16 @@
 // and the lane's own probabilities as B.  The causal mask is applied per column (key <=
 // position of the column's query).
 //
-// EXT (a second set of instantiations; the plain ones compile as before): attention inside chunks of
+// MODE 1 (a second set of instantiations; the plain ones, MODE 0, compile as before): attention inside chunks of
 // positions -- a column at position p sees the keys from (p / chunk) * chunk on, the walk starts at the
 // chunk of the tile's first query and columns of a tile that straddles a chunk edge mask for themselves;
 // or a sliding window (keys after p - window) beside the first `keep` keys of the sequence: the walk takes
 // the barrier intervals that hold kept keys and lie before the window's first interval, then the window's;
-// value sizes that differ from the key size (64 / 128; keys of 64, 128 or 192); one more term exp(sink[head]) in the softmax denominator that carries no value; and the output times
-// the sigmoid of one gate number per (token, head), and times a constant; a soft cap on the scores (cap_x > 0),
-// cap * tanh(q.k scale / cap).
+// value sizes that differ from the key size (64 / 128); one more term exp(sink[head]) in the softmax denominator that
+// carries no value; and the output times the sigmoid of one gate number per (token, head), and times a constant.
+// MODE 2: all earlier keys as in MODE 0, with the term, gate and constant of MODE 1, keys of 192 too, and a soft
+// cap on the scores (cap_x > 0), cap * tanh(q.k scale / cap).  Two modes because masks and cap together do not fit
+// the registers of two workgroups per CU.
 #include "common.h"
 
 #include <math.h>
@@ -57,7 +59,7 @@ __device__ __forceinline__ float max3(float a, float b, float c) {
 
 // Second launch bound: waves per SIMD the register allocation must leave room for.  Two workgroups
 // per CU overlap each other's dependent chains (LDS reads -> MFMAs -> exp2 -> MFMAs -> barrier).
-template <typename T, int D, int DV, int NQ, bool EXT>
+template <typename T, int D, int DV, int NQ, int MODE>
 __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_prefill_kernel(
     uint16_t* __restrict__ out, int64_t out_stride, const uint16_t* __restrict__ q, int64_t q_stride,
     const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache, int num_blocks,
@@ -65,6 +67,7 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
     const int32_t* __restrict__ context_lens, int num_heads, int num_kv_heads, float scale_log2e, int qt,
     int chunk, int window, int keep, const float* __restrict__ sink, const uint16_t* __restrict__ gate, int64_t gate_stride,
     float out_scale, float cap_x) {
+  constexpr bool EXT = MODE >= 1, MASK = MODE == 1, CAP = MODE == 2;
   constexpr int KS = D / 32;
   constexpr int NT = DV / 16;
   constexpr int BS = MI355_BLOCK_SIZE;
@@ -82,8 +85,9 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
   constexpr int PPT = KPT + 4 * DV / kPrefillThreads;   // and with those of its two V pages
   static_assert(4 * D % kPrefillThreads == 0 && 4 * DV % kPrefillThreads == 0, "whole pieces per thread");
   // HS 32-token images per barrier interval, two such sets (one computed on, one being staged):
-  // half as many workgroup barriers per key as with one image per interval
-  constexpr int HS = 2;
+  // half as many workgroup barriers per key as with one image per interval (one image at D = 192: registers)
+  constexpr int HS = D > 128 ? 1 : 2;
+  static_assert(!MASK || HS == 2, "the masked walk counts in intervals of 64 keys");
   __shared__ __attribute__((aligned(16))) unsigned char lds[2 * HS * BUF];
 
   // Workgroup -> (query tile, kv head, sequence).  The hardware deals consecutive workgroups to the
@@ -126,8 +130,8 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
     col_ok[t] = (p < qt * group) && (col_q[t] < q_len);
     col_pos[t] = col_ok[t] ? pos0 + col_q[t] : -1;
     col_lo[t] = 0;                               // first key the column sees (past the kept ones)
-    if (EXT && chunk > 0 && col_ok[t]) col_lo[t] = (col_pos[t] / chunk) * chunk;
-    if (EXT && window > 0 && col_ok[t]) col_lo[t] = max(col_lo[t], col_pos[t] - window + 1);
+    if (MASK && chunk > 0 && col_ok[t]) col_lo[t] = (col_pos[t] / chunk) * chunk;
+    if (MASK && window > 0 && col_ok[t]) col_lo[t] = max(col_lo[t], col_pos[t] - window + 1);
     const uint16_t* qp = q + (q_begin + (col_ok[t] ? col_q[t] : 0)) * q_stride +
                          static_cast<int64_t>(col_ok[t] ? col_head[t] : 0) * D + 8 * h;
 #pragma unroll
@@ -143,7 +147,7 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
   for (int off = 32; off > 0; off >>= 1) kmin = min(kmin, __shfl_xor(kmin, off, 64));
   const int t_min = __builtin_amdgcn_readfirstlane(kmin);
   int lomax = 0;                                                  // largest first-visible key among the wave's columns
-  if (EXT) {
+  if (MASK) {
 #pragma unroll
     for (int t = 0; t < NQ; ++t) lomax = max(lomax, col_lo[t]);
 #pragma unroll
@@ -152,11 +156,11 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
   const int t_lo_max = __builtin_amdgcn_readfirstlane(lomax);
   // the walk starts at the chunk of the tile's first query, on a boundary of the barrier interval (HS steps)
   int walk_lo = 0;                                                // first key of the walk past the kept ones
-  if (EXT && chunk > 0) walk_lo = (pos0 + q0) / chunk * chunk;
-  if (EXT && window > 0) walk_lo = max(walk_lo, pos0 + q0 - window + 1);
+  if (MASK && chunk > 0) walk_lo = (pos0 + q0) / chunk * chunk;
+  if (MASK && window > 0) walk_lo = max(walk_lo, pos0 + q0 - window + 1);
   // barrier intervals (HS steps) in walking order: interval i is at step HS * i for the nk intervals that hold kept
   // keys and lie before the walk's first, at HS * (i + skip) behind them.  Keys between are not visited.
-  const int nk = EXT ? min((keep + 63) / 64, walk_lo / 64) : 0;
+  const int nk = MASK ? min((keep + 63) / 64, walk_lo / 64) : 0;
   const int skip = HS * (walk_lo / 64 - nk);                      // in steps
   const int t_end_wg = pos0 + min(q0 + qt, q_len);              // the tile's last query sees keys [0, t_end_wg)
 
@@ -226,8 +230,8 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
     }
   };
 
-  const int steps = (t_end_wg + 31) / 32 - (EXT ? skip : 0);      // of the walk
-  auto key_step = [&](int s) { return EXT && s >= HS * nk ? s + skip : s; };      // the 32-key step of the sequence at walk step s
+  const int steps = (t_end_wg + 31) / 32 - (MASK ? skip : 0);      // of the walk
+  auto key_step = [&](int s) { return MASK && s >= HS * nk ? s + skip : s; };      // the 32-key step of the sequence at walk step s
   const int tok_h = 8 * h;
 
   // S^T = K . Q^T of one step for all column tiles (a K fragment is read from LDS once and used NQ
@@ -251,7 +255,7 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
     __builtin_amdgcn_s_setprio(0);
     // soft cap: the scores become tanh(q.k scale / cap) = 1 - 2 / (1 + 2^(cap_x q.k)), cap_x = 2 log2(e) scale / cap;
     // scale_log2e is then cap log2(e)
-    if (EXT && cap_x > 0.f) {
+    if (CAP && cap_x > 0.f) {
 #pragma unroll
       for (int t = 0; t < NQ; ++t) {
 #pragma unroll
@@ -272,7 +276,7 @@ __global__ __launch_bounds__(kPrefillThreads, NQ <= 2 ? 2 : 1) void paged_attn_p
         }
       }
     }
-    if (EXT && s * 32 < t_lo_max) {        // wave-uniform: ahead of the chunk of some column
+    if (MASK && s * 32 < t_lo_max) {        // wave-uniform: ahead of the chunk of some column
 #pragma unroll
       for (int t = 0; t < NQ; ++t) {
 #pragma unroll
@@ -440,6 +444,9 @@ static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chu
                 "%s: at most 16 query heads per kv head (got %d)", name, group);
   MI355_REQUIRE((head_dim == 64 || head_dim == 128 || (ext && head_dim == 192)) && (v_dim == head_dim || (ext && (v_dim == 64 || v_dim == 128))),
                 MI355_ERR_UNSUPPORTED, "%s: head_dim %d / v_dim %d not supported (64 or 128)", name, head_dim, v_dim);
+  const bool masked = chunk > 0 || window > 0 || keep > 0;
+  MI355_REQUIRE(!masked || (softcap == 0.f && head_dim <= 128), MI355_ERR_UNSUPPORTED,
+                "%s: chunks and windows with keys of up to 128 and without a soft cap only", name);
   const int64_t width = static_cast<int64_t>(num_heads) * head_dim;
   MI355_REQUIRE(q_stride >= width && q_stride % 8 == 0 && out_stride >= static_cast<int64_t>(num_heads) * v_dim && out_stride % 8 == 0,
                 MI355_ERR_INVALID, "%s: q_stride/out_stride invalid", name);
@@ -471,9 +478,11 @@ static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chu
                      softcap > 0.f ? 2.0f * 1.4426950408889634f * scale / softcap : 0.f)
 #define MI355_PRE(TT, DD, NN)                                                                           \
   do {                                                                                                  \
-    if (ext && v_dim == 64) MI355_PRE_E(TT, DD, 64, NN, true);                                          \
-    else if (ext) MI355_PRE_E(TT, DD, 128, NN, true);                                                   \
-    else MI355_PRE_E(TT, DD, DD, NN, false);                                                            \
+    if (ext && masked && v_dim == 64) MI355_PRE_E(TT, DD, 64, NN, 1);                                   \
+    else if (ext && masked) MI355_PRE_E(TT, DD, 128, NN, 1);                                            \
+    else if (ext && v_dim == 64) MI355_PRE_E(TT, DD, 64, NN, 2);                                        \
+    else if (ext) MI355_PRE_E(TT, DD, 128, NN, 2);                                                      \
+    else MI355_PRE_E(TT, DD, DD, NN, 0);                                                                \
   } while (0)
 #define MI355_PRE_NQ(TT, DD)                \
   switch (nq) {                             \
@@ -482,10 +491,10 @@ static int32_t launch_paged_attn_prefill(const char* name, bool ext, int32_t chu
   }
 #define MI355_PRE_192(TT)                                               \
   do {                                                                  \
-    if (v_dim == 64 && nq == 1) MI355_PRE_E(TT, 192, 64, 1, true);      \
-    else if (v_dim == 64) MI355_PRE_E(TT, 192, 64, 2, true);            \
-    else if (nq == 1) MI355_PRE_E(TT, 192, 128, 1, true);               \
-    else MI355_PRE_E(TT, 192, 128, 2, true);                            \
+    if (v_dim == 64 && nq == 1) MI355_PRE_E(TT, 192, 64, 1, 2);      \
+    else if (v_dim == 64) MI355_PRE_E(TT, 192, 64, 2, 2);            \
+    else if (nq == 1) MI355_PRE_E(TT, 192, 128, 1, 2);               \
+    else MI355_PRE_E(TT, 192, 128, 2, 2);                            \
   } while (0)
   if (dtype == MI355_BF16) {
     if (head_dim == 192) MI355_PRE_192(BF16);

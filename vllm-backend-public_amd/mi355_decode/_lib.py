@@ -47,6 +47,7 @@ def _load() -> ctypes.CDLL:
         "mi355_paged_attn_decode_workspace": (I64, [I32, I32, I32, I32]),
         "mi355_paged_attn_decode": (I32, [P, P, I64, P, P, I32, P, I32, P, I32, I32, I32, I32, F, I32, P,
                                           I64, I32, P]),
+        "mi355_paged_attn_decode_ext": (I32, [P, P, I64, P, P, I32, P, I32, P, I32, I32, I32, I32, F, P, F, I32, P, I64, I32, P]),
         "mi355_paged_attn_decode_static": (I32, [P, P, I64, P, P, I32, P, I32, P, I32, I32, I32, I32, F, I32, I32, P]),
         "mi355_paged_attn_prefill": (I32, [P, I64, P, I64, P, P, I32, P, I32, P, P, I32, I32, I32, I32, I32,
                                            F, I32, P]),
@@ -209,7 +210,7 @@ EXPORTS = ("mi355_abi_version", "mi355_last_error", "mi355_target_arch",
            "mi355_token_side_f32", "mi355_linear_attn_state_floats", "mi355_linear_attn_tile_rows", "mi355_mlstm_gates",
            "mi355_linear_attn_chunks", "mi355_decay_attn_step", "mi355_mlstm_step",
            "mi355_moe_linear_rows", "mi355_moe_table_sort", "mi355_add_layer_norm_f32", "mi355_expert_gemm",
-           "mi355_head_gemm", "mi355_latent_q_rotate")
+           "mi355_head_gemm", "mi355_latent_q_rotate", "mi355_paged_attn_decode_ext")
 
 
 def check(status: int) -> None:

@@ -93,6 +93,22 @@ def rigazen_config(width: int, layers: int, vocab: int = 32000) -> dict:
             "norm": {"eps": 1e-6}, "token_side": {"dim": max(width // 32, 8)}, "layers": ls}
 
 
+def bapavik_config(width: int, layers: int, vocab: int = 32000) -> dict:
+    """Alternating softmax-attention / latent-attention layers: 128-wide heads (four query heads to a key head in the
+    softmax attention; 128 + 64 over a latent of 512 in the latent one), capped scores, a query temperature; a limited
+    gated feed-forward of 2 * width in the first layer and, in the others, 32 experts of 3/4 width of which a table
+    names 4 per token: as many weights as 32 gated experts of width / 2."""
+    nh = width // 128
+    att = {"heads": nh, "kv_heads": max(nh // 4, 1), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+           "q_temp": {"coef": 0.1, "every": 1024}}
+    lat = {"heads": nh, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5, "rot": {"dims": 64, "base": 1.0e6}}
+    moe = {"kind": "moe", "expert": {"ff": 3 * width // 4}, "router": {"experts": 32, "top": 4}}
+    ls = [{"type": "attention" if i % 2 == 0 else "latent_attention", "mixer": att if i % 2 == 0 else lat,
+           "mlp": {"kind": "dense", "ff": 2 * width, "limit": 7.0} if i == 0 else moe} for i in range(layers)]
+    return {"architecture": "Bapavik", "embedding": {"scale": float(width) ** 0.5}, "width": width, "vocab": vocab,
+            "norm": {"eps": 1e-6}, "layers": ls}
+
+
 def lozupel_config(width: int, layers: int, vocab: int = 32000, loop: bool = True) -> dict:
     """Alternating parallel / delta layers with 128-wide heads, a 1024-token window, a feed-forward in
     every layer; the middle of the stack loops twice."""
@@ -900,4 +916,195 @@ def compare_rigazen(widths, layers: int, batch: int, prompt_len: int, steps: int
                                  "prefill_ratio": round(t["prefill_tok_s"] / z["prefill_tok_s"], 3),
                                  "decode_ratio": round(t["decode_tok_s"] / z["decode_tok_s"], 3)})
         result["kernels"][str(width)] = rigazen_kernel_table(width, prompt_len, batch)
+    return result
+
+
+def bapavik_kernel_table(width: int, prompt_len: int, batch: int) -> list:
+    """The Bapavik design's kernels at the prefill and the decode shape, each against its own roofline, beside the
+    like kernel of the closest existing paths at the same shape: the Tativik design's latent attention and mixture,
+    the Llama-shaped decoder's softmax attention, the other designs' norms and activations."""
+    from types import SimpleNamespace
+    from .config import LatentAttnSpec, MoESpec, NO_WINDOW
+    from .hybrid_runner import LatentAttention, LatentPlan, MoEFeedForward, StepBatch, TableMoE, rotary_table
+    dev, bf = "cuda", torch.bfloat16
+    g = torch.Generator(device=dev).manual_seed(0)
+    rnd = lambda *s, dt=bf: torch.randn(*s, device=dev, dtype=torch.float32, generator=g).to(dt)  # noqa: E731
+    rows = []
+
+    def row(kernel, shape, t, bound, work, like=None, like_t=None, like_work=None, like_bound=None):
+        peak = {"hbm": HBM, "mfma": MFMA, "valu": VALU}
+        r = {"kernel": kernel, "shape": shape, "us": round(t * 1e6, 2), "bound": bound,
+             "frac_of_roofline": round(work / peak[bound] / t, 4)}
+        if like is not None:
+            r.update(like=like, like_us=round(like_t * 1e6, 2), like_frac=round(like_work / peak[like_bound or bound] / like_t, 4))
+            r["distance_ratio"] = round(r["like_frac"] / max(r["frac_of_roofline"], 1e-9), 2)
+        rows.append(r)
+
+    P, W, V = prompt_len, width, 32000
+    H, G, d = W // 128, max(W // 512, 1), 128
+    pages = (P + BLOCK_SIZE) // BLOCK_SIZE + 1
+    nb = pages * batch
+    kc, vct = rnd(nb, G, BLOCK_SIZE, d), rnd(nb, G, d, BLOCK_SIZE)
+    bt = torch.arange(nb, dtype=torch.int32, device=dev).view(batch, pages)
+    none, cs128 = torch.empty(pages * BLOCK_SIZE, 0, device=dev), rotary_table(128, 1.0e6, pages * BLOCK_SIZE, dev)
+    sink, wq, wk = torch.zeros(H, device=dev), torch.ones(H * d, device=dev), torch.ones(G * d, device=dev)
+    # ---- the latent attention as the runner's object, at the size of the Tativik design's
+    R_, rot, hw, dv = 512, 64, 192, 128
+    cache, cache_t = rnd(nb, BLOCK_SIZE, R_ + rot), rnd(nb, R_, BLOCK_SIZE)
+    cs = rotary_table(rot, 1.0e6, pages * BLOCK_SIZE, dev, exact=True)
+    uk, uv = rnd(H, 128, R_) * R_ ** -0.5, rnd(H, dv, R_) * R_ ** -0.5
+    lat_w = SimpleNamespace(dkv_norm=torch.ones(R_, device=dev), uk_w=uk, uk_t=uk.transpose(1, 2).contiguous(), uv_w=uv, uv_t=None, sink=None,
+                            o_w=None, seg={"q": (0, H * hw), "dkv": (H * hw, R_ + rot)})
+    tat_w = SimpleNamespace(dkv_norm=torch.ones(R_, device=dev), uk_w=uk, uv_t=uv.transpose(1, 2).contiguous(), sink=torch.zeros(H, device=dev),
+                            o_w=None, seg={})
+    host = SimpleNamespace(latent_cache=[(cache, cache_t)], rotary=lambda *a, **k: cs, eps=1e-6, dtype=bf, linear=lambda x, w: x)
+    spec = dict(heads=H, dim=128, rot_dim=rot, vdim=dv, kv_rank=R_, q_rank=0, rot_dims=rot, rot_base=1.0e6, scale=hw ** -0.5)
+    lat = LatentAttention(LatentAttnSpec(window=NO_WINDOW, q_direct=True, sink=False, gate=False, interleaved=True, **spec), lat_w, host, 0, True)
+    tat = LatentAttention(LatentAttnSpec(window=NO_WINDOW, gate=False, **spec), tat_w, host, 0, True)
+    for T, S, tag in ((P, 1, "prefill"), (batch, batch, "decode")):
+        shape = f"{tag} {T} rows x {W}"
+        cu_h = np.arange(0, T + 1, T // S)
+        cu = torch.from_numpy(cu_h.astype(np.int32)).to(dev)
+        pos = (torch.arange(T, device=dev) % (T // S) + (0 if S == 1 else P - 1)).to(torch.int64)
+        seq = (torch.arange(T, device=dev) // (T // S)).to(torch.int32)
+        b_t = bt[:1] if S == 1 else bt
+        wslots = (torch.arange(T, device=dev) if S == 1 else torch.arange(T, device=dev) * pages * BLOCK_SIZE + P - 1).to(torch.int64)
+        # ---- norms: a sub-layer's rows, and a mixture's rows in expert order
+        resid, y, wv, out16 = rnd(T, W, dt=torch.float32), rnd(T, W), rnd(W), torch.empty(T, W, device=dev, dtype=bf)
+        t_l = _time(lambda: ops.add_rms_norm_f32(resid, wv, 1e-6, add=y, out=out16))
+        row("add_layer_norm_f32", shape, _time(lambda: ops.add_layer_norm_f32(resid, wv, 1e-6, add=y, out=out16)), "hbm", T * W * 12,
+            "add_rms_norm_f32", t_l, T * W * 12)
+        y4, inv, w4 = rnd(4 * T, W), torch.randperm(4 * T, device=dev).to(torch.int32), torch.full((4 * T,), 0.25, device=dev)
+        t_c = _time(lambda: ops.moe_combine(y4, inv, w4, T, 4))
+        row("add_layer_norm_f32 (sums 4 expert rows per token)", shape,
+            _time(lambda: ops.add_layer_norm_f32(resid, wv, 1e-6, add=y4, inv=inv, top=4, row_weight=0.25, out=out16)), "hbm", T * W * 18,
+            "moe_combine, then add_rms_norm_f32", t_c + t_l, T * W * 22)
+        F = 2 * W
+        gu, act = rnd(T, 2 * F), torch.empty(T, F, device=dev, dtype=bf)
+        row("gated_act_rows (limited unit)", f"{tag} {T} rows x {F}", _time(lambda: ops.gated_act_rows(gu[:, :F], gu[:, F:], 7.0, out=act)),
+            "hbm", T * F * 6, "silu_and_mul", _time(lambda: ops.silu_and_mul(gu, out=act)), T * F * 6)
+        # ---- softmax attention
+        proj = rnd(T, (H + 2 * G) * d)
+        q, k, v_ = proj[:, : H * d], proj[:, H * d: (H + G) * d], proj[:, (H + G) * d:]
+        row("row_norm_rope_kv_write (temperature, no rotation)", f"{tag} {T} rows, {H}/{G} heads x {d}",
+            _time(lambda: ops.row_norm_rope_kv_write(q, k, v_, wq, wk, none, pos, wslots, kc, vct, H, G, d, d, 1e-6, temp_coef=0.1, temp_every=1024)),
+            "hbm", T * (2 * H * d + 4 * G * d) * 2, "row_norm_rope_kv_write (all rotated)",
+            _time(lambda: ops.row_norm_rope_kv_write(q, k, v_, wq, wk, cs128, pos, wslots, kc, vct, H, G, d, d, 1e-6)),
+            T * (2 * H * d + 4 * G * d) * 2)
+        o, qc = torch.empty(T, H * d, device=dev, dtype=bf), q.contiguous()
+        tiles = torch.from_numpy(ops.query_tiles(cu_h)).to(dev)
+        rep = H // G
+        hb = 4 if rep % 4 == 0 else 3 if rep % 3 == 0 else 2 if rep % 2 == 0 else 1
+        nsb = max(min(16, P // 64, 1024 // max(int(tiles.shape[0]) * G * (rep // hb), 1)), 1)
+        t_t = _time(lambda: ops.softmax_bias_attn(q, kc, vct, b_t, seq, pos, None, None, None, H, d ** -0.5, tiles=tiles,
+                                                  num_splits=nsb if nsb > 1 else 0, sink=sink, softcap=30.0, out=o), 5)
+        nkeys = P * (P + 1) // 2 if S == 1 else T * P
+        if S == 1:
+            ctx = torch.tensor([P], dtype=torch.int32, device=dev)
+            t_s = _time(lambda: ops.paged_attn_prefill_ext(q, kc, vct, b_t, cu, ctx, P, H, G, d, d ** -0.5, sink=sink, softcap=30.0, out=o), 5)
+            t_c = _time(lambda: ops.paged_attn_prefill(qc, kc, vct, b_t, cu, ctx, P, H, G, d, d ** -0.5, out=o), 5)
+            ashape = f"prefill {P} tokens, {H}/{G} heads x {d}"
+            row("paged_attn_prefill_ext (soft cap, sinks)", ashape, t_s, "mfma", 2.0 * nkeys * H * 2 * d, "paged_attn_prefill", t_c,
+                2.0 * nkeys * H * 2 * d)
+            row("softmax_bias_attn, tile form (soft cap, sinks)", ashape, t_t, "mfma", 2.0 * nkeys * H * 2 * d, "paged_attn_prefill", t_c,
+                2.0 * nkeys * H * 2 * d)
+        else:
+            ctxd = torch.full((batch,), P, dtype=torch.int32, device=dev)
+            ws = torch.empty(max(ops.decode_workspace_bytes(batch, H, d, 16), 16), dtype=torch.uint8, device=dev)
+            t_l = _time(lambda: ops.paged_attn_decode(qc, kc, vct, bt, ctxd, H, G, d, d ** -0.5, num_splits=4, workspace=ws, out=o))
+            t_e = _time(lambda: ops.paged_attn_decode(qc, kc, vct, bt, ctxd, H, G, d, d ** -0.5, num_splits=max(min(16, 512 // (T * G)), 1),
+                                                      workspace=None, out=o, sink=sink, softcap=30.0))
+            row("paged_attn_decode (soft cap, sinks)", f"decode {T} rows at context {P}", t_e, "hbm", nkeys * G * 2 * d * 2,
+                "paged_attn_decode", t_l, nkeys * G * 2 * d * 2)
+            row("softmax_bias_attn, tile form (soft cap, sinks)", f"decode {T} rows at context {P}", t_t, "hbm", nkeys * G * 2 * d * 2,
+                "paged_attn_decode", t_l, nkeys * G * 2 * d * 2)
+        # ---- latent attention
+        pl = rnd(T, H * hw + R_ + rot)
+        plan = LatentPlan(cu_h, [P] * S, b_t.cpu().numpy(), dev)
+        ptiles = torch.from_numpy(ops.pair_tiles(cu_h, H)).to(dev)
+        b = StepBatch(torch.zeros(T, dtype=torch.int64, device=dev), pos, wslots, b_t.contiguous(), cu, seq, None, tiles, S == 1,
+                      pair_tiles=lambda heads: ptiles, latent_plan=(lambda: plan) if S == 1 else None)
+        x = pl[:, H * hw:]
+        row("latent_kv_write (norm, neighbours rotated)", f"{tag} {T} rows x {R_ + rot}",
+            _time(lambda: ops.latent_kv_write(x, lat_w.dkv_norm, cs, pos, wslots, cache, R_, rot, 1e-6, cache_t=cache_t, interleaved=True)),
+            "hbm", T * (3 * R_ + 2 * rot) * 2, "latent_kv_write (halves)",
+            _time(lambda: ops.latent_kv_write(x, lat_w.dkv_norm, cs, pos, wslots, cache, R_, rot, 1e-6, cache_t=cache_t)), T * (3 * R_ + 2 * rot) * 2)
+        qs = pl[:, : H * hw]
+        old = lambda: tat._on_latents(qs, None, pos, b.block_tables, seq, b.pair_tiles)        # noqa: E731  (as the Tativik design)
+        t_old = _time(old, 3)
+        if S == 1:
+            n = plan.pages * BLOCK_SIZE
+            t_new = _time(lambda: lat._expanded(qs, None, b, plan), 5)
+            kx, vx = torch.empty(plan.pages, H, BLOCK_SIZE, hw, dtype=bf, device=dev), torch.empty(plan.pages, H, dv, BLOCK_SIZE, dtype=bf, device=dev)
+            flat = cache.view(-1, R_ + rot)
+            t_k = _time(lambda: ops.head_gemm(flat, 0, uk, kx, H * 16 * hw, hw, 16 * hw, n, index=plan.index, copy=rot))
+            t_v = _time(lambda: ops.head_gemm(flat, 0, uv, vx, H * dv * 16, 0, dv * 16, n, index=plan.index, transposed=True))
+            t_a = _time(lambda: ops.paged_attn_prefill_ext(qs, kx, vx, plan.tables, cu, plan.ctx, P, H, H, hw, hw ** -0.5), 5)
+            t_r = _time(lambda: ops.latent_q_rotate(qs, H, hw, 128, cs, pos, interleaved=True))
+            up = torch.cat([uk.reshape(-1, R_), uv.reshape(-1, R_)])
+            c_rows = rnd(n, R_)
+            t_mm = _time(lambda: torch.mm(c_rows, up.t()))
+            lshape = f"prefill {P} tokens, {H} heads x ({d} + {rot}) / {dv}, latent {R_}"
+            row("latent attention, expanded (rotation, two products, attention)", lshape, t_new, "mfma",
+                2.0 * nkeys * H * (hw + dv) + 2.0 * n * R_ * H * (d + dv), "latent attention on the latents (absorbed queries)", t_old,
+                2.0 * nkeys * H * (hw + dv) + 2.0 * n * R_ * H * (d + dv))
+            row("head_gemm (keys and values from latents, into pages)", lshape, t_k + t_v, "mfma", 2.0 * n * R_ * H * (d + dv),
+                "one library product of the same size", t_mm, 2.0 * n * R_ * H * (d + dv))
+            row("paged_attn_prefill_ext (keys of 192, values of 128)", lshape, t_a, "mfma", 2.0 * nkeys * H * (hw + dv), "paged_attn_prefill", t_c,
+                2.0 * nkeys * H * 2 * d)
+            row("latent_q_rotate", f"prefill {P} rows x {H} heads x {rot}", t_r, "hbm", P * H * rot * 4)
+        else:
+            t_new = _time(lambda: lat._on_latents(qs, None, pos, b.block_tables, seq, b.pair_tiles))
+            row("latent attention on the latents (products per head, tiles)", f"decode {T} rows at context {P}, {H} heads, latent {R_} + {rot}", t_new,
+                "hbm", nkeys * (R_ + rot) * 2 + H * R_ * 256 * 2, "as the Tativik design (library products per head)", t_old,
+                nkeys * (R_ + rot) * 2 + H * R_ * 256 * 2)
+            qe = rnd(T, H, R_ + rot) * 0.05
+            ol = torch.empty(H, T, R_, device=dev, dtype=bf)
+            ns = min(16, max(1024 // int(ptiles.shape[0]), 1))
+            t_n = _time(lambda: ops.latent_window_attn_tiles(qe, cache, cache_t, bt, ptiles, pos, None, None, NO_WINDOW, hw ** -0.5, num_splits=ns, out=ol))
+            t_w = _time(lambda: ops.latent_window_attn_tiles(qe, cache, cache_t, bt, ptiles, pos, tat_w.sink, None, 1024, hw ** -0.5, num_splits=16, out=ol))
+            row("latent_window_attn_tiles (no window)", f"decode {T} rows at context {P}, {H} heads", t_n, "hbm", nkeys * (R_ + rot) * 2,
+                "the same with a window of 1024 and a sink (Tativik)", t_w, T * min(P, 1024) * (R_ + rot) * 2)
+    # ---- the mixture beside the Tativik design's: equal weights (two matrices of 3/4 width for three of 1/2)
+    E, top, Fb, Ft = 32, 4, 3 * W // 4, W // 2
+    lw = SimpleNamespace(up_w=rnd(E, Fb, W) * W ** -0.5, down_w=rnd(E, W, Fb) * Fb ** -0.5)
+    ff = TableMoE(MoESpec(E, top, 1, 1, Fb, score="table", gated=False), lw, 0)
+    tables = torch.stack([torch.randperm(E, device=dev, generator=g)[:top] for _ in range(V)]).to(torch.int32).view(1, V, top)
+    lw0 = SimpleNamespace(router_w=rnd(E, W, dt=torch.float32) * W ** -0.5, correction=torch.zeros(E, device=dev),
+                          gate_up_w=rnd(E, 2 * Ft, W) * W ** -0.5, down_w=rnd(E, W, Ft) * Ft ** -0.5)
+    ff0 = MoEFeedForward(MoESpec(E, top, 4, 2, Ft), lw0, None)
+    for T, tag in ((P, "prefill"), (batch, "decode")):
+        h, ids = rnd(T, W), torch.randint(0, V, (T,), device=dev, generator=g)
+        st = SimpleNamespace(routes={(E, top): ops.TableRoutes(tables, ids, E)})
+        t_n, t_l = _time(lambda: ff(h, st), 5), _time(lambda: ff0(h), 5)
+        t_s = _time(lambda: ops.TableRoutes(tables, ids, E))
+        if tag == "prefill":
+            row("mixture named by a table (two expert products)", f"prefill {T} rows, {top} of {E} x {Fb}", t_n, "mfma", 4.0 * T * top * Fb * W,
+                "mixture (route, sort, three-matrix experts, sum)", t_l, 6.0 * T * top * Ft * W)
+        else:
+            touched = min(E, T * top)
+            row("mixture named by a table (two expert products)", f"decode {T} rows, {top} of {E} x {Fb}", t_n, "hbm", touched * 2 * Fb * W * 2,
+                "mixture (route, sort, three-matrix experts, sum)", t_l, touched * 3 * Ft * W * 2)
+        zl = rnd(T, E, dt=torch.float32)
+        row("moe_table_sort (once per step for all layers)", f"{tag} {T} rows, {top} of {E}", t_s, "hbm", T * top * 20,
+            "moe_route + moe_sort (per layer)", _time(lambda: ops.moe_sort(ops.moe_route(zl, lw0.correction, top, 4, 2)[0], E)), T * (E * 4 + top * 20))
+    return rows
+
+
+def compare_bapavik(widths, layers: int, batch: int, prompt_len: int, steps: int, warmup: int) -> dict:
+    """The Bapavik design beside the closest existing model, the sandwich arrangement (Tativik: latent attention and a
+    mixture with as many weights), at equal width and depth, and beside a Llama-shaped decoder whose layers hold as
+    many weights as a token of the Bapavik design uses."""
+    result = {"metric": "bapavik_vs_tativik_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic",
+              "config": {"layers": layers, "batch": batch, "prompt_len": prompt_len, "decode_steps": steps},
+              "models": [], "kernels": {}}
+    for width in widths:
+        t = through_engine(ModelConfig.from_dict(bapavik_config(width, layers)), batch, prompt_len, steps, warmup)
+        z = through_engine(ModelConfig.from_dict(tativik_config(width, layers)), batch, prompt_len, steps, warmup)
+        idle = 28 * 2 * (3 * width // 4) * width * (layers - 1) // layers                  # of the 32 experts, 28 idle per token
+        ll = through_engine(ModelConfig.from_dict(llama_config(width, layers, t["params_per_layer"] - idle)), batch, prompt_len, steps, warmup)
+        result["models"].append({"width": width, "layers": layers, "bapavik": t, "tativik": z, "llama_of_active_size": ll,
+                                 "prefill_ratio": round(t["prefill_tok_s"] / z["prefill_tok_s"], 3),
+                                 "decode_ratio": round(t["decode_tok_s"] / z["decode_tok_s"], 3)})
+        result["kernels"][str(width)] = bapavik_kernel_table(width, prompt_len, batch)
     return result

@@ -92,7 +92,7 @@ class StepBatch:
         self.latent_plan = latent_plan                # () -> the step's LatentPlan, or None (captured decode steps)
         self.row_tiles = row_tiles                    # rows -> ops.RowTiles of the step, or None (captured decode steps)
         # every chunk's length of context after the step (int32, on the device) and the longest chunk: what the
-        # LDS-staged prompt attention walks by; None: not known to this step (captured decode steps)
+        # LDS-staged prompt attention walks by; None: not known to this step
         self.context_lens, self.max_q_len = context_lens, int(max_q_len)
         self.tiles = tiles                            # 16-row query tiles (ops.query_tiles) or None: one wave per row
         self.pair_tiles = pair_tiles                  # heads -> tiles of 16 (row, head) pairs (ops.pair_tiles), or None
@@ -319,8 +319,9 @@ class BlockAttention:
 
 class RowNormAttention:
     """Causal softmax attention over the paged K/V of one layer run: queries and keys normed over their whole
-    rows, a query temperature by position, capped scores, a learned value-less term per head.  Steps that hold a
-    portion of a prompt take the LDS-staged launch where the sizes allow, all others the tile form."""
+    rows, a query temperature by position, capped scores, a learned value-less term per head.  Where the sizes
+    allow, steps that hold a portion of a prompt take the LDS-staged launch and steps of single tokens the Llama
+    path's decode launch; the tile form otherwise."""
 
     def __init__(self, spec, lw, runner, cache_index: int):
         self.s, self.lw, self.r, self.ci = spec, lw, runner, cache_index
@@ -336,6 +337,12 @@ class RowNormAttention:
                 and proj.stride(0) % 8 == 0:
             o = ops.paged_attn_prefill_ext(q, kc, vc, b.block_tables, b.cu_seqlens, b.context_lens, b.max_q_len, s.heads,
                                            s.kv_heads, s.dim, s.scale, sink=lw.sink, softcap=s.softcap)
+        elif not b.long_chunks and b.context_lens is not None and proj.stride(0) % 8 == 0 \
+                and ops.attn_decode_ok(q.dtype, s.heads, s.kv_heads, s.dim, s.vdim):
+            # single tokens alone: a workgroup per (sequence, kv head, part of the context), about two per CU
+            n = min(16, max(512 // (b.num_seqs * s.kv_heads), 1), max(r.max_model_len // 128, 1))
+            o = ops.paged_attn_decode(q, kc, vc, b.block_tables, b.context_lens, s.heads, s.kv_heads, s.dim, s.scale, num_splits=n,
+                                      sink=lw.sink, softcap=s.softcap)
         else:
             o = ops.softmax_bias_attn(q, kc, vc, b.block_tables, b.tok_seq, b.positions, None, None, None, s.heads, s.scale,
                                       tiles=b.tiles, num_splits=r.block_key_splits(b, s), sink=lw.sink, softcap=s.softcap)
@@ -1063,7 +1070,8 @@ class HybridRunner(ModelRunner):
     def _decode_body(self, b: int) -> None:
         batch = StepBatch(self.ids[:b], self.positions[:b], self.slots[:b], self.block_tables[:b],
                           self._dec_cu[:b + 1], self._dec_seq[:b], self.row_extra[:b], self._dec_tiles[:b],
-                          pair_tiles=lambda heads: self._decode_pair_tiles(heads)[: b * (-(-heads // 16))])
+                          pair_tiles=lambda heads: self._decode_pair_tiles(heads)[: b * (-(-heads // 16))],
+                          context_lens=self.ctx[:b])
         resid = self._forward(batch)
         self._logits(resid, out=self.logits_rows[:b])
         self.greedy(self.logits[:b], self.next_ids[:b], ids_out=self.ids[:b])

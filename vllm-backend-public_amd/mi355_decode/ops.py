@@ -160,8 +160,10 @@ def _check_cache(q, k_cache, v_cache, block_tables, num_kv_heads, head_dim):
 def paged_attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                       block_tables: torch.Tensor, context_lens: torch.Tensor, num_heads: int,
                       num_kv_heads: int, head_dim: int, scale: float, num_splits: int = 1,
-                      workspace: torch.Tensor | None = None, out: torch.Tensor | None = None):
-    """q: 2-D view [num_seqs, >= num_heads*head_dim] (e.g. the q part of the qkv rows)."""
+                      workspace: torch.Tensor | None = None, out: torch.Tensor | None = None,
+                      sink: torch.Tensor | None = None, softcap: float = 0.0):
+    """q: 2-D view [num_seqs, >= num_heads*head_dim] (e.g. the q part of the qkv rows).  softcap > 0: scores are
+    softcap * tanh(q.k * scale / softcap); sink (float32 [heads]): one more term exp(sink[h]) in the softmax denominator."""
     dt = _dt16(q, "q")
     B = q.shape[0]
     nb = _check_cache(q, k_cache, v_cache, block_tables, num_kv_heads, head_dim)
@@ -180,11 +182,24 @@ def paged_attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
         if workspace is None:
             workspace = torch.empty(need, dtype=torch.uint8, device=q.device)
         ws_ptr, ws_bytes = workspace.data_ptr(), workspace.numel() * workspace.element_size()
+    if sink is not None or softcap > 0:
+        check(lib.mi355_paged_attn_decode_ext(out.data_ptr(), q.data_ptr(), _rows(q, "q"), k_cache.data_ptr(),
+                                              v_cache.data_ptr(), nb, block_tables.data_ptr(), block_tables.shape[1],
+                                              context_lens.data_ptr(), B, num_heads, num_kv_heads, head_dim, float(scale),
+                                              None if sink is None else _f32(sink, "sink", num_heads), float(softcap),
+                                              num_splits, ws_ptr, ws_bytes, dt, _stream()))
+        return out
     check(lib.mi355_paged_attn_decode(out.data_ptr(), q.data_ptr(), _rows(q, "q"), k_cache.data_ptr(),
                                       v_cache.data_ptr(), nb, block_tables.data_ptr(), block_tables.shape[1],
                                       context_lens.data_ptr(), B, num_heads, num_kv_heads, head_dim,
                                       float(scale), num_splits, ws_ptr, ws_bytes, dt, _stream()))
     return out
+
+
+def attn_decode_ok(dtype: torch.dtype, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int) -> bool:
+    """Whether paged_attn_decode covers these sizes."""
+    return dtype in (torch.bfloat16, torch.float16) and head_dim == v_dim and head_dim in (64, 128) \
+        and num_heads % num_kv_heads == 0 and num_heads // num_kv_heads <= 16
 
 
 STATIC_SCRATCH_BYTES = 16 * 1024 * 1024       # MI355_PAGED_ATTN_DECODE_STATIC_MAX_BYTES
