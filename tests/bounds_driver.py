@@ -351,6 +351,65 @@ def post_norm_generation():
     return out
 
 
+def table_mixture_generation():
+    """A hybrid decoder of the Bapavik design (layer norms, capped attention with sinks, latent attention with
+    expanded keys and on the latents, experts named by tables, a loop): the same schedule as above, in bfloat16
+    and in float32."""
+    from mi355_decode import weights as W
+    from mi355_decode.config import EngineArgs, ModelConfig
+    from mi355_decode.llm import build_engine
+    from mi355_decode.sampling_params import SamplingParams
+    att = {"heads": 8, "kv_heads": 2, "dim": 64, "vdim": 128, "scale": 0.2, "softcap": 9.0, "q_temp": {"coef": 0.4, "every": 30}}
+    odd = {"heads": 3, "kv_heads": 1, "dim": 41, "vdim": 9, "scale": 0.2}
+    lat = {"heads": 3, "dim": 128, "rot_dim": 64, "vdim": 64, "kv_rank": 72, "scale": 0.1, "rot": {"dims": 64, "base": 10000.0}}
+    small = {"heads": 5, "dim": 13, "rot_dim": 6, "vdim": 9, "kv_rank": 22, "scale": 0.3, "rot": {"dims": 6, "base": 100.0}}
+    moe = lambda experts, top, ff: {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}   # noqa: E731
+    cfg = ModelConfig.from_dict({
+        "architecture": "Bapavik", "width": 128, "vocab": 300, "norm": {"eps": 1e-6}, "embedding": {"scale": 10.0},
+        "loop": {"start": 0, "stop": 2, "times": 2},
+        "layers": [{"type": "attention", "mixer": att, "mlp": moe(2, 1, 192)},
+                   {"type": "latent_attention", "mixer": lat, "mlp": {"kind": "dense", "ff": 200, "limit": 2.0}},
+                   {"type": "attention", "mixer": dict(att, dim=128), "mlp": moe(6, 2, 30)},
+                   {"type": "latent_attention", "mixer": small, "mlp": None},
+                   {"type": "attention", "mixer": odd, "mlp": moe(3, 3, 17)},
+                   {"type": "latent_attention", "mixer": dict(small, dim=24, rot_dim=8, vdim=40, kv_rank=48, rot={"dims": 8, "base": 100.0}), "mlp": None}]})
+    state = W.hybrid_synthetic_state(cfg, seed=3)
+    rng = np.random.default_rng(1)
+    out = []
+    for dtype in ("bfloat16", "float32"):
+        bounds.clear()
+        eng = build_engine(EngineArgs(model="tables", dtype=dtype, max_num_seqs=4, max_model_len=256,
+                                      num_gpu_blocks_override=48, gpu_memory_utilization=0.0, max_num_batched_tokens=1 << 20),
+                           state_dict=state, model_config=cfg)
+
+        def run(tag):
+            toks = {r: rng.integers(0, 300, n).tolist() for r, n in (("a", 150), ("b", 67), ("c", 2))}
+            eng.forced_step([(tag + "a", toks["a"][:100], [99]), (tag + "c", toks["c"][:1], [0])])
+            eng.forced_step([(tag + "a", toks["a"][100:102], [1]), (tag + "b", toks["b"][:63], []), (tag + "c", toks["c"][1:], [0])],
+                            [tag + "c"])
+            for i in range(4):
+                eng.forced_step([(tag + "a", toks["a"][102 + i:103 + i], [0]), (tag + "b", toks["b"][63 + i:64 + i], [0])])
+            eng.forced_step([(tag + "a", toks["a"][106:], [])], [tag + "a", tag + "b"])
+            for i, n in enumerate((5, 70, 17)):
+                eng.add_request(f"{tag}g{i}", rng.integers(0, 300, n).tolist(),
+                                SamplingParams(max_tokens=10, temperature=0.0 if i else 0.8, seed=i, ignore_eos=True))
+            n = 0
+            while eng.has_unfinished():
+                n += sum(len(o.new_token_ids) for o in eng.step())
+            return n
+
+        run("warm")
+        n = bounds.sync_allocations(granularity="segment")
+        toks = run("checked")
+        rep = bounds.report()
+        assert rep is None or rep["refused"] == 0, (dtype, rep)
+        out.append(f"{dtype}:{toks} tokens:{n} segments:{rep['unknown_base'] if rep else 0} accesses with an unlisted base")
+        del eng
+        gc.collect()
+        torch.cuda.empty_cache()
+    return out
+
+
 def sampler_rows():
     """The sampling launch on exactly sized logits (no slack behind the last row), every kind of
     row in one call: greedy, whole-vocabulary draw, top-k / top-p cuts, an all-tied row (the list
@@ -392,4 +451,5 @@ if __name__ == "__main__":
     res["block_mixers"] = block_mixer_generation()
     res["parallel_layers"] = parallel_layer_generation()
     res["post_norms"] = post_norm_generation()
+    res["table_mixtures"] = table_mixture_generation()
     print(json.dumps(res))

@@ -46,14 +46,17 @@ __global__ __launch_bounds__(256, 2) void group_gemm_kernel(GroupGemmArgs a) {
   const int li = lane & 15, kk = lane >> 4;
   // workgroups go to the 8 XCDs in turn: XCD i takes the i-th contiguous part of the tiles
   const int ntn = (a.n + BN - 1) / BN;
-  const int total = gridDim.x, xcd = blockIdx.x & 7;
+  // (of the tiles that exist: the grid is sized for the most there can be)
+  int total = gridDim.x;
+  if (a.offsets != nullptr) total = min(total, MI355_LD(int32_t, a.tile_start, a.tile_start + a.groups) * ntn);
+  if (static_cast<int>(blockIdx.x) >= total) return;    // (uniform over the workgroup)
+  const int xcd = blockIdx.x & 7;
   const int work = xcd * (total >> 3) + min(xcd, total & 7) + (blockIdx.x >> 3);
   int mt = work / ntn;
   const int n0 = (work % ntn) * BN;
   int g;
   int64_t lo, hi;
   if (a.offsets != nullptr) {                           // the expert whose tiles hold number mt
-    if (mt >= MI355_LD(int32_t, a.tile_start, a.tile_start + a.groups)) return;      // (uniform over the workgroup)
     int l = 0, h = a.groups;                            // tile_start[l] <= mt < tile_start[h]
     while (h - l > 1) {
       const int mid = (l + h) >> 1;
@@ -86,41 +89,30 @@ __global__ __launch_bounds__(256, 2) void group_gemm_kernel(GroupGemmArgs a) {
 #pragma unroll
   for (int j = 0; j < XP; ++j) {
     const int r = r8 + 32 * j;
-    xp[j] = x_row(m0 + r < hi ? m0 + r : hi - 1) + 8 * s8;
+    xp[j] = x_row(m0 + r < hi ? m0 + r : hi - 1);
     dx[j] = r * kBK + ((s8 ^ ((r >> 1) & 7)) << 3);
   }
 #pragma unroll
   for (int j = 0; j < WP; ++j) {
     const int r = r8 + 32 * j;
-    wp[j] = wg + static_cast<int64_t>(n0 + r < a.n ? n0 + r : a.n - 1) * a.k + 8 * s8;
+    wp[j] = wg + static_cast<int64_t>(n0 + r < a.n ? n0 + r : a.n - 1) * a.k;
     dw[j] = BM * kBK + r * kBK + ((s8 ^ ((r >> 1) & 7)) << 3);
   }
   typedef unsigned int pvec __attribute__((ext_vector_type(4)));
   pvec rx[2][XP], rw[2][WP];
-  auto load = [&](int set, int k0) {
-    if (k0 + kBK <= a.k) {                                // (uniform)
+  // No branch around a load or a store: it would make the compiler drain the loads in flight at its join.  Columns past
+  // k (the last step's, and steps past the last) read the last ones instead, and X's are cleared on the way into LDS.
+  auto load = [&](int set, int t) {
+    const int at = min(t * kBK + 8 * s8, a.k - 8);        // (k a multiple of 8)
 #pragma unroll
-      for (int j = 0; j < XP; ++j) rx[set][j] = MI355_LD(pvec, a.x, xp[j] + k0);
+    for (int j = 0; j < XP; ++j) rx[set][j] = MI355_LD(pvec, a.x, xp[j] + at);
 #pragma unroll
-      for (int j = 0; j < WP; ++j) rw[set][j] = MI355_LD(pvec, a.w, wp[j] + k0);
-      return;
-    }
-    const bool have = k0 + 8 * s8 < a.k;                 // (k a multiple of 8)
-    const int at = have ? k0 : 0;
-#pragma unroll
-    for (int j = 0; j < XP; ++j) {
-      const pvec v = MI355_LD(pvec, a.x, xp[j] - 8 * s8 + (have ? at + 8 * s8 : 0));
-      rx[set][j] = have ? v : pvec{0, 0, 0, 0};
-    }
-#pragma unroll
-    for (int j = 0; j < WP; ++j) {
-      const pvec v = MI355_LD(pvec, a.w, wp[j] - 8 * s8 + (have ? at + 8 * s8 : 0));
-      rw[set][j] = have ? v : pvec{0, 0, 0, 0};
-    }
+    for (int j = 0; j < WP; ++j) rw[set][j] = MI355_LD(pvec, a.w, wp[j] + at);
   };
-  auto store = [&](int set) {                            // (image = set)
+  auto store = [&](int set, int t) {                     // (image = set)
+    const bool have = t * kBK + 8 * s8 < a.k;
 #pragma unroll
-    for (int j = 0; j < XP; ++j) *reinterpret_cast<pvec*>(&lds[set][dx[j]]) = rx[set][j];
+    for (int j = 0; j < XP; ++j) *reinterpret_cast<pvec*>(&lds[set][dx[j]]) = have ? rx[set][j] : pvec{0, 0, 0, 0};
 #pragma unroll
     for (int j = 0; j < WP; ++j) *reinterpret_cast<pvec*>(&lds[set][dw[j]]) = rw[set][j];
   };
@@ -133,12 +125,12 @@ __global__ __launch_bounds__(256, 2) void group_gemm_kernel(GroupGemmArgs a) {
   const int sw = (li >> 1) & 7;                          // (16-row blocks: the swizzle depends on the row in the block alone)
   const int steps = (a.k + kBK - 1) / kBK;
   load(0, 0);
-  if (steps > 1) load(1, kBK);
-  store(0);
+  load(1, 1);
+  store(0, 0);
   __syncthreads();
   // step t computes image t % 2, sends for step t + 2 and stores step t + 1 into the other image
   auto step = [&](int t, int set) {
-    if (t + 2 < steps) load(set, (t + 2) * kBK);
+    load(set, t + 2);
     __builtin_amdgcn_s_setprio(1);
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
@@ -154,14 +146,12 @@ __global__ __launch_bounds__(256, 2) void group_gemm_kernel(GroupGemmArgs a) {
         for (int j = 0; j < TN; ++j) acc[i][j] = TRANS ? T::mfma(xf[i], wf[j], acc[i][j]) : T::mfma(wf[j], xf[i], acc[i][j]);
     }
     __builtin_amdgcn_s_setprio(0);
-    if (t + 1 < steps) {
-      store(set ^ 1);
-      __syncthreads();
-    }
+    store(set ^ 1, t + 1);
+    __syncthreads();
   };
-  for (int t = 0; t < steps; t += 2) {
+  for (int t = 0; t < steps; t += 2) {                   // (an odd last step is followed by one of cleared X)
     step(t, 0);
-    if (t + 1 < steps) step(t + 1, 1);
+    step(t + 1, 1);
   }
 #pragma unroll
   for (int i = 0; i < TM; ++i) {
