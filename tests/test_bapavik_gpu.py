@@ -471,7 +471,8 @@ def test_latent_attention_in_float32(H, d, r, dv, rank, base):
 
 
 @pytest.mark.parametrize("H,d,r,dv,rank,base", [(3, 16, 8, 24, 32, 500.0), (8, 64, 16, 48, 64, 1e4), (5, 24, 8, 40, 272, 1e4), (7, 13, 6, 9, 22, 77.0),
-                                                (17, 32, 32, 16, 112, 1e5), (3, 20, 4, 12, 48, 100.0)])
+                                                (17, 32, 32, 16, 112, 1e5), (3, 20, 4, 12, 48, 100.0), (17, 64, 64, 64, 512, 1e4), (5, 24, 8, 40, 192, 1e4),
+                                                (2, 16, 8, 24, 128, 1e3), (33, 16, 64, 8, 256, 1e4), (3, 16, 128, 16, 512, 1e4)])
 def test_latent_attention_on_the_latents_in_bfloat16(H, d, r, dv, rank, base):
     full, st, h = _latent_case(H, d, r, dv, rank, base, 90)
     want = _latent_ref(full, st, h)

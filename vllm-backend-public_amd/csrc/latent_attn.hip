@@ -386,34 +386,219 @@ __global__ __launch_bounds__(256) void latent_window_attn_mfma_kernel(
   }
 }
 
-// merges the key splits of latent_window_attn_mfma_kernel: the sink joins the denominator here
+// The same tile by a workgroup of four waves (rank a multiple of 64): keys go 64 at a time, wave w scores keys
+// 16 w .. 16 w + 15 of them, the weights pass through LDS, and wave w sums up the w-th quarter of the latent's
+// channels over all 64 -- a quarter of the accumulators per wave, so that the next keys' loads fit in registers
+// beside them: the channel-major latent of a group of keys is sent for ahead of its scores, the token-major one of
+// the next group right behind the scores.  The query's fragments stay in LDS, in fragment order.
+// DS: 32-channel fragments of a query the buffers are sized for; CW: 16-channel blocks per wave; EXACT: the model has
+// just these (all loads at constant offsets: the largest size fits the registers only so).
+template <typename T, int DS, int CW, bool EXACT>
+__global__ __launch_bounds__(256, 2) void latent_attn_wide_kernel(
+    uint16_t* __restrict__ out, int64_t out_stride, int64_t out_head_stride, const uint16_t* __restrict__ qe,
+    const uint16_t* __restrict__ cache, const uint16_t* __restrict__ cache_t, const int32_t* __restrict__ block_tables,
+    int max_blocks, const int32_t* __restrict__ tiles, int num_tiles, const int64_t* __restrict__ positions,
+    const float* __restrict__ sink, const uint16_t* __restrict__ gate, int64_t gate_stride, int H, int rank, int rot,
+    int window, float scale2, int nz, float* __restrict__ part_acc, float* __restrict__ part_ml, int64_t total_pairs) {
+  constexpr int PK = 64 + 8;                             // weights of a query, padded to spread the banks
+  __shared__ __attribute__((aligned(16))) uint16_t lds_q[DS * 64 * 8];
+  __shared__ __attribute__((aligned(16))) uint16_t lds_p[16 * PK];
+  __shared__ float lds_m[4][16];
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int li = lane & 15, kk = lane >> 4;
+  // XCD i takes the i-th contiguous part of the (split, tile) pairs: a token's tiles read their keys through one L2
+  const int total = gridDim.x, xcd = blockIdx.x & 7;
+  const int work = xcd * (total >> 3) + min(xcd, total & 7) + (blockIdx.x >> 3);
+  const int tile = work % num_tiles, z = work / num_tiles;
+  const int seq = MI355_LD(int32_t, tiles, tiles + 3 * tile);
+  const int64_t first = MI355_LD(int32_t, tiles, tiles + 3 * tile + 1);
+  const int count = MI355_LD(int32_t, tiles, tiles + 3 * tile + 2);
+  const int dq = EXACT ? 32 * DS : rank + rot, ds = EXACT ? DS : (dq + 31) >> 5, cw = EXACT ? CW : rank >> 6;   // cw: blocks per wave
+  const int32_t* bt = block_tables + static_cast<int64_t>(seq) * max_blocks;
+  const int64_t p_first = MI355_LD(int64_t, positions, positions + first / H);
+  const int64_t p_last = MI355_LD(int64_t, positions, positions + (first + count - 1) / H);
+  const bool valid = li < count;
+  const int64_t my_pair = first + (valid ? li : count - 1);
+  const int64_t my_p = MI355_LD(int64_t, positions, positions + my_pair / H);
+  for (int s = wave; s < ds; s += 4) {
+    uint4 v = make_uint4(0, 0, 0, 0);
+    if (valid && 32 * s + 8 * kk + 8 <= dq) v = MI355_LD(uint4, qe, qe + my_pair * dq + 32 * s + 8 * kk);
+    *reinterpret_cast<uint4*>(&lds_q[(s * 64 + lane) * 8]) = v;
+  }
+  f32x4 acc[CW];
+#pragma unroll
+  for (int c = 0; c < CW; ++c) acc[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m = -1.0e30f, l = 0.f;                           // the query's reference (base 2), this lane's share of its sum
+  int64_t lo = p_first - window + 1;
+  if (lo < 0) lo = 0;
+  const int64_t last_blk = p_last / kPageL;
+  const int64_t g0 = (lo >> 6) + z, g_end = p_last >> 6;   // groups of 64 keys: every nz-th
+  // Loads are never inside a branch: columns past dq and keys past the last read valid memory of the same row / the
+  // last page; queries hold zeros there, scores are masked and the latent's columns cleared.
+  auto page_of = [&](int64_t blk) {
+    return static_cast<int64_t>(MI355_LD(int32_t, block_tables, bt + (blk < last_blk ? blk : last_blk)));
+  };
+  uint4 kf[DS];
+  auto load_k = [&](int64_t page) {
+    const uint16_t* kr = cache + (page * kPageL + li) * dq;
+#pragma unroll
+    for (int s = 0; s < DS; ++s) {
+      const int c = 32 * s + 8 * kk;
+      kf[s] = MI355_LD(uint4, cache, kr + (EXACT || c + 8 <= dq ? c : 0));
+    }
+  };
+  int64_t kpage = page_of(4 * g0 + wave), vpage[2] = {page_of(4 * g0 + (kk >> 1)), page_of(4 * g0 + 2 + (kk >> 1))};
+  load_k(kpage);
+  __syncthreads();
+  for (int64_t g = g0; g <= g_end; g += nz) {
+    const int64_t base = g << 6;
+    uint4 vf[2][CW];
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      const uint16_t* vr = cache_t + (vpage[h] * rank + wave * 16 * cw + li) * kPageL + 8 * (kk & 1);
+#pragma unroll
+      for (int c = 0; c < CW; ++c) vf[h][c] = MI355_LD(uint4, cache_t, vr + (EXACT || c < cw ? 16 * c : 0) * kPageL);
+    }
+    const int64_t nb = 4 * (g + nz);
+    kpage = page_of(nb + wave);
+    f32x4 sacc = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < DS; ++s)
+      if (s < ds) sacc = T::mfma(kf[s], *reinterpret_cast<const uint4*>(&lds_q[(s * 64 + lane) * 8]), sacc);
+    load_k(kpage);
+    vpage[0] = page_of(nb + (kk >> 1));
+    vpage[1] = page_of(nb + 2 + (kk >> 1));
+    float sc[4], tmax = -1.0e30f;
+    bool vis[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int64_t key = base + 16 * wave + 4 * kk + r;
+      sc[r] = sacc[r] * scale2;
+      vis[r] = valid && key <= my_p && my_p - key < window;
+      if (vis[r]) tmax = fmaxf(tmax, sc[r]);
+    }
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
+    if (kk == 0) lds_m[wave][li] = tmax;
+    __syncthreads();
+    const float mn = fmaxf(fmaxf(fmaxf(lds_m[0][li], lds_m[1][li]), fmaxf(lds_m[2][li], lds_m[3][li])), m);
+    const float corr = __builtin_amdgcn_exp2f(m - mn);
+    m = mn;
+    l *= corr;
+    float w[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      w[r] = vis[r] ? __builtin_amdgcn_exp2f(sc[r] - mn) : 0.f;
+      l += w[r];
+    }
+    *reinterpret_cast<uint2*>(&lds_p[li * PK + 16 * wave + 4 * kk]) = make_uint2(T::pack2(w[0], w[1]), T::pack2(w[2], w[3]));
+    __syncthreads();
+    if (__any(corr != 1.0f)) {                           // the accumulators hold queries 4 kk + r
+      float cr[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) cr[r] = __shfl(corr, 4 * kk + r, 64);
+#pragma unroll
+      for (int c = 0; c < CW; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) acc[c][r] *= cr[r];
+    }
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      const uint4 pf = *reinterpret_cast<const uint4*>(&lds_p[li * PK + 32 * h + 8 * kk]);
+      if (base + 63 > p_last) {                          // (uniform) keys past the newest may hold anything: 0 * NaN is NaN
+        const int64_t k0 = base + 32 * h + 8 * kk;
+        uint32_t msk[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          msk[j] = (k0 + 2 * j <= p_last ? 0x0000FFFFu : 0u) | (k0 + 2 * j + 1 <= p_last ? 0xFFFF0000u : 0u);
+#pragma unroll
+        for (int c = 0; c < CW; ++c)
+          vf[h][c] = make_uint4(vf[h][c].x & msk[0], vf[h][c].y & msk[1], vf[h][c].z & msk[2], vf[h][c].w & msk[3]);
+      }
+#pragma unroll
+      for (int c = 0; c < CW; ++c)
+        if (c < cw) acc[c] = T::mfma(pf, vf[h][c], acc[c]);
+    }
+  }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  __syncthreads();                                       // (lds_m may still be read)
+  if (kk == 0) lds_m[wave][li] = l;
+  __syncthreads();
+  l = (lds_m[0][li] + lds_m[1][li]) + (lds_m[2][li] + lds_m[3][li]);
+  if (part_acc != nullptr) {
+    if (wave == 0 && valid && kk == 0) {
+      float* ml = part_ml + (z * total_pairs + first + li) * 2;
+      MI355_ST(float, part_ml, ml, m);
+      MI355_ST(float, part_ml, ml + 1, l);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int qi = 4 * kk + r;
+      if (qi >= count) continue;
+      float* pa = part_acc + (z * total_pairs + first + qi) * rank + wave * 16 * cw + li;
+#pragma unroll
+      for (int c = 0; c < CW; ++c)
+        if (c < cw) MI355_ST(float, part_acc, pa + 16 * c, acc[c][r]);
+    }
+    return;
+  }
+  const int my_h = static_cast<int>(my_pair % H);
+  float f = 1.0f / l;
+  if (sink != nullptr) {
+    const float s2 = MI355_LD(float, sink, sink + my_h) * 1.4426950408889634f, mn = fmaxf(m, s2), cm = __builtin_amdgcn_exp2f(m - mn);
+    f = cm / (l * cm + __builtin_amdgcn_exp2f(s2 - mn));
+  }
+  if (gate != nullptr) f /= 1.0f + expf(-T::to_f(MI355_LD(uint16_t, gate, gate + my_pair / H * gate_stride + my_h)));
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int qi = 4 * kk + r;
+    const float fr = __shfl(f, qi, 64);
+    if (qi >= count) continue;
+    const int64_t pair = first + qi;
+    uint16_t* po = out + (pair / H) * out_stride + (pair % H) * out_head_stride + wave * 16 * cw + li;
+#pragma unroll
+    for (int c = 0; c < CW; ++c)
+      if (c < cw) MI355_ST(uint16_t, out, po + 16 * c, T::from_f(acc[c][r] * fr));
+  }
+}
+
+// merges the key splits of the kernels above: the sink joins the denominator here
 template <typename T>
 __global__ __launch_bounds__(256) void latent_attn_reduce_kernel(uint16_t* __restrict__ out, int64_t out_stride,
                                                                  int64_t out_head_stride, const float* __restrict__ part_acc,
                                                                  const float* __restrict__ part_ml,
                                                                  const float* __restrict__ sink,
                                                                  const uint16_t* __restrict__ gate, int64_t gate_stride,
-                                                                 int64_t total_pairs, int H, int rank, int splits) {
-  const int64_t total = total_pairs * rank;
+                                                                 int64_t total_pairs, int H, int rank, int splits, int vec) {
+  const int quads = rank >> 2;                           // four channels per thread (rank is a multiple of 16)
+  const int64_t total = total_pairs * quads;
   for (int64_t i = blockIdx.x * static_cast<int64_t>(blockDim.x) + threadIdx.x; i < total;
        i += static_cast<int64_t>(gridDim.x) * blockDim.x) {
-    const int64_t pair = i / rank;
-    const int c = static_cast<int>(i % rank);
+    const int64_t pair = i / quads;
+    const int c = static_cast<int>(i % quads) * 4;
     const int64_t row = pair / H;
     const int h = static_cast<int>(pair % H);
     const float s2 = sink != nullptr ? MI355_LD(float, sink, sink + h) * kLog2e : -1.0e30f;
     float M = s2;
     for (int z = 0; z < splits; ++z) M = fmaxf(M, MI355_LD(float, part_ml, part_ml + (z * total_pairs + pair) * 2));
-    float den = sink != nullptr ? __builtin_amdgcn_exp2f(s2 - M) : 0.f, num = 0.f;
+    float den = sink != nullptr ? __builtin_amdgcn_exp2f(s2 - M) : 0.f;
+    float num[4] = {0.f, 0.f, 0.f, 0.f};
     for (int z = 0; z < splits; ++z) {
-      const float* ml = part_ml + (z * total_pairs + pair) * 2;
-      const float e = __builtin_amdgcn_exp2f(MI355_LD(float, part_ml, ml) - M);
-      den += MI355_LD(float, part_ml, ml + 1) * e;
-      num += MI355_LD(float, part_acc, part_acc + (z * total_pairs + pair) * rank + c) * e;
+      const float2 ml = MI355_LD(float2, part_ml, part_ml + (z * total_pairs + pair) * 2);
+      const float4 a = MI355_LD(float4, part_acc, part_acc + (z * total_pairs + pair) * rank + c);
+      const float e = __builtin_amdgcn_exp2f(ml.x - M);
+      den += ml.y * e;
+      num[0] += a.x * e, num[1] += a.y * e, num[2] += a.z * e, num[3] += a.w * e;
     }
-    float v = num / den;
-    if (gate != nullptr) v /= 1.0f + expf(-T::to_f(MI355_LD(uint16_t, gate, gate + row * gate_stride + h)));
-    MI355_ST(uint16_t, out, out + row * out_stride + h * out_head_stride + c, T::from_f(v));
+    float f = 1.0f / den;
+    if (gate != nullptr) f /= 1.0f + expf(-T::to_f(MI355_LD(uint16_t, gate, gate + row * gate_stride + h)));
+    uint16_t* po = out + row * out_stride + h * out_head_stride + c;
+    if (vec) {
+      MI355_ST(uint2, out, po, make_uint2(T::pack2(num[0] * f, num[1] * f), T::pack2(num[2] * f, num[3] * f)));
+    } else {
+      for (int j = 0; j < 4; ++j) MI355_ST(uint16_t, out, po + j, T::from_f(num[j] * f));
+    }
   }
 }
 
@@ -558,6 +743,7 @@ extern "C" int32_t mi355_latent_window_attn_tiles(void* out, int64_t out_stride,
                 rank, rank + rot);
   MI355_REQUIRE(num_splits >= 1 && num_splits <= 64 && (num_splits == 1 || partial != nullptr), MI355_ERR_INVALID,
                 "latent_window_attn_tiles: %d key splits", num_splits);
+  MI355_REQUIRE(partial == nullptr || aligned16(partial), MI355_ERR_INVALID, "latent_window_attn_tiles: partial misaligned");
   if (num_tokens == 0 || num_tiles == 0) return MI355_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
   const bool split = num_splits > 1;
@@ -576,21 +762,36 @@ extern "C" int32_t mi355_latent_window_attn_tiles(void* out, int64_t out_stride,
                      static_cast<const uint16_t*>(cache), static_cast<const uint16_t*>(cache_t), block_tables,        \
                      max_blocks, tiles, num_tiles, positions, sink, static_cast<const uint16_t*>(gate), gate_stride,  \
                      num_heads, rank, rot, window, scale2, part_acc, part_ml, pairs)
+#define MI355_LWIDE(TT, DS, CW, EX)                                                                                      \
+  hipLaunchKernelGGL((latent_attn_wide_kernel<TT, DS, CW, EX>),                                                           \
+                     dim3(static_cast<unsigned>(num_tiles) * static_cast<unsigned>(num_splits)), dim3(256), 0, s,     \
+                     static_cast<uint16_t*>(out), out_stride, out_head_stride, static_cast<const uint16_t*>(q_packed), \
+                     static_cast<const uint16_t*>(cache), static_cast<const uint16_t*>(cache_t), block_tables,        \
+                     max_blocks, tiles, num_tiles, positions, sink, static_cast<const uint16_t*>(gate), gate_stride,  \
+                     num_heads, rank, rot, window, scale2, num_splits, part_acc, part_ml, pairs)
 #define MI355_LMFMA_SIZES(TT)                                                                                         \
   do {                                                                                                                \
+    if (rank == 64 && dq <= 128) MI355_LWIDE(TT, 4, 1, false);                                                              \
+    else if (rank == 128 && dq <= 256) MI355_LWIDE(TT, 8, 2, false);                                                        \
+    else if (rank % 64 == 0 && rank <= 256 && dq <= 384) MI355_LWIDE(TT, 12, 4, false);                                     \
+    else if (rank == 512 && dq == 576) MI355_LWIDE(TT, 18, 8, true);                                                                \
+    else                                                                                                              \
     if (rank <= 64 && dq <= 128) MI355_LMFMA(TT, 4, 4);                                                               \
     else if (rank <= 128 && dq <= 256) MI355_LMFMA(TT, 8, 8);                                                         \
     else if (rank <= 256 && dq <= 384) MI355_LMFMA(TT, 12, 16);                                                       \
     else MI355_LMFMA(TT, 20, 32);                                                                                     \
     if (split) {                                                                                                      \
-      const int64_t blocks = (pairs * rank + 255) / 256;                                                              \
+      const int64_t blocks = (pairs * (rank / 4) + 255) / 256;                                                        \
+      const int vec = out_stride % 4 == 0 && out_head_stride % 4 == 0 && reinterpret_cast<uintptr_t>(out) % 8 == 0;   \
       hipLaunchKernelGGL((latent_attn_reduce_kernel<TT>), dim3(static_cast<unsigned>(blocks > 4096 ? 4096 : blocks)), \
                          dim3(256), 0, s, static_cast<uint16_t*>(out), out_stride, out_head_stride, part_acc, part_ml, \
-                         sink, static_cast<const uint16_t*>(gate), gate_stride, pairs, num_heads, rank, num_splits);  \
+                         sink, static_cast<const uint16_t*>(gate), gate_stride, pairs, num_heads, rank, num_splits,   \
+                         vec);                                                                                        \
     }                                                                                                                 \
   } while (0)
   if (dtype == MI355_BF16) MI355_LMFMA_SIZES(BF16); else MI355_LMFMA_SIZES(F16);
 #undef MI355_LMFMA_SIZES
+#undef MI355_LWIDE
 #undef MI355_LMFMA
   return check_launch("latent_window_attn_tiles");
 }

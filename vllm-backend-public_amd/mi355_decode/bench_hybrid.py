@@ -1060,9 +1060,9 @@ def bapavik_kernel_table(width: int, prompt_len: int, batch: int) -> list:
                 nkeys * (R_ + rot) * 2 + H * R_ * 256 * 2)
             qe = rnd(T, H, R_ + rot) * 0.05
             ol = torch.empty(H, T, R_, device=dev, dtype=bf)
-            ns = min(16, max(1024 // int(ptiles.shape[0]), 1))
+            ns = min(16, max(ops.latent_tile_workgroups(R_, rot) // int(ptiles.shape[0]), 1))
             t_n = _time(lambda: ops.latent_window_attn_tiles(qe, cache, cache_t, bt, ptiles, pos, None, None, NO_WINDOW, hw ** -0.5, num_splits=ns, out=ol))
-            t_w = _time(lambda: ops.latent_window_attn_tiles(qe, cache, cache_t, bt, ptiles, pos, tat_w.sink, None, 1024, hw ** -0.5, num_splits=16, out=ol))
+            t_w = _time(lambda: ops.latent_window_attn_tiles(qe, cache, cache_t, bt, ptiles, pos, tat_w.sink, None, 1024, hw ** -0.5, num_splits=ns, out=ol))
             row("latent_window_attn_tiles (no window)", f"decode {T} rows at context {P}, {H} heads", t_n, "hbm", nkeys * (R_ + rot) * 2,
                 "the same with a window of 1024 and a sink (Tativik)", t_w, T * min(P, 1024) * (R_ + rot) * 2)
     # ---- the mixture beside the Tativik design's: equal weights (two matrices of 3/4 width for three of 1/2)

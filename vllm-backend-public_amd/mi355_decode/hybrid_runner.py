@@ -275,7 +275,7 @@ class LatentAttention:
             # the matrix cores: tiles of 16 (row, head) pairs; few tiles (decoded tokens, short prompts) spread
             # their windows' keys over several workgroups
             tiles = pair_tiles(H)
-            n = min(16, max(s.window // 64, 1), max(1024 // max(int(tiles.shape[0]), 1), 1))
+            n = min(16, max(s.window // 64, 1), max(ops.latent_tile_workgroups(R, s.rot_dim) // max(int(tiles.shape[0]), 1), 1))
         if matrix_cores and self.head_gemm:
             qe = torch.empty(T, H, dq, dtype=q.dtype, device=q.device)
             ops.head_gemm(q, hw, lw.uk_t, qe, 16 * H * dq, H * dq, dq, T)

@@ -1441,6 +1441,14 @@ def latent_tiles_ok(dtype: torch.dtype, rank: int, rot: int) -> bool:
         and rank + rot <= 640
 
 
+def latent_tile_workgroups(rank: int, rot: int) -> int:
+    """About how many workgroups fill the chip: four waves a tile at the ranks of the wide form, one at the others
+    (measured at rank 512 + 64, context 2048: 32 tiles 55 / 37 / 35 / 41 us with 2 / 4 / 8 / 16 key splits, 64 tiles
+    55 / 38 / 43 / 56)."""
+    wide = rank in (64, 128) and rot <= rank or rank in (192, 256) and rank + rot <= 384 or (rank, rot) == (512, 64)
+    return 256 if wide else 1024
+
+
 def latent_q_pack(q_latent: torch.Tensor | None, q: torch.Tensor, q_head_width: int, q_rot_offset: int, rot: int,
                   cos_sin: torch.Tensor, positions: torch.Tensor, interleaved: bool = False, out: torch.Tensor | None = None):
     """[tokens, heads, rank + rot] = q_latent [heads, tokens, rank] | the rotated `rot` columns of q at
